@@ -5,4 +5,5 @@ from .novosun import NovosunConfig
 from .ditazen import DitazenConfig
 from .noresun import NoresunConfig
 from .zovozen import ZovozenConfig
+from .guduzen import GuduzenConfig
 from .presets import preset, preset_names

@@ -63,8 +63,9 @@ __device__ __forceinline__ float block_sum(float v, float* red) {
 }
 
 // The law of a gated activation act(gate, up), the epilogue of a product over [gate; up]:
-//   limit <= 0:  silu(g) u
+//   limit 0:     silu(g) u
 //   limit > 0:   g' sigmoid(slope g') (u' + shift) with g' = min(g, limit), u' = clamp(u, -limit, limit)
+//   limit < 0:   gelu(g) u, the gelu's tanh form
 // A struct of zeros is the first law.
 struct GateLaw { float limit, slope, shift; };
 
@@ -74,6 +75,8 @@ __device__ __forceinline__ float gated_activation(float g, float u, const GateLa
         u = fminf(fmaxf(u, -law.limit), law.limit);
         return g / (1.0f + expf(-law.slope * g)) * (u + law.shift);
     }
+    if (law.limit < 0.f)      // (0.5 (1 + tanh z) = 1 / (1 + exp(-2 z)))
+        return g / (1.0f + expf(-1.5957691216057308f * (g + 0.044715f * g * g * g))) * u;
     return g / (1.0f + expf(-g)) * u;
 }
 

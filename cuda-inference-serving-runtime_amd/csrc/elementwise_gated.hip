@@ -169,15 +169,13 @@ extern "C" int cisr_post_norm_add(float* x, const float* a, const float* wa, con
 // gu[r] = [gate (inter) | up (inter)]; arithmetic in float.
 template <typename T>
 __global__ void glu_clamped_kernel(const T* __restrict__ gu, T* __restrict__ act, int inter, size_t n,
-                                   float limit, float slope, float shift) {
+                                   GateLaw law) {
     const size_t i = (size_t)blockIdx.x * 256 + threadIdx.x;
     if (i >= n) return;
     const size_t row = i / inter;
     const int col = (int)(i % inter);
     const T* base = gu + row * (size_t)(2 * inter);
-    const float g = fminf(load_f32(base + col), limit);
-    const float u = fminf(fmaxf(load_f32(base + inter + col), -limit), limit);
-    store_f32(act + i, g / (1.0f + expf(-slope * g)) * (u + shift));
+    store_f32(act + i, gated_activation(load_f32(base + col), load_f32(base + inter + col), law));
 }
 
 // the same for bf16, eight elements a thread with 16-byte accesses (inter % 8 == 0, aligned pointers)
@@ -203,15 +201,15 @@ extern "C" int cisr_glu_clamped(const void* gu, void* act, int rows, int inter, 
                                 int dtype, hipStream_t stream) {
     const size_t n = (size_t)rows * inter;
     if (n == 0) return 0;
-    if (dtype == DT_BF16 && limit > 0.f && inter % 8 == 0 && ((uintptr_t)gu) % 16 == 0 && ((uintptr_t)act) % 16 == 0) {
+    if (dtype == DT_BF16 && inter % 8 == 0 && ((uintptr_t)gu) % 16 == 0 && ((uintptr_t)act) % 16 == 0) {
         const size_t n8 = n / 8;
         glu_clamped_bf16x8_kernel<<<(unsigned)((n8 + 255) / 256), 256, 0, stream>>>((const bf16_t*)gu, (bf16_t*)act, inter / 8, n8,
                                                                                   GateLaw{limit, slope, shift});
         return CISR_LAUNCH_CHECK();
     }
     const unsigned blocks = (unsigned)((n + 255) / 256);
-    if (dtype == DT_F32) glu_clamped_kernel<float><<<blocks, 256, 0, stream>>>((const float*)gu, (float*)act, inter, n, limit, slope, shift);
-    else glu_clamped_kernel<bf16_t><<<blocks, 256, 0, stream>>>((const bf16_t*)gu, (bf16_t*)act, inter, n, limit, slope, shift);
+    if (dtype == DT_F32) glu_clamped_kernel<float><<<blocks, 256, 0, stream>>>((const float*)gu, (float*)act, inter, n, GateLaw{limit, slope, shift});
+    else glu_clamped_kernel<bf16_t><<<blocks, 256, 0, stream>>>((const bf16_t*)gu, (bf16_t*)act, inter, n, GateLaw{limit, slope, shift});
     return CISR_LAUNCH_CHECK();
 }
 
@@ -220,32 +218,35 @@ extern "C" int cisr_glu_clamped(const void* gu, void* act, int rows, int inter, 
 // k: kv_heads x dim | v: kv_heads x vdim | ...].  Queries go to q_out [T, heads, pad] (coordinates dim..pad-1 zero),
 // keys to kcache [pages, kv_heads, page_size, pad] (likewise), values transposed to vcache [pages, kv_heads, pad,
 // page_size] (coordinates vdim..pad-1 zero): heads of `pad` coordinates are what the attention kernels read.
-// wq / wk null: that side is not normed.
-template <typename T>
+// wq / wk null: that side is not normed, or with `plain` normed without a weight.  The rows may be float where the pages are
+// bf16 (TI, T); `bias` (float, over the q, k and v columns, or null) is added before everything else.  has_kv 0: the rows
+// hold queries only (a layer that reads the keys of another).
+template <typename TI, typename T>
 __global__ void __launch_bounds__(256)
-qk_norm_scatter_kernel(const T* __restrict__ qkv, int ld, const float* __restrict__ wq, const float* __restrict__ wk,
+qk_norm_scatter_kernel(const TI* __restrict__ qkv, int ld, const float* __restrict__ bias, const float* __restrict__ wq, const float* __restrict__ wk,
                        T* __restrict__ q_out, T* __restrict__ kcache, T* __restrict__ vcache,
                        const int* __restrict__ slots, int heads, int kv_heads, int dim, int vdim, int pad,
-                       int page_size, float eps) {
+                       int page_size, float eps, int plain, int has_kv) {
     const int row = blockIdx.x, wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
-    const T* src = qkv + (size_t)row * ld;
+    const TI* src = qkv + (size_t)row * ld;
     const int slot = slots ? slots[row] : -1;
-    const int items = heads + 2 * kv_heads;
+    const int items = heads + (has_kv ? 2 * kv_heads : 0);
     for (int item = blockIdx.y * 4 + wave; item < items; item += 4 * gridDim.y) {
         if (item < heads + kv_heads) {
             const bool is_q = item < heads;
             const int head = is_q ? item : item - heads;
             if (!is_q && slot < 0) continue;
-            const T* v = src + (size_t)item * dim;         // (queries and keys have the same size: one run of heads)
+            const TI* v = src + (size_t)item * dim;        // (queries and keys have the same size: one run of heads)
+            const float* b = bias ? bias + (size_t)item * dim : nullptr;
             const float* w = is_q ? wq : wk;
             float vals[4], ss = 0.f;
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
                 const int d = lane + WAVE * i;
-                vals[i] = d < dim ? load_f32(v + d) : 0.f;
+                vals[i] = d < dim ? load_f32(v + d) + (b ? b[d] : 0.f) : 0.f;
                 ss += vals[i] * vals[i];
             }
-            const float scale = w ? 1.0f / sqrtf(wave_sum(ss) / (float)dim + eps) : 1.0f;
+            const float scale = w || plain ? 1.0f / sqrtf(wave_sum(ss) / (float)dim + eps) : 1.0f;
             T* dst = is_q ? q_out + ((size_t)row * heads + head) * pad
                           : kcache + (((size_t)(slot / page_size) * kv_heads + head) * page_size + slot % page_size) * pad;
 #pragma unroll
@@ -256,27 +257,31 @@ qk_norm_scatter_kernel(const T* __restrict__ qkv, int ld, const float* __restric
         } else {
             if (slot < 0) continue;
             const int head = item - heads - kv_heads;
-            const T* v = src + (size_t)(heads + kv_heads) * dim + (size_t)head * vdim;
+            const size_t at = (size_t)(heads + kv_heads) * dim + (size_t)head * vdim;
+            const TI* v = src + at;
+            const float* b = bias ? bias + at : nullptr;
             T* dst = vcache + ((size_t)(slot / page_size) * kv_heads + head) * pad * page_size + slot % page_size;
-            for (int d = lane; d < pad; d += WAVE) store_f32(dst + (size_t)d * page_size, d < vdim ? load_f32(v + d) : 0.f);
+            for (int d = lane; d < pad; d += WAVE) store_f32(dst + (size_t)d * page_size, d < vdim ? load_f32(v + d) + (b ? b[d] : 0.f) : 0.f);
         }
     }
 }
 
-extern "C" int cisr_qk_norm_scatter(const void* qkv, int ld, const float* wq, const float* wk, void* q_out, void* kcache,
-                                    void* vcache, const int* slots, int rows, int heads, int kv_heads, int dim, int vdim,
-                                    int pad, int page_size, float eps, int dtype, hipStream_t stream) {
+// in_dtype / dtype: the rows' and the pages' storage (float rows may go to bf16 pages)
+extern "C" int cisr_qk_norm_scatter(const void* qkv, int ld, const float* bias, const float* wq, const float* wk, void* q_out,
+                                    void* kcache, void* vcache, const int* slots, int rows, int heads, int kv_heads, int dim,
+                                    int vdim, int pad, int page_size, float eps, int plain, int has_kv, int in_dtype, int dtype,
+                                    hipStream_t stream) {
     if (rows <= 0) return 0;
-    if (dim <= 0 || vdim <= 0 || dim > pad || vdim > pad || pad > 256 || page_size <= 0 ||
-        ld < (heads + kv_heads) * dim + kv_heads * vdim)
+    if (dim <= 0 || vdim <= 0 || dim > pad || vdim > pad || pad > 256 || page_size <= 0 || (in_dtype == DT_BF16 && dtype == DT_F32) ||
+        ld < heads * dim + (has_kv ? kv_heads * (dim + vdim) : 0) || (has_kv && (!kcache || !vcache || !slots)))
         return (int)hipErrorInvalidValue;
-    const dim3 grid(rows, min((heads + 2 * kv_heads + 3) / 4, 65535));
-    if (dtype == DT_F32)
-        qk_norm_scatter_kernel<float><<<grid, 256, 0, stream>>>((const float*)qkv, ld, wq, wk, (float*)q_out, (float*)kcache,
-            (float*)vcache, slots, heads, kv_heads, dim, vdim, pad, page_size, eps);
-    else
-        qk_norm_scatter_kernel<bf16_t><<<grid, 256, 0, stream>>>((const bf16_t*)qkv, ld, wq, wk, (bf16_t*)q_out, (bf16_t*)kcache,
-            (bf16_t*)vcache, slots, heads, kv_heads, dim, vdim, pad, page_size, eps);
+    const dim3 grid(rows, min((heads + (has_kv ? 2 * kv_heads : 0) + 3) / 4, 65535));
+#define QK_NORM_SCATTER(TI, T) qk_norm_scatter_kernel<TI, T><<<grid, 256, 0, stream>>>((const TI*)qkv, ld, bias, wq, wk, (T*)q_out, \
+        (T*)kcache, (T*)vcache, slots, heads, kv_heads, dim, vdim, pad, page_size, eps, plain, has_kv)
+    if (dtype == DT_F32) QK_NORM_SCATTER(float, float);
+    else if (in_dtype == DT_F32) QK_NORM_SCATTER(float, bf16_t);
+    else QK_NORM_SCATTER(bf16_t, bf16_t);
+#undef QK_NORM_SCATTER
     return CISR_LAUNCH_CHECK();
 }
 

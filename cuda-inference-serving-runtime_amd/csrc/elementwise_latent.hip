@@ -153,7 +153,8 @@ template <typename T>
 __global__ void __launch_bounds__(256) latent_keys_kernel(LatentArgs p) {
     __shared__ float red[4];
     const int t = blockIdx.x, tid = threadIdx.x;
-    const int pos = min(max(p.positions[t], 0), p.max_pos - 1), half = p.rot / 2;
+    const int half = p.rot / 2;                     // (0: a latent without a turning part)
+    const int pos = half ? min(max(p.positions[t], 0), p.max_pos - 1) : 0;
     const float* cs = p.cos + (size_t)pos * half;
     const float* sn = p.sin + (size_t)pos * half;
     const float* row = p.down + (size_t)t * p.ld + p.first;
@@ -211,7 +212,7 @@ extern "C" int cisr_latent_keys(const float* down, int ld, int first, const floa
                                 int rank, int pad, int page, int max_pos, int interleaved, float eps, int dtype,
                                 hipStream_t stream) {
     if (rows <= 0) return 0;
-    if (rot <= 0 || rot % 2 || rot > rot_dim || rank + rot_dim > pad || page <= 0 || max_pos <= 0 || first < 0 ||
+    if (rot < 0 || rot % 2 || rot > rot_dim || rank + rot_dim > pad || page <= 0 || (rot > 0 && max_pos <= 0) || first < 0 ||
         first + rank + rot_dim > ld || heads <= 0)
         return (int)hipErrorInvalidValue;
     LatentArgs p{down, ld, first, weight, q, ldq, q_out, kcache, vcache, positions, slots, cos, sin,

@@ -187,6 +187,7 @@ extern "C" int cisr_decay_gate(const float* z, int ld, const float* bias, float*
 //   u = y[t, i] + (skip ? skip[i / skip_span] * x[t * ldx + i] : 0)
 //   GATE_FIRST:  u *= silu(gate[t * ldg + i]);  out = u / rms(part) * w[shared ? d : i]
 //   else:        out = u / rms(part) * w[shared ? d : i] * silu(gate[t * ldg + i])
+// with `sigmoid` the gate's law is sigmoid instead of silu.
 // A block of NT threads a (row, part): a wave for parts of up to 256 elements, four waves up to 2,048, sixteen beyond.
 // KEEP: the part's elements (after the skip term and the gate before the norm) wait in LDS for their scale, so every
 // input is read once; else (parts of more than 12,288 elements) they are made a second time.
@@ -194,7 +195,7 @@ template <typename T, bool GATE_FIRST, int NT, bool KEEP>
 __global__ void __launch_bounds__(NT)
 group_norm_gate_kernel(const float* __restrict__ y, const float* __restrict__ gate, int ldg, const float* __restrict__ w,
                        int shared, const float* __restrict__ skip, int skip_span, const float* __restrict__ x, int ldx,
-                       T* __restrict__ out, int size, float eps) {
+                       T* __restrict__ out, int size, float eps, int sigmoid) {
     __shared__ float red[NT / WAVE];
     extern __shared__ float kept[];
     const int t = blockIdx.x, g = blockIdx.y, groups = gridDim.y, lane = threadIdx.x;
@@ -203,7 +204,7 @@ group_norm_gate_kernel(const float* __restrict__ y, const float* __restrict__ ga
     auto element = [&](int d) {
         float u = y[base + d];
         if (skip) u += skip[(col0 + d) / skip_span] * x[(size_t)t * ldx + col0 + d];
-        if (GATE_FIRST) { const float z = gate[(size_t)t * ldg + col0 + d]; u *= z / (1.0f + expf(-z)); }
+        if (GATE_FIRST) { const float z = gate[(size_t)t * ldg + col0 + d]; u *= (sigmoid ? 1.0f : z) / (1.0f + expf(-z)); }
         return u;
     };
     float ss = 0.f;
@@ -215,7 +216,7 @@ group_norm_gate_kernel(const float* __restrict__ y, const float* __restrict__ ga
     const float scale = 1.0f / sqrtf((NT == WAVE ? wave_sum(ss) : block_sum<NT>(ss, red)) / (float)size + eps);
     for (int d = lane; d < size; d += NT) {
         float u = (KEEP ? kept[d] : element(d)) * scale * w[shared ? d : col0 + d];     // (a thread reads back what it wrote)
-        if (!GATE_FIRST) { const float z = gate[(size_t)t * ldg + col0 + d]; u *= z / (1.0f + expf(-z)); }
+        if (!GATE_FIRST) { const float z = gate[(size_t)t * ldg + col0 + d]; u *= (sigmoid ? 1.0f : z) / (1.0f + expf(-z)); }
         store_f32(out + base + d, u);
     }
 }
@@ -223,10 +224,10 @@ group_norm_gate_kernel(const float* __restrict__ y, const float* __restrict__ ga
 template <typename T, bool GATE_FIRST>
 static void launch_group_norm_gate(const float* y, const float* gate, int ldg, const float* w, int shared, const float* skip,
                                    int skip_span, const float* x, int ldx, T* out, int rows, int groups, int size, float eps,
-                                   hipStream_t stream) {
+                                   int sigmoid, hipStream_t stream) {
     const dim3 grid(rows, groups);
     const size_t lds = (size_t)size * sizeof(float);
-#define GNG(NT, KEEP) group_norm_gate_kernel<T, GATE_FIRST, NT, KEEP><<<grid, NT, KEEP ? lds : 0, stream>>>(y, gate, ldg, w, shared, skip, skip_span, x, ldx, out, size, eps)
+#define GNG(NT, KEEP) group_norm_gate_kernel<T, GATE_FIRST, NT, KEEP><<<grid, NT, KEEP ? lds : 0, stream>>>(y, gate, ldg, w, shared, skip, skip_span, x, ldx, out, size, eps, sigmoid)
     if (size <= 256) GNG(64, true);
     else if (size <= 2048) GNG(256, true);
     else if (size <= 12288) GNG(1024, true);
@@ -236,15 +237,15 @@ static void launch_group_norm_gate(const float* y, const float* gate, int ldg, c
 
 extern "C" int cisr_group_norm_gate(const float* y, const float* gate, int ldg, const float* w, int shared, const float* skip,
                                     int skip_span, const float* x, int ldx, void* out, int rows, int groups, int size,
-                                    float eps, int gate_first, int dtype, hipStream_t stream) {
+                                    float eps, int gate_first, int sigmoid, int dtype, hipStream_t stream) {
     if (rows <= 0) return 0;
     if (groups <= 0 || groups > 65535 || size <= 0 || (skip && (skip_span <= 0 || !x))) return (int)hipErrorInvalidValue;
     if (dtype == DT_F32) {
-        if (gate_first) launch_group_norm_gate<float, true>(y, gate, ldg, w, shared, skip, skip_span, x, ldx, (float*)out, rows, groups, size, eps, stream);
-        else launch_group_norm_gate<float, false>(y, gate, ldg, w, shared, skip, skip_span, x, ldx, (float*)out, rows, groups, size, eps, stream);
+        if (gate_first) launch_group_norm_gate<float, true>(y, gate, ldg, w, shared, skip, skip_span, x, ldx, (float*)out, rows, groups, size, eps, sigmoid, stream);
+        else launch_group_norm_gate<float, false>(y, gate, ldg, w, shared, skip, skip_span, x, ldx, (float*)out, rows, groups, size, eps, sigmoid, stream);
     } else {
-        if (gate_first) launch_group_norm_gate<bf16_t, true>(y, gate, ldg, w, shared, skip, skip_span, x, ldx, (bf16_t*)out, rows, groups, size, eps, stream);
-        else launch_group_norm_gate<bf16_t, false>(y, gate, ldg, w, shared, skip, skip_span, x, ldx, (bf16_t*)out, rows, groups, size, eps, stream);
+        if (gate_first) launch_group_norm_gate<bf16_t, true>(y, gate, ldg, w, shared, skip, skip_span, x, ldx, (bf16_t*)out, rows, groups, size, eps, sigmoid, stream);
+        else launch_group_norm_gate<bf16_t, false>(y, gate, ldg, w, shared, skip, skip_span, x, ldx, (bf16_t*)out, rows, groups, size, eps, sigmoid, stream);
     }
     return CISR_LAUNCH_CHECK();
 }

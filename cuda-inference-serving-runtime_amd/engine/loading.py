@@ -74,6 +74,8 @@ def random_model(config, seed=0, dtype="bfloat16", device="cuda:0", std=0.02):
         values = torch.randn(spec.drawn_shape(), generator=generator, device=device, dtype=torch.float32) * std
         if spec.init == "one_plus_normal":
             values += 1.0
+        elif spec.init == "identity_plus_normal":
+            values += torch.eye(*spec.drawn_shape(), device=device)
         tensors[spec.name] = values.to(torch.bfloat16 if dtype == torch.bfloat16 else torch.float32)
     model.bind(tensors, dtype, torch.device(device))
     return model

@@ -71,7 +71,7 @@ def _declare(h):
         "cisr_gemm_bf16_gated": [p, i, p, i, p, i, i, i, i, i, f, f, f, p],
         "cisr_post_norm_add": [p, p, p, p, p, p, i, i, f, f, p, f, p, i, i, i, f, f, p, p],
         "cisr_glu_clamped": [p, p, i, i, f, f, f, i, p],
-        "cisr_qk_norm_scatter": [p, i, p, p, p, p, p, p, i, i, i, i, i, i, i, f, i, p],
+        "cisr_qk_norm_scatter": [p, i, p, p, p, p, p, p, p, i, i, i, i, i, i, i, f, i, i, i, i, p],
         "cisr_head_gate": [p, p, i, p, i, i, i, i, i, p],
         "cisr_layernorm": [p, p, p, p, p, i, i, f, i, p],
         "cisr_rms_slice": [p, i, i, p, p, i, i, f, i, p],
@@ -94,6 +94,10 @@ def _declare(h):
         "cisr_experts_combine": [p, p, p, p, i, p, p, i, i, i, i, p],
         "cisr_bias_act": [p, p, p, ll, i, i, i, p],
         "cisr_experts_rows_ok": [i, i, i],
+        "cisr_streams_read": [p, p, p, f, p, p, i, i, i, i, p],
+        "cisr_streams_step": [p, p, i, p, p, p, p, f, p, i, i, i, i, p],
+        "cisr_streams_embed": [p, p, p, p, p, f, p, i, i, i, i, i, p],
+        "cisr_softcap": [p, ll, f, p],
     }
     for name, args in sig.items():
         fn = getattr(h, name)
@@ -723,9 +727,13 @@ def gemm_normed(x, norm, w, out):
     return out
 
 
+GELU_TANH_LAW = (-1.0, 0.0, 0.0)      # the law of gemm_swiglu and glu_clamped that gates by the tanh form of gelu
+
+
 def gemm_swiglu(a, w_gate_up, out, gate_up=None, norm=None, scratch=None, law=None):
     """out[M, I] = silu(a . Wg^T) * (a . Wu^T) with w_gate_up = [Wg; Wu] ([2I, K]); with `law` = (limit, slope, shift)
-    the activation is g sigmoid(slope g) (u + shift), g = min(gate, limit), u = clamp(up, -limit, limit) instead.
+    the activation is g sigmoid(slope g) (u + shift), g = min(gate, limit), u = clamp(up, -limit, limit) instead, or with
+    GELU_TANH_LAW gelu(gate) u, the gelu's tanh form.
     Few rows of bf16 run one fused weight-streaming kernel (with `norm` = (weight, eps, None), `a` is the float
     residual and RMSNorm is fused too); otherwise the product goes to `gate_up` [M, 2I] and the activation is
     a second kernel.  `scratch`: the ScratchPool of the caller's steps."""
@@ -1073,7 +1081,8 @@ def post_norm_add(x, y, weight, eps, mult, second=None, following=None):
 
 
 def glu_clamped(gate_up, out, limit, slope=1.702, shift=1.0):
-    """out[r, i] = g sigmoid(slope g) (u + shift), g = min(gate_up[r, i], limit), u = clamp(gate_up[r, I + i], -limit, limit)."""
+    """out[r, i] = g sigmoid(slope g) (u + shift), g = min(gate_up[r, i], limit), u = clamp(gate_up[r, I + i], -limit, limit);
+    by the signs of `limit` also the other laws of a gated activation: 0 silu(g) u, negative (GELU_TANH_LAW) gelu(g) u."""
     rows, two_i = gate_up.shape
     if two_i % 2:
         raise KernelError("glu_clamped: input width must be even")
@@ -1083,22 +1092,33 @@ def glu_clamped(gate_up, out, limit, slope=1.702, shift=1.0):
     return out
 
 
-def qk_norm_scatter(qkv, q_norm, k_norm, q_out, kcache, vcache, slots, heads, kv_heads, dim, vdim, pad, page_size, eps):
+def qk_norm_scatter(qkv, q_norm, k_norm, q_out, kcache, vcache, slots, heads, kv_heads, dim, vdim, pad, page_size, eps, bias=None,
+                    plain_norm=False):
     """Rows of a fused projection [q: heads x dim | k: kv_heads x dim | v: kv_heads x vdim | ...]: queries and keys
-    RMS-normed per head (weights float [dim], or None: left as they are), queries into q_out [T, heads * pad], keys and
-    values into the cache at `slots`, all as heads of `pad` coordinates whose rest is zero (keys [pages, kv_heads,
-    page_size, pad], values transposed in a page, [pages, kv_heads, pad, page_size])."""
+    RMS-normed per head (weights float [dim]; None: left as they are, or with `plain_norm` normed without a weight), queries
+    into q_out [T, heads * pad], keys and values into the cache at `slots`, all as heads of `pad` coordinates whose rest is
+    zero (keys [pages, kv_heads, page_size, pad], values transposed in a page, [pages, kv_heads, pad, page_size]).  qkv has
+    the cache's dtype, or is float.  `bias`: float over the q, k and v columns, added before everything else.  kcache None:
+    the rows have queries only (a layer that reads another's cache)."""
     rows, ld = qkv.shape
-    if dim > pad or vdim > pad or pad > 256 or ld < (heads + kv_heads) * dim + kv_heads * vdim:
+    has_kv = kcache is not None
+    columns = heads * dim + (kv_heads * (dim + vdim) if has_kv else 0)
+    if dim > pad or vdim > pad or pad > 256 or ld < columns:
         raise KernelError(f"qk_norm_scatter: heads of {dim} / {vdim} do not fit rows of {ld} or pages of {pad}")
-    pages = kcache.shape[0]
+    if qkv.dtype not in (q_out.dtype, torch.float32):
+        raise KernelError("qk_norm_scatter: the rows have the queries' dtype, or are float")
     wq = None if q_norm is None else _dev(q_norm, "q_norm", torch.float32, (dim,))
     wk = None if k_norm is None else _dev(k_norm, "k_norm", torch.float32, (dim,))
-    _check(lib().cisr_qk_norm_scatter(_dev(qkv, "qkv"), ld, wq, wk, _dev(q_out, "q_out", qkv.dtype, (rows, heads * pad)),
-                                      _dev(kcache, "kcache", qkv.dtype, (pages, kv_heads, page_size, pad)),
-                                      _dev(vcache, "vcache", qkv.dtype, (pages, kv_heads, pad, page_size)),
-                                      _dev(slots, "slots", torch.int32, (rows,)), rows, heads, kv_heads, dim, vdim, pad,
-                                      page_size, float(eps), _storage(qkv, "qkv"), _stream()), "qk_norm_scatter")
+    bp = None if bias is None else _dev(bias, "bias", torch.float32, (columns,))
+    kp = vp = sp = None
+    if has_kv:
+        pages = kcache.shape[0]
+        kp = _dev(kcache, "kcache", q_out.dtype, (pages, kv_heads, page_size, pad))
+        vp = _dev(vcache, "vcache", q_out.dtype, (pages, kv_heads, pad, page_size))
+        sp = _dev(slots, "slots", torch.int32, (rows,))
+    _check(lib().cisr_qk_norm_scatter(_dev(qkv, "qkv"), ld, bp, wq, wk, _dev(q_out, "q_out", None, (rows, heads * pad)), kp, vp, sp,
+                                      rows, heads, kv_heads, dim, vdim, pad, page_size, float(eps), int(bool(plain_norm)), int(has_kv),
+                                      _storage(qkv, "qkv"), _storage(q_out, "q_out"), _stream()), "qk_norm_scatter")
     return q_out
 
 
@@ -1152,11 +1172,11 @@ def latent_keys(down, weight, q, q_out, kcache, vcache, positions, slots, cos, s
     key head [c | turned | 0] of `pad` coordinates (kcache [pages, 1, page_size, pad]) and one value head [c | 0]
     (vcache [pages, 1, pad, page_size]).  q [T, heads * (dim + rot_dim)]: the last rot_dim coordinates of each head are
     turned alike and written to q_out[t, h, rank : rank + rot_dim], zeros behind them; q_out[t, h, :rank] is left to
-    the caller (the query's product with the key up-projection)."""
+    the caller (the query's product with the key up-projection).  cos and sin None: nothing turns (rot_dim may be 0)."""
     rows = q_out.shape[0]
     dp, ld = _rows_of(down, "down", rank + rot_dim)
-    max_pos, half = cos.shape
-    if rank + rot_dim > pad or 2 * half > rot_dim or half <= 0:
+    max_pos, half = cos.shape if cos is not None else (0, 0)
+    if rank + rot_dim > pad or 2 * half > rot_dim:
         raise KernelError(f"latent_keys: {rank} + {rot_dim} coordinates do not fit heads of {pad}, or {2 * half} turn among {rot_dim}")
     if q.dim() != 2 or q.stride(1) != 1 or q.shape[1] != heads * (dim + rot_dim) or q.shape[0] != rows or q.dtype != q_out.dtype:
         raise KernelError("latent_keys: q must be [T, heads * (dim + rot_dim)] of the cache's dtype")
@@ -1167,7 +1187,8 @@ def latent_keys(down, weight, q, q_out, kcache, vcache, positions, slots, cos, s
                                   _dev(kcache, "kcache", q_out.dtype, (pages, 1, page_size, pad)),
                                   _dev(vcache, "vcache", q_out.dtype, (pages, 1, pad, page_size)),
                                   _dev(positions, "positions", torch.int32, (rows,)), sp,
-                                  _dev(cos, "cos", torch.float32), _dev(sin, "sin", torch.float32, (max_pos, half)),
+                                  None if cos is None else _dev(cos, "cos", torch.float32),
+                                  None if cos is None else _dev(sin, "sin", torch.float32, (max_pos, half)),
                                   rows, heads, dim, rot_dim, 2 * half, rank, pad, page_size, max_pos, int(bool(interleaved)),
                                   float(eps), _storage(q_out, "q_out"), _stream()), "latent_keys")
     return q_out
@@ -1258,9 +1279,11 @@ def _rec():
             "cisr_conv_silu": [p, i, i, p, p, p, ll, p, p, p, p, i, i, i, i, i, i, p, p, p, p, i, p],
             "cisr_decay_gate": [p, i, p, p, i, i, f, p],
             "cisr_decay_gate_low_rank": [p, i, i, p, p, p, i, i, f, p],
-            "cisr_group_norm_gate": [p, p, i, p, i, p, i, p, i, p, i, i, i, f, i, i, p],
+            "cisr_group_norm_gate": [p, p, i, p, i, p, i, p, i, p, i, i, i, f, i, i, i, p],
             "cisr_delta_scan": [p, i, p, i, p, i, p, i, p, i, p, i, p, ll, p, p, i, i, i, i, i, f, i, p],
             "cisr_unit_heads": [p, i, i, i, i, i, f, f, p],
+            "cisr_channel_inputs": [p, i, p, i, p, ll, p, p, p, p, i, i, i, i, i, i, f, i, i, p, p, p, p, i, i, p, p, i, i, p],
+            "cisr_channel_scan": [p, i, p, i, p, i, p, i, p, i, p, i, p, ll, p, p, i, i, i, i, i, f, i, p],
             "cisr_mingru_scan": [p, i, p, p, p, i, p, p, p, i, i, i, i, p, i, i, p],
             "cisr_mlstm_gates": [p, i, p, i, p, p, p, i, p, p, p, p, p, ll, p, p, i, i, i, i, f, i, p],
             "cisr_mlstm_finish": [p, p, p, i, p, p, i, i, i, f, f, i, p],
@@ -1407,11 +1430,12 @@ def decay_gate_low_rank(low, up, bias, out, tau):
     return out
 
 
-def group_norm_gate(y, gate, weight, out, groups, eps, gate_first, shared_weight=False, skip=None):
+def group_norm_gate(y, gate, weight, out, groups, eps, gate_first, shared_weight=False, skip=None, sigmoid=False):
     """Rows of y float [T, groups * size] in `groups` equal parts, each divided by its own root mean square, times
     `weight` ([size] if shared by the parts, else [groups * size]), with silu(gate) multiplied in before the norm
     (`gate_first`) or after it; `skip` = (d [n], x view [T, groups * size]) adds d[i // (groups * size / n)] x[t, i]
-    first.  gate a float view [T, groups * size]; out [T, groups * size] float or bf16."""
+    first.  gate a float view [T, groups * size]; out [T, groups * size] float or bf16.  `sigmoid`: the gate's law is
+    sigmoid instead of silu."""
     T, width = y.shape
     if width % groups:
         raise KernelError("group_norm_gate: the row does not divide into its parts")
@@ -1427,7 +1451,7 @@ def group_norm_gate(y, gate, weight, out, groups, eps, gate_first, shared_weight
         xp, ldx = _rows_of(x, "x", width)
     _check(_rec().cisr_group_norm_gate(_dev(y, "y", torch.float32), gp, ldg, wp, int(shared_weight), dp, span, xp, ldx,
                                        _dev(out, "out", None, (T, width)), T, groups, size, float(eps), int(bool(gate_first)),
-                                       _storage(out, "out"), _stream()), "group_norm_gate")
+                                       int(bool(sigmoid)), _storage(out, "out"), _stream()), "group_norm_gate")
     return out
 
 
@@ -1476,6 +1500,149 @@ def delta_scan(q, k, v, decay, write, out, state, seg_start, state_slots, heads,
                                   _dev(state_slots, "state_slots", torch.int32, (segments,)), segments, heads, R, Cc,
                                   int(share), float(q_scale), cols, _stream()), "delta_scan")
     return out
+
+
+def channel_delta_inputs(proj, taps, conv_state, qkv, seg_of_row, seg_start, state_slots, kv_heads, dim, heads, vdim, decay_at, decay_up,
+                         dt_bias, a_log, decay, gate_at, gate_up, gate, unit_eps=1e-6, single_rows=False):
+    """The operands of channel_delta_scan from the float rows of an input product, proj [T, >= ...]: its first channels =
+    2 kv_heads dim + heads vdim columns [q | k | v] go through the causal convolution (taps float [K, channels], taps[K - 1]
+    weighs the newest input; the K - 1 inputs before a segment from conv_state, a float view [slots, >= (K - 1) channels],
+    which moves on) and silu, and the heads of q and k become unit vectors: qkv float [T, channels].  decay [T, heads * dim]
+    = exp(-exp(a_log) softplus(proj[:, decay_at:] . decay_up + dt_bias)), decay_up [rank, heads * dim]; gate [T, heads * vdim]
+    = proj[:, gate_at:] . gate_up, gate_up [rank, heads * vdim] (both of one dtype, float or bf16; the sums are float)."""
+    T = qkv.shape[0]
+    pp, ld = _rows_of(proj, "proj")
+    K, channels = taps.shape
+    segments = state_slots.shape[0]
+    if proj.shape[0] != T or channels != 2 * kv_heads * dim + heads * vdim or heads % kv_heads:
+        raise KernelError("channel_delta_inputs: the rows do not hold these heads")
+    if (conv_state.dtype != torch.float32 or not conv_state.is_cuda or conv_state.stride(1) != 1
+            or conv_state.shape[1] < (K - 1) * channels):
+        raise KernelError("channel_delta_inputs: the state must be float [slots, >= (K - 1) * channels]")
+    ra, rg = decay_up.shape[0], gate_up.shape[0]
+    if decay_up.dtype != gate_up.dtype or decay_at + ra > proj.shape[1] or gate_at + rg > proj.shape[1]:
+        raise KernelError("channel_delta_inputs: low-rank columns beyond the rows, or matrices of two dtypes")
+    _check(_rec().cisr_channel_inputs(pp, ld, _dev(taps, "taps", torch.float32), K, conv_state.data_ptr(), conv_state.stride(0),
+                                      _dev(qkv, "qkv", torch.float32, (T, channels)), _dev(seg_of_row, "seg_of_row", torch.int32, (T,)),
+                                      _dev(seg_start, "seg_start", torch.int32, (segments + 1,)),
+                                      _dev(state_slots, "state_slots", torch.int32, (segments,)), T, segments, kv_heads, dim, heads, vdim,
+                                      float(unit_eps), int(decay_at), ra, _dev(decay_up, "decay_up", None, (ra, heads * dim)),
+                                      _dev(dt_bias, "dt_bias", torch.float32, (heads * dim,)), _dev(a_log, "a_log", torch.float32, (heads,)),
+                                      _dev(decay, "decay", torch.float32, (T, heads * dim)), int(gate_at), rg,
+                                      _dev(gate_up, "gate_up", None, (rg, heads * vdim)), _dev(gate, "gate", torch.float32, (T, heads * vdim)),
+                                      int(bool(single_rows)), _storage(decay_up, "decay_up"), _stream()), "channel_delta_inputs")
+    return qkv
+
+
+def channel_columns(segments, heads, cols):
+    """Columns of the state that one wave of the delta rule with decays a channel owns (32, 16, 8 or 4): see delta_columns."""
+    for width in (32, 16, 8, 4):
+        if segments * heads * -(-cols // width) >= 1024 or width == 4:
+            return width
+
+
+def channel_delta_scan(q, k, v, decay, write, out, state, seg_start, state_slots, heads, rows_of_state, cols_of_state, share=1,
+                       q_scale=1.0, columns=None):
+    """delta_scan with a decay a head and key channel: per segment and head, over the segment's rows in order, S <- diag(g)
+    S; u = sigmoid(b) (v - S^T k); S <- S + k u^T; o = q_scale S^T q.  decay (g) [T, heads * R]; everything else as there."""
+    R, Cc = int(rows_of_state), int(cols_of_state)
+    T = v.shape[0]
+    segments = state_slots.shape[0]
+    if heads % share or R > 256:
+        raise KernelError("channel_delta_scan: heads must divide into their groups and a state has at most 256 rows")
+    qp, ldq = _rows_of(q, "q", heads // share * R)
+    kp, ldk = _rows_of(k, "k", heads // share * R)
+    vp, ldv = _rows_of(v, "v", heads * Cc)
+    op, ldo = _rows_of(out, "out", heads * Cc)
+    gp, ldg = _rows_of(decay, "decay", heads * R)
+    bp, ldb = _rows_of(write, "write", heads)
+    if any(t.shape[0] != T for t in (q, k, decay, write, out)):
+        raise KernelError("channel_delta_scan: operands differ in rows")
+    if state.dtype != torch.float32 or state.dim() != 2 or state.stride(1) != 1 or state.shape[1] < heads * R * Cc or not state.is_cuda:
+        raise KernelError("channel_delta_scan: the state must be float [slots, >= heads * R * C]")
+    cols = int(columns or channel_columns(segments, heads, Cc))
+    while columns is None and cols > 8 and -(-R // (128 // cols)) > 32:
+        cols //= 2         # (at most 32 rows of its two columns a lane)
+    _check(_rec().cisr_channel_scan(qp, ldq, kp, ldk, vp, ldv, gp, ldg, bp, ldb, op, ldo, state.data_ptr(), state.stride(0),
+                                    _dev(seg_start, "seg_start", torch.int32, (segments + 1,)),
+                                    _dev(state_slots, "state_slots", torch.int32, (segments,)), segments, heads, R, Cc,
+                                    int(share), float(q_scale), cols, _stream()), "channel_delta_scan")
+    return out
+
+
+# -- a residual of several streams (csrc/elementwise_streams.hip) ------------------------------------------------------
+
+MAX_STREAMS = 8
+
+
+def _streams_read_args(read, rows, dim, streams):
+    """(in, weight, eps, out, out dtype) of a read (weights over the streams float [S], norm weight float [H], eps, out [R, H])."""
+    if read is None:
+        return None, None, 0.0, None, F32
+    w_in, weight, eps, out = read
+    return (_dev(w_in, "read weights", torch.float32, (streams,)), _dev(weight, "norm weight", torch.float32, (dim,)), float(eps),
+            _dev(out, "out", None, (rows, dim)), _storage(out, "out"))
+
+
+def _streams_of(x, streams, name):
+    if not 1 <= streams <= MAX_STREAMS or x.dim() != 2 or x.shape[1] % streams:
+        raise KernelError(f"{name}: rows of {tuple(x.shape)} in {streams} streams (at most {MAX_STREAMS})")
+    if x.shape[1] // streams > 16384:
+        raise KernelError(f"{name}: streams of at most 16384 elements")
+    return _dev(x, "x", torch.float32), x.shape[1] // streams
+
+
+def streams_read(x, streams, w_in, weight, eps, out, rows=None):
+    """out[r] = rmsnorm(sum_s w_in[s] x_s[r]) * weight of the rows of x float [T, streams * H] (or of x[rows])."""
+    xp, dim = _streams_of(x, streams, "streams_read")
+    n = out.shape[0]
+    if rows is None and n != x.shape[0]:
+        raise KernelError("streams_read: out rows differ from input rows")
+    rp = None if rows is None else _dev(rows, "rows", torch.int32, (n,))
+    ip, wp, eps, op, dt = _streams_read_args((w_in, weight, eps, out), n, dim, streams)
+    _check(lib().cisr_streams_read(xp, ip, wp, eps, op, rp, n, dim, streams, dt, _stream()), "streams_read")
+    return out
+
+
+def streams_step(x, streams, y, mix, w_out, read=None):
+    """x_t <- sum_s mix[s, t] x_s + w_out[t] y in place, every stream from the old ones: x float [T, streams * H], y float
+    [T, H] or the Partials of such a product, mix float [streams, streams] (from, to), w_out float [streams].  `read` = (w_in
+    float [streams], weight float [H], eps, out [T, H]): what reads the streams next is made by the same kernel,
+    out = rmsnorm(sum_s w_in[s] x_s) * weight of the new streams."""
+    xp, dim = _streams_of(x, streams, "streams_step")
+    rows, slices = x.shape[0], 0
+    if isinstance(y, Partials):
+        if (y.rows, y.cols) != (rows, dim) or y.parts.numel() < y.slices * rows * dim:
+            raise KernelError(f"streams_step: y is not the partial sums of a product [{rows}, {dim}]")
+        yp, slices = _dev(y.parts, "y", torch.float32), y.slices
+    else:
+        yp = _dev(y, "y", torch.float32, (rows, dim))
+    ip, wp, eps, op, dt = _streams_read_args(read, rows, dim, streams)
+    _check(lib().cisr_streams_step(xp, yp, slices, _dev(mix, "mix", torch.float32, (streams, streams)),
+                                   _dev(w_out, "w_out", torch.float32, (streams,)), ip, wp, eps, op, rows, dim, streams, dt, _stream()),
+           "streams_step")
+    return x
+
+
+def streams_embed(tokens, table, x, streams, read=None):
+    """x_s[r] = table[tokens[r]] in every stream, x float [T, streams * H]; `read` as in streams_step (its out has the
+    table's dtype)."""
+    xp, dim = _streams_of(x, streams, "streams_embed")
+    rows, vocab = tokens.shape[0], table.shape[0]
+    if x.shape[0] != rows or (read is not None and read[3].dtype != table.dtype):
+        raise KernelError("streams_embed: a row a token, and a read in the table's dtype")
+    ip, wp, eps, op, _ = _streams_read_args(read, rows, dim, streams)
+    _check(lib().cisr_streams_embed(_dev(tokens, "tokens", torch.int32, (rows,)), _dev(table, "table", None, (vocab, dim)), xp, ip, wp, eps, op,
+                                    rows, dim, streams, vocab, _storage(table, "table"), _stream()), "streams_embed")
+    return x
+
+
+def softcap(x, cap):
+    """x <- cap tanh(x / cap), in place, float."""
+    if not cap > 0:
+        raise KernelError("softcap: the cap must be positive")
+    _check(lib().cisr_softcap(_dev(x, "x", torch.float32), x.numel(), float(cap), _stream()), "softcap")
+    return x
 
 
 # -- layers that norm after the sum, hashed token pairs, whole-projection norms (csrc/elementwise_postnorm.hip) --------

@@ -4,3 +4,4 @@ from .novosun import build_novosun
 from .ditazen import build_ditazen
 from .noresun import build_noresun
 from .zovozen import build_zovozen
+from .guduzen import build_guduzen

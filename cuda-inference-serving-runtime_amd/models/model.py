@@ -123,6 +123,8 @@ class Model:
     def forward(self, ctx):
         """Logits [R, vocab] (float) at ctx.logit_rows; None if no row is wanted
         (the layers still run: they fill the cache)."""
+        first = self.layers[self.schedule[0].layer] if self.schedule else None
+        ctx.next_norm = first.first_norm() if hasattr(first, "first_norm") else None     # (an embedding may make the first norm)
         x = self.embedding.forward(ctx)
         last = len(self.schedule) - 1
         for index, entry in enumerate(self.schedule):

@@ -128,9 +128,13 @@ class PagedAttention(Mixer):
 
 class NormedGatedAttention(Mixer):
     """Grouped-query softmax attention over the paged cache whose positions do not enter the scores: queries and keys
-    are RMS-normed per head (a weight of size `dim` each, shared by the heads; `qk_norm` False: not normed), the score
-    is (q . k) * scale, keys and values may differ in size (`dim`, `vdim`), and each head's result is multiplied by
-    sigmoid of a projection of the mixer's input, one number a head (`head_gate`).
+    are RMS-normed per head (a weight of size `dim` each, shared by the heads; `qk_norm` False: not normed, "plain": normed
+    without a weight), the score is (q . k) * scale, keys and values may differ in size (`dim`, `vdim`), and each head's
+    result is multiplied by sigmoid of a projection of the mixer's input, one number a head (`head_gate`).  A row sees
+    itself and the `window` - 1 keys before it (None: all).  With `bias` the projections of q, k and v add
+    `<tensor>.b`; their results are then float until they are normed (`float_rows`, on its own: without biases too).
+    `own_kv` False: the layer has no key and value tensors and reads the cache another layer wrote.  `keep`: the window
+    the layer's own cache keeps, where layers that read it look further back than it does itself.
 
     The pages hold heads of `pad` = max(dim, vdim) coordinates (rounded up to a multiple of 8), the rest zero: zero
     coordinates add nothing to a score and give result coordinates that are not read, so the attention kernels
@@ -139,7 +143,7 @@ class NormedGatedAttention(Mixer):
     NAMES = {"q": "q", "k": "k", "v": "v", "o": "o", "gate": "g", "q_norm": "q.norm", "k_norm": "k.norm"}
 
     def __init__(self, name, hidden, heads, kv_heads, dim, vdim, scale, eps, qk_norm=True, head_gate=True, window=None,
-                 names=None, tuning=None):
+                 names=None, tuning=None, bias=False, float_rows=None, own_kv=True, keep="own"):
         if heads % kv_heads:
             raise ValueError(f"{heads} query heads are not a multiple of {kv_heads} key/value heads")
         self.pad = -(-max(dim, vdim) // 8) * 8
@@ -148,10 +152,17 @@ class NormedGatedAttention(Mixer):
         if not scale > 0:
             raise ValueError("the score scale must be positive")
         self.name, self.hidden, self.heads, self.kv_heads, self.dim, self.vdim = name, hidden, heads, kv_heads, dim, vdim
-        self.scale, self.eps, self.qk_norm, self.head_gate, self.window = float(scale), float(eps), bool(qk_norm), bool(head_gate), window
+        self.scale, self.eps, self.qk_norm, self.head_gate, self.window = float(scale), float(eps), qk_norm, bool(head_gate), window
+        self.bias, self.own_kv = bool(bias), bool(own_kv)
+        self.float_rows = self.bias if float_rows is None else bool(float_rows)
+        if self.float_rows and self.head_gate:
+            raise ValueError("the heads' gates are read in the activations' type: no float rows beside them")
+        self.keep = window if keep == "own" else keep
+        if self.keep is not None and (window is None or window > self.keep):
+            raise ValueError("a layer's cache keeps at least the keys the layer itself looks back over")
         self.names = {**self.NAMES, **(names or {})}
         self.tuning = tuning or kernel.DEFAULT_TUNING
-        self.w_in = self.w_out = self.q_weight = self.k_weight = None
+        self.w_in = self.w_out = self.q_weight = self.k_weight = self.b_in = None
 
     def _tensor(self, which):
         return f"{self.name}.{self.names[which]}"
@@ -163,29 +174,42 @@ class NormedGatedAttention(Mixer):
         return [kernel.SingleRows(self.tuning.split_single_from), kernel.RowsLongestFirst()]
 
     def cache_need(self):
-        return KVNeed(self.kv_heads, self.pad, self.window)
+        return KVNeed(self.kv_heads, self.pad, self.keep) if self.own_kv else None
+
+    def cache_read(self):
+        return None if self.own_kv else KVNeed(self.kv_heads, self.pad, self.window)
+
+    def _projections(self):
+        nh, nkv, D, V = self.heads, self.kv_heads, self.dim, self.vdim
+        return {"q": nh * D, "k": nkv * D, "v": nkv * V} if self.own_kv else {"q": nh * D}
 
     def tensor_specs(self):
-        H, nh, nkv, D, V = self.hidden, self.heads, self.kv_heads, self.dim, self.vdim
-        specs = [TensorSpec(self._tensor("q"), (nh * D, H)), TensorSpec(self._tensor("k"), (nkv * D, H)),
-                 TensorSpec(self._tensor("v"), (nkv * V, H)), TensorSpec(self._tensor("o"), (H, nh * V))]
+        H, nh, D, V = self.hidden, self.heads, self.dim, self.vdim
+        specs = [TensorSpec(self._tensor(p), (rows, H)) for p, rows in self._projections().items()]
+        if self.bias:
+            specs += [TensorSpec(self._tensor(p) + ".b", (rows,)) for p, rows in self._projections().items()]
+        specs.append(TensorSpec(self._tensor("o"), (H, nh * V)))
         if self.head_gate:
             specs.append(TensorSpec(self._tensor("gate"), (nh, H)))
-        if self.qk_norm:
-            specs += [TensorSpec(self._tensor("q_norm"), (D,), init="one_plus_normal"),
-                      TensorSpec(self._tensor("k_norm"), (D,), init="one_plus_normal")]
+        if self.qk_norm and self.qk_norm != "plain":
+            specs.append(TensorSpec(self._tensor("q_norm"), (D,), init="one_plus_normal"))
+            if self.own_kv:
+                specs.append(TensorSpec(self._tensor("k_norm"), (D,), init="one_plus_normal"))
         return specs
 
     def bind(self, tensors, dtype):
-        parts = [matrix_operand(tensors[self._tensor(p)], dtype) for p in (("q", "k", "v", "gate") if self.head_gate else ("q", "k", "v"))]
+        inputs = list(self._projections())
+        parts = [matrix_operand(tensors[self._tensor(p)], dtype) for p in inputs + (["gate"] if self.head_gate else [])]
         rows = sum(p.shape[0] for p in parts)
         if rows % 8:      # rows of the fused projection are a multiple of 16 bytes: zero rows at the end
             parts.append(torch.zeros(8 - rows % 8, self.hidden, dtype=parts[0].dtype, device=parts[0].device))
         self.w_in = torch.cat(parts, dim=0).contiguous()
         self.w_out = matrix_operand(tensors[self._tensor("o")], dtype)
-        if self.qk_norm:
+        if self.bias:
+            self.b_in = torch.cat([tensors[self._tensor(p) + ".b"].to(torch.float32) for p in inputs]).contiguous()
+        if self.qk_norm and self.qk_norm != "plain":
             self.q_weight = tensors[self._tensor("q_norm")].to(torch.float32).contiguous()
-            self.k_weight = tensors[self._tensor("k_norm")].to(torch.float32).contiguous()
+            self.k_weight = tensors[self._tensor("k_norm")].to(torch.float32).contiguous() if self.own_kv else None
 
     def output(self, h, ctx, site):
         """The mixer's result, float [T, hidden], without the residual sum."""
@@ -193,14 +217,18 @@ class NormedGatedAttention(Mixer):
         nh, nkv, D, V, pad = self.heads, self.kv_heads, self.dim, self.vdim, self.pad
         gid, kcache, vcache = ctx.cache.pages_of_site(site)
         view = ctx.kv[gid]
-        qkv = ops.gemm(h, self.w_in, ctx.buffer("gattn.qkv", (T, self.w_in.shape[0]), ctx.dtype), scratch=ctx.scratch)
-        q = ops.qk_norm_scatter(qkv, self.q_weight, self.k_weight, ctx.buffer("gattn.q", (T, nh * pad), ctx.dtype), kcache, vcache,
-                                view.slots, nh, nkv, D, V, pad, view.page_size, self.eps)
+        qkv = ctx.buffer("gattn.qkv", (T, self.w_in.shape[0]), torch.float32 if self.float_rows else ctx.dtype)
+        ops.gemm(h, self.w_in, qkv, scratch=ctx.scratch)
+        written = (kcache, vcache, view.slots) if self.own_kv else (None, None, None)
+        q = ops.qk_norm_scatter(qkv, self.q_weight, self.k_weight, ctx.buffer("gattn.q", (T, nh * pad), ctx.dtype), *written,
+                                nh, nkv, D, V, pad, view.page_size, self.eps, bias=self.b_in, plain_norm=self.qk_norm == "plain")
         out = ctx.buffer("gattn.out", (T, nh * pad), ctx.dtype)
         kernel.paged_attention(ctx, q, nh * pad, kcache, vcache, view, out, nh, nkv, pad, self.window, self.scale, tuning=self.tuning)
-        first_gate = (nh + nkv) * D + nkv * V
+        first_gate = sum(self._projections().values())
         gates = qkv[:, first_gate:first_gate + nh] if self.head_gate else None
-        act = ops.head_gate(out, gates, ctx.buffer("gattn.act", (T, nh * V), ctx.dtype), nh, V, pad)
+        act = out
+        if gates is not None or pad != V:
+            act = ops.head_gate(out, gates, ctx.buffer("gattn.act", (T, nh * V), ctx.dtype), nh, V, pad)
         return ctx.product_for_norm(act, self.w_out, "gattn.y")
 
     def forward(self, h, residual, ctx, site, norm=None):
@@ -224,7 +252,8 @@ class LatentAttention(Mixer):
     run as they are; the weighted sum of latents then goes through Wuv_j.  The pages therefore hold what the design
     says must be kept, c and kr, and nothing a head.  Up to 256 coordinates the matrix-core kernels serve (bfloat16); a
     larger latent (up to 640 with its turning part) runs the exact row-wise kernel in both dtypes.  `position` turns the first `position.rotary_dim` of the rot_dim
-    coordinates.  `names`: the tensors' names under `name`."""
+    coordinates; `position` None (and rot_dim 0): positions do not enter the scores.  `names`: the tensors' names under
+    `name`."""
 
     NAMES = {"q": "q", "dq": "dq", "dq_norm": "dq.norm", "uq": "uq", "dkv": "dkv", "dkv_norm": "dkv.norm", "uk": "uk",
              "uv": "uv", "gate": "g", "o": "o"}
@@ -236,7 +265,9 @@ class LatentAttention(Mixer):
             raise ValueError(f"a latent of {kv_rank} and {rot_dim} turning coordinates: at most {ops.ROWWISE_MAX_HEAD} together")
         if not scale > 0:
             raise ValueError("the score scale must be positive")
-        if position.rotary_dim > rot_dim:
+        if position is None and rot_dim:
+            raise ValueError("turning coordinates need a position part")
+        if position is not None and position.rotary_dim > rot_dim:
             raise ValueError(f"{position.rotary_dim} coordinates turn, the queries and keys have {rot_dim} for it")
         self.name, self.hidden, self.heads, self.dim, self.rot_dim, self.vdim = name, hidden, heads, dim, rot_dim, vdim
         self.kv_rank, self.scale, self.eps, self.position = kv_rank, float(scale), float(eps), position
@@ -293,14 +324,16 @@ class LatentAttention(Mixer):
                 raise ValueError(f"{self.name}: the query latent's projections and norm disagree about its size")
 
     def prepare(self, device, dtype):
-        self.position.prepare(device, dtype)
+        if self.position is not None:
+            self.position.prepare(device, dtype)
 
-    def forward(self, h, residual, ctx, site, norm=None):
+    def _heads_result(self, h, ctx, site):
+        """The operand of the output projection [T, heads * vdim]."""
         T = h.shape[0]
         nh, D, R, V, r, pad = self.heads, self.dim, self.rot_dim, self.vdim, self.kv_rank, self.pad
         gid, kcache, vcache = ctx.cache.pages_of_site(site)
         view = ctx.kv[gid]
-        cos, sin = self.position.tables()
+        cos, sin = self.position.tables() if self.position is not None else (None, None)
         small = ops.gemm(h, self.w_small, ctx.buffer("lat.small", (T, self.w_small.shape[0]), torch.float32), scratch=ctx.scratch)
         first = 0
         if self.q_rank is not None:
@@ -315,13 +348,19 @@ class LatentAttention(Mixer):
             ops.gemm(h, self.w_q, q, scratch=ctx.scratch)
         qa = ctx.buffer("lat.qa", (T, nh * pad), ctx.dtype)
         ops.latent_keys(small[:, first:first + r + R], self.kv_weight, q, qa, kcache, vcache, ctx.positions, view.slots, cos, sin,
-                        nh, D, R, r, pad, view.page_size, self.eps, interleaved=self.position.pairing == "interleaved")
+                        nh, D, R, r, pad, view.page_size, self.eps, interleaved=getattr(self.position, "pairing", None) == "interleaved")
         ops.heads_product(q, D + R, self.w_absorb, qa, pad)
         out = ctx.buffer("lat.out", (T, nh * pad), ctx.dtype)
         kernel.paged_attention(ctx, qa, nh * pad, kcache, vcache, view, out, nh, 1, pad, self.window, self.scale, tuning=self.tuning)
         gates = small[:, first + r + R:first + r + R + nh] if self.head_gate else None
-        act = ops.heads_product(out, pad, self.w_value, ctx.buffer("lat.act", (T, nh * V), ctx.dtype), V, gate=gates)
-        return ctx.add_product(act, self.w_out, residual)
+        return ops.heads_product(out, pad, self.w_value, ctx.buffer("lat.act", (T, nh * V), ctx.dtype), V, gate=gates)
+
+    def output(self, h, ctx, site):
+        """The mixer's result, float [T, hidden], without the residual sum."""
+        return ctx.product_for_norm(self._heads_result(h, ctx, site), self.w_out, "lat.y")
+
+    def forward(self, h, residual, ctx, site, norm=None):
+        return ctx.add_product(self._heads_result(h, ctx, site), self.w_out, residual)
 
 
 class SigmoidAttention(Mixer):

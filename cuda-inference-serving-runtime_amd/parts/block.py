@@ -4,7 +4,8 @@ the residual stream x kept in float.  SandwichBlock norms each sublayer's result
 and scales it: x = x + m norm1b(mixer(norm1(x))); x = x + m norm2b(ffn(norm2(x))); without the norms in front
 (`reads_stream`) its sublayers read x itself: x = x + m norm1b(mixer(x)).  PostNormBlock norms after the
 sum, and its sublayers read the stream itself: x = norm1(a x + g1 mixer(x)); x = norm2(a x + g2 ffn(x)), with
-optional gates g = sigmoid(W x + b) element by element."""
+optional gates g = sigmoid(W x + b) element by element.  HyperConnectedBlock keeps several streams instead of one x,
+with weights that read, mix and write them around every sublayer."""
 import torch
 
 from ..kernels import ops
@@ -334,6 +335,90 @@ class PostNormBlock(Part):
         return residual
 
 
+class HyperConnectedBlock(Part):
+    """A residual of `streams` streams x_1 .. x_s (rows [T, streams * hidden], one stream after the other) and, around each
+    sublayer q (1: mixer, 2: feed-forward), weights over them: u = sum_s in[s] x_s; y = sublayer(norm(u)); then, every stream
+    from the old ones, x_t <- sum_s mix[s, t] x_s + out[t] y (mix is indexed [from, to]).  Tensors
+    `<name>.<names[q]>.in|out|mix`.  `mixer_norm` and `ffn_norm` are StreamsNorm parts: they own `in` and make the read.
+    The write of a sublayer's result and the read of whatever reads the streams next (this block's feed-forward, or the
+    following block) are one kernel (ops.streams_step).  Mixer and feed-forward give their result without a residual sum
+    (`output`).  `ffn` None: a layer without a feed-forward."""
+
+    def __init__(self, name, streams, mixer_norm, mixer, ffn_norm=None, ffn=None, names=("hc1", "hc2")):
+        if (ffn is None) != (ffn_norm is None):
+            raise ValueError("a feed-forward comes with the norm before it, or not at all")
+        for norm in (mixer_norm, ffn_norm):
+            if norm is not None and getattr(norm, "reads_streams", None) != streams:
+                raise ValueError(f"the norms of this arrangement read {streams} streams")
+        if not hasattr(mixer, "output") or (ffn is not None and not hasattr(ffn, "output")):
+            raise ValueError("the sublayers of this arrangement must give their result without the residual sum (output)")
+        self.name, self.streams, self.names = name, int(streams), tuple(names)
+        self.mixer_norm, self.mixer, self.ffn_norm, self.ffn = mixer_norm, mixer, ffn_norm, ffn
+        self.writes = []       # per sublayer (mix [streams, streams], out [streams]), float
+
+    def parts(self):
+        return [p for p in (self.mixer_norm, self.mixer, self.ffn_norm, self.ffn) if p is not None]
+
+    def _sublayers(self):
+        return 1 if self.ffn is None else 2
+
+    def tensor_specs(self):
+        specs, S = [s for p in self.parts() for s in p.tensor_specs()], self.streams
+        for q in self.names[:self._sublayers()]:
+            specs += [TensorSpec(f"{self.name}.{q}.out", (S,), init="one_plus_normal"),
+                      TensorSpec(f"{self.name}.{q}.mix", (S, S), init="identity_plus_normal")]
+        return specs
+
+    def bind(self, tensors, dtype):
+        for p in self.parts():
+            p.bind(tensors, dtype)
+        self.writes = [tuple(tensors[f"{self.name}.{q}.{w}"].to(torch.float32).contiguous() for w in ("mix", "out"))
+                       for q in self.names[:self._sublayers()]]
+
+    def prepare(self, device, dtype):
+        for p in self.parts():
+            p.prepare(device, dtype)
+
+    def cache_need(self):
+        return self.mixer.cache_need()
+
+    def cache_read(self):
+        return self.mixer.cache_read() if hasattr(self.mixer, "cache_read") else None
+
+    def state_need(self):
+        return self.mixer.state_need()
+
+    def kernel_units(self, dtype):
+        return [u for p in self.parts() if hasattr(p, "kernel_units") for u in p.kernel_units(dtype)]
+
+    def step_arrays(self):
+        return [a for p in self.parts() if hasattr(p, "step_arrays") for a in p.step_arrays()]
+
+    def first_norm(self):
+        return self.mixer_norm
+
+    def _write(self, x, result, sublayer, reader, ctx):
+        """The streams take a sublayer's result; returns what `reader` reads of them (None: it does not read streams)."""
+        mix, out = self.writes[sublayer]
+        read = reader.read_args(x.shape[0], ctx) if getattr(reader, "reads_streams", None) == self.streams else None
+        ops.streams_step(x, self.streams, result, mix, out, read=read)
+        return None if read is None else read[3]
+
+    def forward(self, residual, ctx, site):
+        after = ctx.next_norm
+        ctx.next_norm = None          # (no product of this block is left to a later norm)
+        h = ctx.take_normed(self.mixer_norm, residual)
+        if h is None:
+            h = self.mixer_norm.forward(residual, ctx)
+        h = self._write(residual, self.mixer.output(h, ctx, site), 0, after if self.ffn is None else self.ffn_norm, ctx)
+        if self.ffn is not None:
+            h = self._write(residual, self.ffn.output(h, ctx, unfinished=True), 1, after, ctx)
+        if h is not None:
+            ctx.leave_normed(after, residual, h)
+        return residual
+
+
+register_part("block", "hyper_connected", HyperConnectedBlock)
 register_part("block", "postnorm", PostNormBlock)
 register_part("block", "prenorm", PreNormBlock)
 register_part("block", "sandwich", SandwichBlock)

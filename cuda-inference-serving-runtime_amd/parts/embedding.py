@@ -29,6 +29,25 @@ class TokenEmbedding(Part):
         return ops.embedding(ctx.tokens, self.weight, out)
 
 
+class StreamsEmbedding(TokenEmbedding):
+    """The embedding of a model whose residual is `streams` streams: every stream of a row starts as the token's row, and
+    the first sublayer's read of them (a norm that says `reads_streams`) is made on the way."""
+
+    def __init__(self, name, vocab, hidden, streams, tensor=None):
+        super().__init__(name, vocab, hidden, tensor=tensor)
+        self.streams = int(streams)
+
+    def forward(self, ctx):
+        T = ctx.tokens.shape[0]
+        x = ctx.buffer("residual", (T, self.streams * self.hidden), torch.float32)
+        reader = ctx.next_norm
+        read = reader.read_args(T, ctx) if getattr(reader, "reads_streams", None) == self.streams else None
+        ops.streams_embed(ctx.tokens, self.weight, x, self.streams, read=read)
+        if read is not None:
+            ctx.leave_normed(reader, x, read[3])
+        return x
+
+
 STATE_SITE = "embedding"      # the key of the embedding's state among the cache manager's state sites
 
 
@@ -77,8 +96,11 @@ class PairHashEmbedding(TokenEmbedding):
 
 
 class LMHead(Part):
-    def __init__(self, name, vocab, hidden, tied_to=None, tensor=None):
-        self.name, self.vocab, self.hidden, self.tied_to = name, vocab, hidden, tied_to
+    def __init__(self, name, vocab, hidden, tied_to=None, tensor=None, softcap=None):
+        """`softcap`: the logits become cap tanh(logits / cap)."""
+        if softcap is not None and not softcap > 0:
+            raise ValueError("the logits' cap must be positive")
+        self.name, self.vocab, self.hidden, self.tied_to, self.softcap = name, vocab, hidden, tied_to, softcap
         self.tensor = tensor if tensor is not None else name + ".weight"
         self.weight = None
 
@@ -96,5 +118,7 @@ class LMHead(Part):
         n = ctx.logit_rows.shape[0] if norm is not None else h.shape[0]
         logits = ctx.buffer("logits", (n, self.vocab), torch.float32)
         if norm is not None:
-            return ops.gemm_normed(residual, (norm.weight, norm.eps, ctx.logit_rows), self.weight, logits)
-        return ops.gemm(h, self.weight, logits, after_norm=True, scratch=ctx.scratch)
+            ops.gemm_normed(residual, (norm.weight, norm.eps, ctx.logit_rows), self.weight, logits)
+        else:
+            ops.gemm(h, self.weight, logits, after_norm=True, scratch=ctx.scratch)
+        return logits if self.softcap is None else ops.softcap(logits, self.softcap)

@@ -9,11 +9,16 @@ from .base import FeedForward, TensorSpec, matrix_operand, register_part
 
 
 class GatedMLP(FeedForward):
+    LAWS = {"silu": None, "gelu_tanh": ops.GELU_TANH_LAW}      # what the kernels take as the gate's law (None: silu)
+
     def __init__(self, name, hidden, intermediate, activation="silu", bias=False, names=None):
         """`names` = (gate, up, down): the matrices' full names under `name` where they are not `<x>_proj.weight`
-        (no biases then)."""
-        if activation != "silu":
-            raise ValueError(f"activation {activation!r}: only silu has a kernel")
+        (no biases then).  `activation`: "silu", or "gelu_tanh" (the gelu's tanh form)."""
+        if activation not in self.LAWS:
+            raise ValueError(f"activation {activation!r}: one of {sorted(self.LAWS)}")
+        if activation != "silu" and bias:
+            raise ValueError("biases come with silu")
+        self.law = self.LAWS[activation]
         if names is not None and bias:
             raise ValueError("biases come with the default tensor names")
         self.name, self.hidden, self.intermediate = name, hidden, intermediate
@@ -39,7 +44,7 @@ class GatedMLP(FeedForward):
             self.b_down = tensors[f"{self.name}.down_proj.bias"].contiguous()
 
     def fuses_norm(self, norm, residual, ctx):
-        return not self.bias and getattr(norm, "fusable_as", None) == "rms" and ops.fused_norm_ok(residual, self.w_gate_up, residual.shape[0])
+        return not self.bias and self.law is None and getattr(norm, "fusable_as", None) == "rms" and ops.fused_norm_ok(residual, self.w_gate_up, residual.shape[0])
 
     def forward(self, h, residual, ctx, norm=None):
         T = residual.shape[0]
@@ -51,21 +56,26 @@ class GatedMLP(FeedForward):
         if norm is not None:
             ops.gemm_swiglu(residual, self.w_gate_up, act, norm=(norm.weight, norm.eps, None), scratch=ctx.scratch)
         elif ops.swiglu_fused_ok(h, self.w_gate_up):
-            ops.gemm_swiglu(h, self.w_gate_up, act, scratch=ctx.scratch)   # one kernel: product and activation
+            ops.gemm_swiglu(h, self.w_gate_up, act, scratch=ctx.scratch, law=self.law)   # one kernel: product and activation
         else:
-            ops.gemm_swiglu(h, self.w_gate_up, act, gate_up=ctx.buffer("ffn.gate_up", (T, 2 * self.intermediate), ctx.dtype), scratch=ctx.scratch)
+            ops.gemm_swiglu(h, self.w_gate_up, act, gate_up=ctx.buffer("ffn.gate_up", (T, 2 * self.intermediate), ctx.dtype),
+                            scratch=ctx.scratch, law=self.law)
         return ctx.add_product(act, self.w_down, residual)
 
-    def output(self, h, ctx, tag="ffn"):
-        """The feed-forward's result, float [T, hidden], without the residual sum (no biases)."""
+    def output(self, h, ctx, tag="ffn", unfinished=False):
+        """The feed-forward's result, float [T, hidden], without the residual sum (no biases); `unfinished`: it may be
+        left as partial sums (ops.Partials) for a reader that adds them."""
         if self.bias:
             raise NotImplementedError("the result without the residual sum is made for the form without biases")
         T = h.shape[0]
         act = ctx.buffer(tag + ".act", (T, self.intermediate), ctx.dtype)
         if ops.swiglu_fused_ok(h, self.w_gate_up):
-            ops.gemm_swiglu(h, self.w_gate_up, act, scratch=ctx.scratch)
+            ops.gemm_swiglu(h, self.w_gate_up, act, scratch=ctx.scratch, law=self.law)
         else:
-            ops.gemm_swiglu(h, self.w_gate_up, act, gate_up=ctx.buffer(tag + ".gate_up", (T, 2 * self.intermediate), ctx.dtype), scratch=ctx.scratch)
+            ops.gemm_swiglu(h, self.w_gate_up, act, gate_up=ctx.buffer(tag + ".gate_up", (T, 2 * self.intermediate), ctx.dtype),
+                            scratch=ctx.scratch, law=self.law)
+        if unfinished:
+            return ctx.product_for_norm(act, self.w_down, tag + ".out")
         return ops.gemm(act, self.w_down, ctx.buffer(tag + ".out", (T, self.hidden), torch.float32), scratch=ctx.scratch)
 
 

@@ -1,5 +1,6 @@
 """RMSNorm: y = x * rsqrt(mean(x^2) + eps) * w in float
 (reference: runtime/reference.py:5-6, kernels/ops.cu:3-19).
+StreamsNorm: the RMSNorm of a weighted sum of a residual's streams.
 LayerNorm: y = (x - mean) * rsqrt(var + eps) * w (+ b), var the mean of the squared deviations, in float."""
 import torch
 
@@ -13,17 +14,20 @@ class RMSNorm(Part):
     fusable_as = "rms"
     adds_partials = True    # forward adds the partial sums of a product left unfinished before it (ctx.add_product)
 
-    def __init__(self, name, dim, eps, tensor=None):
-        """`tensor`: the weight's full name where it is not `<name>.weight`."""
-        self.name, self.dim, self.eps = name, dim, float(eps)
+    def __init__(self, name, dim, eps, tensor=None, around_zero=False):
+        """`tensor`: the weight's full name where it is not `<name>.weight`.  `around_zero`: the stored weight is the
+        deviation from one (y = x * rsqrt(...) * (1 + w)); the sum is made once, in float, at bind."""
+        self.name, self.dim, self.eps, self.around_zero = name, dim, float(eps), bool(around_zero)
         self.tensor = tensor if tensor is not None else name + ".weight"
         self.weight = None
 
     def tensor_specs(self):
-        return [TensorSpec(self.tensor, (self.dim,), init="one_plus_normal")]
+        return [TensorSpec(self.tensor, (self.dim,), init="normal" if self.around_zero else "one_plus_normal")]
 
     def bind(self, tensors, dtype):
         self.weight = tensors[self.tensor].to(torch.float32).contiguous()  # exact widening
+        if self.around_zero:
+            self.weight = self.weight + 1.0
 
     def forward(self, x, ctx, rows=None, tag="norm"):
         n_out = x.shape[0] if rows is None else rows.shape[0]
@@ -65,5 +69,38 @@ class LayerNorm(Part):
         return ops.layernorm(x, self.weight, ctx.buffer(tag, (n_out, self.dim), ctx.dtype), self.eps, rows, bias=self.bias)
 
 
+class StreamsNorm(RMSNorm):
+    """The RMS norm of a weighted sum of a residual's streams (rows [T, streams * dim], one stream after the other):
+    y = rmsnorm(sum_s in[s] x_s) * w, in[s] the tensor `reads` [streams], or 1 for every stream (None).  What a sublayer
+    of a model with hyper-connections reads, and what its head reads.  `reads_streams` says so to whoever writes the
+    streams before: that kernel can make this read on its way (`read_args`)."""
+    fusable_as = None
+    adds_partials = False
+
+    def __init__(self, name, dim, eps, streams, reads=None, tensor=None, around_zero=False):
+        super().__init__(name, dim, eps, tensor=tensor, around_zero=around_zero)
+        self.reads_streams, self.reads, self.w_in = int(streams), reads, None
+
+    def tensor_specs(self):
+        own = [] if self.reads is None else [TensorSpec(self.reads, (self.reads_streams,), init="one_plus_normal")]
+        return super().tensor_specs() + own
+
+    def bind(self, tensors, dtype):
+        super().bind(tensors, dtype)
+        if self.reads is not None:
+            self.w_in = tensors[self.reads].to(torch.float32).contiguous()
+        else:
+            self.w_in = torch.ones(self.reads_streams, dtype=torch.float32, device=self.weight.device)
+
+    def read_args(self, rows, ctx, tag="streams.read"):
+        """The `read` of ops.streams_step / streams_embed: weights, norm, and the buffer [rows, dim] it goes to."""
+        return (self.w_in, self.weight, self.eps, ctx.buffer(tag, (rows, self.dim), ctx.dtype))
+
+    def forward(self, x, ctx, rows=None, tag="norm"):
+        n_out = x.shape[0] if rows is None else rows.shape[0]
+        return ops.streams_read(x, self.reads_streams, self.w_in, self.weight, self.eps, ctx.buffer(tag, (n_out, self.dim), ctx.dtype), rows)
+
+
+register_part("norm", "streams_norm", StreamsNorm)
 register_part("norm", "rmsnorm", RMSNorm)
 register_part("norm", "layernorm", LayerNorm)

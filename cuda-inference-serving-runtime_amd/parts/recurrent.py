@@ -18,6 +18,10 @@ the state in the cache manager's state slots, in float in every mode:
                          part of the state), q and k are made unit vectors per head, q scaled by dim^(-1/2); each
                          head's result RMS-normed, times silu of a gate projection, then the output projection.
 
+  ChannelDeltaRule       the same rule with a decay a head and key channel (ops.channel_delta_scan): g_t = exp(-exp(A_log)
+                         softplus(Wa2 Wa1 h + dt_bias)) from a low-rank projection, acting on the rows of S; the result's
+                         gate is sigmoid of a low-rank projection.
+
   MinGRU                 no heads and no matrix state: S_t = (1 - z_t) S_(t-1) + z_t c_t element by element over `width`
                          channels, z_t = sigmoid(Wz h + bz), c_t = cand(Wx h + bx) with cand(u) = u + 1/2 for u >= 0 and
                          sigmoid(u) below (the gates read the current token only); the result is Wo (S_t silu(Wg h)).
@@ -257,6 +261,68 @@ class GatedDeltaRule(Mixer):
         return ctx.add_product(self._normed_result(h, ctx, site), self.w_out, residual)
 
 
+class ChannelDeltaRule(GatedDeltaRule):
+    """The gated delta rule with a decay a head and key channel.  Decays and the result's gate come from low-rank
+    projections whose inner sizes the file decides; the convolution, the unit vectors, the decays and the gates are one
+    kernel (ops.channel_delta_inputs).  The state is that of the rule with a decay a head."""
+
+    NAMES = {"q": "q", "k": "k", "v": "v", "write": "b", "decay_down": "a1", "decay_up": "a2", "dt_bias": "dt_bias", "a_log": "A_log",
+             "gate_down": "g1", "gate_up": "g2", "norm": "norm", "o": "o", "conv": "conv"}
+
+    def __init__(self, name, hidden, heads, kv_heads, dim, vdim, taps, eps, unit_eps=1e-6, rank=None, names=None):
+        """`rank`: the inner size of the low-rank projections where no file says it (`dim` unless given)."""
+        super().__init__(name, hidden, heads, kv_heads, dim, vdim, taps, eps, unit_eps=unit_eps, names=names)
+        self.rank = int(rank) if rank is not None else dim
+
+    def tensor_specs(self):
+        H, t, conv, rank = self.hidden, self._tensor, self.names["conv"], AnySize(self.rank)
+        return [TensorSpec(t("q"), (self.qk, H)), TensorSpec(t("k"), (self.qk, H)), TensorSpec(t("v"), (self.inner, H)),
+                TensorSpec(f"{t('q')}.{conv}", (self.qk, self.taps)), TensorSpec(f"{t('k')}.{conv}", (self.qk, self.taps)),
+                TensorSpec(f"{t('v')}.{conv}", (self.inner, self.taps)), TensorSpec(t("write"), (self.heads, H)),
+                TensorSpec(t("decay_down"), (rank, H)), TensorSpec(t("decay_up"), (self.heads * self.dim, rank)),
+                TensorSpec(t("dt_bias"), (self.heads * self.dim,)), TensorSpec(t("a_log"), (self.heads,)),
+                TensorSpec(t("gate_down"), (rank, H)), TensorSpec(t("gate_up"), (self.inner, rank)),
+                TensorSpec(t("norm"), (self.vdim,), init="one_plus_normal"), TensorSpec(t("o"), (H, self.inner))]
+
+    def bind(self, tensors, dtype):
+        t, conv = self._tensor, self.names["conv"]
+        # one product with float results: [q | k | v | write | decay's first half | gate's first half]
+        inputs = ("q", "k", "v", "write", "decay_down", "gate_down")
+        parts = [matrix_operand(tensors[t(p)], dtype) for p in inputs]
+        starts = [sum(p.shape[0] for p in parts[:i]) for i in range(len(parts) + 1)]
+        self.at = dict(zip(inputs, starts))
+        if starts[-1] % 8:
+            parts.append(torch.zeros(8 - starts[-1] % 8, self.hidden, dtype=parts[0].dtype, device=parts[0].device))
+        self.w_in = torch.cat(parts, dim=0).contiguous()
+        self.w_out = matrix_operand(tensors[t("o")], dtype)
+        # the second halves by columns, [rank, columns]: neighbouring threads own neighbouring columns
+        self.decay_up = matrix_operand(tensors[t("decay_up")], dtype).t().contiguous()
+        self.gate_up = matrix_operand(tensors[t("gate_up")], dtype).t().contiguous()
+        for down, up in (("decay_down", self.decay_up), ("gate_down", self.gate_up)):
+            if tensors[t(down)].shape[0] != up.shape[0]:
+                raise ValueError(f"{self.name}: the projections {self.names[down]} and its second half disagree about their inner size")
+        self.conv = torch.cat([_float(tensors[f"{t(p)}.{conv}"]) for p in ("q", "k", "v")], dim=0).t().contiguous()     # [taps, channels]
+        self.dt_bias, self.a_log = _float(tensors[t("dt_bias")]), _float(tensors[t("a_log")])
+        self.norm_weight = _float(tensors[t("norm")])
+
+    def _normed_result(self, h, ctx, site):
+        T = h.shape[0]
+        qk, inner, ch, nh = self.qk, self.inner, self.channels, self.heads
+        proj = ops.gemm(h, self.w_in, ctx.buffer("cdelta.proj", (T, self.w_in.shape[0]), torch.float32), scratch=ctx.scratch)
+        state = ctx.cache.state_storage[site]
+        qkv, decay, gate = (ctx.buffer("cdelta." + n, (T, size), torch.float32)
+                            for n, size in (("qkv", ch), ("decay", nh * self.dim), ("gate", inner)))
+        ops.channel_delta_inputs(proj, self.conv, state[:, nh * self.dim * self.vdim:], qkv, ctx.seg_of_row, ctx.seg_start, ctx.state_slots,
+                                 self.kv_heads, self.dim, nh, self.vdim, self.at["decay_down"], self.decay_up, self.dt_bias, self.a_log, decay,
+                                 self.at["gate_down"], self.gate_up, gate, unit_eps=self.unit_eps, single_rows=ctx.decode_only)
+        o = ctx.buffer("cdelta.o", (T, inner), torch.float32)
+        write = self.at["write"]
+        ops.channel_delta_scan(qkv[:, :qk], qkv[:, qk:2 * qk], qkv[:, 2 * qk:], decay, proj[:, write:write + nh], o, state,
+                               ctx.seg_start, ctx.state_slots, nh, self.dim, self.vdim, share=nh // self.kv_heads, q_scale=self.dim ** -0.5)
+        return ops.group_norm_gate(o, gate, self.norm_weight, ctx.buffer("cdelta.act", (T, inner), ctx.dtype), nh, self.eps,
+                                   gate_first=False, shared_weight=True, sigmoid=True)
+
+
 class MinGRU(Mixer):
     """The minimal gated recurrent unit over `width` channels (see the module's text).  State: float [width] a request,
     zero at the start.  `ride(weight)`: further rows for the input product, whose float results are then `rider`.
@@ -459,5 +525,6 @@ register_part("mixer", "gated_linear_attention", GatedLinearAttention)
 register_part("mixer", "state_space_duality", StateSpaceDuality)
 register_part("mixer", "side_by_side", SideBySide)
 register_part("mixer", "gated_delta_rule", GatedDeltaRule)
+register_part("mixer", "channel_delta_rule", ChannelDeltaRule)
 register_part("mixer", "mingru", MinGRU)
 register_part("mixer", "matrix_memory", MatrixMemory)

@@ -47,7 +47,7 @@ class AnySize:
 class TensorSpec:
     name: str
     shape: Tuple[object, ...]   # sizes; an AnySize stands for a dimension that the file decides
-    init: str = "normal"        # "normal": N(0, std); "one_plus_normal": 1 + N(0, std)  (random-weights mode)
+    init: str = "normal"        # "normal": N(0, std); "one_plus_normal": 1 + N(0, std); "identity_plus_normal": I + N(0, std)  (random-weights mode)
     integer: bool = False       # an integer table (kept as int32)
 
     def fits(self, shape):

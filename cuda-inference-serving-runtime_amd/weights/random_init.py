@@ -1,7 +1,7 @@
 """Random-weights mode: writes a model folder (config.json, model.safetensors)
 from a configuration and a seed.
 
-Matrices are N(0, 0.02); norm weights are 1 + N(0, 0.02).  Tensors are drawn in
+Matrices are N(0, 0.02); norm weights are 1 + N(0, 0.02); what mixes the streams of a residual is I + N(0, 0.02).  Tensors are drawn in
 the order of their names with one generator, so a folder is a function of
 (config, seed, stored dtype) only.  (The reference's own toy weights are
 N(0,1)/sqrt(in) with norms of exactly 1, runtime/model.py:38-55; the recipe here
@@ -28,6 +28,8 @@ def random_tensors(specs, seed, dtype=torch.bfloat16, std=STD):
         values = rng.standard_normal(size=spec.drawn_shape(), dtype=np.float32) * np.float32(std)
         if spec.init == "one_plus_normal":
             values = values + np.float32(1.0)
+        elif spec.init == "identity_plus_normal":
+            values = values + np.eye(*spec.drawn_shape(), dtype=np.float32)
         out[spec.name] = torch.from_numpy(values).to(dtype)
     return out
 
