@@ -283,7 +283,7 @@ def main():
     ap.add_argument("--check", type=int, default=1, choices=[0, 1], help="compare the timed way of running with the plain one first")
     ap.add_argument("--widths", default="1024,2048,4096", help="designs workload: model widths to time (comma separated)")
     ap.add_argument("--design-layers", type=int, default=4, help="designs workload: layers of each model")
-    ap.add_argument("--designs", default="llama,novosun,ditazen,noresun,zovozen", help="designs workload: which designs to time (comma separated)")
+    ap.add_argument("--designs", default="llama,novosun,ditazen,noresun,zovozen,guduzen", help="designs workload: which designs to time (comma separated)")
     args = ap.parse_args()
     if args.gpus != 1:
         print(f"bench.py measures one GPU only; --gpus {args.gpus} is not run")
@@ -388,8 +388,8 @@ def main():
 
 
 def design_configs(width, layers, context):
-    """A Llama, a Novosun, a Ditazen, a Noresun and a Zovozen configuration of the same width, depth and vocabulary.  The Novosun
-    layers alternate: softmax attention (heads of 64 for keys, 128 for values, a quarter as many key/value heads) beside
+    """A Llama, a Novosun, a Ditazen, a Noresun, a Zovozen and a Guduzen configuration of the same width, depth and vocabulary.  The
+    Novosun layers alternate: softmax attention (heads of 64 for keys, 128 for values, a quarter as many key/value heads) beside
     a state-space layer (inner size twice the width in heads of 64, 128 states, a convolution of 4 taps), then gated
     linear attention (key size half the width, value size the width, in heads of 128 x 256)."""
     ff, vocab = 4 * width, 32768
@@ -440,11 +440,24 @@ def design_configs(width, layers, context):
               "shared": {"ff": width}}
     zovozen = {"architecture": "Zovozen", "vocab": vocab, "width": width, "norm": {"eps": 1e-5}, "max_positions": context,
                "layers": [{"type": "parallel", "mixer": pair, "mlp": dense if i % 2 == 0 else scored} for i in range(layers)]}
-    return {"llama": llama, "novosun": novosun, "ditazen": ditazen, "noresun": noresun, "zovozen": zovozen}
+    # Guduzen: a residual of four streams; attention over a window of 1,024 keys without positions (heads of 128, a quarter as many
+    # key/value heads, biases), the delta rule with a decay a channel (twice as many value heads as query/key heads, all of 128, a
+    # convolution of 4 taps), latent attention without positions over every earlier key (latents of 256, as many coordinates as
+    # Ditazen caches a token), and attention over the same window that reads the first layer's keys; feed-forwards as Llama's
+    glu = {"kind": "dense", "ff": ff}
+    slide = {"heads": heads, "kv_heads": max(1, width // 512), "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "mask": {"size": 1024}}
+    order = [{"type": "attention", "mixer": slide, "mlp": glu},
+             {"type": "channel_delta", "mixer": {"heads": 2 * heads, "kv_heads": heads, "dim": 128, "vdim": 128, "conv": 4}, "mlp": glu},
+             {"type": "latent_attention", "mixer": {"heads": heads, "dim": 128, "vdim": 128, "kv_rank": 256, "q_rank": 3 * width // 4,
+                                                    "scale": 128 ** -0.5}, "mlp": glu},
+             {"type": "attention", "mixer": {**slide, "kv_from": 0}, "mlp": glu}]
+    guduzen = {"architecture": "Guduzen", "vocab": vocab, "width": width, "streams": 4, "logit_softcap": 30.0, "norm": {"eps": 1e-5},
+               "layers": [order[i % 4] for i in range(layers)], "max_positions": context}
+    return {"llama": llama, "novosun": novosun, "ditazen": ditazen, "noresun": noresun, "zovozen": zovozen, "guduzen": guduzen}
 
 
 def designs(args):
-    """Prompt steps and decode steps of the Novosun, Ditazen, Noresun and Zovozen designs beside the Llama design at equal width, depth
+    """Prompt steps and decode steps of the Novosun, Ditazen, Noresun, Zovozen and Guduzen designs beside the Llama design at equal width, depth
     and vocabulary (random weights drawn on the device): tokens a second of a whole prompt of --prompt tokens and
     of decode steps of 1, 8 and 64 requests after such prompts, through the step function with captured programs and
     the greedy pick."""
@@ -499,7 +512,7 @@ def designs(args):
             result["prefill"] = {"tokens": prompt, "ms": round(pf * 1e3, 3), "tokens_per_s": round(prompt / pf, 1)}
             out.setdefault(str(width), {})[design] = result
             del runner, model
-    return {"metric": f"prompt and decode tokens/s of the Novosun, Ditazen, Noresun and Zovozen designs beside Llama at equal width, {args.design_layers} layers",
+    return {"metric": f"prompt and decode tokens/s of the Novosun, Ditazen, Noresun, Zovozen and Guduzen designs beside Llama at equal width, {args.design_layers} layers",
             "unit": "tokens/s", "n_gpus": 1, "dtype": "bf16" if args.dtype == "bfloat16" else "fp32", "steps": steps,
             "data": "synthetic (random weights N(0,0.02), uniform-random token ids)", "prompt_len": prompt,
             "execution": args.execution, "widths": out}
