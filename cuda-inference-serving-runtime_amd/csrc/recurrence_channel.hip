@@ -4,8 +4,10 @@
 //   S <- diag(g_t) S;  u = beta_t (v_t - S^T k_t);  S <- S + k_t u^T;  o_t = S^T q_t
 //
 // g_t a decay a head and key channel, beta_t = sigmoid(b_t) one write strength a head, q and k shared by `share` heads.
-// Two kernels: the operands (short convolution with silu of q, k, v, unit vectors of q and k, decays and gates from
-// their low-rank projections) and the scan.  All float.
+// The operands (short convolution with silu of q, k, v, unit vectors of q and k,
+// decays and gates from their low-rank projections) are one kernel; the recurrence comes in three forms: a scan row by
+// row, a step of single rows with the result's norm and gate in it, and for prompt portions a walk chunk by chunk on
+// the matrix cores (recurrence_chunk.hip).  All float.
 #include "common.h"
 
 #define MAX_TAPS 16
@@ -19,101 +21,182 @@ struct ChannelInputs {
     const int* seg_of_row; const int* seg_start; const int* state_slots;
     int rows, G, R, H, C;
     float unit_eps;
-    // decays: exp(-exp(a_log[h]) softplus(sum_r up_a[r, h R + c] in[t, off_a + r] + dt_bias[h R + c]))
+    // decays: exp(-exp(a_log[h]) softplus(sum_r up_a[h R + c, r] in[t, off_a + r] + dt_bias[h R + c]))
     int off_a, rank_a; const void* up_a; const float* dt_bias; const float* a_log; float* decay;      // [T, H R]
-    // gates: sum_r up_g[r, h C + c] in[t, off_g + r]
+    // gates: sum_r up_g[h C + c, r] in[t, off_g + r]
     int off_g, rank_g; const void* up_g; float* gate;                                                 // [T, H C]
+    int ldu_a, ldu_g;                          // row strides of up_a, up_g: the ranks rounded up to 32, the rest zero
     int conv_blocks, row_tiles;                // how the grid divides: conv_blocks, then row_tiles x column blocks
 };
 
-#define RANK_CHUNK 64
+typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8_t;
+typedef __attribute__((ext_vector_type(4))) float f32x4_t;
 
-// A block is four waves.  The first conv_blocks blocks: a wave a (row, item), an item being a q head, a k head (both made
-// unit vectors) or up to 256 channels of v.  The others: a tile of RT rows by 256 columns of the decays or of the gates,
-// a thread a column, the rows' low-rank coordinates in LDS.  SINGLE: every segment has one row, and the wave of a
-// (row, channel) moves that channel's state on itself.
-template <bool SINGLE, int RT, typename TW>
-__global__ void __launch_bounds__(256) channel_inputs_kernel(ChannelInputs p) {
+__device__ __forceinline__ float channel_decay(float z, float rate) {
+    return expf(-rate * (fmaxf(z, 0.f) + log1pf(expf(-fabsf(z)))));
+}
+
+// An item of the convolution for the rows t .. t + n - 1 (n <= RB): a q head, a k head (both made unit vectors) or up to 256
+// channels of v; four channels a lane.  TAPS > 0: that many taps, the rows' inputs and those before them asked for at
+// once; rows whose inputs reach back before their segment, and TAPS 0 (any number of taps), take them one by one, from
+// the state where they lie before the segment.  SINGLE: every segment has one row, and the lane of a (row, channel)
+// moves that channel's state on itself.
+template <bool SINGLE, int TAPS>
+__device__ __forceinline__ void conv_item(const ChannelInputs& p, int t0, int n_rows, int item, int lane) {
+    constexpr int RB = TAPS ? 8 : 1, BACK = TAPS ? TAPS - 1 : 0;
     const int qk = p.G * p.R, inner = p.H * p.C, channels = 2 * qk + inner;
-    if ((int)blockIdx.x < p.conv_blocks) {
-        const int v_items = (inner + 255) / 256, per_row = 2 * p.G + v_items;
-        const int work = blockIdx.x * 4 + threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
-        const int t = work / per_row, item = work % per_row;
-        if (t >= p.rows) return;
-        const int seg = p.seg_of_row[t];
-        if (seg < 0) return;
-        const bool head = item < 2 * p.G;
-        const int first = head ? item * p.R : 2 * qk + (item - 2 * p.G) * 256;
-        const int n = head ? p.R : min(256, channels - first);
-        const int rel = t - p.seg_start[seg];
-        float* st = p.conv_state + (long long)p.state_slots[seg] * p.slot_stride;
-        float y[4], ss = 0.f;
+    const bool head = item < 2 * p.G;
+    const int first = head ? item * p.R : 2 * qk + (item - 2 * p.G) * 256;
+    const int n = head ? p.R : min(256, channels - first);
+    float x[RB + BACK][4], w[TAPS ? TAPS : 1][4];
+    if (TAPS) {
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
-            const int at = lane + WAVE * i, ch = first + at;
-            y[i] = 0.f;
-            if (at >= n) continue;
-            for (int j = 0; j < p.taps; ++j) {
-                const int src = rel - (p.taps - 1) + j;
-                const float x = src >= 0 ? p.in[(size_t)(t - rel + src) * p.ld + ch] : st[(size_t)(p.taps - 1 + src) * channels + ch];
-                y[i] += p.taps_w[(size_t)j * channels + ch] * x;
-                if (SINGLE && j > 0) st[(size_t)(j - 1) * channels + ch] = x;     // (input j of this row is input j - 1 of the next)
+            const int ch = first + min(lane + WAVE * i, n - 1);
+#pragma unroll
+            for (int r = 0; r < RB + BACK; ++r) x[r][i] = p.in[(size_t)min(max(t0 - BACK + r, 0), p.rows - 1) * p.ld + ch];
+#pragma unroll
+            for (int j = 0; j < TAPS; ++j) w[j][i] = p.taps_w[(size_t)j * channels + ch];
+        }
+    }
+#pragma unroll
+    for (int r = 0; r < RB; ++r) {
+        if (r >= n_rows) break;
+        const int t = t0 + r, seg = p.seg_of_row[t];
+        if (seg < 0) continue;
+        const int rel = t - p.seg_start[seg];
+        float y[4] = {0.f, 0.f, 0.f, 0.f}, ss = 0.f;
+        if (TAPS && rel >= BACK) {
+#pragma unroll
+            for (int i = 0; i < 4; ++i)
+#pragma unroll
+                for (int j = 0; j < (TAPS ? TAPS : 1); ++j) y[i] += w[j][i] * x[r + (TAPS ? j : 0)][i];
+        } else {
+            float* st = p.conv_state + (long long)p.state_slots[seg] * p.slot_stride;
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                const int ch = first + lane + WAVE * i;
+                if (lane + WAVE * i >= n) continue;
+                for (int j = 0; j < p.taps; ++j) {
+                    const int src = rel - (p.taps - 1) + j;
+                    const float a = src >= 0 ? p.in[(size_t)(t - rel + src) * p.ld + ch] : st[(size_t)(p.taps - 1 + src) * channels + ch];
+                    y[i] += p.taps_w[(size_t)j * channels + ch] * a;
+                    if (SINGLE && j > 0) st[(size_t)(j - 1) * channels + ch] = a;     // (input j of this row is input j - 1 of the next)
+                }
             }
-            y[i] = y[i] / (1.0f + expf(-y[i]));
+        }
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            y[i] = lane + WAVE * i < n ? y[i] / (1.0f + expf(-y[i])) : 0.f;
             ss += y[i] * y[i];
         }
         const float f = head ? 1.0f / sqrtf(wave_sum(ss) + p.unit_eps) : 1.0f;
 #pragma unroll
         for (int i = 0; i < 4; ++i)
             if (lane + WAVE * i < n) p.qkv[(size_t)t * channels + first + lane + WAVE * i] = y[i] * f;
+    }
+}
+
+// A block is four waves.  The first conv_blocks blocks: a wave an (item, run of rows) of the convolution.  The others make a
+// tile of rows by 256 columns of the decays or of the gates.
+//   bf16 matrices: 16 RT rows, on the matrix cores, a wave four tiles of 16 columns; the low-rank coordinates, float,
+//   as the sum of two bf16 numbers each (16 bits of mantissa), so two products.
+//   float matrices: RT rows, a thread a column, float sums in the order of the coordinates.
+#define RANK_CHUNK 64
+
+template <bool SINGLE, int TAPS, int RT, typename TW>
+__global__ void __launch_bounds__(256) channel_inputs_kernel(ChannelInputs p) {
+    const int inner = p.H * p.C;
+    const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
+    if ((int)blockIdx.x < p.conv_blocks) {
+        constexpr int RB = TAPS ? 8 : 1;
+        const int per_run = 2 * p.G + (inner + 255) / 256;
+        const int work = blockIdx.x * 4 + wave, t0 = work / per_run * RB;
+        if (t0 < p.rows) conv_item<SINGLE, TAPS>(p, t0, min(RB, p.rows - t0), work % per_run, lane);
         return;
     }
-    __shared__ __attribute__((aligned(16))) float low[RT][RANK_CHUNK];
     const int b = blockIdx.x - p.conv_blocks, tid = threadIdx.x;
-    const int t0 = (b % p.row_tiles) * RT, col_block = b / p.row_tiles;
+    const int col_block = b / p.row_tiles;
     const int a_cols = p.H * p.R, a_blocks = (a_cols + 255) / 256;
     const bool is_decay = col_block < a_blocks;
     const int cols = is_decay ? a_cols : inner, rank = is_decay ? p.rank_a : p.rank_g, off = is_decay ? p.off_a : p.off_g;
-    const int c = (is_decay ? col_block : col_block - a_blocks) * 256 + tid, cc = min(c, cols - 1);
-    const TW* up = (const TW*)(is_decay ? p.up_a : p.up_g) + cc;
-    float acc[RT];
+    const int ldu = is_decay ? p.ldu_a : p.ldu_g;
+    const TW* up = (const TW*)(is_decay ? p.up_a : p.up_g);
+    const int c_first = (is_decay ? col_block : col_block - a_blocks) * 256;
+    float* out = is_decay ? p.decay : p.gate;
+    if constexpr (sizeof(TW) == 2) {
+        const int t0 = (b % p.row_tiles) * 16 * RT, m = lane % 16, kg = lane / 16;
+        const int n_tiles = min(4, (cols - c_first - wave * 64 + 15) / 16);           // this wave's tiles of 16 columns
+        if (n_tiles <= 0) return;
+        f32x4_t acc[4][RT];
 #pragma unroll
-    for (int j = 0; j < RT; ++j) acc[j] = 0.f;
-    for (int r0 = 0; r0 < rank; r0 += RANK_CHUNK) {
-        __syncthreads();                                       // (the chunk before is used up)
-        for (int i = tid; i < RT * RANK_CHUNK; i += 256) {
-            const int j = i / RANK_CHUNK, r = r0 + i % RANK_CHUNK;
-            low[j][i % RANK_CHUNK] = r < rank ? p.in[(size_t)min(t0 + j, p.rows - 1) * p.ld + off + r] : 0.f;
+        for (int c = 0; c < 4; ++c)
+#pragma unroll
+            for (int j = 0; j < RT; ++j) acc[c][j] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
+        for (int k0 = 0; k0 < rank; k0 += 32) {
+            bf16x8_t hi[RT], lo[RT], wt[4];
+            const int k = k0 + kg * 8;
+#pragma unroll
+            for (int c = 0; c < 4; ++c)
+                wt[c] = *(const bf16x8_t*)(up + (size_t)min(c_first + wave * 64 + c * 16 + m, cols - 1) * ldu + k);
+#pragma unroll
+            for (int j = 0; j < RT; ++j) {
+                const float* row = p.in + (size_t)min(t0 + j * 16 + m, p.rows - 1) * p.ld + off + k;
+#pragma unroll
+                for (int e = 0; e < 8; ++e) {
+                    const float a = k + e < rank ? row[e] : 0.f;
+                    const __bf16 h = (__bf16)a;
+                    hi[j][e] = h;
+                    lo[j][e] = (__bf16)(a - (float)h);
+                }
+            }
+#pragma unroll
+            for (int c = 0; c < 4; ++c)
+#pragma unroll
+                for (int j = 0; j < RT; ++j) {
+                    acc[c][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(lo[j], wt[c], acc[c][j], 0, 0, 0);
+                    acc[c][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(hi[j], wt[c], acc[c][j], 0, 0, 0);
+                }
         }
-        __syncthreads();
-        const int m = min(RANK_CHUNK, rank - r0);
-        int r = 0;
-        for (; r + 8 <= m; r += 8) {
-            float w[8];
 #pragma unroll
-            for (int k = 0; k < 8; ++k) w[k] = load_f32(up + (size_t)(r0 + r + k) * cols);
+        for (int c = 0; c < 4; ++c) {
+            const int col = c_first + wave * 64 + c * 16 + m;
+            if (col >= cols) continue;
+            const float bias = is_decay ? p.dt_bias[col] : 0.f, rate = is_decay ? expf(p.a_log[col / p.R]) : 0.f;
 #pragma unroll
             for (int j = 0; j < RT; ++j)
 #pragma unroll
-                for (int k = 0; k < 8; ++k) acc[j] += w[k] * low[j][r + k];
+                for (int i = 0; i < 4; ++i) {
+                    const int t = t0 + j * 16 + kg * 4 + i;
+                    if (t < p.rows) out[(size_t)t * cols + col] = is_decay ? channel_decay(acc[c][j][i] + bias, rate) : acc[c][j][i];
+                }
         }
-        for (; r < m; ++r) {
-            const float w = load_f32(up + (size_t)(r0 + r) * cols);
+    } else {
+        __shared__ __attribute__((aligned(16))) float low[RT][RANK_CHUNK];
+        const int t0 = (b % p.row_tiles) * RT, c = c_first + tid, cc = min(c, cols - 1);
+        float acc[RT];
 #pragma unroll
-            for (int j = 0; j < RT; ++j) acc[j] += w * low[j][r];
+        for (int j = 0; j < RT; ++j) acc[j] = 0.f;
+        for (int r0 = 0; r0 < rank; r0 += RANK_CHUNK) {
+            __syncthreads();                                       // (the chunk before is used up)
+            for (int i = tid; i < RT * RANK_CHUNK; i += 256) {
+                const int j = i / RANK_CHUNK, r = r0 + i % RANK_CHUNK;
+                low[j][i % RANK_CHUNK] = r < rank ? p.in[(size_t)min(t0 + j, p.rows - 1) * p.ld + off + r] : 0.f;
+            }
+            __syncthreads();
+            const int m = min(RANK_CHUNK, rank - r0);
+            for (int r = 0; r < m; ++r) {
+                const float w = load_f32(up + (size_t)cc * ldu + r0 + r);
+#pragma unroll
+                for (int j = 0; j < RT; ++j) acc[j] += w * low[j][r];
+            }
         }
-    }
-    if (c >= cols) return;
-    const float bias = is_decay ? p.dt_bias[c] : 0.f, rate = is_decay ? expf(p.a_log[c / p.R]) : 0.f;
+        if (c >= cols) return;
+        const float bias = is_decay ? p.dt_bias[c] : 0.f, rate = is_decay ? expf(p.a_log[c / p.R]) : 0.f;
 #pragma unroll
-    for (int j = 0; j < RT; ++j) {
-        if (t0 + j >= p.rows) break;
-        if (is_decay) {
-            const float z = acc[j] + bias;
-            const float soft = fmaxf(z, 0.f) + log1pf(expf(-fabsf(z)));
-            p.decay[(size_t)(t0 + j) * cols + c] = expf(-rate * soft);
-        } else {
-            p.gate[(size_t)(t0 + j) * cols + c] = acc[j];
+        for (int j = 0; j < RT; ++j) {
+            if (t0 + j >= p.rows) break;
+            out[(size_t)(t0 + j) * cols + c] = is_decay ? channel_decay(acc[j] + bias, rate) : acc[j];
         }
     }
 }
@@ -140,38 +223,49 @@ channel_conv_state_kernel(const float* __restrict__ in, int ld, float* __restric
     }
 }
 
-template <bool SINGLE, typename TW>
-static int launch_channel_inputs(ChannelInputs& p, hipStream_t stream) {
-    const int inner = p.H * p.C, a_cols = p.H * p.R;
-    const long long items = (long long)p.rows * (2 * p.G + (inner + 255) / 256);
+template <bool SINGLE, int TAPS, typename TW>
+static int launch_channel_inputs_of(ChannelInputs& p, hipStream_t stream) {
+    const int inner = p.H * p.C, a_cols = p.H * p.R, run = TAPS ? 8 : 1;
+    const long long items = (long long)((p.rows + run - 1) / run) * (2 * p.G + (inner + 255) / 256);
     const int col_blocks = (a_cols + 255) / 256 + (inner + 255) / 256;
-    const int rt = p.rows >= 256 ? 16 : p.rows > 2 ? 4 : 1;       // rows a tile: many rows share a column's weights
+    constexpr int unit = sizeof(TW) == 2 ? 16 : 1;                // rows of a step of RT
+    const int rt = sizeof(TW) == 2 ? (p.rows > 128 ? 2 : 1) : (p.rows > 16 ? 16 : 1);      // many rows share a column's weights
     p.conv_blocks = (int)((items + 3) / 4);
-    p.row_tiles = (p.rows + rt - 1) / rt;
+    p.row_tiles = (p.rows + rt * unit - 1) / (rt * unit);
     const long long blocks = p.conv_blocks + (long long)p.row_tiles * col_blocks;
     if (blocks > 0x7fffffff) return (int)hipErrorInvalidValue;
-    if (rt == 16) channel_inputs_kernel<SINGLE, 16, TW><<<(unsigned)blocks, 256, 0, stream>>>(p);
-    else if (rt == 4) channel_inputs_kernel<SINGLE, 4, TW><<<(unsigned)blocks, 256, 0, stream>>>(p);
-    else channel_inputs_kernel<SINGLE, 1, TW><<<(unsigned)blocks, 256, 0, stream>>>(p);
+    if (rt == 1) channel_inputs_kernel<SINGLE, TAPS, 1, TW><<<(unsigned)blocks, 256, 0, stream>>>(p);
+    else channel_inputs_kernel<SINGLE, TAPS, sizeof(TW) == 2 ? 2 : 16, TW><<<(unsigned)blocks, 256, 0, stream>>>(p);
     return CISR_LAUNCH_CHECK();
 }
 
+template <typename TW>
+static int launch_channel_inputs(ChannelInputs& p, bool single, hipStream_t stream) {
+    if (single) return launch_channel_inputs_of<true, 0, TW>(p, stream);
+    if (p.taps == 2) return launch_channel_inputs_of<false, 2, TW>(p, stream);
+    if (p.taps == 3) return launch_channel_inputs_of<false, 3, TW>(p, stream);
+    if (p.taps == 4) return launch_channel_inputs_of<false, 4, TW>(p, stream);
+    return launch_channel_inputs_of<false, 0, TW>(p, stream);
+}
+
+// up_a [heads * R, ldu_a], up_g [heads * C, ldu_g]: rows of rank_a / rank_g coordinates, then zeros up to ldu; bf16 matrices
+// are read in 16-byte words of 32 coordinates a step, so their ldu is a multiple of 32 and they are 16-byte aligned.
 extern "C" int cisr_channel_inputs(const float* in, int ld, const float* taps_w, int taps, float* conv_state, long long slot_stride,
                                    float* qkv, const int* seg_of_row, const int* seg_start, const int* state_slots, int rows,
                                    int segments, int kv_heads, int R, int heads, int C, float unit_eps, int off_a, int rank_a,
-                                   const void* up_a, const float* dt_bias, const float* a_log, float* decay, int off_g, int rank_g,
-                                   const void* up_g, float* gate, int single_rows, int weight_dtype, hipStream_t stream) {
+                                   const void* up_a, int ldu_a, const float* dt_bias, const float* a_log, float* decay, int off_g,
+                                   int rank_g, const void* up_g, int ldu_g, float* gate, int single_rows, int weight_dtype, hipStream_t stream) {
     if (rows <= 0 || segments <= 0) return 0;
     const int channels = 2 * kv_heads * R + heads * C;
     if (kv_heads <= 0 || heads <= 0 || R <= 0 || R > 256 || C <= 0 || taps < 1 || taps > MAX_TAPS || rank_a <= 0 || rank_g <= 0 ||
-        channels > ld || off_a < 0 || off_a + rank_a > ld || off_g < 0 || off_g + rank_g > ld || segments > 65535)
+        channels > ld || off_a < 0 || off_a + rank_a > ld || off_g < 0 || off_g + rank_g > ld || segments > 65535 || ldu_a < rank_a ||
+        ldu_g < rank_g)
         return (int)hipErrorInvalidValue;
+    if (weight_dtype == DT_BF16 && (ldu_a % 32 || ldu_g % 32 || (uintptr_t)up_a % 16 || (uintptr_t)up_g % 16)) return (int)hipErrorInvalidValue;
     ChannelInputs p{in, ld, taps_w, taps, conv_state, slot_stride, qkv, seg_of_row, seg_start, state_slots, rows, kv_heads, R, heads, C,
-                    unit_eps, off_a, rank_a, up_a, dt_bias, a_log, decay, off_g, rank_g, up_g, gate, 0, 0};
-    if (single_rows)
-        return weight_dtype == DT_F32 ? launch_channel_inputs<true, float>(p, stream) : launch_channel_inputs<true, bf16_t>(p, stream);
-    const int err = weight_dtype == DT_F32 ? launch_channel_inputs<false, float>(p, stream) : launch_channel_inputs<false, bf16_t>(p, stream);
-    if (err || taps == 1) return err;
+                    unit_eps, off_a, rank_a, up_a, dt_bias, a_log, decay, off_g, rank_g, up_g, gate, ldu_a, ldu_g, 0, 0};
+    const int err = weight_dtype == DT_F32 ? launch_channel_inputs<float>(p, single_rows, stream) : launch_channel_inputs<bf16_t>(p, single_rows, stream);
+    if (err || taps == 1 || single_rows) return err;
     channel_conv_state_kernel<<<dim3(segments, (channels + 255) / 256), 256, 0, stream>>>(in, ld, conv_state, slot_stride, seg_start,
                                                                                        state_slots, channels, taps);
     return CISR_LAUNCH_CHECK();
@@ -362,4 +456,124 @@ extern "C" int cisr_channel_scan(const float* q, int ldq, const float* k, int ld
     if (cols == 8) return launch_channel_scan<16, 2>(p, segments, stream);
     if (cols == 16) return launch_channel_scan<8, 2>(p, segments, stream);
     return launch_channel_scan<4, 2>(p, segments, stream);
+}
+
+// ------------------------------------------------------------------------------------------------ a step of single rows
+// One row a segment: a block of 256 threads takes a head's whole state.  A thread owns four neighbouring columns of RPT
+// rows (16-byte accesses, runs of a whole row of the state), the 256 / (C / 4) groups of rows meet through LDS for S^T k
+// and for S^T q, and the block ends with the head's result, so it norms and gates it too:
+// act = o / rms(o) * weight * sigmoid(gate).
+struct ChannelStep {
+    ChannelScan s;
+    const float* gate; int ldgate;    // gate[t * ldgate + head * C + c]
+    const float* weight; float eps;   // [C]
+    void* act; int ldact;
+};
+
+template <int RPT, typename T>
+__global__ void __launch_bounds__(256) channel_step_kernel(ChannelStep a) {
+    const ChannelScan& p = a.s;
+    __shared__ float sk[256], sq[256], sg[256], red[4];
+    __shared__ __attribute__((aligned(16))) float4 part[256];
+    const int seg = blockIdx.x, head = blockIdx.y, tid = threadIdx.x;
+    const int t = p.seg_start[seg];
+    if (p.seg_start[seg + 1] <= t) return;
+    const int R = p.R, C = p.C, quads = C / 4, groups = 256 / quads;
+    const int quad = tid % quads, group = tid / quads;
+    const bool on = group < groups;                    // (256 need not be a multiple of the quads)
+    float4* state = (float4*)(p.state + (long long)p.state_slots[seg] * p.slot_stride + (size_t)head * R * C);
+    float4 S[RPT];
+#pragma unroll
+    for (int i = 0; i < RPT; ++i) {
+        const int r = group * RPT + i;
+        S[i] = on && r < R ? state[(size_t)r * quads + quad] : make_float4(0.f, 0.f, 0.f, 0.f);
+    }
+    if (tid < R) {
+        sk[tid] = p.k[(size_t)t * p.ldk + (size_t)(head / p.share) * R + tid];
+        sq[tid] = p.q[(size_t)t * p.ldq + (size_t)(head / p.share) * R + tid] * p.q_scale;
+        sg[tid] = p.g[(size_t)t * p.ldg + (size_t)head * R + tid];
+    } else {
+        sk[tid] = sq[tid] = sg[tid] = 0.f;
+    }
+    const float beta = 1.0f / (1.0f + expf(-p.b[(size_t)t * p.ldb + head]));
+    const float4 v = tid < quads ? make_float4(p.v[(size_t)t * p.ldv + (size_t)head * C + 4 * tid], p.v[(size_t)t * p.ldv + (size_t)head * C + 4 * tid + 1],
+                                               p.v[(size_t)t * p.ldv + (size_t)head * C + 4 * tid + 2], p.v[(size_t)t * p.ldv + (size_t)head * C + 4 * tid + 3])
+                                 : make_float4(0.f, 0.f, 0.f, 0.f);
+    __syncthreads();
+    // the sum of x over the groups, for the quad of this thread if it is one of the first `quads`
+    auto meet = [&](float4 x) {
+        part[tid] = x;
+        __syncthreads();
+        float4 sum = make_float4(0.f, 0.f, 0.f, 0.f);
+        if (tid < quads)
+            for (int g = 0; g < groups; ++g) {
+                const float4 y = part[g * quads + tid];
+                sum.x += y.x; sum.y += y.y; sum.z += y.z; sum.w += y.w;
+            }
+        return sum;
+    };
+    float4 d = make_float4(0.f, 0.f, 0.f, 0.f);
+#pragma unroll
+    for (int i = 0; i < RPT; ++i) {
+        const int r = min(group * RPT + i, 255);
+        const float g = sg[r], k = sk[r];
+        S[i].x *= g; S[i].y *= g; S[i].z *= g; S[i].w *= g;
+        d.x += S[i].x * k; d.y += S[i].y * k; d.z += S[i].z * k; d.w += S[i].w * k;
+    }
+    d = meet(d);
+    __syncthreads();
+    if (tid < quads) part[tid] = make_float4(beta * (v.x - d.x), beta * (v.y - d.y), beta * (v.z - d.z), beta * (v.w - d.w));
+    __syncthreads();
+    const float4 u = part[quad];
+    __syncthreads();
+    float4 o = make_float4(0.f, 0.f, 0.f, 0.f);
+#pragma unroll
+    for (int i = 0; i < RPT; ++i) {
+        const int r = group * RPT + i, rc = min(r, 255);
+        const float k = sk[rc], q = sq[rc];
+        S[i].x += k * u.x; S[i].y += k * u.y; S[i].z += k * u.z; S[i].w += k * u.w;
+        o.x += S[i].x * q; o.y += S[i].y * q; o.z += S[i].z * q; o.w += S[i].w * q;
+        if (on && r < R) state[(size_t)r * quads + quad] = S[i];
+    }
+    o = meet(o);
+    const float scale = 1.0f / sqrtf(block_sum<256>(o.x * o.x + o.y * o.y + o.z * o.z + o.w * o.w, red) / (float)C + a.eps);
+    if (tid >= quads) return;
+    const float* z = a.gate + (size_t)t * a.ldgate + (size_t)head * C + 4 * tid;
+    const float* w = a.weight + 4 * tid;
+    T* out = (T*)a.act + (size_t)t * a.ldact + (size_t)head * C + 4 * tid;
+    store_f32(out, o.x * scale * w[0] / (1.0f + expf(-z[0])));
+    store_f32(out + 1, o.y * scale * w[1] / (1.0f + expf(-z[1])));
+    store_f32(out + 2, o.z * scale * w[2] / (1.0f + expf(-z[2])));
+    store_f32(out + 3, o.w * scale * w[3] / (1.0f + expf(-z[3])));
+}
+
+// Rows of the state a thread owns, or 0 if the step kernel does not take these sizes.
+static int channel_step_rows(int R, int C, long long slot_stride) {
+    if (C % 4 || C < 4 || C > 1024 || R > 256 || slot_stride % 4) return 0;
+    const int groups = 256 / (C / 4), per = (R + groups - 1) / groups;
+    return per <= 4 ? 4 : per <= 8 ? 8 : per <= 16 ? 16 : per <= 32 ? 32 : 0;
+}
+
+extern "C" int cisr_channel_step_ok(int R, int C, long long slot_stride) { return channel_step_rows(R, C, slot_stride) > 0; }
+
+extern "C" int cisr_channel_step(const float* q, int ldq, const float* k, int ldk, const float* v, int ldv, const float* g, int ldg,
+                                 const float* b, int ldb, float* state, long long slot_stride, const int* seg_start,
+                                 const int* state_slots, int segments, int heads, int R, int C, int share, float q_scale,
+                                 const float* gate, int ldgate, const float* weight, float eps, void* act, int ldact, int dtype,
+                                 hipStream_t stream) {
+    if (segments <= 0 || heads <= 0) return 0;
+    const int per = channel_step_rows(R, C, slot_stride);
+    if (!per || R <= 0 || share <= 0 || heads % share || heads > 65535 || (uintptr_t)state % 16) return (int)hipErrorInvalidValue;
+    ChannelStep a{{q, ldq, k, ldk, v, ldv, g, ldg, b, ldb, nullptr, 0, state, slot_stride, seg_start, state_slots, R, C, share, heads, q_scale},
+                  gate, ldgate, weight, eps, act, ldact};
+    const dim3 grid(segments, heads);
+#define CHANNEL_STEP(RPT) \
+    if (dtype == DT_F32) channel_step_kernel<RPT, float><<<grid, 256, 0, stream>>>(a); \
+    else channel_step_kernel<RPT, bf16_t><<<grid, 256, 0, stream>>>(a)
+    if (per == 4) { CHANNEL_STEP(4); }
+    else if (per == 8) { CHANNEL_STEP(8); }
+    else if (per == 16) { CHANNEL_STEP(16); }
+    else { CHANNEL_STEP(32); }
+#undef CHANNEL_STEP
+    return CISR_LAUNCH_CHECK();
 }

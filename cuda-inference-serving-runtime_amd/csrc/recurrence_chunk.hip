@@ -1,0 +1,303 @@
+// The gated delta rule with a decay a key channel over prompt portions, chunk by chunk on the matrix cores (float operands,
+// v_mfma_f32_16x16x4_f32).  A segment's rows in chunks of 16; with D(t, i) the product of a chunk's decays g_(i+1) .. g_t,
+// channel by channel, D(t) that of g_0 .. g_t, and S0 the state at the chunk's start:
+//
+//   A[t, i] = beta_t sum_r k_t k_i D(t, i), i < t          P[t, i] = sum_r q_t k_i D(t, i), i <= t
+//   M = (I + A)^-1 diag(beta)
+//   U = M (V - Kg S0),   Kg_t = D(t) k_t                      (the rows' writes u_t)
+//   o_t = (D(t) q_t)^T S0 + sum_i P[t, i] u_i
+//   S  <- D(15) S0 + sum_i (D(15, i) k_i) u_i^T
+//
+// Every product of decays is made by multiplying decays along the rows: no quotients and no differences of logarithms, so a
+// channel whose decays vanish within a chunk costs neither range nor precision.  A first kernel makes, chunk by chunk and
+// all side by side, what does not need the state: M V, M Kg, D q, P, D(15, i) k and D(15); a second walks a segment's chunks
+// in order, a block a (head, 16 columns of S): its four waves own the rows of S in turn, two products with S0, one meeting
+// through LDS, one product into S.  Rows behind a segment's end count as k = q = v = 0 with decays of one.
+#include "common.h"
+
+#define CHUNK 16
+
+typedef __attribute__((ext_vector_type(4))) float f32x4_t;
+
+struct ChunkArgs {
+    const float* q; int ldq;          // q[t * ldq + (head / share) * R + r]
+    const float* k; int ldk;
+    const float* v; int ldv;          // v[t * ldv + head * C + c]
+    const float* g; int ldg;          // g[t * ldg + head * R + r]
+    const float* b; int ldb;          // b[t * ldb + head], beta = sigmoid(b)
+    float* out; int ldo;
+    float* state; long long slot_stride;
+    const int* seg_start; const int* state_slots;
+    int R, C, share, heads, segments;
+    float q_scale;
+    int Rp, Cp;                       // R and C rounded up to 16
+    int slot0, slots;                 // this launch's chunk slots (a chunk's slot: seg_start / 16 + segment + its number)
+    float* work;                      // [slots][heads][chunk_floats]
+};
+
+// Floats of a (chunk, head): M Kg and D q as [16][Rp], D(15, i) k as [Rp][16], M V as [Cp][16], P as [16][16], D(15) [Rp].
+__host__ __device__ __forceinline__ int chunk_floats(int Rp, int Cp) { return 3 * CHUNK * Rp + CHUNK * Cp + CHUNK * CHUNK + Rp; }
+
+// The segment whose chunk slots hold `slot` (segments without rows own a slot without a chunk).
+__device__ __forceinline__ int segment_of_slot(const int* seg_start, int segments, int slot) {
+    int lo = 0, hi = segments - 1;
+    while (lo < hi) {
+        const int mid = (lo + hi + 1) / 2;
+        if (seg_start[mid] / CHUNK + mid <= slot) lo = mid; else hi = mid - 1;
+    }
+    return lo;
+}
+
+template <int CTRL>
+__device__ __forceinline__ float lanes_moved(float x) {
+    return __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(x), CTRL, 0xF, 0xF, false));
+}
+
+// the sum over the 16 lanes of an aligned row, in each of them
+__device__ __forceinline__ float row_sum(float x) {
+    x += lanes_moved<0xB1>(x);                   // quad_perm [1, 0, 3, 2]
+    x += lanes_moved<0x4E>(x);                   // quad_perm [2, 3, 0, 1]
+    x += lanes_moved<0x141>(x);                  // row_half_mirror
+    x += lanes_moved<0x140>(x);                  // row_mirror
+    return x;
+}
+
+__global__ void __launch_bounds__(256, 3) channel_chunk_kernel(ChunkArgs p) {
+    extern __shared__ __attribute__((aligned(16))) float lds[];
+    __shared__ float sA[CHUNK][CHUNK + 1], sM[CHUNK][CHUNK], sBeta[CHUNK];
+    const int slot = p.slot0 + blockIdx.y, head = blockIdx.x, tid = threadIdx.x;
+    const int seg = segment_of_slot(p.seg_start, p.segments, slot);
+    const int t0 = p.seg_start[seg] + (slot - p.seg_start[seg] / CHUNK - seg) * CHUNK, t1 = p.seg_start[seg + 1];
+    if (t0 >= t1 || t0 < p.seg_start[seg]) return;
+    const int n = min(CHUNK, t1 - t0), R = p.R, C = p.C, Rp = p.Rp, RS = Rp + 4;
+    float* sk = lds;
+    float* sq = sk + CHUNK * RS;
+    float* sg = sq + CHUNK * RS;
+    const float* kh = p.k + (size_t)(head / p.share) * R;
+    const float* qh = p.q + (size_t)(head / p.share) * R;
+    const float* gh = p.g + (size_t)head * R;
+    for (int r = tid; r < Rp; r += 256) {        // a thread a channel
+#pragma unroll
+        for (int i = 0; i < CHUNK; ++i) {
+            const size_t t = (size_t)(t0 + min(i, n - 1));
+            const bool in = r < R && i < n;
+            const int rr = min(r, R - 1);
+            const float k = kh[t * p.ldk + rr], q = qh[t * p.ldq + rr], g = gh[t * p.ldg + rr];
+            sk[i * RS + r] = in ? k : 0.f;
+            sq[i * RS + r] = in ? q * p.q_scale : 0.f;
+            sg[i * RS + r] = in ? g : 1.f;
+        }
+    }
+    if (tid < CHUNK) sBeta[tid] = tid < n ? 1.0f / (1.0f + expf(-p.b[(size_t)(t0 + tid) * p.ldb + head])) : 0.f;
+    __syncthreads();
+    float* work = p.work + ((size_t)blockIdx.y * p.heads + head) * chunk_floats(Rp, p.Cp);
+    float* wP = work + 3 * CHUNK * Rp + CHUNK * p.Cp;
+    // column i of A and P: sixteen neighbouring threads, each with every sixteenth run of four channels, carry k_i down the
+    // rows behind i (times their decays) and meet
+    {
+        const int i = tid / 16, part = tid % 16;
+        float a[CHUNK], b[CHUNK];
+#pragma unroll
+        for (int t = 0; t < CHUNK; ++t) a[t] = b[t] = 0.f;
+        for (int r = 4 * part; r < Rp; r += 64) {
+            f32x4_t x = *(const f32x4_t*)(sk + i * RS + r);
+#pragma unroll
+            for (int t = 0; t < CHUNK; ++t) {
+                if (t < i) continue;
+                const f32x4_t q = *(const f32x4_t*)(sq + t * RS + r);
+                if (t > i) {
+                    const f32x4_t k = *(const f32x4_t*)(sk + t * RS + r);
+                    x *= *(const f32x4_t*)(sg + t * RS + r);
+                    a[t] += (x[0] * k[0] + x[1] * k[1]) + (x[2] * k[2] + x[3] * k[3]);
+                }
+                b[t] += (x[0] * q[0] + x[1] * q[1]) + (x[2] * q[2] + x[3] * q[3]);
+            }
+        }
+#pragma unroll
+        for (int t = 0; t < CHUNK; ++t) {
+            const float at = row_sum(a[t]), bt = row_sum(b[t]);
+            if (part == t) {
+                if (t > i) sA[t][i] = sBeta[t] * at;
+                wP[t * CHUNK + i] = t >= i ? bt : 0.f;
+            }
+        }
+    }
+    __syncthreads();
+    // column j of the inverse of the unit triangle I + A by forward substitution, times beta_j
+    if (tid < CHUNK) {
+        float x[CHUNK];
+#pragma unroll
+        for (int t = 0; t < CHUNK; ++t) {
+            float s = t == tid ? 1.f : 0.f;
+#pragma unroll
+            for (int i = 0; i < t; ++i) s -= sA[t][i] * x[i];
+            x[t] = s;
+        }
+#pragma unroll
+        for (int t = 0; t < CHUNK; ++t) sM[t][tid] = x[t] * sBeta[tid];
+    }
+    __syncthreads();
+    // a thread a channel (M Kg and the other operands over the state's rows) or a column of v (M V)
+    for (int idx = tid; idx < Rp + p.Cp; idx += 256) {
+        const bool key = idx < Rp;
+        const int c = key ? idx : idx - Rp;
+        float x[CHUNK];
+        if (key) {
+            float* wq = work + CHUNK * Rp + c;
+            float* wk = work + 2 * CHUNK * Rp + (size_t)c * CHUNK;
+            float d = 1.f, kd[CHUNK];
+#pragma unroll
+            for (int i = 0; i < CHUNK; ++i) {
+                d *= sg[i * RS + c];
+                x[i] = sk[i * RS + c] * d;
+                wq[(size_t)i * Rp] = sq[i * RS + c] * d;
+            }
+            work[3 * CHUNK * Rp + CHUNK * p.Cp + CHUNK * CHUNK + c] = d;
+            d = 1.f;
+#pragma unroll
+            for (int i = CHUNK - 1; i >= 0; --i) {
+                kd[i] = sk[i * RS + c] * d;
+                d *= sg[i * RS + c];
+            }
+#pragma unroll
+            for (int i = 0; i < CHUNK; i += 4) *(f32x4_t*)(wk + i) = (f32x4_t){kd[i], kd[i + 1], kd[i + 2], kd[i + 3]};
+        } else {
+#pragma unroll
+            for (int i = 0; i < CHUNK; ++i) x[i] = i < n && c < C ? p.v[(size_t)(t0 + min(i, n - 1)) * p.ldv + (size_t)head * C + min(c, C - 1)] : 0.f;
+        }
+        float y[CHUNK];
+#pragma unroll
+        for (int t = 0; t < CHUNK; ++t) {
+            float s = 0.f;
+#pragma unroll
+            for (int i = 0; i <= t; ++i) s += sM[t][i] * x[i];
+            y[t] = s;
+        }
+        if (key) {
+#pragma unroll
+            for (int t = 0; t < CHUNK; ++t) work[(size_t)t * Rp + c] = y[t];
+        } else {
+            float* wv = work + 3 * CHUNK * Rp + (size_t)c * CHUNK;
+#pragma unroll
+            for (int t = 0; t < CHUNK; t += 4) *(f32x4_t*)(wv + t) = (f32x4_t){y[t], y[t + 1], y[t + 2], y[t + 3]};
+        }
+    }
+}
+
+// A block a (head, segment, 16 columns).  The state's rows in tiles of 16: wave w owns the tiles w NT .. w NT + NT - 1, in
+// the matrix instruction's result layout (lane l: rows 4 (l / 16) + i of the tile, column l % 16), which serves as its
+// right operand as it is when the left operand's inner index runs alike: every operand is a 16-byte load.
+template <int NT>
+__global__ void __launch_bounds__(256) channel_walk_kernel(ChunkArgs p) {
+    __shared__ f32x4_t meet[2][2][4][WAVE];         // [chunk parity][M Kg S0, (D q) S0][wave][lane]
+    const int head = blockIdx.x, seg = blockIdx.z, wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
+    const int t0 = p.seg_start[seg], t1 = p.seg_start[seg + 1];
+    if (t1 <= t0) return;
+    const int base = t0 / CHUNK + seg, chunks = (t1 - t0 + CHUNK - 1) / CHUNK;
+    const int first = max(base, p.slot0), last = min(base + chunks, p.slot0 + p.slots);
+    if (first >= last) return;
+    const int m = lane % 16, kg = lane / 16, R = p.R, C = p.C, Rp = p.Rp;
+    const int c = blockIdx.y * 16 + m;
+    float* state = p.state + (long long)p.state_slots[seg] * p.slot_stride + (size_t)head * R * C;
+    f32x4_t S[NT];
+#pragma unroll
+    for (int j = 0; j < NT; ++j)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            const int r = (wave * NT + j) * 16 + 4 * kg + i;
+            S[j][i] = r < R && c < C ? state[(size_t)r * C + c] : 0.f;
+        }
+    struct Operands { f32x4_t kg[NT], qg[NT], kd[NT], g[NT], u, pr; } now, next;
+    const size_t per = (size_t)chunk_floats(Rp, p.Cp);
+    auto fetch = [&](Operands& o, int slot) {
+        const float* w = p.work + ((size_t)(slot - p.slot0) * p.heads + head) * per;
+#pragma unroll
+        for (int j = 0; j < NT; ++j) {
+            const int r = min((wave * NT + j) * 16, Rp - 16);          // (a wave without this tile reads another: its S is zero)
+            o.kg[j] = *(const f32x4_t*)(w + (size_t)m * Rp + r + 4 * kg);
+            o.qg[j] = *(const f32x4_t*)(w + (size_t)(CHUNK + m) * Rp + r + 4 * kg);
+            o.kd[j] = *(const f32x4_t*)(w + (size_t)2 * CHUNK * Rp + (size_t)(r + m) * CHUNK + 4 * kg);
+            o.g[j] = *(const f32x4_t*)(w + (size_t)3 * CHUNK * Rp + (size_t)CHUNK * p.Cp + CHUNK * CHUNK + r + 4 * kg);
+        }
+        o.u = *(const f32x4_t*)(w + (size_t)3 * CHUNK * Rp + (size_t)c * CHUNK + 4 * kg);
+        o.pr = *(const f32x4_t*)(w + (size_t)3 * CHUNK * Rp + (size_t)CHUNK * p.Cp + m * CHUNK + 4 * kg);
+    };
+    fetch(now, first);
+    for (int slot = first; slot < last; ++slot) {
+        const int par = slot & 1;
+        if (slot + 1 < last) fetch(next, slot + 1);
+        f32x4_t w = {0.f, 0.f, 0.f, 0.f}, o = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int j = 0; j < NT; ++j)
+#pragma unroll
+            for (int i = 0; i < 4; ++i) w = __builtin_amdgcn_mfma_f32_16x16x4f32(now.kg[j][i], S[j][i], w, 0, 0, 0);
+        meet[par][0][wave][lane] = w;
+#pragma unroll
+        for (int j = 0; j < NT; ++j)
+#pragma unroll
+            for (int i = 0; i < 4; ++i) o = __builtin_amdgcn_mfma_f32_16x16x4f32(now.qg[j][i], S[j][i], o, 0, 0, 0);
+        meet[par][1][wave][lane] = o;
+        __syncthreads();                       // (the other parity's buffers were read before the barrier before this one's writes)
+        f32x4_t u = now.u - ((meet[par][0][0][lane] + meet[par][0][1][lane]) + (meet[par][0][2][lane] + meet[par][0][3][lane]));
+#pragma unroll
+        for (int j = 0; j < NT; ++j) {
+            const bool own = (wave * NT + j) * 16 < Rp;
+            S[j] *= now.g[j];
+            if (own)
+#pragma unroll
+                for (int i = 0; i < 4; ++i) S[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(now.kd[j][i], u[i], S[j], 0, 0, 0);
+        }
+        if (wave == (slot & 3)) {              // (the waves finish a chunk's result in turn)
+            f32x4_t y = (meet[par][1][0][lane] + meet[par][1][1][lane]) + (meet[par][1][2][lane] + meet[par][1][3][lane]);
+#pragma unroll
+            for (int i = 0; i < 4; ++i) y = __builtin_amdgcn_mfma_f32_16x16x4f32(now.pr[i], u[i], y, 0, 0, 0);
+            const int row = t0 + (slot - base) * CHUNK + 4 * kg;
+#pragma unroll
+            for (int i = 0; i < 4; ++i)
+                if (row + i < t1 && c < C) p.out[(size_t)(row + i) * p.ldo + (size_t)head * C + c] = y[i];
+        }
+        now = next;
+    }
+#pragma unroll
+    for (int j = 0; j < NT; ++j)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            const int r = (wave * NT + j) * 16 + 4 * kg + i;
+            if (r < R && c < C) state[(size_t)r * C + c] = S[j][i];
+        }
+}
+
+// Chunk slots of a step, and floats of `work` a slot takes.
+extern "C" int cisr_channel_chunk_slots(int rows, int segments) { return rows / CHUNK + segments; }
+extern "C" long long cisr_channel_chunk_floats(int heads, int R, int C) {
+    return (long long)heads * chunk_floats((R + 15) / 16 * 16, (C + 15) / 16 * 16);
+}
+
+// The step's rows in launches of `slab` chunk slots each (two kernels a slab); work: slab * cisr_channel_chunk_floats floats.
+extern "C" int cisr_channel_chunks(const float* q, int ldq, const float* k, int ldk, const float* v, int ldv, const float* g, int ldg,
+                                   const float* b, int ldb, float* out, int ldo, float* state, long long slot_stride,
+                                   const int* seg_start, const int* state_slots, int rows, int segments, int heads, int R, int C,
+                                   int share, float q_scale, float* work, int slab, hipStream_t stream) {
+    if (rows <= 0 || segments <= 0 || heads <= 0) return 0;
+    if (R <= 0 || R > 256 || C <= 0 || share <= 0 || heads % share || segments > 65535 || (C + 15) / 16 > 65535 || slab <= 0 || slab > 65535 ||
+        (uintptr_t)work % 16)
+        return (int)hipErrorInvalidValue;
+    ChunkArgs p{q, ldq, k, ldk, v, ldv, g, ldg, b, ldb, out, ldo, state, slot_stride, seg_start, state_slots, R, C, share, heads, segments,
+                q_scale, (R + 15) / 16 * 16, (C + 15) / 16 * 16, 0, 0, work};
+    const int total = rows / CHUNK + segments, nt = (p.Rp / 16 + 3) / 4;
+    const size_t lds = (size_t)3 * CHUNK * (p.Rp + 4) * sizeof(float);
+    for (p.slot0 = 0; p.slot0 < total; p.slot0 += slab) {
+        p.slots = min(slab, total - p.slot0);
+        channel_chunk_kernel<<<dim3(heads, p.slots), 256, lds, stream>>>(p);
+        int err = CISR_LAUNCH_CHECK();
+        if (err) return err;
+        const dim3 grid(heads, p.Cp / 16, segments);
+        if (nt == 1) channel_walk_kernel<1><<<grid, 256, 0, stream>>>(p);
+        else if (nt == 2) channel_walk_kernel<2><<<grid, 256, 0, stream>>>(p);
+        else if (nt == 3) channel_walk_kernel<3><<<grid, 256, 0, stream>>>(p);
+        else channel_walk_kernel<4><<<grid, 256, 0, stream>>>(p);
+        err = CISR_LAUNCH_CHECK();
+        if (err) return err;
+    }
+    return 0;
+}

@@ -1282,7 +1282,11 @@ def _rec():
             "cisr_group_norm_gate": [p, p, i, p, i, p, i, p, i, p, i, i, i, f, i, i, i, p],
             "cisr_delta_scan": [p, i, p, i, p, i, p, i, p, i, p, i, p, ll, p, p, i, i, i, i, i, f, i, p],
             "cisr_unit_heads": [p, i, i, i, i, i, f, f, p],
-            "cisr_channel_inputs": [p, i, p, i, p, ll, p, p, p, p, i, i, i, i, i, i, f, i, i, p, p, p, p, i, i, p, p, i, i, p],
+            "cisr_channel_inputs": [p, i, p, i, p, ll, p, p, p, p, i, i, i, i, i, i, f, i, i, p, i, p, p, p, i, i, p, i, p, i, i, p],
+            "cisr_channel_step": [p, i, p, i, p, i, p, i, p, i, p, ll, p, p, i, i, i, i, i, f, p, i, p, f, p, i, i, p],
+            "cisr_channel_step_ok": [i, i, ll],
+            "cisr_channel_chunks": [p, i, p, i, p, i, p, i, p, i, p, i, p, ll, p, p, i, i, i, i, i, i, f, p, i, p],
+            "cisr_channel_chunk_slots": [i, i],
             "cisr_channel_scan": [p, i, p, i, p, i, p, i, p, i, p, i, p, ll, p, p, i, i, i, i, i, f, i, p],
             "cisr_mingru_scan": [p, i, p, p, p, i, p, p, p, i, i, i, i, p, i, i, p],
             "cisr_mlstm_gates": [p, i, p, i, p, p, p, i, p, p, p, p, p, ll, p, p, i, i, i, i, f, i, p],
@@ -1294,6 +1298,8 @@ def _rec():
             fn.restype = C.c_int
         h.cisr_linear_scan_carry.argtypes = [i, i, i, i, i, i, C.POINTER(ll)]
         h.cisr_linear_scan_carry.restype = ll
+        h.cisr_channel_chunk_floats.argtypes = [i, i, i]
+        h.cisr_channel_chunk_floats.restype = ll
         _recurrence = h
     return _recurrence
 
@@ -1502,14 +1508,26 @@ def delta_scan(q, k, v, decay, write, out, state, seg_start, state_slots, heads,
     return out
 
 
+def low_rank_rows(w):
+    """The second half of a low-rank projection, [columns, rank], as channel_delta_inputs reads it: bf16 rows padded with
+    zeros to a multiple of 32 coordinates (a view of the rank, whose row stride says so); float rows as they are."""
+    if w.dtype != torch.bfloat16:
+        return w.contiguous()
+    rank = w.shape[1]
+    out = torch.zeros(w.shape[0], -(-rank // 32) * 32, dtype=w.dtype, device=w.device)
+    out[:, :rank] = w
+    return out[:, :rank]
+
+
 def channel_delta_inputs(proj, taps, conv_state, qkv, seg_of_row, seg_start, state_slots, kv_heads, dim, heads, vdim, decay_at, decay_up,
                          dt_bias, a_log, decay, gate_at, gate_up, gate, unit_eps=1e-6, single_rows=False):
-    """The operands of channel_delta_scan from the float rows of an input product, proj [T, >= ...]: its first channels =
-    2 kv_heads dim + heads vdim columns [q | k | v] go through the causal convolution (taps float [K, channels], taps[K - 1]
-    weighs the newest input; the K - 1 inputs before a segment from conv_state, a float view [slots, >= (K - 1) channels],
-    which moves on) and silu, and the heads of q and k become unit vectors: qkv float [T, channels].  decay [T, heads * dim]
-    = exp(-exp(a_log) softplus(proj[:, decay_at:] . decay_up + dt_bias)), decay_up [rank, heads * dim]; gate [T, heads * vdim]
-    = proj[:, gate_at:] . gate_up, gate_up [rank, heads * vdim] (both of one dtype, float or bf16; the sums are float)."""
+    """The operands of the delta rule with a decay a channel from the float rows of an input product, proj [T, >= ...]: its
+    first channels = 2 kv_heads dim + heads vdim columns [q | k | v] go through the causal convolution (taps float [K,
+    channels], taps[K - 1] weighs the newest input; the K - 1 inputs before a segment from conv_state, a float view [slots, >=
+    (K - 1) channels], which moves on) and silu, and the heads of q and k become unit vectors: qkv float [T, channels].
+    decay [T, heads * dim] = exp(-exp(a_log) softplus(proj[:, decay_at:] . decay_up^T + dt_bias)), decay_up [heads * dim,
+    rank]; gate [T, heads * vdim] = proj[:, gate_at:] . gate_up^T, gate_up [heads * vdim, rank] (both as low_rank_rows makes
+    them, float or bf16; with bf16 matrices the projections' coordinates enter as two bf16 numbers each, on the matrix cores)."""
     T = qkv.shape[0]
     pp, ld = _rows_of(proj, "proj")
     K, channels = taps.shape
@@ -1519,17 +1537,24 @@ def channel_delta_inputs(proj, taps, conv_state, qkv, seg_of_row, seg_start, sta
     if (conv_state.dtype != torch.float32 or not conv_state.is_cuda or conv_state.stride(1) != 1
             or conv_state.shape[1] < (K - 1) * channels):
         raise KernelError("channel_delta_inputs: the state must be float [slots, >= (K - 1) * channels]")
-    ra, rg = decay_up.shape[0], gate_up.shape[0]
+
+    def up(w, cols, name):
+        if not w.is_cuda or w.dim() != 2 or w.shape[0] != cols or w.stride(1) != 1 or w.stride(0) < w.shape[1] or w.untyped_storage().nbytes() < (
+                w.storage_offset() + cols * w.stride(0)) * w.element_size():
+            raise KernelError(f"channel_delta_inputs: {name} must be the rows [{cols}, rank] that low_rank_rows makes")
+        return w.data_ptr(), w.stride(0), w.shape[1]
+
+    ap, lda, ra = up(decay_up, heads * dim, "decay_up")
+    gp, ldg, rg = up(gate_up, heads * vdim, "gate_up")
     if decay_up.dtype != gate_up.dtype or decay_at + ra > proj.shape[1] or gate_at + rg > proj.shape[1]:
         raise KernelError("channel_delta_inputs: low-rank columns beyond the rows, or matrices of two dtypes")
     _check(_rec().cisr_channel_inputs(pp, ld, _dev(taps, "taps", torch.float32), K, conv_state.data_ptr(), conv_state.stride(0),
                                       _dev(qkv, "qkv", torch.float32, (T, channels)), _dev(seg_of_row, "seg_of_row", torch.int32, (T,)),
                                       _dev(seg_start, "seg_start", torch.int32, (segments + 1,)),
                                       _dev(state_slots, "state_slots", torch.int32, (segments,)), T, segments, kv_heads, dim, heads, vdim,
-                                      float(unit_eps), int(decay_at), ra, _dev(decay_up, "decay_up", None, (ra, heads * dim)),
-                                      _dev(dt_bias, "dt_bias", torch.float32, (heads * dim,)), _dev(a_log, "a_log", torch.float32, (heads,)),
-                                      _dev(decay, "decay", torch.float32, (T, heads * dim)), int(gate_at), rg,
-                                      _dev(gate_up, "gate_up", None, (rg, heads * vdim)), _dev(gate, "gate", torch.float32, (T, heads * vdim)),
+                                      float(unit_eps), int(decay_at), ra, ap, lda, _dev(dt_bias, "dt_bias", torch.float32, (heads * dim,)),
+                                      _dev(a_log, "a_log", torch.float32, (heads,)), _dev(decay, "decay", torch.float32, (T, heads * dim)),
+                                      int(gate_at), rg, gp, ldg, _dev(gate, "gate", torch.float32, (T, heads * vdim)),
                                       int(bool(single_rows)), _storage(decay_up, "decay_up"), _stream()), "channel_delta_inputs")
     return qkv
 
@@ -1541,32 +1566,89 @@ def channel_columns(segments, heads, cols):
             return width
 
 
+def _channel_operands(name, q, k, v, decay, write, state, seg_start, state_slots, heads, R, C_, share):
+    """Checked pointers and strides that the forms of the delta rule with decays a channel share."""
+    T, segments = v.shape[0], state_slots.shape[0]
+    if heads % share or R > 256:
+        raise KernelError(f"{name}: heads must divide into their groups and a state has at most 256 rows")
+    args = (*_rows_of(q, "q", heads // share * R), *_rows_of(k, "k", heads // share * R), *_rows_of(v, "v", heads * C_),
+            *_rows_of(decay, "decay", heads * R), *_rows_of(write, "write", heads))
+    if any(t.shape[0] != T for t in (q, k, decay, write)):
+        raise KernelError(f"{name}: operands differ in rows")
+    if state.dtype != torch.float32 or state.dim() != 2 or state.stride(1) != 1 or state.shape[1] < heads * R * C_ or not state.is_cuda:
+        raise KernelError(f"{name}: the state must be float [slots, >= heads * R * C]")
+    return args, (state.data_ptr(), state.stride(0), _dev(seg_start, "seg_start", torch.int32, (segments + 1,)),
+                  _dev(state_slots, "state_slots", torch.int32, (segments,)))
+
+
 def channel_delta_scan(q, k, v, decay, write, out, state, seg_start, state_slots, heads, rows_of_state, cols_of_state, share=1,
                        q_scale=1.0, columns=None):
     """delta_scan with a decay a head and key channel: per segment and head, over the segment's rows in order, S <- diag(g)
     S; u = sigmoid(b) (v - S^T k); S <- S + k u^T; o = q_scale S^T q.  decay (g) [T, heads * R]; everything else as there."""
     R, Cc = int(rows_of_state), int(cols_of_state)
-    T = v.shape[0]
     segments = state_slots.shape[0]
-    if heads % share or R > 256:
-        raise KernelError("channel_delta_scan: heads must divide into their groups and a state has at most 256 rows")
-    qp, ldq = _rows_of(q, "q", heads // share * R)
-    kp, ldk = _rows_of(k, "k", heads // share * R)
-    vp, ldv = _rows_of(v, "v", heads * Cc)
+    args, where = _channel_operands("channel_delta_scan", q, k, v, decay, write, state, seg_start, state_slots, heads, R, Cc, share)
     op, ldo = _rows_of(out, "out", heads * Cc)
-    gp, ldg = _rows_of(decay, "decay", heads * R)
-    bp, ldb = _rows_of(write, "write", heads)
-    if any(t.shape[0] != T for t in (q, k, decay, write, out)):
+    if out.shape[0] != v.shape[0]:
         raise KernelError("channel_delta_scan: operands differ in rows")
-    if state.dtype != torch.float32 or state.dim() != 2 or state.stride(1) != 1 or state.shape[1] < heads * R * Cc or not state.is_cuda:
-        raise KernelError("channel_delta_scan: the state must be float [slots, >= heads * R * C]")
     cols = int(columns or channel_columns(segments, heads, Cc))
     while columns is None and cols > 8 and -(-R // (128 // cols)) > 32:
         cols //= 2         # (at most 32 rows of its two columns a lane)
-    _check(_rec().cisr_channel_scan(qp, ldq, kp, ldk, vp, ldv, gp, ldg, bp, ldb, op, ldo, state.data_ptr(), state.stride(0),
-                                    _dev(seg_start, "seg_start", torch.int32, (segments + 1,)),
-                                    _dev(state_slots, "state_slots", torch.int32, (segments,)), segments, heads, R, Cc,
-                                    int(share), float(q_scale), cols, _stream()), "channel_delta_scan")
+    _check(_rec().cisr_channel_scan(*args, op, ldo, *where, segments, heads, R, Cc, int(share), float(q_scale), cols, _stream()),
+           "channel_delta_scan")
+    return out
+
+
+CHANNEL_CHUNK_ROWS = 32       # rows beyond one a segment from which a step's portions are walked chunk by chunk
+CHANNEL_SLAB = 160            # chunks whose operands wait in memory at one time (2,048 rows of one request and some)
+
+
+def channel_chunked(rows, segments, decode_only):
+    """Whether a step walks the delta rule with decays a channel chunk by chunk (channel_delta_chunks): portions long
+    enough that some 16-row chunks fill; short ones are walked row by row."""
+    return not decode_only and rows - segments >= CHANNEL_CHUNK_ROWS
+
+
+def channel_chunk_work(rows, segments, heads, rows_of_state, cols_of_state, slab=CHANNEL_SLAB):
+    """Floats of `work` that channel_delta_chunks needs for a step of `rows` rows in `segments` segments."""
+    slots = int(_rec().cisr_channel_chunk_slots(int(rows), int(segments)))
+    return min(slots, int(slab)) * int(_rec().cisr_channel_chunk_floats(int(heads), int(rows_of_state), int(cols_of_state)))
+
+
+def channel_delta_chunks(q, k, v, decay, write, out, state, seg_start, state_slots, heads, rows_of_state, cols_of_state, work, share=1,
+                         q_scale=1.0, slab=CHANNEL_SLAB):
+    """channel_delta_scan in chunks of 16 rows on the matrix cores with float operands: the same results up to rounding.
+    work: float, at least channel_chunk_work(...) elements; `slab`: chunks that one pair of launches takes."""
+    R, Cc = int(rows_of_state), int(cols_of_state)
+    T, segments = v.shape[0], state_slots.shape[0]
+    args, where = _channel_operands("channel_delta_chunks", q, k, v, decay, write, state, seg_start, state_slots, heads, R, Cc, share)
+    op, ldo = _rows_of(out, "out", heads * Cc)
+    if out.shape[0] != T or work.numel() < channel_chunk_work(T, segments, heads, R, Cc, slab):
+        raise KernelError("channel_delta_chunks: too few result rows, or too little work space")
+    _check(_rec().cisr_channel_chunks(*args, op, ldo, *where, T, segments, heads, R, Cc, int(share), float(q_scale),
+                                      _dev(work, "work", torch.float32), int(slab), _stream()), "channel_delta_chunks")
+    return out
+
+
+def channel_step_ok(state, rows_of_state, cols_of_state):
+    """Whether channel_delta_step takes states of these sizes."""
+    return state.data_ptr() % 16 == 0 and bool(_rec().cisr_channel_step_ok(int(rows_of_state), int(cols_of_state), int(state.stride(0))))
+
+
+def channel_delta_step(q, k, v, decay, write, gate, weight, out, state, seg_start, state_slots, heads, rows_of_state, cols_of_state,
+                       eps, share=1, q_scale=1.0):
+    """channel_delta_scan over segments of one row each (the caller vouches for that), with the result's norm and gate in
+    the same kernel: out[t, h] = o / rms(o) * weight * sigmoid(gate), rms over the head's columns with eps; gate a float
+    view [T, heads * C], weight float [C], out [T, heads * C] float or bf16."""
+    R, Cc = int(rows_of_state), int(cols_of_state)
+    T, segments = v.shape[0], state_slots.shape[0]
+    args, where = _channel_operands("channel_delta_step", q, k, v, decay, write, state, seg_start, state_slots, heads, R, Cc, share)
+    gp, ldg = _rows_of(gate, "gate", heads * Cc)
+    if not channel_step_ok(state, R, Cc) or gate.shape[0] != T or tuple(out.shape) != (T, heads * Cc) or out.stride(1) != 1 or not out.is_cuda:
+        raise KernelError("channel_delta_step: sizes not supported")
+    _check(_rec().cisr_channel_step(*args, *where, segments, heads, R, Cc, int(share), float(q_scale), gp, ldg,
+                                    _dev(weight, "weight", torch.float32, (Cc,)), float(eps), out.data_ptr(), out.stride(0),
+                                    _storage(out, "out"), _stream()), "channel_delta_step")
     return out
 
 

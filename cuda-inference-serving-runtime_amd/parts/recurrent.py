@@ -264,7 +264,8 @@ class GatedDeltaRule(Mixer):
 class ChannelDeltaRule(GatedDeltaRule):
     """The gated delta rule with a decay a head and key channel.  Decays and the result's gate come from low-rank
     projections whose inner sizes the file decides; the convolution, the unit vectors, the decays and the gates are one
-    kernel (ops.channel_delta_inputs).  The state is that of the rule with a decay a head."""
+    kernel (ops.channel_delta_inputs); portions are walked chunk by chunk on the matrix cores, short ones row by row, single
+    rows by a kernel that norms and gates the result as well.  The state is that of the rule with a decay a head."""
 
     NAMES = {"q": "q", "k": "k", "v": "v", "write": "b", "decay_down": "a1", "decay_up": "a2", "dt_bias": "dt_bias", "a_log": "A_log",
              "gate_down": "g1", "gate_up": "g2", "norm": "norm", "o": "o", "conv": "conv"}
@@ -295,11 +296,9 @@ class ChannelDeltaRule(GatedDeltaRule):
             parts.append(torch.zeros(8 - starts[-1] % 8, self.hidden, dtype=parts[0].dtype, device=parts[0].device))
         self.w_in = torch.cat(parts, dim=0).contiguous()
         self.w_out = matrix_operand(tensors[t("o")], dtype)
-        # the second halves by columns, [rank, columns]: neighbouring threads own neighbouring columns
-        self.decay_up = matrix_operand(tensors[t("decay_up")], dtype).t().contiguous()
-        self.gate_up = matrix_operand(tensors[t("gate_up")], dtype).t().contiguous()
+        self.decay_up, self.gate_up = (ops.low_rank_rows(matrix_operand(tensors[t(p)], dtype)) for p in ("decay_up", "gate_up"))
         for down, up in (("decay_down", self.decay_up), ("gate_down", self.gate_up)):
-            if tensors[t(down)].shape[0] != up.shape[0]:
+            if tensors[t(down)].shape[0] != up.shape[1]:
                 raise ValueError(f"{self.name}: the projections {self.names[down]} and its second half disagree about their inner size")
         self.conv = torch.cat([_float(tensors[f"{t(p)}.{conv}"]) for p in ("q", "k", "v")], dim=0).t().contiguous()     # [taps, channels]
         self.dt_bias, self.a_log = _float(tensors[t("dt_bias")]), _float(tensors[t("a_log")])
@@ -315,12 +314,21 @@ class ChannelDeltaRule(GatedDeltaRule):
         ops.channel_delta_inputs(proj, self.conv, state[:, nh * self.dim * self.vdim:], qkv, ctx.seg_of_row, ctx.seg_start, ctx.state_slots,
                                  self.kv_heads, self.dim, nh, self.vdim, self.at["decay_down"], self.decay_up, self.dt_bias, self.a_log, decay,
                                  self.at["gate_down"], self.gate_up, gate, unit_eps=self.unit_eps, single_rows=ctx.decode_only)
-        o = ctx.buffer("cdelta.o", (T, inner), torch.float32)
         write = self.at["write"]
-        ops.channel_delta_scan(qkv[:, :qk], qkv[:, qk:2 * qk], qkv[:, 2 * qk:], decay, proj[:, write:write + nh], o, state,
-                               ctx.seg_start, ctx.state_slots, nh, self.dim, self.vdim, share=nh // self.kv_heads, q_scale=self.dim ** -0.5)
-        return ops.group_norm_gate(o, gate, self.norm_weight, ctx.buffer("cdelta.act", (T, inner), ctx.dtype), nh, self.eps,
-                                   gate_first=False, shared_weight=True, sigmoid=True)
+        operands = (qkv[:, :qk], qkv[:, qk:2 * qk], qkv[:, 2 * qk:], decay, proj[:, write:write + nh])
+        where, sizes = (state, ctx.seg_start, ctx.state_slots), (nh, self.dim, self.vdim)
+        law = dict(share=nh // self.kv_heads, q_scale=self.dim ** -0.5)
+        act = ctx.buffer("cdelta.act", (T, inner), ctx.dtype)
+        if ctx.decode_only and ops.channel_step_ok(state, self.dim, self.vdim):
+            # single rows: the step of the state, the result's norm and its gate are one kernel
+            return ops.channel_delta_step(*operands, gate, self.norm_weight, act, *where, *sizes, self.eps, **law)
+        o = ctx.buffer("cdelta.o", (T, inner), torch.float32)
+        if ops.channel_chunked(T, ctx.n_segments, ctx.decode_only):
+            work = ctx.buffer("cdelta.work", (ops.channel_chunk_work(T, ctx.n_segments, *sizes),), torch.float32)
+            ops.channel_delta_chunks(*operands, o, *where, *sizes, work, **law)
+        else:
+            ops.channel_delta_scan(*operands, o, *where, *sizes, **law)
+        return ops.group_norm_gate(o, gate, self.norm_weight, act, nh, self.eps, gate_first=False, shared_weight=True, sigmoid=True)
 
 
 class MinGRU(Mixer):

@@ -211,11 +211,14 @@ def test_delta_rule_with_a_decay_a_channel_over_segments_with_states_carried_and
     state = torch.zeros(4, size + (taps - 1) * ch, device="cuda")
     fresh = lambda: (np.zeros((heads, dim, vdim)), np.zeros((taps - 1, ch)))
     kept = {s: fresh() for s in range(4)}
-    ua, ug = dev(up_a, td).t().contiguous(), dev(up_g, td).t().contiguous()
+    ua, ug = ops.low_rank_rows(dev(up_a, td)), ops.low_rank_rows(dev(up_g, td))
+    chunk_state, step_state = state.clone(), state.clone()
+    eqv = ops.channel_step_ok(step_state, dim, vdim)
     steps = [([7, 1, 300, 2], [2, 0, 3, 1]), ([1, 1, 1, 1], [3, 1, 0, 2]), ([1, 2, 33], [1, 2, 0]), ([1, 1], [3, 0])]
     for n, (counts, slots) in enumerate(steps):
         if n == 2:
-            state[1].zero_()
+            for st in (state, chunk_state, step_state):
+                st[1].zero_()
             kept[1] = fresh()
         single = all(c == 1 for c in counts)
         T = sum(counts) + 2                                      # two padding rows, which belong to no segment
@@ -227,8 +230,19 @@ def test_delta_rule_with_a_decay_a_channel_over_segments_with_states_carried_and
         args = (ints(start), ints(slots))
         ops.channel_delta_inputs(dp, dev(taps_w.T), state[:, size:], qkv, ints(seg_of_row), *args, kv_heads, dim, heads, vdim, at_a, ua,
                                  dev(dt_bias), dev(a_log), decay, at_g, ug, gate, single_rows=single)
-        ops.channel_delta_scan(qkv[:, :qk], qkv[:, qk:2 * qk], qkv[:, 2 * qk:], decay, dp[:, at_b:at_b + heads], o, state, *args, heads, dim, vdim,
-                               share=share, q_scale=dim ** -0.5, columns=columns)
+        operands = (qkv[:, :qk], qkv[:, qk:2 * qk], qkv[:, 2 * qk:], decay, dp[:, at_b:at_b + heads])
+        law = dict(share=share, q_scale=dim ** -0.5)
+        ops.channel_delta_scan(*operands, o, state, *args, heads, dim, vdim, columns=columns, **law)
+        # the same chunk by chunk, a few chunks a launch
+        chunked = torch.full((T, inner), float("nan"), device="cuda")
+        work = torch.full((ops.channel_chunk_work(T, len(counts), heads, dim, vdim, slab=7),), float("nan"), device="cuda")
+        ops.channel_delta_chunks(*operands, chunked, chunk_state, *args, heads, dim, vdim, work, slab=7, **law)
+        if eqv:       # single rows with norm and gate in the kernel; the other steps move its state on row by row
+            stepped = torch.full((T, inner), float("nan"), dtype=td, device="cuda")
+            if single:
+                ops.channel_delta_step(*operands, gate, dev(weight), stepped, step_state, *args, heads, dim, vdim, eps, **law)
+            else:
+                ops.channel_delta_scan(*operands, o.clone(), step_state, *args, heads, dim, vdim, **law)
         out = torch.full((T, inner), float("nan"), device="cuda")
         ops.group_norm_gate(o, gate, dev(weight), out, heads, eps, gate_first=False, shared_weight=True, sigmoid=True)
         pr = rounded(proj)
@@ -237,8 +251,9 @@ def test_delta_rule_with_a_decay_a_channel_over_segments_with_states_carried_and
         gz = pr[:, at_g:at_g + rg] @ rounded(up_g, dtype).T
         beta = P.sigmoid(pr[:, at_b:at_b + heads])
         rows = slice(0, sum(counts))
-        close(decay.cpu().numpy()[rows], g.reshape(T, -1)[rows], 2e-5)
-        close(gate.cpu().numpy()[rows], gz[rows], 2e-5)
+        close(decay.cpu().numpy()[rows], g.reshape(T, -1)[rows], 2e-5 if dtype == "float32" else 4e-5)
+        g = decay.double().cpu().numpy().reshape(T, heads, dim)              # (the recurrence from the decays as they came out)
+        close(gate.cpu().numpy()[rows], gz[rows], 2e-5 if dtype == "float32" else 4e-5)
         for s, slot in enumerate(slots):
             S, past = kept[slot]
             own = pr[start[s]:start[s + 1]]
@@ -256,12 +271,16 @@ def test_delta_rule_with_a_decay_a_channel_over_segments_with_states_carried_and
                     S[h] = S[h] + np.outer(k[i, h // share], beta[t, h] * (v[i, h] - k[i, h // share] @ S[h]))
                     want[i, h] = q[i, h // share] @ S[h] * dim ** -0.5
             close(o.cpu().numpy()[start[s]:start[s + 1]], want.reshape(-1, inner), 3e-5)
-            want = P.rms(want, eps) * rounded(weight) * P.sigmoid(gz[start[s]:start[s + 1]].reshape(-1, heads, vdim))
+            close(chunked.cpu().numpy()[start[s]:start[s + 1]], want.reshape(-1, inner), 3e-5)
+            want = P.rms(want, eps) * rounded(weight) * P.sigmoid(gate.double().cpu().numpy()[start[s]:start[s + 1]].reshape(-1, heads, vdim))
             close(out.cpu().numpy()[start[s]:start[s + 1]], want.reshape(-1, inner), 1e-4)
+            if eqv and single:
+                close(stepped.float().cpu().numpy()[start[s]:start[s + 1]], want.reshape(-1, inner), 1e-4 if dtype == "float32" else 6e-3)
             kept[slot] = (S, x[len(x) - (taps - 1):] if taps > 1 else past)
         for slot in range(4):
             have = state[slot].cpu().numpy()
-            close(have[:size].reshape(heads, dim, vdim) + 1.0, kept[slot][0] + 1.0, 2e-5)
+            for st in (state, chunk_state, step_state) if eqv else (state, chunk_state):
+                close(st[slot, :size].cpu().numpy().reshape(heads, dim, vdim) + 1.0, kept[slot][0] + 1.0, 2e-5)
             if taps > 1:
                 close(have[size:].reshape(taps - 1, ch) + 1.0, kept[slot][1] + 1.0, 1e-6)
 
