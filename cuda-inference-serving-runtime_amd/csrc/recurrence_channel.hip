@@ -38,48 +38,61 @@ __device__ __forceinline__ float channel_decay(float z, float rate) {
 
 // An item of the convolution for the rows t .. t + n - 1 (n <= RB): a q head, a k head (both made unit vectors) or up to 256
 // channels of v; four channels a lane.  TAPS > 0: that many taps, the rows' inputs and those before them asked for at
-// once; rows whose inputs reach back before their segment, and TAPS 0 (any number of taps), take them one by one, from
-// the state where they lie before the segment.  SINGLE: every segment has one row, and the lane of a (row, channel)
+// once (of a single row from the state); rows whose inputs reach back before their segment, and TAPS 0 (any number of taps),
+// take them one by one, from the state where they lie before the segment.  SINGLE: every segment has one row, and the lane of a (row, channel)
 // moves that channel's state on itself.
 template <bool SINGLE, int TAPS>
 __device__ __forceinline__ void conv_item(const ChannelInputs& p, int t0, int n_rows, int item, int lane) {
-    constexpr int RB = TAPS ? 8 : 1, BACK = TAPS ? TAPS - 1 : 0;
+    constexpr int RB = TAPS && !SINGLE ? 8 : 1, BACK = TAPS ? TAPS - 1 : 0, TN = TAPS ? TAPS : 1;
     const int qk = p.G * p.R, inner = p.H * p.C, channels = 2 * qk + inner;
     const bool head = item < 2 * p.G;
     const int first = head ? item * p.R : 2 * qk + (item - 2 * p.G) * 256;
     const int n = head ? p.R : min(256, channels - first);
-    float x[RB + BACK][4], w[TAPS ? TAPS : 1][4];
+    int seg[RB], rel[RB];
+#pragma unroll
+    for (int r = 0; r < RB; ++r) seg[r] = p.seg_of_row[min(t0 + r, p.rows - 1)];
+    float x[RB + BACK][4], w[TN][4];
+    float* single = nullptr;
     if (TAPS) {
+        if (SINGLE) {
+            if (seg[0] < 0) return;
+            single = p.conv_state + (long long)p.state_slots[seg[0]] * p.slot_stride;
+        }
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
             const int ch = first + min(lane + WAVE * i, n - 1);
 #pragma unroll
-            for (int r = 0; r < RB + BACK; ++r) x[r][i] = p.in[(size_t)min(max(t0 - BACK + r, 0), p.rows - 1) * p.ld + ch];
+            for (int r = 0; r < RB + BACK; ++r)
+                x[r][i] = SINGLE && r < BACK ? single[(size_t)r * channels + ch] : p.in[(size_t)min(max(t0 - BACK + r, 0), p.rows - 1) * p.ld + ch];
 #pragma unroll
             for (int j = 0; j < TAPS; ++j) w[j][i] = p.taps_w[(size_t)j * channels + ch];
         }
     }
 #pragma unroll
+    for (int r = 0; r < RB; ++r) rel[r] = SINGLE || seg[r] < 0 ? 0 : t0 + r - p.seg_start[seg[r]];
+#pragma unroll
     for (int r = 0; r < RB; ++r) {
         if (r >= n_rows) break;
-        const int t = t0 + r, seg = p.seg_of_row[t];
-        if (seg < 0) continue;
-        const int rel = t - p.seg_start[seg];
+        const int t = t0 + r;
+        if (seg[r] < 0) continue;
         float y[4] = {0.f, 0.f, 0.f, 0.f}, ss = 0.f;
-        if (TAPS && rel >= BACK) {
+        if (TAPS && (SINGLE || rel[r] >= BACK)) {
 #pragma unroll
             for (int i = 0; i < 4; ++i)
 #pragma unroll
-                for (int j = 0; j < (TAPS ? TAPS : 1); ++j) y[i] += w[j][i] * x[r + (TAPS ? j : 0)][i];
+                for (int j = 0; j < TN; ++j) {
+                    y[i] += w[j][i] * x[TAPS ? r + j : 0][i];
+                    if (SINGLE && j > 0 && lane + WAVE * i < n) single[(size_t)(j - 1) * channels + first + lane + WAVE * i] = x[TAPS ? j : 0][i];
+                }
         } else {
-            float* st = p.conv_state + (long long)p.state_slots[seg] * p.slot_stride;
+            float* st = p.conv_state + (long long)p.state_slots[seg[r]] * p.slot_stride;
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
                 const int ch = first + lane + WAVE * i;
                 if (lane + WAVE * i >= n) continue;
                 for (int j = 0; j < p.taps; ++j) {
-                    const int src = rel - (p.taps - 1) + j;
-                    const float a = src >= 0 ? p.in[(size_t)(t - rel + src) * p.ld + ch] : st[(size_t)(p.taps - 1 + src) * channels + ch];
+                    const int src = rel[r] - (p.taps - 1) + j;
+                    const float a = src >= 0 ? p.in[(size_t)(t - rel[r] + src) * p.ld + ch] : st[(size_t)(p.taps - 1 + src) * channels + ch];
                     y[i] += p.taps_w[(size_t)j * channels + ch] * a;
                     if (SINGLE && j > 0) st[(size_t)(j - 1) * channels + ch] = a;     // (input j of this row is input j - 1 of the next)
                 }
@@ -104,18 +117,21 @@ __device__ __forceinline__ void conv_item(const ChannelInputs& p, int t0, int n_
 //   float matrices: RT rows, a thread a column, float sums in the order of the coordinates.
 #define RANK_CHUNK 64
 
-template <bool SINGLE, int TAPS, int RT, typename TW>
+// A step of single rows runs both parts in one launch (PART 0), others each in a launch of its own (1, 2: two kernels with
+// the registers that each needs).
+template <int PART, bool SINGLE, int TAPS, int RT, typename TW>
 __global__ void __launch_bounds__(256) channel_inputs_kernel(ChannelInputs p) {
     const int inner = p.H * p.C;
     const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
-    if ((int)blockIdx.x < p.conv_blocks) {
-        constexpr int RB = TAPS ? 8 : 1;
+    if (PART == 1 || (PART == 0 && (int)blockIdx.x < p.conv_blocks)) {
+        constexpr int RB = TAPS && !SINGLE ? 8 : 1;
         const int per_run = 2 * p.G + (inner + 255) / 256;
         const int work = blockIdx.x * 4 + wave, t0 = work / per_run * RB;
         if (t0 < p.rows) conv_item<SINGLE, TAPS>(p, t0, min(RB, p.rows - t0), work % per_run, lane);
         return;
     }
-    const int b = blockIdx.x - p.conv_blocks, tid = threadIdx.x;
+    if (PART == 1) return;
+    const int b = PART == 0 ? blockIdx.x - p.conv_blocks : blockIdx.x, tid = threadIdx.x;
     const int col_block = b / p.row_tiles;
     const int a_cols = p.H * p.R, a_blocks = (a_cols + 255) / 256;
     const bool is_decay = col_block < a_blocks;
@@ -133,6 +149,7 @@ __global__ void __launch_bounds__(256) channel_inputs_kernel(ChannelInputs p) {
         for (int c = 0; c < 4; ++c)
 #pragma unroll
             for (int j = 0; j < RT; ++j) acc[c][j] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
         for (int k0 = 0; k0 < rank; k0 += 32) {
             bf16x8_t hi[RT], lo[RT], wt[4];
             const int k = k0 + kg * 8;
@@ -142,9 +159,12 @@ __global__ void __launch_bounds__(256) channel_inputs_kernel(ChannelInputs p) {
 #pragma unroll
             for (int j = 0; j < RT; ++j) {
                 const float* row = p.in + (size_t)min(t0 + j * 16 + m, p.rows - 1) * p.ld + off + k;
+                f32x4_t v[2];                      // (16-byte words; the last one may reach into the row's next columns)
+                v[0] = k < rank ? *(const f32x4_t*)row : (f32x4_t){0.f, 0.f, 0.f, 0.f};
+                v[1] = k + 4 < rank ? *(const f32x4_t*)(row + 4) : (f32x4_t){0.f, 0.f, 0.f, 0.f};
 #pragma unroll
                 for (int e = 0; e < 8; ++e) {
-                    const float a = k + e < rank ? row[e] : 0.f;
+                    const float a = k + e < rank ? v[e / 4][e % 4] : 0.f;
                     const __bf16 h = (__bf16)a;
                     hi[j][e] = h;
                     lo[j][e] = (__bf16)(a - (float)h);
@@ -225,31 +245,43 @@ channel_conv_state_kernel(const float* __restrict__ in, int ld, float* __restric
 
 template <bool SINGLE, int TAPS, typename TW>
 static int launch_channel_inputs_of(ChannelInputs& p, hipStream_t stream) {
-    const int inner = p.H * p.C, a_cols = p.H * p.R, run = TAPS ? 8 : 1;
+    const int inner = p.H * p.C, a_cols = p.H * p.R, run = TAPS && !SINGLE ? 8 : 1;
     const long long items = (long long)((p.rows + run - 1) / run) * (2 * p.G + (inner + 255) / 256);
     const int col_blocks = (a_cols + 255) / 256 + (inner + 255) / 256;
     constexpr int unit = sizeof(TW) == 2 ? 16 : 1;                // rows of a step of RT
     const int rt = sizeof(TW) == 2 ? (p.rows > 128 ? 2 : 1) : (p.rows > 16 ? 16 : 1);      // many rows share a column's weights
     p.conv_blocks = (int)((items + 3) / 4);
     p.row_tiles = (p.rows + rt * unit - 1) / (rt * unit);
-    const long long blocks = p.conv_blocks + (long long)p.row_tiles * col_blocks;
-    if (blocks > 0x7fffffff) return (int)hipErrorInvalidValue;
-    if (rt == 1) channel_inputs_kernel<SINGLE, TAPS, 1, TW><<<(unsigned)blocks, 256, 0, stream>>>(p);
-    else channel_inputs_kernel<SINGLE, TAPS, sizeof(TW) == 2 ? 2 : 16, TW><<<(unsigned)blocks, 256, 0, stream>>>(p);
+    const long long tiles = (long long)p.row_tiles * col_blocks;
+    if (p.conv_blocks + tiles > 0x7fffffff) return (int)hipErrorInvalidValue;
+    constexpr int MANY = sizeof(TW) == 2 ? 2 : 16;
+    if (SINGLE) {
+        const unsigned blocks = (unsigned)(p.conv_blocks + tiles);
+        if (rt == 1) channel_inputs_kernel<0, SINGLE, TAPS, 1, TW><<<blocks, 256, 0, stream>>>(p);
+        else channel_inputs_kernel<0, SINGLE, TAPS, MANY, TW><<<blocks, 256, 0, stream>>>(p);
+        return CISR_LAUNCH_CHECK();
+    }
+    channel_inputs_kernel<1, SINGLE, TAPS, 1, TW><<<(unsigned)p.conv_blocks, 256, 0, stream>>>(p);
+    const int err = CISR_LAUNCH_CHECK();
+    if (err) return err;
+    if (rt == 1) channel_inputs_kernel<2, SINGLE, 0, 1, TW><<<(unsigned)tiles, 256, 0, stream>>>(p);
+    else channel_inputs_kernel<2, SINGLE, 0, MANY, TW><<<(unsigned)tiles, 256, 0, stream>>>(p);
     return CISR_LAUNCH_CHECK();
 }
 
 template <typename TW>
 static int launch_channel_inputs(ChannelInputs& p, bool single, hipStream_t stream) {
-    if (single) return launch_channel_inputs_of<true, 0, TW>(p, stream);
-    if (p.taps == 2) return launch_channel_inputs_of<false, 2, TW>(p, stream);
-    if (p.taps == 3) return launch_channel_inputs_of<false, 3, TW>(p, stream);
-    if (p.taps == 4) return launch_channel_inputs_of<false, 4, TW>(p, stream);
-    return launch_channel_inputs_of<false, 0, TW>(p, stream);
+#define CHANNEL_INPUTS(TAPS) single ? launch_channel_inputs_of<true, TAPS, TW>(p, stream) : launch_channel_inputs_of<false, TAPS, TW>(p, stream)
+    if (p.taps == 2) return CHANNEL_INPUTS(2);
+    if (p.taps == 3) return CHANNEL_INPUTS(3);
+    if (p.taps == 4) return CHANNEL_INPUTS(4);
+    return CHANNEL_INPUTS(0);
+#undef CHANNEL_INPUTS
 }
 
 // up_a [heads * R, ldu_a], up_g [heads * C, ldu_g]: rows of rank_a / rank_g coordinates, then zeros up to ldu; bf16 matrices
-// are read in 16-byte words of 32 coordinates a step, so their ldu is a multiple of 32 and they are 16-byte aligned.
+// are read in 16-byte words, 32 coordinates a step, so their ldu is a multiple of 32 and they are 16-byte aligned, and so are
+// the rows' low-rank coordinates.
 extern "C" int cisr_channel_inputs(const float* in, int ld, const float* taps_w, int taps, float* conv_state, long long slot_stride,
                                    float* qkv, const int* seg_of_row, const int* seg_start, const int* state_slots, int rows,
                                    int segments, int kv_heads, int R, int heads, int C, float unit_eps, int off_a, int rank_a,
@@ -261,6 +293,7 @@ extern "C" int cisr_channel_inputs(const float* in, int ld, const float* taps_w,
         channels > ld || off_a < 0 || off_a + rank_a > ld || off_g < 0 || off_g + rank_g > ld || segments > 65535 || ldu_a < rank_a ||
         ldu_g < rank_g)
         return (int)hipErrorInvalidValue;
+    if (weight_dtype == DT_BF16 && (off_a % 4 || off_g % 4 || ld % 4 || (uintptr_t)in % 16)) return (int)hipErrorInvalidValue;
     if (weight_dtype == DT_BF16 && (ldu_a % 32 || ldu_g % 32 || (uintptr_t)up_a % 16 || (uintptr_t)up_g % 16)) return (int)hipErrorInvalidValue;
     ChannelInputs p{in, ld, taps_w, taps, conv_state, slot_stride, qkv, seg_of_row, seg_start, state_slots, rows, kv_heads, R, heads, C,
                     unit_eps, off_a, rank_a, up_a, dt_bias, a_log, decay, off_g, rank_g, up_g, gate, ldu_a, ldu_g, 0, 0};

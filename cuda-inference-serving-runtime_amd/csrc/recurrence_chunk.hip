@@ -62,9 +62,10 @@ __device__ __forceinline__ float row_sum(float x) {
     return x;
 }
 
-__global__ void __launch_bounds__(256, 3) channel_chunk_kernel(ChunkArgs p) {
+__global__ void __launch_bounds__(256, 4) channel_chunk_kernel(ChunkArgs p) {
     extern __shared__ __attribute__((aligned(16))) float lds[];
-    __shared__ float sA[CHUNK][CHUNK + 1], sM[CHUNK][CHUNK], sBeta[CHUNK];
+    __shared__ float sA[CHUNK][CHUNK + 1], sBeta[CHUNK];
+    __shared__ __attribute__((aligned(16))) float sM[CHUNK][CHUNK];
     const int slot = p.slot0 + blockIdx.y, head = blockIdx.x, tid = threadIdx.x;
     const int seg = segment_of_slot(p.seg_start, p.segments, slot);
     const int t0 = p.seg_start[seg] + (slot - p.seg_start[seg] / CHUNK - seg) * CHUNK, t1 = p.seg_start[seg + 1];
@@ -73,20 +74,16 @@ __global__ void __launch_bounds__(256, 3) channel_chunk_kernel(ChunkArgs p) {
     float* sk = lds;
     float* sq = sk + CHUNK * RS;
     float* sg = sq + CHUNK * RS;
-    const float* kh = p.k + (size_t)(head / p.share) * R;
-    const float* qh = p.q + (size_t)(head / p.share) * R;
-    const float* gh = p.g + (size_t)head * R;
-    for (int r = tid; r < Rp; r += 256) {        // a thread a channel
-#pragma unroll
-        for (int i = 0; i < CHUNK; ++i) {
-            const size_t t = (size_t)(t0 + min(i, n - 1));
-            const bool in = r < R && i < n;
-            const int rr = min(r, R - 1);
-            const float k = kh[t * p.ldk + rr], q = qh[t * p.ldq + rr], g = gh[t * p.ldg + rr];
-            sk[i * RS + r] = in ? k : 0.f;
-            sq[i * RS + r] = in ? q * p.q_scale : 0.f;
-            sg[i * RS + r] = in ? g : 1.f;
-        }
+    const float* kh = p.k + (size_t)t0 * p.ldk + (size_t)(head / p.share) * R;
+    const float* qh = p.q + (size_t)t0 * p.ldq + (size_t)(head / p.share) * R;
+    const float* gh = p.g + (size_t)t0 * p.ldg + (size_t)head * R;
+    for (int idx = tid; idx < CHUNK * Rp; idx += 256) {
+        const int i = idx / Rp, r = idx % Rp, tt = min(i, n - 1), rr = min(r, R - 1);
+        const bool in = r < R && i < n;
+        const float k = kh[tt * p.ldk + rr], q = qh[tt * p.ldq + rr], g = gh[tt * p.ldg + rr];
+        sk[i * RS + r] = in ? k : 0.f;
+        sq[i * RS + r] = in ? q * p.q_scale : 0.f;
+        sg[i * RS + r] = in ? g : 1.f;
     }
     if (tid < CHUNK) sBeta[tid] = tid < n ? 1.0f / (1.0f + expf(-p.b[(size_t)(t0 + tid) * p.ldb + head])) : 0.f;
     __syncthreads();
@@ -96,29 +93,26 @@ __global__ void __launch_bounds__(256, 3) channel_chunk_kernel(ChunkArgs p) {
     // rows behind i (times their decays) and meet
     {
         const int i = tid / 16, part = tid % 16;
-        float a[CHUNK], b[CHUNK];
+        f32x4_t x[4];
 #pragma unroll
-        for (int t = 0; t < CHUNK; ++t) a[t] = b[t] = 0.f;
-        for (int r = 4 * part; r < Rp; r += 64) {
-            f32x4_t x = *(const f32x4_t*)(sk + i * RS + r);
-#pragma unroll
-            for (int t = 0; t < CHUNK; ++t) {
-                if (t < i) continue;
-                const f32x4_t q = *(const f32x4_t*)(sq + t * RS + r);
-                if (t > i) {
-                    const f32x4_t k = *(const f32x4_t*)(sk + t * RS + r);
-                    x *= *(const f32x4_t*)(sg + t * RS + r);
-                    a[t] += (x[0] * k[0] + x[1] * k[1]) + (x[2] * k[2] + x[3] * k[3]);
-                }
-                b[t] += (x[0] * q[0] + x[1] * q[1]) + (x[2] * q[2] + x[3] * q[3]);
-            }
-        }
-#pragma unroll
+        for (int j = 0; j < 4; ++j) x[j] = 64 * j + 4 * part < Rp ? *(const f32x4_t*)(sk + i * RS + 64 * j + 4 * part) : (f32x4_t){0.f, 0.f, 0.f, 0.f};
         for (int t = 0; t < CHUNK; ++t) {
-            const float at = row_sum(a[t]), bt = row_sum(b[t]);
+            float a = 0.f, b = 0.f;
+#pragma unroll
+            for (int j = 0; j < 4; ++j) {
+                const int r = 64 * j + 4 * part;
+                if (64 * j >= Rp) break;                           // (uniform)
+                if (r >= Rp || t < i) continue;
+                const f32x4_t k = *(const f32x4_t*)(sk + t * RS + r), q = *(const f32x4_t*)(sq + t * RS + r);
+                if (t > i) x[j] *= *(const f32x4_t*)(sg + t * RS + r);
+                a += (x[j][0] * k[0] + x[j][1] * k[1]) + (x[j][2] * k[2] + x[j][3] * k[3]);
+                b += (x[j][0] * q[0] + x[j][1] * q[1]) + (x[j][2] * q[2] + x[j][3] * q[3]);
+            }
+            a = row_sum(a);
+            b = row_sum(b);
             if (part == t) {
-                if (t > i) sA[t][i] = sBeta[t] * at;
-                wP[t * CHUNK + i] = t >= i ? bt : 0.f;
+                sA[t][i] = sBeta[t] * a;                           // (only i < t is read)
+                wP[t * CHUNK + i] = b;                             // (0 for i > t)
             }
         }
     }
@@ -132,6 +126,7 @@ __global__ void __launch_bounds__(256, 3) channel_chunk_kernel(ChunkArgs p) {
 #pragma unroll
             for (int i = 0; i < t; ++i) s -= sA[t][i] * x[i];
             x[t] = s;
+            __builtin_amdgcn_sched_barrier(0);                     // (the rows' operands are not asked for all at once: registers)
         }
 #pragma unroll
         for (int t = 0; t < CHUNK; ++t) sM[t][tid] = x[t] * sBeta[tid];
@@ -172,6 +167,7 @@ __global__ void __launch_bounds__(256, 3) channel_chunk_kernel(ChunkArgs p) {
 #pragma unroll
             for (int i = 0; i <= t; ++i) s += sM[t][i] * x[i];
             y[t] = s;
+            __builtin_amdgcn_sched_barrier(0);
         }
         if (key) {
 #pragma unroll
@@ -187,8 +183,10 @@ __global__ void __launch_bounds__(256, 3) channel_chunk_kernel(ChunkArgs p) {
 // A block a (head, segment, 16 columns).  The state's rows in tiles of 16: wave w owns the tiles w NT .. w NT + NT - 1, in
 // the matrix instruction's result layout (lane l: rows 4 (l / 16) + i of the tile, column l % 16), which serves as its
 // right operand as it is when the left operand's inner index runs alike: every operand is a 16-byte load.
-template <int NT>
-__global__ void __launch_bounds__(256) channel_walk_kernel(ChunkArgs p) {
+// AHEAD chunks' operands are in flight (an even number).  The loads of a chunk are kept together in program order: they
+// return in order, so a chunk's wait then leaves those of the chunks behind it in flight.
+template <int NT, int AHEAD>
+__global__ void __launch_bounds__(256, 2) channel_walk_kernel(ChunkArgs p) {
     __shared__ f32x4_t meet[2][2][4][WAVE];         // [chunk parity][M Kg S0, (D q) S0][wave][lane]
     const int head = blockIdx.x, seg = blockIdx.z, wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
     const int t0 = p.seg_start[seg], t1 = p.seg_start[seg + 1];
@@ -207,25 +205,41 @@ __global__ void __launch_bounds__(256) channel_walk_kernel(ChunkArgs p) {
             const int r = (wave * NT + j) * 16 + 4 * kg + i;
             S[j][i] = r < R && c < C ? state[(size_t)r * C + c] : 0.f;
         }
-    struct Operands { f32x4_t kg[NT], qg[NT], kd[NT], g[NT], u, pr; } now, next;
+    struct Operands { f32x4_t kg[NT], qg[NT], kd[NT], g[NT], u, pr; } ring[AHEAD];
     const size_t per = (size_t)chunk_floats(Rp, p.Cp);
+    // byte offsets of this lane's words from a chunk's operands (a uniform address): 32 bits
+    unsigned at_k[NT], at_d[NT], at_g[NT];
+    const unsigned q_words = CHUNK * Rp * 4u, at_u = (3u * CHUNK * Rp + c * CHUNK + 4 * kg) * 4u,
+                   at_p = (3u * CHUNK * Rp + CHUNK * p.Cp + m * CHUNK + 4 * kg) * 4u;
+#pragma unroll
+    for (int j = 0; j < NT; ++j) {
+        const unsigned r = min((wave * NT + j) * 16, Rp - 16);          // (a wave without this tile reads another: its S is zero)
+        at_k[j] = (m * Rp + r + 4 * kg) * 4u;
+        at_d[j] = (2u * CHUNK * Rp + (r + m) * CHUNK + 4 * kg) * 4u;
+        at_g[j] = (3u * CHUNK * Rp + CHUNK * p.Cp + CHUNK * CHUNK + r + 4 * kg) * 4u;
+    }
     auto fetch = [&](Operands& o, int slot) {
-        const float* w = p.work + ((size_t)(slot - p.slot0) * p.heads + head) * per;
+        slot = min(slot, last - 1);
+        const char* w = (const char*)(p.work + ((size_t)(slot - p.slot0) * p.heads + head) * per);
 #pragma unroll
         for (int j = 0; j < NT; ++j) {
-            const int r = min((wave * NT + j) * 16, Rp - 16);          // (a wave without this tile reads another: its S is zero)
-            o.kg[j] = *(const f32x4_t*)(w + (size_t)m * Rp + r + 4 * kg);
-            o.qg[j] = *(const f32x4_t*)(w + (size_t)(CHUNK + m) * Rp + r + 4 * kg);
-            o.kd[j] = *(const f32x4_t*)(w + (size_t)2 * CHUNK * Rp + (size_t)(r + m) * CHUNK + 4 * kg);
-            o.g[j] = *(const f32x4_t*)(w + (size_t)3 * CHUNK * Rp + (size_t)CHUNK * p.Cp + CHUNK * CHUNK + r + 4 * kg);
+            o.kg[j] = *(const f32x4_t*)(w + at_k[j]);
+            o.qg[j] = *(const f32x4_t*)(w + q_words + at_k[j]);
         }
-        o.u = *(const f32x4_t*)(w + (size_t)3 * CHUNK * Rp + (size_t)c * CHUNK + 4 * kg);
-        o.pr = *(const f32x4_t*)(w + (size_t)3 * CHUNK * Rp + (size_t)CHUNK * p.Cp + m * CHUNK + 4 * kg);
+        o.u = *(const f32x4_t*)(w + at_u);
+#pragma unroll
+        for (int j = 0; j < NT; ++j) {
+            o.g[j] = *(const f32x4_t*)(w + at_g[j]);
+            o.kd[j] = *(const f32x4_t*)(w + at_d[j]);
+        }
+        o.pr = *(const f32x4_t*)(w + at_p);
     };
-    fetch(now, first);
-    for (int slot = first; slot < last; ++slot) {
-        const int par = slot & 1;
-        if (slot + 1 < last) fetch(next, slot + 1);
+#pragma unroll
+    for (int d = 0; d < AHEAD; ++d) {
+        fetch(ring[d], first + d);
+        __builtin_amdgcn_sched_barrier(0);
+    }
+    auto walk = [&](Operands& now, int slot, int par) {
         f32x4_t w = {0.f, 0.f, 0.f, 0.f}, o = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int j = 0; j < NT; ++j)
@@ -238,14 +252,13 @@ __global__ void __launch_bounds__(256) channel_walk_kernel(ChunkArgs p) {
             for (int i = 0; i < 4; ++i) o = __builtin_amdgcn_mfma_f32_16x16x4f32(now.qg[j][i], S[j][i], o, 0, 0, 0);
         meet[par][1][wave][lane] = o;
         __syncthreads();                       // (the other parity's buffers were read before the barrier before this one's writes)
-        f32x4_t u = now.u - ((meet[par][0][0][lane] + meet[par][0][1][lane]) + (meet[par][0][2][lane] + meet[par][0][3][lane]));
+        const f32x4_t u = now.u - ((meet[par][0][0][lane] + meet[par][0][1][lane]) + (meet[par][0][2][lane] + meet[par][0][3][lane]));
 #pragma unroll
         for (int j = 0; j < NT; ++j) {
-            const bool own = (wave * NT + j) * 16 < Rp;
             S[j] *= now.g[j];
-            if (own)
+            const float mine = (wave * NT + j) * 16 < Rp ? 1.f : 0.f;          // (a tile beyond the state's rows stays zero)
 #pragma unroll
-                for (int i = 0; i < 4; ++i) S[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(now.kd[j][i], u[i], S[j], 0, 0, 0);
+            for (int i = 0; i < 4; ++i) S[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(now.kd[j][i] * mine, u[i], S[j], 0, 0, 0);
         }
         if (wave == (slot & 3)) {              // (the waves finish a chunk's result in turn)
             f32x4_t y = (meet[par][1][0][lane] + meet[par][1][1][lane]) + (meet[par][1][2][lane] + meet[par][1][3][lane]);
@@ -256,8 +269,17 @@ __global__ void __launch_bounds__(256) channel_walk_kernel(ChunkArgs p) {
             for (int i = 0; i < 4; ++i)
                 if (row + i < t1 && c < C) p.out[(size_t)(row + i) * p.ldo + (size_t)head * C + c] = y[i];
         }
-        now = next;
-    }
+    };
+    // (a turn past the last chunk loads a chunk again and does nothing: no way out of the unrolled loop, so that the waits of
+    // every turn stay exact)
+    for (int turn = first; turn < last; turn += AHEAD)
+#pragma unroll
+        for (int d = 0; d < AHEAD; ++d) {
+            if (turn + d < last) walk(ring[d], turn + d, d & 1);          // (uniform over the block)
+            __builtin_amdgcn_sched_barrier(0);
+            fetch(ring[d], turn + d + AHEAD);
+            __builtin_amdgcn_sched_barrier(0);
+        }
 #pragma unroll
     for (int j = 0; j < NT; ++j)
 #pragma unroll
@@ -292,10 +314,10 @@ extern "C" int cisr_channel_chunks(const float* q, int ldq, const float* k, int 
         int err = CISR_LAUNCH_CHECK();
         if (err) return err;
         const dim3 grid(heads, p.Cp / 16, segments);
-        if (nt == 1) channel_walk_kernel<1><<<grid, 256, 0, stream>>>(p);
-        else if (nt == 2) channel_walk_kernel<2><<<grid, 256, 0, stream>>>(p);
-        else if (nt == 3) channel_walk_kernel<3><<<grid, 256, 0, stream>>>(p);
-        else channel_walk_kernel<4><<<grid, 256, 0, stream>>>(p);
+        if (nt == 1) channel_walk_kernel<1, 4><<<grid, 256, 0, stream>>>(p);
+        else if (nt == 2) channel_walk_kernel<2, 4><<<grid, 256, 0, stream>>>(p);
+        else if (nt == 3) channel_walk_kernel<3, 2><<<grid, 256, 0, stream>>>(p);
+        else channel_walk_kernel<4, 2><<<grid, 256, 0, stream>>>(p);
         err = CISR_LAUNCH_CHECK();
         if (err) return err;
     }

@@ -1527,7 +1527,8 @@ def channel_delta_inputs(proj, taps, conv_state, qkv, seg_of_row, seg_start, sta
     (K - 1) channels], which moves on) and silu, and the heads of q and k become unit vectors: qkv float [T, channels].
     decay [T, heads * dim] = exp(-exp(a_log) softplus(proj[:, decay_at:] . decay_up^T + dt_bias)), decay_up [heads * dim,
     rank]; gate [T, heads * vdim] = proj[:, gate_at:] . gate_up^T, gate_up [heads * vdim, rank] (both as low_rank_rows makes
-    them, float or bf16; with bf16 matrices the projections' coordinates enter as two bf16 numbers each, on the matrix cores)."""
+    them, float or bf16; with bf16 matrices the projections' coordinates enter as two bf16 numbers each, on the matrix cores,
+    and their columns and the rows of proj start at 16-byte words)."""
     T = qkv.shape[0]
     pp, ld = _rows_of(proj, "proj")
     K, channels = taps.shape

@@ -289,11 +289,15 @@ class ChannelDeltaRule(GatedDeltaRule):
         t, conv = self._tensor, self.names["conv"]
         # one product with float results: [q | k | v | write | decay's first half | gate's first half]
         inputs = ("q", "k", "v", "write", "decay_down", "gate_down")
-        parts = [matrix_operand(tensors[t(p)], dtype) for p in inputs]
-        starts = [sum(p.shape[0] for p in parts[:i]) for i in range(len(parts) + 1)]
-        self.at = dict(zip(inputs, starts))
-        if starts[-1] % 8:
-            parts.append(torch.zeros(8 - starts[-1] % 8, self.hidden, dtype=parts[0].dtype, device=parts[0].device))
+        parts, self.at, rows = [], {}, 0
+        for p in inputs:
+            part = matrix_operand(tensors[t(p)], dtype)
+            parts.append(part)
+            self.at[p] = rows
+            rows += part.shape[0]
+            if p in inputs[2:] and rows % 8:      # (behind the convolution's channels every part starts at a 32-byte word)
+                parts.append(torch.zeros(8 - rows % 8, self.hidden, dtype=part.dtype, device=part.device))
+                rows += 8 - rows % 8
         self.w_in = torch.cat(parts, dim=0).contiguous()
         self.w_out = matrix_operand(tensors[t("o")], dtype)
         self.decay_up, self.gate_up = (ops.low_rank_rows(matrix_operand(tensors[t(p)], dtype)) for p in ("decay_up", "gate_up"))

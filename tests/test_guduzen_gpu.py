@@ -202,8 +202,10 @@ def test_delta_rule_with_a_decay_a_channel_over_segments_with_states_carried_and
     td, eps, share = TORCH[dtype], 1e-5, heads // kv_heads
     qk, inner = kv_heads * dim, heads * vdim
     ch, (ra, rg) = 2 * qk + inner, ranks
-    at_b, at_a, at_g = ch, ch + heads, ch + heads + ra
-    width = -(-(at_g + rg) // 8) * 8
+    up4 = lambda n: -(-n // 4) * 4
+    at_b, at_a = ch, up4(ch + heads)
+    at_g = up4(at_a + ra)
+    width = up4(at_g + rg)
     taps_w, up_a, up_g = rng.standard_normal((ch, taps)), rng.standard_normal((heads * dim, ra)) / ra ** 0.5, rng.standard_normal((inner, rg)) / rg ** 0.5
     dt_bias, a_log, weight = rng.standard_normal(heads * dim) - 1, rng.standard_normal(heads) - 1, 1 + 0.1 * rng.standard_normal(vdim)
     dt_bias[0] = 30.0                                            # softplus far from zero: a decay that is nothing
