@@ -32,8 +32,12 @@ struct ChannelInputs {
 typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8_t;
 typedef __attribute__((ext_vector_type(4))) float f32x4_t;
 
+// exp(-rate softplus(z)), softplus(z) = max(z, 0) + log(1 + e), e = exp(-|z|); log(1 + e) = log(u) e / (u - 1) with the rounded
+// u = 1 + e: the rounding of u cancels, so small e keep their precision.
 __device__ __forceinline__ float channel_decay(float z, float rate) {
-    return expf(-rate * (fmaxf(z, 0.f) + log1pf(expf(-fabsf(z)))));
+    const float e = __expf(-fabsf(z)), u = 1.0f + e;
+    const float l = u == 1.0f ? e : __logf(u) * e * __builtin_amdgcn_rcpf(u - 1.0f);
+    return __expf(-rate * (fmaxf(z, 0.f) + l));
 }
 
 // An item of the convolution for the rows t .. t + n - 1 (n <= RB): a q head, a k head (both made unit vectors) or up to 256

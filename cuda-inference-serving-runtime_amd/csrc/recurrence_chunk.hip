@@ -11,8 +11,8 @@
 // Every product of decays is made by multiplying decays along the rows: no quotients and no differences of logarithms, so a
 // channel whose decays vanish within a chunk costs neither range nor precision.  A first kernel makes, chunk by chunk and
 // all side by side, what does not need the state: M V, M Kg, D q, P, D(15, i) k and D(15); a second walks a segment's chunks
-// in order, a block a (head, 16 columns of S): its four waves own the rows of S in turn, two products with S0, one meeting
-// through LDS, one product into S.  Rows behind a segment's end count as k = q = v = 0 with decays of one.
+// in order, a block a (head, 16 columns of S): its waves own the rows of S in turn, two products with S0, one meeting through
+// LDS, one product into S.  Rows behind a segment's end count as k = q = v = 0 with decays of one.
 #include "common.h"
 
 #define CHUNK 16
@@ -180,14 +180,16 @@ __global__ void __launch_bounds__(256, 4) channel_chunk_kernel(ChunkArgs p) {
     }
 }
 
-// A block a (head, segment, 16 columns).  The state's rows in tiles of 16: wave w owns the tiles w NT .. w NT + NT - 1, in
-// the matrix instruction's result layout (lane l: rows 4 (l / 16) + i of the tile, column l % 16), which serves as its
-// right operand as it is when the left operand's inner index runs alike: every operand is a 16-byte load.
+// A block a (head, segment, 16 columns), five waves.  The state's rows in tiles of 16: wave w < 4 owns the tiles w NT ..
+// w NT + NT - 1, in the matrix instruction's result layout (lane l: rows 4 (l / 16) + i of the tile, column l % 16), which
+// serves as its right operand as it is when the left operand's inner index runs alike: every operand is a 16-byte load.
+// A chunk is M Kg S0 (each wave its rows' share), the meeting of the four shares through LDS, (D q) S0 while they travel,
+// and the new S; the fifth wave adds the shares of (D q) S0 and P U, one chunk behind, and writes the results.
 // AHEAD chunks' operands are in flight (an even number).  The loads of a chunk are kept together in program order: they
 // return in order, so a chunk's wait then leaves those of the chunks behind it in flight.
 template <int NT, int AHEAD>
-__global__ void __launch_bounds__(256, 2) channel_walk_kernel(ChunkArgs p) {
-    __shared__ f32x4_t meet[2][2][4][WAVE];         // [chunk parity][M Kg S0, (D q) S0][wave][lane]
+__global__ void __launch_bounds__(320) __attribute__((amdgpu_waves_per_eu(2, 2))) channel_walk_kernel(ChunkArgs p) {
+    __shared__ f32x4_t share_w[2][4][WAVE], share_o[2][4][WAVE];         // [chunk parity][wave][lane]
     const int head = blockIdx.x, seg = blockIdx.z, wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
     const int t0 = p.seg_start[seg], t1 = p.seg_start[seg + 1];
     if (t1 <= t0) return;
@@ -196,6 +198,48 @@ __global__ void __launch_bounds__(256, 2) channel_walk_kernel(ChunkArgs p) {
     if (first >= last) return;
     const int m = lane % 16, kg = lane / 16, R = p.R, C = p.C, Rp = p.Rp;
     const int c = blockIdx.y * 16 + m;
+    const size_t per = (size_t)chunk_floats(Rp, p.Cp);
+    auto operands = [&](int slot) { return (const char*)(p.work + ((size_t)(min(slot, last - 1) - p.slot0) * p.heads + head) * per); };
+    // byte offsets of this lane's words from a chunk's operands (a uniform address): 32 bits
+    const unsigned at_u = (3u * CHUNK * Rp + c * CHUNK + 4 * kg) * 4u;
+    auto writes = [&](f32x4_t u, int par) {          // the rows' writes: M V - M Kg S0
+        return u - ((share_w[par][0][lane] + share_w[par][1][lane]) + (share_w[par][2][lane] + share_w[par][3][lane]));
+    };
+    if (wave == 4) {
+        const unsigned at_p = (3u * CHUNK * Rp + CHUNK * p.Cp + m * CHUNK + 4 * kg) * 4u;
+        struct Result { f32x4_t u, pr; } ring[AHEAD];
+        auto fetch = [&](Result& r, int slot) {
+            const char* w = operands(slot);
+            r.u = *(const f32x4_t*)(w + at_u);
+            r.pr = *(const f32x4_t*)(w + at_p);
+        };
+#pragma unroll
+        for (int d = 0; d < AHEAD; ++d) fetch(ring[d], first + d);
+        f32x4_t u = {0.f, 0.f, 0.f, 0.f}, pr = u;
+        auto finish = [&](int slot, int par) {       // o of the chunk before, whose shares are there now
+            f32x4_t y = (share_o[par][0][lane] + share_o[par][1][lane]) + (share_o[par][2][lane] + share_o[par][3][lane]);
+#pragma unroll
+            for (int i = 0; i < 4; ++i) y = __builtin_amdgcn_mfma_f32_16x16x4f32(pr[i], u[i], y, 0, 0, 0);
+            const int row = t0 + (slot - base) * CHUNK + 4 * kg;
+#pragma unroll
+            for (int i = 0; i < 4; ++i)
+                if (row + i < t1 && c < C) p.out[(size_t)(row + i) * p.ldo + (size_t)head * C + c] = y[i];
+        };
+        for (int turn = first; turn < last; turn += AHEAD)
+#pragma unroll
+            for (int d = 0; d < AHEAD; ++d) {
+                if (turn + d < last) {
+                    __syncthreads();
+                    if (turn + d > first) finish(turn + d - 1, (d + 1) & 1);
+                    u = writes(ring[d].u, d & 1);
+                    pr = ring[d].pr;
+                }
+                fetch(ring[d], turn + d + AHEAD);
+            }
+        __syncthreads();
+        finish(last - 1, (last - 1 - first) & 1);
+        return;
+    }
     float* state = p.state + (long long)p.state_slots[seg] * p.slot_stride + (size_t)head * R * C;
     f32x4_t S[NT];
 #pragma unroll
@@ -205,81 +249,68 @@ __global__ void __launch_bounds__(256, 2) channel_walk_kernel(ChunkArgs p) {
             const int r = (wave * NT + j) * 16 + 4 * kg + i;
             S[j][i] = r < R && c < C ? state[(size_t)r * C + c] : 0.f;
         }
-    struct Operands { f32x4_t kg[NT], qg[NT], kd[NT], g[NT], u, pr; } ring[AHEAD];
-    const size_t per = (size_t)chunk_floats(Rp, p.Cp);
-    // byte offsets of this lane's words from a chunk's operands (a uniform address): 32 bits
+    struct Operands { f32x4_t kg[NT], qg[NT], kd[NT], g[NT], u; } ring[AHEAD];
     unsigned at_k[NT], at_d[NT], at_g[NT];
-    const unsigned q_words = CHUNK * Rp * 4u, at_u = (3u * CHUNK * Rp + c * CHUNK + 4 * kg) * 4u,
-                   at_p = (3u * CHUNK * Rp + CHUNK * p.Cp + m * CHUNK + 4 * kg) * 4u;
+    float mine[NT];
+    const unsigned q_words = CHUNK * Rp * 4u;
 #pragma unroll
     for (int j = 0; j < NT; ++j) {
-        const unsigned r = min((wave * NT + j) * 16, Rp - 16);          // (a wave without this tile reads another: its S is zero)
+        const unsigned r = min((wave * NT + j) * 16, Rp - 16);          // (a wave without this tile reads another: its S stays zero)
+        mine[j] = (wave * NT + j) * 16 < Rp ? 1.f : 0.f;
         at_k[j] = (m * Rp + r + 4 * kg) * 4u;
         at_d[j] = (2u * CHUNK * Rp + (r + m) * CHUNK + 4 * kg) * 4u;
         at_g[j] = (3u * CHUNK * Rp + CHUNK * p.Cp + CHUNK * CHUNK + r + 4 * kg) * 4u;
     }
     auto fetch = [&](Operands& o, int slot) {
-        slot = min(slot, last - 1);
-        const char* w = (const char*)(p.work + ((size_t)(slot - p.slot0) * p.heads + head) * per);
+        const char* w = operands(slot);
 #pragma unroll
-        for (int j = 0; j < NT; ++j) {
-            o.kg[j] = *(const f32x4_t*)(w + at_k[j]);
-            o.qg[j] = *(const f32x4_t*)(w + q_words + at_k[j]);
-        }
+        for (int j = 0; j < NT; ++j) o.kg[j] = *(const f32x4_t*)(w + at_k[j]);
+#pragma unroll
+        for (int j = 0; j < NT; ++j) o.qg[j] = *(const f32x4_t*)(w + q_words + at_k[j]);
         o.u = *(const f32x4_t*)(w + at_u);
 #pragma unroll
         for (int j = 0; j < NT; ++j) {
             o.g[j] = *(const f32x4_t*)(w + at_g[j]);
             o.kd[j] = *(const f32x4_t*)(w + at_d[j]);
         }
-        o.pr = *(const f32x4_t*)(w + at_p);
+    };
+    auto walk = [&](Operands& now, int par) {
+        f32x4_t w = {0.f, 0.f, 0.f, 0.f}, o = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int j = 0; j < NT; ++j)
+#pragma unroll
+            for (int i = 0; i < 4; ++i) w = __builtin_amdgcn_mfma_f32_16x16x4f32(now.kg[j][i], S[j][i], w, 0, 0, 0);
+        share_w[par][wave][lane] = w;
+        __syncthreads();           // (the other parity's shares were read before the barrier before this one's writes)
+        const f32x4_t u = writes(now.u, par);
+#pragma unroll
+        for (int j = 0; j < NT; ++j)
+#pragma unroll
+            for (int i = 0; i < 4; ++i) o = __builtin_amdgcn_mfma_f32_16x16x4f32(now.qg[j][i], S[j][i], o, 0, 0, 0);
+        share_o[par][wave][lane] = o;
+#pragma unroll
+        for (int j = 0; j < NT; ++j) S[j] *= now.g[j];
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+#pragma unroll
+            for (int j = 0; j < NT; ++j) S[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(now.kd[j][i] * mine[j], u[i], S[j], 0, 0, 0);
     };
 #pragma unroll
     for (int d = 0; d < AHEAD; ++d) {
         fetch(ring[d], first + d);
         __builtin_amdgcn_sched_barrier(0);
     }
-    auto walk = [&](Operands& now, int slot, int par) {
-        f32x4_t w = {0.f, 0.f, 0.f, 0.f}, o = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-        for (int j = 0; j < NT; ++j)
-#pragma unroll
-            for (int i = 0; i < 4; ++i) w = __builtin_amdgcn_mfma_f32_16x16x4f32(now.kg[j][i], S[j][i], w, 0, 0, 0);
-        meet[par][0][wave][lane] = w;
-#pragma unroll
-        for (int j = 0; j < NT; ++j)
-#pragma unroll
-            for (int i = 0; i < 4; ++i) o = __builtin_amdgcn_mfma_f32_16x16x4f32(now.qg[j][i], S[j][i], o, 0, 0, 0);
-        meet[par][1][wave][lane] = o;
-        __syncthreads();                       // (the other parity's buffers were read before the barrier before this one's writes)
-        const f32x4_t u = now.u - ((meet[par][0][0][lane] + meet[par][0][1][lane]) + (meet[par][0][2][lane] + meet[par][0][3][lane]));
-#pragma unroll
-        for (int j = 0; j < NT; ++j) {
-            S[j] *= now.g[j];
-            const float mine = (wave * NT + j) * 16 < Rp ? 1.f : 0.f;          // (a tile beyond the state's rows stays zero)
-#pragma unroll
-            for (int i = 0; i < 4; ++i) S[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(now.kd[j][i] * mine, u[i], S[j], 0, 0, 0);
-        }
-        if (wave == (slot & 3)) {              // (the waves finish a chunk's result in turn)
-            f32x4_t y = (meet[par][1][0][lane] + meet[par][1][1][lane]) + (meet[par][1][2][lane] + meet[par][1][3][lane]);
-#pragma unroll
-            for (int i = 0; i < 4; ++i) y = __builtin_amdgcn_mfma_f32_16x16x4f32(now.pr[i], u[i], y, 0, 0, 0);
-            const int row = t0 + (slot - base) * CHUNK + 4 * kg;
-#pragma unroll
-            for (int i = 0; i < 4; ++i)
-                if (row + i < t1 && c < C) p.out[(size_t)(row + i) * p.ldo + (size_t)head * C + c] = y[i];
-        }
-    };
     // (a turn past the last chunk loads a chunk again and does nothing: no way out of the unrolled loop, so that the waits of
     // every turn stay exact)
     for (int turn = first; turn < last; turn += AHEAD)
 #pragma unroll
         for (int d = 0; d < AHEAD; ++d) {
-            if (turn + d < last) walk(ring[d], turn + d, d & 1);          // (uniform over the block)
+            if (turn + d < last) walk(ring[d], d & 1);          // (uniform over the block)
             __builtin_amdgcn_sched_barrier(0);
             fetch(ring[d], turn + d + AHEAD);
             __builtin_amdgcn_sched_barrier(0);
         }
+    __syncthreads();               // (the last chunk's shares of (D q) S0 are there)
 #pragma unroll
     for (int j = 0; j < NT; ++j)
 #pragma unroll
@@ -314,10 +345,10 @@ extern "C" int cisr_channel_chunks(const float* q, int ldq, const float* k, int 
         int err = CISR_LAUNCH_CHECK();
         if (err) return err;
         const dim3 grid(heads, p.Cp / 16, segments);
-        if (nt == 1) channel_walk_kernel<1, 4><<<grid, 256, 0, stream>>>(p);
-        else if (nt == 2) channel_walk_kernel<2, 4><<<grid, 256, 0, stream>>>(p);
-        else if (nt == 3) channel_walk_kernel<3, 2><<<grid, 256, 0, stream>>>(p);
-        else channel_walk_kernel<4, 2><<<grid, 256, 0, stream>>>(p);
+        if (nt == 1) channel_walk_kernel<1, 4><<<grid, 320, 0, stream>>>(p);
+        else if (nt == 2) channel_walk_kernel<2, 4><<<grid, 320, 0, stream>>>(p);
+        else if (nt == 3) channel_walk_kernel<3, 2><<<grid, 320, 0, stream>>>(p);
+        else channel_walk_kernel<4, 2><<<grid, 320, 0, stream>>>(p);
         err = CISR_LAUNCH_CHECK();
         if (err) return err;
     }
