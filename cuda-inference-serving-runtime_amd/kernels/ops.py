@@ -374,6 +374,10 @@ def attention_rowwise(q, q_row_stride, kcache, vcache, tables, seg_of_row, posit
 LIBRARY_MIN_ROWS = 65
 LIBRARY_MIN_BYTES = 8 << 20
 LIBRARY_GATED_MIN_ROWS, LIBRARY_GATED_MIN_BYTES = 33, 64 << 20
+# Products that end with their store (no residual sum or activation that a kernel here has in its epilogue) go there already
+# with 2 MB of weights: at 2,048 rows 1,792 x 2,048 takes 21 us there and 35 in the tiled kernel here (float results; the
+# same with bf16), 2,048 x 1,536 18 and 28, 1,024 x 1,024 10 and 14; at 128 rows 6.8 and 12.7, 5.8 and 9.9, 5.3 and 6.9.
+LIBRARY_PLAIN_MIN_BYTES = 2 << 20
 
 
 def attention_talking(q, q_row_stride, kcache, vcache, tables, seg_of_row, positions, out, heads, kv_heads, vdim, pad, page_size,
@@ -500,16 +504,17 @@ class ScratchPool:
 DEFAULT_SCRATCH = ScratchPool()
 
 
-def library_ok(m, w, gated=False):
-    """`gated`: the product of gate and up, whose activation is a kernel of its own after the library's product.  With
+def library_ok(m, w, gated=False, plain=False):
+    """`plain`: the product ends with its store.  `gated`: the product of gate and up, whose activation is a kernel of its own after the library's product.  With
     weights of 64 MB and more it goes there from 33 rows on: 64 rows against the 8B sizes' 235 MB take 60.7 us there and
     69.7 in the wide kernel here (58.4 against 63.0 at 33 rows; 23.0 against 26.5 at the 1.7B sizes), the activation
     included; the other products of 33 to 64 rows are as fast here."""
     least = LIBRARY_MIN_ROWS
     if gated and w.numel() * 2 >= LIBRARY_GATED_MIN_BYTES:
         least = min(least, LIBRARY_GATED_MIN_ROWS)
+    least_bytes = LIBRARY_PLAIN_MIN_BYTES if plain and w.shape[0] % 8 == 0 and w.shape[1] % 8 == 0 else LIBRARY_MIN_BYTES
     return (LIBRARY_MIN_ROWS > 0 and m >= least and w.dtype == torch.bfloat16 and w.is_contiguous()
-            and w.numel() * 2 >= LIBRARY_MIN_BYTES)
+            and w.numel() * 2 >= least_bytes)
 
 
 def _scratch_bf16(scratch, device, rows, cols):
@@ -541,7 +546,7 @@ def gemm(a, w, out, residual=None, after_norm=False, scratch=None):
             raise KernelError("gemm: float operands need a float output")
         code = lib().cisr_gemm_f32(a.data_ptr(), a.stride(0), w.data_ptr(), w.stride(0), out.data_ptr(), out.stride(0),
                                    rp, ldr, m, n, k, _stream())
-    elif (a.dtype == torch.bfloat16 and library_ok(m, w) and a.is_contiguous() and out.is_contiguous()
+    elif (a.dtype == torch.bfloat16 and library_ok(m, w, plain=residual is None) and a.is_contiguous() and out.is_contiguous()
           and (residual is None or residual is out)):
         if residual is None:
             # (float results are the library's float accumulators as they are: 2,048 rows against 10,240 x 2,048 take 83 us
@@ -934,21 +939,23 @@ def gemm_merged_ok(m, w, heads, dim, splits):
             and w.data_ptr() % 16 == 0 and bool(lib().cisr_gemm_merged_ok(int(m), int(w.shape[0]), int(heads), int(dim), int(splits))))
 
 
-def gemm_merged(partials, heads, dim, w, out, residual):
-    """out[M, N] = residual + merge(partials) . w^T in float: the output projection of a decode step whose attention
+def gemm_merged(partials, heads, dim, w, out, residual=None):
+    """out[M, N] = residual + merge(partials) . w^T in float (residual None: the product alone): the output projection of a decode step whose attention
     was split over `splits` blocks along the keys and left unmerged (attention_mfma with merge=False).
     partials = (bf16 [M, heads, splits, dim] normalised partial outputs, float [M, heads, splits, 2] statistics, splits)."""
     part_o, part_ml, splits = partials
     m, n = out.shape
     if not gemm_merged_ok(m, w, heads, dim, splits) or w.shape[0] != n:
         raise KernelError("gemm_merged: shape not supported by the fused kernel")
-    if out.dtype != torch.float32 or out.stride(1) != 1 or tuple(residual.shape) != (m, n) or residual.dtype != torch.float32 or residual.stride(1) != 1:
+    if out.dtype != torch.float32 or out.stride(1) != 1 or (residual is not None and (
+            tuple(residual.shape) != (m, n) or residual.dtype != torch.float32 or residual.stride(1) != 1)):
         raise KernelError("gemm_merged: float output and residual [M, N]")
     if part_o.numel() < m * heads * splits * dim or part_ml.numel() < m * heads * splits * 2:
         raise KernelError("gemm_merged: partial results too small")
     _check(lib().cisr_gemm_merged_bf16(_dev(part_o, "part_o", torch.bfloat16), _dev(part_ml, "part_ml", torch.float32), int(splits),
                                        int(heads), int(dim), w.data_ptr(), w.stride(0), out.data_ptr(), out.stride(0),
-                                       residual.data_ptr(), residual.stride(0), m, n, _stream()), "gemm_merged")
+                                       *((None, 0) if residual is None else (residual.data_ptr(), residual.stride(0))), m, n,
+                                       _stream()), "gemm_merged")
     return out
 
 

@@ -223,7 +223,12 @@ class NormedGatedAttention(Mixer):
         q = ops.qk_norm_scatter(qkv, self.q_weight, self.k_weight, ctx.buffer("gattn.q", (T, nh * pad), ctx.dtype), *written,
                                 nh, nkv, D, V, pad, view.page_size, self.eps, bias=self.b_in, plain_norm=self.qk_norm == "plain")
         out = ctx.buffer("gattn.out", (T, nh * pad), ctx.dtype)
-        kernel.paged_attention(ctx, q, nh * pad, kcache, vcache, view, out, nh, nkv, pad, self.window, self.scale, tuning=self.tuning)
+        # a decode step of few rows may leave the partial results of its split keys to the output projection
+        merges = None if self.head_gate or pad != V else (lambda splits: ops.gemm_merged_ok(T, self.w_out, nh, V, splits))
+        unmerged = kernel.paged_attention(ctx, q, nh * pad, kcache, vcache, view, out, nh, nkv, pad, self.window, self.scale,
+                                          defer_merge=merges, tuning=self.tuning)
+        if unmerged is not None:
+            return ops.gemm_merged(unmerged, nh, V, self.w_out, ctx.buffer("gattn.y", (T, self.hidden), torch.float32))
         first_gate = sum(self._projections().values())
         gates = qkv[:, first_gate:first_gate + nh] if self.head_gate else None
         act = out
