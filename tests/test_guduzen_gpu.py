@@ -163,6 +163,23 @@ def test_biases_and_norms_without_a_weight_land_in_the_pages(dtype, float_rows, 
     assert torch.equal(alone, q_out)
 
 
+@pytest.mark.parametrize("m, n, heads, dim, splits", [(1, 96, 4, 64, 8), (3, 200, 2, 128, 4), (8, 192, 6, 64, 8), (14, 64, 3, 32, 4), (1, 4096, 16, 128, 8)])
+def test_a_product_that_merges_split_attention_without_a_residual(m, n, heads, dim, splits):
+    from runtime.kernels import ops
+    gen = torch.Generator(device="cuda").manual_seed(m * n)
+    k = heads * dim
+    w = (torch.randn(n, k, generator=gen, device="cuda") / k ** 0.5).to(torch.bfloat16)
+    assert ops.gemm_merged_ok(m, w, heads, dim, splits)
+    part = torch.randn(m, heads, splits, dim, generator=gen, device="cuda").to(torch.bfloat16)
+    ml = torch.stack([torch.randn(m, heads, splits, generator=gen, device="cuda"), 0.5 + torch.rand(m, heads, splits, generator=gen, device="cuda")], dim=-1).contiguous()
+    out = torch.full((m, n), float("nan"), device="cuda")
+    ops.gemm_merged((part, ml, splits), heads, dim, w, out)
+    share = torch.exp2((ml[..., 0] - ml[..., 0].amax(dim=-1, keepdim=True)).double()) * ml[..., 1].double()
+    share = share / share.sum(dim=-1, keepdim=True)
+    want = (share[..., None] * part.double()).sum(dim=2).reshape(m, k).cpu() @ w.double().cpu().t()
+    close(out.cpu().numpy(), want.numpy(), 1e-2)
+
+
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("rank", [13, 40, 96, 300])
 def test_latents_without_a_turning_part_land_in_the_pages(dtype, rank):
@@ -377,6 +394,36 @@ def test_long_decoding_from_the_first_token(folders, name, dtype, execution):
     assert_close(np.concatenate(got), plain_logits(folders[name], first), dtype, "decoded from the first token")
     assert_close(np.concatenate(got2), plain_logits(folders[name], second), dtype, "the late one")
     runner.cache.check()
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_a_prompt_of_thousands_of_tokens_then_single_tokens(tmp_path, dtype, no_gemv):
+    """Long enough that the rule's chunks take several launches (one call's operands wait in a bounded memory), that the
+    attention of a decoded token is split along its keys and merged by the output projection, and that a window of a
+    thousand keys has passed; with the first tokens still in the state."""
+    from guduzen_models import attention, config, delta, latent
+    from runtime.engine import StepEntry
+    from runtime.kernels import ops
+    cfg = config(150, 192, 2, 12.0, 1e-5, [attention(6, 3, 64, 64, 0.125, 1000, ff=160), delta(3, 1, 64, 48, 4), latent(3, 32, 24, 96, 64, 0.2, ff=96),
+                                           attention(6, 3, 64, 64, 0.125, None, kv_from=0)])
+    cfg["layers"][3]["mixer"]["mask"] = {"size": 1400}
+    folder = write_folder(tmp_path / "m", cfg, 91, sharp=True, ranks=(20, 24))
+    n = ops.CHANNEL_SLAB * 16 + 140
+    tokens = random_tokens(17, n + 8, cfg["vocab"])
+    want = plain_logits(folder, tokens)
+    merged = []
+    plain_merge = ops.gemm_merged
+    runner = make_runner(folder, dtype, pages=-(-len(tokens) // 16) + 2)
+    runner.create("r")
+    places = list(range(5)) + list(range(990, 1010)) + list(range(1390, 1410)) + list(range(n - 40, n))
+    got = [runner.step([StepEntry("r", tokens[:n], places)]).cpu().numpy()]
+    try:
+        ops.gemm_merged = lambda *a, **k: (merged.append(1), plain_merge(*a, **k))[1]
+        got += [runner.step([StepEntry("r", [t], [0])]).cpu().numpy() for t in tokens[n:]]
+    finally:
+        ops.gemm_merged = plain_merge
+    assert dtype == "float32" or merged, "no output projection merged the split keys: the test does not test it"
+    assert_close(np.concatenate(got), want[places + list(range(n, n + 8))], dtype, "a long prompt and what follows")
 
 
 def mixed(V, seed, lengths=(70, 33, 120, 9, 64, 97, 40, 130), live_at_once=4):
