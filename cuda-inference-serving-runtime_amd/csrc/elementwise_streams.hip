@@ -2,7 +2,7 @@
 // after the other, x[t, s * H + d], float.  Around a sublayer,
 //
 //   u = sum_s in[s] x_s,  h = rmsnorm(u) * w          what the sublayer reads
-//   x_t <- sum_s mix[s, t] x_s + out[t] y             every stream from the old ones (mix is indexed [from, to])
+//   x_t <- sum_s mix[s, t] x_s + out[t] y             the right side as it was (row s of mix: where x_s goes)
 //
 // and the two meet in one kernel: the write of a sublayer's result y and the read (and norm) of the sublayer that comes
 // next, so a row of streams makes one trip to memory a sublayer.  y is finished float rows or the partial sums of a cut

@@ -1695,8 +1695,8 @@ def streams_read(x, streams, w_in, weight, eps, out, rows=None):
 
 
 def streams_step(x, streams, y, mix, w_out, read=None):
-    """x_t <- sum_s mix[s, t] x_s + w_out[t] y in place, every stream from the old ones: x float [T, streams * H], y float
-    [T, H] or the Partials of such a product, mix float [streams, streams] (from, to), w_out float [streams].  `read` = (w_in
+    """x_t <- sum_s mix[s, t] x_s + w_out[t] y in place, the right side as it was: x float [T, streams * H], y float
+    [T, H] or the Partials of such a product, mix float [streams, streams], w_out float [streams].  `read` = (w_in
     float [streams], weight float [H], eps, out [T, H]): what reads the streams next is made by the same kernel,
     out = rmsnorm(sum_s w_in[s] x_s) * weight of the new streams."""
     xp, dim = _streams_of(x, streams, "streams_step")

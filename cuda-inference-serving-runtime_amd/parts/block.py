@@ -337,8 +337,8 @@ class PostNormBlock(Part):
 
 class HyperConnectedBlock(Part):
     """A residual of `streams` streams x_1 .. x_s (rows [T, streams * hidden], one stream after the other) and, around each
-    sublayer q (1: mixer, 2: feed-forward), weights over them: u = sum_s in[s] x_s; y = sublayer(norm(u)); then, every stream
-    from the old ones, x_t <- sum_s mix[s, t] x_s + out[t] y (mix is indexed [from, to]).  Tensors
+    sublayer q (1: mixer, 2: feed-forward), weights over them: u = sum_s in[s] x_s; y = sublayer(norm(u));
+    x_t <- sum_s mix[s, t] x_s + out[t] y for all t, the right side as it was (row s of mix: where x_s goes).  Tensors
     `<name>.<names[q]>.in|out|mix`.  `mixer_norm` and `ffn_norm` are StreamsNorm parts: they own `in` and make the read.
     The write of a sublayer's result and the read of whatever reads the streams next (this block's feed-forward, or the
     following block) are one kernel (ops.streams_step).  Mixer and feed-forward give their result without a residual sum

@@ -19,7 +19,7 @@ the state in the cache manager's state slots, in float in every mode:
                          head's result RMS-normed, times silu of a gate projection, then the output projection.
 
   ChannelDeltaRule       the same rule with a decay a head and key channel (ops.channel_delta_scan): g_t = exp(-exp(A_log)
-                         softplus(Wa2 Wa1 h + dt_bias)) from a low-rank projection, acting on the rows of S; the result's
+                         softplus(Wa2 Wa1 h + dt_bias)) from a low-rank projection, row r of S shrinking by g_t[r]; the result's
                          gate is sigmoid of a low-rank projection.
 
   MinGRU                 no heads and no matrix state: S_t = (1 - z_t) S_(t-1) + z_t c_t element by element over `width`

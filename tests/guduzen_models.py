@@ -96,7 +96,7 @@ def tensor_shapes(c, ranks=(16, 24)):
 
 
 def make_weights(c, seed, sharp=False, ranks=(16, 24)):
-    """Matrices N(0, 1/in), biases N(0, 0.3), norms stored around zero N(0, 0.2), the other norms 1 + N(0, 0.1), streams read
+    """Matrices N(0, 1/in), biases N(0, 0.3), norms that add one to their weight N(0, 0.2), the other norms 1 + N(0, 0.1), streams read
     with 1/s + N(0, 0.2), written with 1 + N(0, 0.2) and mixed with 0.8 I + N(0, 0.09/s), convolutions N(0, 1/taps), A_log N(-1, 1), dt_bias
     N(-1, 1), embedding rows N(0, 16/width).  `sharp`: the query latents' norms times 2.5 (a query's result hangs on single keys),
     A_log N(-5, 0.5) (the state keeps the first tokens)."""

@@ -26,7 +26,7 @@ def rmsnorm(x, weight, eps):
 
 
 def rmsnorm_around_zero(x, weight, eps):
-    """The norm whose stored weight is the deviation from one."""
+    """The RMS norm with weight 1 + w."""
     return rms(x, eps) * (1.0 + np.asarray(weight, np.float64))
 
 
@@ -72,7 +72,7 @@ def read_streams(X, w_in):
 
 
 def write_streams(X, mix, w_out, y):
-    """X_t <- sum_s mix[s, t] X_s + out[t] y, every stream from the old ones (mix is indexed [from, to])."""
+    """X_t <- sum_s mix[s, t] X_s + out[t] y, with the X_s as they were (row s of mix: where X_s goes)."""
     mix, w_out = np.asarray(mix, np.float64), np.asarray(w_out, np.float64)
     return np.stack([sum(mix[s, t] * X[s] for s in range(X.shape[0])) + w_out[t] * y for t in range(X.shape[0])])
 
@@ -122,7 +122,7 @@ def latent_attention(h, w, p, m, eps):
 # -- the delta rule with a decay a key channel --------------------------------------------------------------------
 
 def short_conv(x, taps):
-    """y[t, c] = silu(sum_j taps[c, j] x[t - (n - 1) + j, c]), zeros before the start."""
+    """y[t, c] = silu(sum_j taps[c, j] x[t - (n - 1) + j, c]), x zero at negative times."""
     taps = np.asarray(taps, np.float64)
     n = taps.shape[1]
     padded = np.concatenate([np.zeros((n - 1, x.shape[1])), x])

@@ -19,7 +19,7 @@ def test_streams_are_read_mixed_and_written_from_the_old_ones():
     w_in, w_out, mix, y = rng.standard_normal(3), rng.standard_normal(3), rng.standard_normal((3, 3)), rng.standard_normal((4, 5))
     np.testing.assert_allclose(P.read_streams(X, w_in), w_in[0] * X[0] + w_in[1] * X[1] + w_in[2] * X[2], rtol=1e-12)
     got = P.write_streams(X, mix, w_out, y)
-    for t in range(3):                        # [from, to]: stream t takes column t of the mix
+    for t in range(3):                        # stream t takes column t of the mix
         np.testing.assert_allclose(got[t], mix[0, t] * X[0] + mix[1, t] * X[1] + mix[2, t] * X[2] + w_out[t] * y, rtol=1e-12)
     # with one stream, weights of one: the plain residual sum
     one = P.spread(X[0], 1)
