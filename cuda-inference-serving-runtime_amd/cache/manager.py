@@ -246,14 +246,15 @@ class CacheManager:
     def most_pages_held(self, tokens, portion):
         """Per group, the most pages one request holds at any time while it grows to `tokens` cached tokens in
         steps of at most `portion`: all of them where every key is kept; where only a window is kept, the pages
-        that a window and a portion can touch (a portion is placed after the pages behind its first token's
+        that the kept first keys, a window and a portion can touch (a portion is placed after the pages behind its first token's
         window went back)."""
         P = self.page_size
         out = []
         for group in self.groups:
             pages = -(-tokens // P)
             if group.need.window is not None:
-                pages = min(pages, (group.need.window + max(1, portion) - 1) // P + 2)
+                kept = -(-getattr(group.need, "keep_first", 0) // P)
+                pages = min(pages, kept + (group.need.window + max(1, portion) - 1) // P + 2)
             out.append(pages)
         return out
 

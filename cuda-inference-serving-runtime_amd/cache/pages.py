@@ -69,6 +69,13 @@ class ChunkNeed(KVNeed):
 
 
 @dataclass(frozen=True)
+class KeptWindowNeed(KVNeed):
+    """Keys and values of a mixer whose rows see the last `window` keys and, for ever, the first `keep_first` of the
+    sequence: the pages that hold only keys between the two go back."""
+    keep_first: int = 0
+
+
+@dataclass(frozen=True)
 class StateNeed:
     """A fixed-size state per request."""
     shape: tuple
@@ -125,14 +132,15 @@ class CacheGroup:
 
     # -- planning -------------------------------------------------------
     def _dead_pages(self, request, length):
-        """Logical pages that no later query can see (window groups only)."""
+        """Logical pages that no later query can see, a range (window groups only)."""
+        P = self.page_size
         rule = getattr(self.need, "first_visible", None)
         if rule is not None:               # (a need with a rule of its own: blocks of positions)
-            return rule(length) // self.page_size
+            return range(0, rule(length) // P)
         if self.need.window is None:
-            return 0
+            return range(0)
         first_visible = max(0, length - self.need.window + 1)  # the next token sits at `length`
-        return first_visible // self.page_size
+        return range(-(-getattr(self.need, "keep_first", 0) // P), first_visible // P)
 
     def pages_needed(self, request, length, n_new):
         """Fresh pages an append of n_new tokens takes (after trimming)."""
@@ -146,8 +154,8 @@ class CacheGroup:
 
     def trimmable(self, request, length):
         table = self.tables[request]
-        return sum(1 for j in range(min(self._dead_pages(request, length), len(table)))
-                   if table[j] >= 0 and self.pool.refs[table[j]] == 1)
+        return sum(1 for j in self._dead_pages(request, length)
+                   if j < len(table) and table[j] >= 0 and self.pool.refs[table[j]] == 1)
 
     # -- mutation -------------------------------------------------------
     def _touch(self, request):
@@ -156,8 +164,8 @@ class CacheGroup:
 
     def trim(self, request, length):
         table = self.tables[request]
-        for j in range(min(self._dead_pages(request, length), len(table))):
-            if table[j] >= 0:
+        for j in self._dead_pages(request, length):
+            if j < len(table) and table[j] >= 0:
                 self.pool.drop(table[j])
                 table[j] = -1
                 self._touch(request)

@@ -6,4 +6,5 @@ from .ditazen import DitazenConfig
 from .noresun import NoresunConfig
 from .zovozen import ZovozenConfig
 from .guduzen import GuduzenConfig
+from .movazen import MovazenConfig
 from .presets import preset, preset_names

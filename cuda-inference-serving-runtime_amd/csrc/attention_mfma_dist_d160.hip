@@ -1,0 +1,4 @@
+// Matrix-core attention whose scores fall with the distance, heads of up to 160 coordinates (see attention_mfma.inc).
+#define ATTN_DISTANCE
+#define DPAD 160
+#include "attention_mfma.inc"

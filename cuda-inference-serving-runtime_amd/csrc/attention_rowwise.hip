@@ -17,6 +17,9 @@
 
 // SIGMOID: the weight of a visible key is sigmoid(score + head_bias[head]) and the weights are not normed over the keys
 // (no maximum, no denominator: a row's result is the plain sum, and the partial results of splits are added).
+// Of the softmax law only: `slopes` (float [heads] or null): slopes[head] * (position - key) is taken off a score;
+// `sink` (float [heads] or null): a score that joins the denominator and has no value; `keep_first`: with a window, the
+// first keys that are seen besides it.
 template <typename T, bool SIGMOID>
 __global__ void __launch_bounds__(64)
 attn_rowwise_kernel(const T* __restrict__ q, int q_row_stride, const T* __restrict__ kcache,
@@ -24,7 +27,8 @@ attn_rowwise_kernel(const T* __restrict__ q, int q_row_stride, const T* __restri
                     const int* __restrict__ seg_of_row, const int* __restrict__ positions,
                     T* __restrict__ out, float* __restrict__ part_o, float* __restrict__ part_ml,
                     int heads, int kv_heads, int dim, int page_size, int width, int window,
-                    float scale, int splits, const float* __restrict__ head_bias) {
+                    float scale, int splits, const float* __restrict__ head_bias, const float* __restrict__ slopes,
+                    const float* __restrict__ sink, int keep_first) {
     __shared__ float qs[MAX_HEAD_DIM];
     __shared__ float ps[WAVE];
     __shared__ long long rowoff[WAVE];   // offset of a key's first value element (values are [D, page_size] in a page)
@@ -38,13 +42,15 @@ attn_rowwise_kernel(const T* __restrict__ q, int q_row_stride, const T* __restri
 #pragma unroll
     for (int c = 0; c < MAX_COORDS; ++c) acc[c] = 0.f;
     float m = -INFINITY, l = 0.f;
-    int begin = 0, end = 0;
+    // the visible keys in order, numbered from `lo - kept`: the kept first ones, then lo .. p
+    int begin = 0, end = 0, lo = 0, kept = 0, p = 0;
     if (seg >= 0) {
-        const int p = positions[row];
-        const int lo = (window > 0 && p + 1 > window) ? p + 1 - window : 0;
+        p = positions[row];
+        lo = (window > 0 && p + 1 > window) ? p + 1 - window : 0;
+        kept = min(keep_first, lo);
         const int hi = p + 1;
-        const int chunk = (hi - lo + splits - 1) / splits;
-        begin = lo + split * chunk;
+        const int chunk = (hi - lo + kept + splits - 1) / splits;
+        begin = lo - kept + split * chunk;
         end = min(hi, begin + chunk);
     }
     if (begin < end) {
@@ -53,8 +59,8 @@ attn_rowwise_kernel(const T* __restrict__ q, int q_row_stride, const T* __restri
         __syncthreads();
         const int* table = tables + (size_t)seg * width;
         for (int base = begin; base < end; base += WAVE) {
-            const int t = base + lane;
-            const bool valid = t < end;
+            const bool valid = base + lane < end;
+            const int t = base + lane < lo ? base + lane - (lo - kept) : base + lane;       // the key's position
             float s = -INFINITY;
             long long off = 0;
             if (valid) {
@@ -65,6 +71,7 @@ attn_rowwise_kernel(const T* __restrict__ q, int q_row_stride, const T* __restri
                 float dot = 0.f;
                 for (int d = 0; d < dim; ++d) dot += qs[d] * load_f32(kr + d);
                 s = dot * scale;
+                if (!SIGMOID && slopes) s -= slopes[head] * (float)(p - t);
             }
             float pj, alpha;
             if (SIGMOID) {
@@ -95,6 +102,14 @@ attn_rowwise_kernel(const T* __restrict__ q, int q_row_stride, const T* __restri
                 }
             }
         }
+    }
+    if (!SIGMOID && sink && split == 0 && seg >= 0) {       // (counted once: by the first wave along the keys)
+        const float m_new = fmaxf(m, sink[head]);
+        const float alpha = expf(m - m_new);
+#pragma unroll
+        for (int c = 0; c < MAX_COORDS; ++c) acc[c] *= alpha;
+        l = l * alpha + expf(sink[head] - m_new);
+        m = m_new;
     }
     const float inv = SIGMOID ? 1.0f : l > 0.f ? 1.0f / l : 0.f;
     if (splits == 1) {
@@ -236,11 +251,11 @@ extern "C" int cisr_attn_rowwise_sigmoid(const void* q, int q_row_stride, const 
     if (dtype == DT_F32)
         attn_rowwise_kernel<float, true><<<grid, 64, 0, stream>>>((const float*)q, q_row_stride, (const float*)kcache,
             (const float*)vcache, tables, seg_of_row, positions, (float*)out, part_o, part_ml, heads, kv_heads,
-            dim, page_size, width, window, scale, splits, head_bias);
+            dim, page_size, width, window, scale, splits, head_bias, nullptr, nullptr, 0);
     else
         attn_rowwise_kernel<bf16_t, true><<<grid, 64, 0, stream>>>((const bf16_t*)q, q_row_stride, (const bf16_t*)kcache,
             (const bf16_t*)vcache, tables, seg_of_row, positions, (bf16_t*)out, part_o, part_ml, heads, kv_heads,
-            dim, page_size, width, window, scale, splits, head_bias);
+            dim, page_size, width, window, scale, splits, head_bias, nullptr, nullptr, 0);
     int err = CISR_LAUNCH_CHECK();
     if (err || splits == 1) return err;
     if (dtype == DT_F32) attn_merge_sum_kernel<float><<<dim3(rows, heads), merge_threads(dim), 0, stream>>>(part_o, (float*)out, heads, dim, splits);
@@ -252,19 +267,20 @@ extern "C" int cisr_attn_rowwise(const void* q, int q_row_stride, const void* kc
                                  const int* tables, const int* seg_of_row, const int* positions, void* out,
                                  float* part_o, float* part_ml, int rows, int heads, int kv_heads, int dim,
                                  int page_size, int width, int window, float scale, int splits, int dtype,
-                                 hipStream_t stream) {
+                                 const float* slopes, const float* sink, int keep_first, hipStream_t stream) {
     if (rows <= 0) return 0;
-    if (dim > MAX_HEAD_DIM || dim <= 0 || heads % kv_heads || splits < 1 || splits > 65535 || heads > 65535)
+    if (dim > MAX_HEAD_DIM || dim <= 0 || heads % kv_heads || splits < 1 || splits > 65535 || heads > 65535 || keep_first < 0 ||
+        (keep_first > 0 && window <= 0))
         return (int)hipErrorInvalidValue;
     dim3 grid(rows, heads, splits);
     if (dtype == DT_F32)
         attn_rowwise_kernel<float, false><<<grid, 64, 0, stream>>>((const float*)q, q_row_stride, (const float*)kcache,
             (const float*)vcache, tables, seg_of_row, positions, (float*)out, part_o, part_ml, heads, kv_heads,
-            dim, page_size, width, window, scale, splits, nullptr);
+            dim, page_size, width, window, scale, splits, nullptr, slopes, sink, keep_first);
     else
         attn_rowwise_kernel<bf16_t, false><<<grid, 64, 0, stream>>>((const bf16_t*)q, q_row_stride, (const bf16_t*)kcache,
             (const bf16_t*)vcache, tables, seg_of_row, positions, (bf16_t*)out, part_o, part_ml, heads, kv_heads,
-            dim, page_size, width, window, scale, splits, nullptr);
+            dim, page_size, width, window, scale, splits, nullptr, slopes, sink, keep_first);
     int err = CISR_LAUNCH_CHECK();
     if (err || splits == 1) return err;
     const int threads = merge_threads(dim);

@@ -4,7 +4,7 @@
 //                                                    and with the next norm of x made on the way)
 //   act = g sigmoid(slope g) (u + shift), g = min(gate, limit), u = clamp(up, -limit, limit)
 //   q, k normed per head, q into a buffer of padded heads, k and v into the pages of the cache
-//   out[t, h, :] = attn[t, h, :vdim] * sigmoid(gate[t, h])
+//   out[t, h, :] = attn[t, h, :vdim] * sigmoid(gate[t, h])        (or a gate an element)
 // Statistics and the residual stream are float; `T` is the storage type of activations (float or bf16).
 #include "common.h"
 
@@ -220,16 +220,18 @@ extern "C" int cisr_glu_clamped(const void* gu, void* act, int rows, int inter, 
 // page_size] (coordinates vdim..pad-1 zero): heads of `pad` coordinates are what the attention kernels read.
 // wq / wk null: that side is not normed, or with `plain` normed without a weight.  The rows may be float where the pages are
 // bf16 (TI, T); `bias` (float, over the q, k and v columns, or null) is added before everything else.  has_kv 0: the rows
-// hold queries only (a layer that reads the keys of another).
+// hold queries only (a layer that reads the keys of another).  `every` > 0: queries (after the bias and the norm) are
+// multiplied by 1 + coef ln(floor((position + 1) / every) + 1).
 template <typename TI, typename T>
 __global__ void __launch_bounds__(256)
 qk_norm_scatter_kernel(const TI* __restrict__ qkv, int ld, const float* __restrict__ bias, const float* __restrict__ wq, const float* __restrict__ wk,
                        T* __restrict__ q_out, T* __restrict__ kcache, T* __restrict__ vcache,
                        const int* __restrict__ slots, int heads, int kv_heads, int dim, int vdim, int pad,
-                       int page_size, float eps, int plain, int has_kv) {
+                       int page_size, float eps, int plain, int has_kv, const int* __restrict__ positions, float coef, int every) {
     const int row = blockIdx.x, wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
     const TI* src = qkv + (size_t)row * ld;
     const int slot = slots ? slots[row] : -1;
+    const float warmth = every > 0 ? 1.0f + coef * logf((float)((positions[row] + 1) / every + 1)) : 1.0f;
     const int items = heads + (has_kv ? 2 * kv_heads : 0);
     for (int item = blockIdx.y * 4 + wave; item < items; item += 4 * gridDim.y) {
         if (item < heads + kv_heads) {
@@ -246,7 +248,8 @@ qk_norm_scatter_kernel(const TI* __restrict__ qkv, int ld, const float* __restri
                 vals[i] = d < dim ? load_f32(v + d) + (b ? b[d] : 0.f) : 0.f;
                 ss += vals[i] * vals[i];
             }
-            const float scale = w || plain ? 1.0f / sqrtf(wave_sum(ss) / (float)dim + eps) : 1.0f;
+            float scale = w || plain ? 1.0f / sqrtf(wave_sum(ss) / (float)dim + eps) : 1.0f;
+            if (is_q) scale *= warmth;
             T* dst = is_q ? q_out + ((size_t)row * heads + head) * pad
                           : kcache + (((size_t)(slot / page_size) * kv_heads + head) * page_size + slot % page_size) * pad;
 #pragma unroll
@@ -270,14 +273,15 @@ qk_norm_scatter_kernel(const TI* __restrict__ qkv, int ld, const float* __restri
 extern "C" int cisr_qk_norm_scatter(const void* qkv, int ld, const float* bias, const float* wq, const float* wk, void* q_out,
                                     void* kcache, void* vcache, const int* slots, int rows, int heads, int kv_heads, int dim,
                                     int vdim, int pad, int page_size, float eps, int plain, int has_kv, int in_dtype, int dtype,
-                                    hipStream_t stream) {
+                                    const int* positions, float coef, int every, hipStream_t stream) {
     if (rows <= 0) return 0;
     if (dim <= 0 || vdim <= 0 || dim > pad || vdim > pad || pad > 256 || page_size <= 0 || (in_dtype == DT_BF16 && dtype == DT_F32) ||
-        ld < heads * dim + (has_kv ? kv_heads * (dim + vdim) : 0) || (has_kv && (!kcache || !vcache || !slots)))
+        ld < heads * dim + (has_kv ? kv_heads * (dim + vdim) : 0) || (has_kv && (!kcache || !vcache || !slots)) ||
+        every < 0 || (every > 0 && !positions))
         return (int)hipErrorInvalidValue;
     const dim3 grid(rows, min((heads + (has_kv ? 2 * kv_heads : 0) + 3) / 4, 65535));
 #define QK_NORM_SCATTER(TI, T) qk_norm_scatter_kernel<TI, T><<<grid, 256, 0, stream>>>((const TI*)qkv, ld, bias, wq, wk, (T*)q_out, \
-        (T*)kcache, (T*)vcache, slots, heads, kv_heads, dim, vdim, pad, page_size, eps, plain, has_kv)
+        (T*)kcache, (T*)vcache, slots, heads, kv_heads, dim, vdim, pad, page_size, eps, plain, has_kv, positions, coef, every)
     if (dtype == DT_F32) QK_NORM_SCATTER(float, float);
     else if (in_dtype == DT_F32) QK_NORM_SCATTER(float, bf16_t);
     else QK_NORM_SCATTER(bf16_t, bf16_t);
@@ -285,10 +289,11 @@ extern "C" int cisr_qk_norm_scatter(const void* qkv, int ld, const float* bias, 
     return CISR_LAUNCH_CHECK();
 }
 
-// ------------------------------------------------------------------ one gate a head
+// ------------------------------------------------------------------ one gate a head, or one an element
 // out[t, h, d] = attn[t, h, d] * sigmoid(gate[t * ld_gate + h]) for d < vdim; attn has heads of `pad` coordinates.
-template <typename T>
-__global__ void head_gate_kernel(const T* __restrict__ attn, const T* __restrict__ gate, int ld_gate,
+// per_element: the gate is gate[t * ld_gate + h * vdim + d].  The gates may be float beside bf16 activations (TG, T).
+template <typename TG, typename T>
+__global__ void head_gate_kernel(const T* __restrict__ attn, const TG* __restrict__ gate, int ld_gate, int per_element,
                                  T* __restrict__ out, int heads, int vdim, int pad, size_t n) {
     const size_t i = (size_t)blockIdx.x * 256 + threadIdx.x;
     if (i >= n) return;
@@ -296,13 +301,14 @@ __global__ void head_gate_kernel(const T* __restrict__ attn, const T* __restrict
     const size_t th = i / vdim;
     const int h = (int)(th % heads);
     const size_t t = th / heads;
-    const float g = gate ? 1.0f / (1.0f + expf(-load_f32(gate + t * ld_gate + h))) : 1.0f;
+    const float g = gate ? 1.0f / (1.0f + expf(-load_f32(gate + t * ld_gate + (per_element ? h * vdim + d : h)))) : 1.0f;
     store_f32(out + i, load_f32(attn + th * pad + d) * g);
 }
 
 // the same for bf16 with vdim and pad multiples of eight: eight elements a thread, 16-byte accesses
+template <typename TG>
 __global__ void __launch_bounds__(256)
-head_gate_bf16x8_kernel(const bf16_t* __restrict__ attn, const bf16_t* __restrict__ gate, int ld_gate, bf16_t* __restrict__ out,
+head_gate_bf16x8_kernel(const bf16_t* __restrict__ attn, const TG* __restrict__ gate, int ld_gate, int per_element, bf16_t* __restrict__ out,
                         int heads, int vdim8, int pad, size_t n8) {
     typedef __attribute__((ext_vector_type(4))) uint32_t u32x4_t;
     const size_t i = (size_t)blockIdx.x * 256 + threadIdx.x;
@@ -311,28 +317,42 @@ head_gate_bf16x8_kernel(const bf16_t* __restrict__ attn, const bf16_t* __restric
     const size_t th = i / vdim8;
     const int h = (int)(th % heads);
     const size_t t = th / heads;
-    const float g = gate ? 1.0f / (1.0f + expf(-bf16_to_f32(gate[t * ld_gate + h]))) : 1.0f;
+    float g[8];
+    if (per_element) {
+#pragma unroll
+        for (int k = 0; k < 8; ++k) g[k] = load_f32(gate + t * ld_gate + (size_t)(h * vdim8 + d8) * 8 + k);
+#pragma unroll
+        for (int k = 0; k < 8; ++k) g[k] = 1.0f / (1.0f + expf(-g[k]));
+    } else {
+        const float one = gate ? 1.0f / (1.0f + expf(-load_f32(gate + t * ld_gate + h))) : 1.0f;
+#pragma unroll
+        for (int k = 0; k < 8; ++k) g[k] = one;
+    }
     const u32x4_t a = *(const u32x4_t*)(attn + th * pad + d8 * 8);
     const uint32_t aw[4] = {a.x, a.y, a.z, a.w};
     uint32_t o[4];
 #pragma unroll
-    for (int k = 0; k < 4; ++k) o[k] = pack_bf16x2(__uint_as_float(aw[k] << 16) * g, __uint_as_float(aw[k] & 0xffff0000u) * g);
+    for (int k = 0; k < 4; ++k) o[k] = pack_bf16x2(__uint_as_float(aw[k] << 16) * g[2 * k], __uint_as_float(aw[k] & 0xffff0000u) * g[2 * k + 1]);
     *(u32x4_t*)(out + i * 8) = (u32x4_t){o[0], o[1], o[2], o[3]};
 }
 
-extern "C" int cisr_head_gate(const void* attn, const void* gate, int ld_gate, void* out, int rows, int heads, int vdim,
-                              int pad, int dtype, hipStream_t stream) {
+extern "C" int cisr_head_gate(const void* attn, const void* gate, int ld_gate, int per_element, void* out, int rows, int heads, int vdim,
+                              int pad, int gate_dtype, int dtype, hipStream_t stream) {
     const size_t n = (size_t)rows * heads * vdim;
     if (n == 0) return 0;
-    if (vdim > pad) return (int)hipErrorInvalidValue;
+    if (vdim > pad || (per_element && !gate) || (gate_dtype == DT_BF16 && dtype == DT_F32)) return (int)hipErrorInvalidValue;
     if (dtype == DT_BF16 && vdim % 8 == 0 && pad % 8 == 0 && ((uintptr_t)attn) % 16 == 0 && ((uintptr_t)out) % 16 == 0) {
         const size_t n8 = n / 8;
-        head_gate_bf16x8_kernel<<<(unsigned)((n8 + 255) / 256), 256, 0, stream>>>((const bf16_t*)attn, (const bf16_t*)gate, ld_gate,
-                                                                                (bf16_t*)out, heads, vdim / 8, pad, n8);
+        const unsigned blocks8 = (unsigned)((n8 + 255) / 256);
+        if (gate_dtype == DT_F32) head_gate_bf16x8_kernel<float><<<blocks8, 256, 0, stream>>>((const bf16_t*)attn, (const float*)gate, ld_gate, per_element,
+                                                                                             (bf16_t*)out, heads, vdim / 8, pad, n8);
+        else head_gate_bf16x8_kernel<bf16_t><<<blocks8, 256, 0, stream>>>((const bf16_t*)attn, (const bf16_t*)gate, ld_gate, per_element,
+                                                                         (bf16_t*)out, heads, vdim / 8, pad, n8);
         return CISR_LAUNCH_CHECK();
     }
     const unsigned blocks = (unsigned)((n + 255) / 256);
-    if (dtype == DT_F32) head_gate_kernel<float><<<blocks, 256, 0, stream>>>((const float*)attn, (const float*)gate, ld_gate, (float*)out, heads, vdim, pad, n);
-    else head_gate_kernel<bf16_t><<<blocks, 256, 0, stream>>>((const bf16_t*)attn, (const bf16_t*)gate, ld_gate, (bf16_t*)out, heads, vdim, pad, n);
+    if (dtype == DT_F32) head_gate_kernel<float, float><<<blocks, 256, 0, stream>>>((const float*)attn, (const float*)gate, ld_gate, per_element, (float*)out, heads, vdim, pad, n);
+    else if (gate_dtype == DT_F32) head_gate_kernel<float, bf16_t><<<blocks, 256, 0, stream>>>((const bf16_t*)attn, (const float*)gate, ld_gate, per_element, (bf16_t*)out, heads, vdim, pad, n);
+    else head_gate_kernel<bf16_t, bf16_t><<<blocks, 256, 0, stream>>>((const bf16_t*)attn, (const bf16_t*)gate, ld_gate, per_element, (bf16_t*)out, heads, vdim, pad, n);
     return CISR_LAUNCH_CHECK();
 }

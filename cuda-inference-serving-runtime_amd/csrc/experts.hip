@@ -96,20 +96,27 @@ extern "C" int cisr_experts_route(const float* logits, int ld, const float* bias
     return CISR_LAUNCH_CHECK();
 }
 
-// Routing by scores: s = softmax of the logits over all `outputs` of the router; the choice goes by s + correction
-// (null: by s), held to the `keep` groups, of `groups` equal groups of neighbours, whose largest choice score is
-// largest (groups 0: no groups); the `top` largest are chosen (the lowest index wins a tie) and weigh s itself, not
-// normed again.  A thread a row; float arithmetic.
+// Routing by scores: s = softmax of the logits over all `outputs` of the router, or with law.sigmoid the sigmoid of each;
+// the choice goes by s + correction (null: by s), held to the `keep` groups, of `groups` equal groups of neighbours, whose
+// score is largest (groups 0: no groups): a group's score is its largest choice score, or with law.pairs the sum of its
+// two largest (of its one, if it has one member); the `top` largest are chosen (the lowest index wins a tie) and weigh s
+// itself, with law.floor >= 0 divided by the sum of the chosen s plus that floor.  A thread a row; float arithmetic.
+struct ScoreLaw { int sigmoid, pairs; float floor; };
+
+__device__ __forceinline__ float logistic(float z) { return 1.0f / (1.0f + expf(-z)); }
+
 __global__ void __launch_bounds__(256)
 route_scored_kernel(const float* __restrict__ logits, int ld, const float* __restrict__ correction, int* __restrict__ chosen,
-                    float* __restrict__ weights, int rows, int outputs, int top, int groups, int keep) {
+                    float* __restrict__ weights, int rows, int outputs, int top, int groups, int keep, ScoreLaw law) {
     const int row = blockIdx.x * 256 + threadIdx.x;
     if (row >= rows) return;
     const float* lr = logits + (size_t)row * ld;
     float largest = -INFINITY, den = 0.f;
-    for (int e = 0; e < outputs; ++e) largest = fmaxf(largest, lr[e]);
-    for (int e = 0; e < outputs; ++e) den += expf(lr[e] - largest);
-    auto score = [&](int e) { return expf(lr[e] - largest) / den; };
+    if (!law.sigmoid) {
+        for (int e = 0; e < outputs; ++e) largest = fmaxf(largest, lr[e]);
+        for (int e = 0; e < outputs; ++e) den += expf(lr[e] - largest);
+    }
+    auto score = [&](int e) { return law.sigmoid ? logistic(lr[e]) : expf(lr[e] - largest) / den; };
     auto choice = [&](int e) { return score(e) + (correction ? correction[e] : 0.f); };
     unsigned long long kept = ~0ull;                       // groups that may be chosen from (at most 64 groups)
     const int per = groups > 0 ? outputs / groups : outputs;
@@ -120,8 +127,13 @@ route_scored_kernel(const float* __restrict__ logits, int ld, const float* __res
             float bv = -INFINITY;
             for (int g = 0; g < groups; ++g) {
                 if ((kept >> g) & 1ull) continue;
-                float gv = -INFINITY;
-                for (int e = g * per; e < (g + 1) * per; ++e) gv = fmaxf(gv, choice(e));
+                float gv = -INFINITY, g2 = -INFINITY;
+                for (int e = g * per; e < (g + 1) * per; ++e) {
+                    const float v = choice(e);
+                    g2 = fmaxf(g2, fminf(gv, v));
+                    gv = fmaxf(gv, v);
+                }
+                if (law.pairs && per > 1) gv += g2;
                 if (best < 0 || gv > bv) { best = g; bv = gv; }
             }
             kept |= 1ull << best;
@@ -143,6 +155,11 @@ route_scored_kernel(const float* __restrict__ logits, int ld, const float* __res
         chosen[(size_t)row * top + k] = best;
         weights[(size_t)row * top + k] = score(best);
     }
+    if (law.floor >= 0.f) {
+        float sum = 0.f;
+        for (int k = 0; k < top; ++k) sum += weights[(size_t)row * top + k];
+        for (int k = 0; k < top; ++k) weights[(size_t)row * top + k] /= sum + law.floor;
+    }
 }
 
 // The same routing with a wave a row (routers of at most 512 outputs): lane l holds the outputs l, l + 64, ...; the
@@ -151,7 +168,8 @@ route_scored_kernel(const float* __restrict__ logits, int ld, const float* __res
 #define ROUTE_PER_LANE 8
 __global__ void __launch_bounds__(256)
 route_scored_wave_kernel(const float* __restrict__ logits, int ld, const float* __restrict__ correction, int* __restrict__ chosen,
-                         float* __restrict__ weights, int rows, int outputs, int top, int groups, int keep) {
+                         float* __restrict__ weights, int rows, int outputs, int top, int groups, int keep, ScoreLaw law) {
+    __shared__ float scores_of[4][WAVE * ROUTE_PER_LANE];      // (law.pairs: a wave's choice scores, by output)
     const int row = blockIdx.x * 4 + threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
     if (row >= rows) return;
     const float* lr = logits + (size_t)row * ld;
@@ -165,8 +183,11 @@ route_scored_wave_kernel(const float* __restrict__ logits, int ld, const float* 
     largest = wave_max(largest);
     float den = 0.f, s[ROUTE_PER_LANE], c[ROUTE_PER_LANE];
 #pragma unroll
-    for (int i = 0; i < ROUTE_PER_LANE; ++i) { s[i] = lane + WAVE * i < outputs ? expf(z[i] - largest) : 0.f; den += s[i]; }
-    den = wave_sum(den);
+    for (int i = 0; i < ROUTE_PER_LANE; ++i) {
+        s[i] = lane + WAVE * i < outputs ? (law.sigmoid ? logistic(z[i]) : expf(z[i] - largest)) : 0.f;
+        den += s[i];
+    }
+    den = law.sigmoid ? 1.0f : wave_sum(den);
 #pragma unroll
     for (int i = 0; i < ROUTE_PER_LANE; ++i) {
         const int e = lane + WAVE * i;
@@ -191,7 +212,36 @@ route_scored_wave_kernel(const float* __restrict__ logits, int ld, const float* 
     if (groups > 0) {
         const int per = outputs / groups;
         unsigned long long kept = 0ull;
-        for (int k = 0; k < keep; ++k) {
+        // by pairs: lane g adds the two largest choice scores of group g (at most 64 groups)
+        float group_score = -INFINITY;
+        if (law.pairs) {
+            float* mine = scores_of[threadIdx.x / WAVE];
+#pragma unroll
+            for (int i = 0; i < ROUTE_PER_LANE; ++i) if (lane + WAVE * i < outputs) mine[lane + WAVE * i] = c[i];
+            __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+            __builtin_amdgcn_wave_barrier();
+            if (lane < groups) {
+                float first = -INFINITY, second = -INFINITY;
+                for (int j = 0; j < per; ++j) {
+                    const float v = mine[lane * per + j];
+                    second = fmaxf(second, fminf(first, v));
+                    first = fmaxf(first, v);
+                }
+                group_score = per > 1 ? first + second : first;
+            }
+        }
+        for (int k = 0; law.pairs && k < keep; ++k) {
+            float bv = lane < groups && !((kept >> lane) & 1ull) ? group_score : -INFINITY;
+            int bg = lane < groups && !((kept >> lane) & 1ull) ? lane : 0x7fffffff;
+#pragma unroll
+            for (int off = 32; off > 0; off >>= 1) {
+                const float ov = __shfl_xor(bv, off, WAVE);
+                const int og = __shfl_xor(bg, off, WAVE);
+                if (ov > bv || (ov == bv && og < bg)) { bv = ov; bg = og; }
+            }
+            kept |= 1ull << bg;
+        }
+        for (int k = 0; !law.pairs && k < keep; ++k) {
             // the group, not kept yet, whose largest choice score is largest (the lowest group wins a tie): a group's
             // largest score is the score of its best member, and of two equal ones the lower index lies in the lower group
             float v[ROUTE_PER_LANE];
@@ -215,6 +265,7 @@ route_scored_wave_kernel(const float* __restrict__ logits, int ld, const float* 
             if (e < outputs && !((kept >> (e / per)) & 1ull)) c[i] = -INFINITY;
         }
     }
+    float total = 0.f, mine_w = 0.f;                             // lane k keeps the k-th choice's score
     for (int k = 0; k < top; ++k) {
         float bv; int be;
         best_of(c, bv, be);
@@ -224,14 +275,17 @@ route_scored_wave_kernel(const float* __restrict__ logits, int ld, const float* 
             if (lane + WAVE * i == be) { share = s[i]; c[i] = -INFINITY; }
         }
         share = wave_sum(share);                                 // (one lane holds it)
-        if (lane == 0) { chosen[(size_t)row * top + k] = be; weights[(size_t)row * top + k] = share; }
+        total += share;
+        if (lane == k) mine_w = share;
+        if (lane == 0) chosen[(size_t)row * top + k] = be;
     }
+    if (lane < top) weights[(size_t)row * top + lane] = law.floor >= 0.f ? mine_w / (total + law.floor) : mine_w;
 }
 
 // `experts` of the router's `outputs` have matrices (the first ones): only their pairs are arranged into tiles.
 extern "C" int cisr_experts_route_scored(const float* logits, int ld, const float* correction, int* chosen, float* weights, int rows,
-                                         int outputs, int experts, int top, int groups, int keep, int max_tiles, int* pair_of_pos,
-                                         int* tile_expert, hipStream_t stream) {
+                                         int outputs, int experts, int top, int groups, int keep, int sigmoid, int group_pairs,
+                                         float floor, int max_tiles, int* pair_of_pos, int* tile_expert, hipStream_t stream) {
     if (rows <= 0) return 0;
     const bool arrange = pair_of_pos != nullptr;
     if (outputs <= 0 || experts <= 0 || experts > outputs || top <= 0 || top > MAX_TOP || top > outputs || experts > 4096 || groups < 0 ||
@@ -239,10 +293,11 @@ extern "C" int cisr_experts_route_scored(const float* logits, int ld, const floa
         (arrange && (!tile_expert || (long long)max_tiles * EX_TILE < (long long)rows * top + (long long)experts * (EX_TILE - 1))))
         return (int)hipErrorInvalidValue;
     // steps of few rows: a wave a row; many rows keep a thread a row (the GPU is full either way, and a thread's chain is short beside the step)
+    const ScoreLaw law = {sigmoid, group_pairs, floor};
     if (outputs <= WAVE * ROUTE_PER_LANE && rows <= 4096)
-        route_scored_wave_kernel<<<(rows + 3) / 4, 256, 0, stream>>>(logits, ld, correction, chosen, weights, rows, outputs, top, groups, keep);
+        route_scored_wave_kernel<<<(rows + 3) / 4, 256, 0, stream>>>(logits, ld, correction, chosen, weights, rows, outputs, top, groups, keep, law);
     else
-        route_scored_kernel<<<(rows + 255) / 256, 256, 0, stream>>>(logits, ld, correction, chosen, weights, rows, outputs, top, groups, keep);
+        route_scored_kernel<<<(rows + 255) / 256, 256, 0, stream>>>(logits, ld, correction, chosen, weights, rows, outputs, top, groups, keep, law);
     int err = CISR_LAUNCH_CHECK();
     if (err || !arrange) return err;
     arrange_kernel<<<1, 1024, 3 * experts * sizeof(int), stream>>>(chosen, rows * top, experts, max_tiles, pair_of_pos, tile_expert);
@@ -278,6 +333,67 @@ extern "C" int cisr_experts_combine(const float* down, const float* weights, con
     if (dim <= 0 || top <= 0 || top > MAX_TOP || experts < 0) return (int)hipErrorInvalidValue;
     if (x_dtype == DT_F32) experts_combine_kernel<float><<<rows, 256, 0, stream>>>(down, weights, chosen, (const float*)x, shared, y, dim, top, experts);
     else experts_combine_kernel<bf16_t><<<rows, 256, 0, stream>>>(down, weights, chosen, (const bf16_t*)x, shared, y, dim, top, experts);
+    return CISR_LAUNCH_CHECK();
+}
+
+// The sum of a row's choices straight into the residual stream: x[row] += sum_k weights[row, k] down[row top + k] +
+// sigmoid(gate[row]) shared[row] (gate null: 1; shared null: nothing), and what reads the stream next on the way: out =
+// rmsnorm(x) * next_w, or with next_w null the new row itself (out null: nothing).  A block a row; the row waits in
+// registers (E floats a thread) while it is summed.  `chosen` outside the experts: that choice adds nothing.
+template <int E, typename TO>
+__global__ void __launch_bounds__(256)
+experts_add_kernel(float* __restrict__ x, const float* __restrict__ down, const float* __restrict__ weights, const int* __restrict__ chosen,
+                   const float* __restrict__ shared, const float* __restrict__ gate, int ld_gate, int dim, int top, int experts,
+                   const float* __restrict__ next_w, float next_eps, TO* __restrict__ out) {
+    __shared__ float red[4];
+    const size_t row = blockIdx.x;
+    float w[MAX_TOP];
+    for (int k = 0; k < top; ++k) {
+        const int e = chosen[row * top + k];
+        w[k] = e >= 0 && e < experts ? weights[row * top + k] : 0.f;
+    }
+    const float sg = shared && gate ? logistic(gate[row * ld_gate]) : 1.0f;
+    float v[E], vx[E], ss = 0.f;
+#pragma unroll
+    for (int e = 0; e < E; ++e) {
+        const int d = threadIdx.x + 256 * e;
+        vx[e] = d < dim ? x[row * dim + d] : 0.f;
+        v[e] = shared && d < dim ? sg * shared[row * dim + d] : 0.f;
+    }
+    for (int k = 0; k < top; ++k)
+#pragma unroll
+        for (int e = 0; e < E; ++e) {
+            const int d = threadIdx.x + 256 * e;
+            if (d < dim && w[k] != 0.f) v[e] += w[k] * down[(row * top + k) * dim + d];
+        }
+#pragma unroll
+    for (int e = 0; e < E; ++e) {
+        const int d = threadIdx.x + 256 * e;
+        vx[e] += v[e];
+        if (d < dim) { x[row * dim + d] = vx[e]; ss += vx[e] * vx[e]; }
+    }
+    if (!out) return;
+    const float rs = next_w ? 1.0f / sqrtf(block_sum<256>(ss, red) / (float)dim + next_eps) : 1.0f;
+#pragma unroll
+    for (int e = 0; e < E; ++e) {
+        const int d = threadIdx.x + 256 * e;
+        if (d < dim) store_f32(out + row * dim + d, vx[e] * rs * (next_w ? next_w[d] : 1.0f));
+    }
+}
+
+extern "C" int cisr_experts_add(float* x, const float* down, const float* weights, const int* chosen, const float* shared, const float* gate,
+                                int ld_gate, int rows, int dim, int top, int experts, const float* next_w, float next_eps, void* out,
+                                int out_dtype, hipStream_t stream) {
+    if (rows <= 0) return 0;
+    if (dim <= 0 || dim > 16384 || top <= 0 || top > MAX_TOP || experts < 0 || (next_w && !out)) return (int)hipErrorInvalidValue;
+#define EX_ADD(E, TO) experts_add_kernel<E, TO><<<rows, 256, 0, stream>>>(x, down, weights, chosen, shared, gate, ld_gate, dim, top, experts, next_w, next_eps, (TO*)out)
+#define EX_ADD_TYPES(E) do { if (out_dtype == DT_F32) EX_ADD(E, float); else EX_ADD(E, bf16_t); } while (0)
+    if (dim <= 1024) EX_ADD_TYPES(4);
+    else if (dim <= 2048) EX_ADD_TYPES(8);
+    else if (dim <= 4096) EX_ADD_TYPES(16);
+    else EX_ADD_TYPES(64);
+#undef EX_ADD_TYPES
+#undef EX_ADD
     return CISR_LAUNCH_CHECK();
 }
 
@@ -492,16 +608,18 @@ expert_gemm_mfma_kernel(const bf16_t* __restrict__ A, int lda, const bf16_t* __r
 // four waves makes 16 columns of one pair's row, a wave 4 of them: the operand row's share of a lane stays in registers
 // (K up to 64 x 8 x EX_ROW_CHUNKS), the four matrix rows are read 16 bytes a lane, all loads of a column quartet in
 // flight together.  C[pair] = act(A[pair / gather_div or pair] . W[chosen[pair]]^T).
+// GATED: an expert's matrix is [gate; up] of N rows each, a wave makes 2 columns of each and C[pair] (N columns) is their
+// gated activation.
 #define EX_ROW_CHUNKS 16
-template <typename TC, int ACT>
+template <typename TC, int ACT, bool GATED = false>
 __global__ void __launch_bounds__(256)
 expert_rows_kernel(const bf16_t* __restrict__ A, int lda, const bf16_t* __restrict__ W, const int* __restrict__ chosen,
-                   int gather_div, TC* __restrict__ C, int ldc, int N, int K, int experts) {
+                   int gather_div, TC* __restrict__ C, int ldc, int N, int K, int experts, GateLaw law = GateLaw{0.f, 0.f, 0.f}) {
     const int pair = blockIdx.y;
     const int e = chosen[pair];
     if (e < 0 || e >= experts) return;                       // (a choice without matrices: its row is left alone)
     const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
-    const int n_first = (blockIdx.x * 4 + wave) * 4;
+    const int n_first = (blockIdx.x * 4 + wave) * (GATED ? 2 : 4);
     if (n_first >= N) return;
     const bf16_t* ar = A + (size_t)(gather_div > 0 ? pair / gather_div : pair) * lda;
     const int chunks = (K + 511) / 512;                      // 16-byte chunks a lane holds of a row
@@ -515,7 +633,10 @@ expert_rows_kernel(const bf16_t* __restrict__ A, int lda, const bf16_t* __restri
     float sum[4] = {0.f, 0.f, 0.f, 0.f};
     const bf16_t* wr[4];
 #pragma unroll
-    for (int j = 0; j < 4; ++j) wr[j] = W + ((size_t)e * N + min(n_first + j, N - 1)) * K;
+    for (int j = 0; j < 4; ++j) {
+        if (GATED) wr[j] = W + ((size_t)e * 2 * N + (j / 2) * N + min(n_first + j % 2, N - 1)) * K;
+        else wr[j] = W + ((size_t)e * N + min(n_first + j, N - 1)) * K;
+    }
 #pragma unroll
     for (int c = 0; c < EX_ROW_CHUNKS; ++c) {
         if (c >= chunks) continue;                           // (uniform; the loop stays unrolled, the row in registers)
@@ -536,6 +657,11 @@ expert_rows_kernel(const bf16_t* __restrict__ A, int lda, const bf16_t* __restri
     }
 #pragma unroll
     for (int j = 0; j < 4; ++j) sum[j] = wave_sum(sum[j]);
+    if (GATED) {
+        if (lane < 2 && n_first + lane < N)
+            store_f32(C + (size_t)pair * ldc + n_first + lane, gated_activation(lane ? sum[1] : sum[0], lane ? sum[3] : sum[2], law));
+        return;
+    }
     if (lane < 4 && n_first + lane < N)
         store_f32(C + (size_t)pair * ldc + n_first + lane, expert_act<ACT>(lane == 0 ? sum[0] : lane == 1 ? sum[1] : lane == 2 ? sum[2] : sum[3]));
 }
@@ -559,6 +685,16 @@ extern "C" int cisr_experts_rows(const void* A, int lda, const void* W, const in
         if (act) expert_rows_kernel<bf16_t, 1><<<grid, 256, 0, stream>>>(a, lda, w, chosen, gather_div, (bf16_t*)C, ldc, N, K, experts);
         else expert_rows_kernel<bf16_t, 0><<<grid, 256, 0, stream>>>(a, lda, w, chosen, gather_div, (bf16_t*)C, ldc, N, K, experts);
     }
+    return CISR_LAUNCH_CHECK();
+}
+
+// The gated form: W [experts, 2 N, K] = [gate; up] of every expert, C [pairs, N] bf16.
+extern "C" int cisr_experts_rows_gated(const void* A, int lda, const void* W, const int* chosen, int gather_div, void* C, int ldc,
+                                       int pairs, int N, int K, int experts, float limit, float slope, float shift, hipStream_t stream) {
+    if (pairs <= 0 || N <= 0) return 0;
+    if (!cisr_experts_rows_ok(K, lda, pairs) || ((uintptr_t)A) % 16 || ((uintptr_t)W) % 16) return (int)hipErrorInvalidValue;
+    expert_rows_kernel<bf16_t, 0, true><<<dim3((N + 7) / 8, pairs), 256, 0, stream>>>((const bf16_t*)A, lda, (const bf16_t*)W, chosen, gather_div,
+                                                                                     (bf16_t*)C, ldc, N, K, experts, GateLaw{limit, slope, shift});
     return CISR_LAUNCH_CHECK();
 }
 

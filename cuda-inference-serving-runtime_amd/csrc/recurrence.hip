@@ -30,20 +30,21 @@ int cisr_scan_launch_c4(const ScanArgs& p, int segments, bool vec, hipStream_t s
 int cisr_scan_launch_c8(const ScanArgs& p, int segments, bool vec, hipStream_t stream);
 int cisr_scan_launch_c16(const ScanArgs& p, int segments, bool vec, hipStream_t stream);
 
+// silu 1: q, k and v are silu of what is stored.  lda 0: decays that do not change from row to row.
 // cols: 4, 8 or 16 columns a wave (the caller's rule: fewer columns are more waves for the same head).  piece > 0:
 // segments longer than `piece` rows are walked in pieces of that many rows side by side (three launches; `rows` is the
 // number of rows of the step, carry / carry_decay as cisr_linear_scan_carry says); piece 0: a wave walks a whole segment.
 extern "C" int cisr_linear_scan(const float* q, int ldq, const float* k, int ldk, const float* v, int ldv,
                                 const float* a, int lda, int vec, const float* vs, int ldvs, float* out, int ldo,
                                 float* state, long long slot_stride, const int* seg_start, const int* state_slots,
-                                int segments, int heads, int R, int C, int share, float q_scale, int cols,
+                                int segments, int heads, int R, int C, int share, float q_scale, int silu, int cols,
                                 int rows, int piece, float* carry, float* carry_decay, hipStream_t stream) {
     if (segments <= 0 || heads <= 0) return 0;
     if (R <= 0 || C <= 0 || share <= 0 || heads % share || heads > 65535 || (cols != 4 && cols != 8 && cols != 16) ||
         piece < 0 || (piece > 0 && (!carry || !carry_decay || rows <= 0)))
         return (int)hipErrorInvalidValue;
     ScanArgs p{q, ldq, k, ldk, v, ldv, a, lda, vs, ldvs, out, ldo, state, slot_stride, seg_start, state_slots, R, C, share, heads,
-               q_scale, piece, piece > 0 ? (rows + piece - 1) / piece : 1, 0, carry, carry_decay};
+               q_scale, silu, piece, piece > 0 ? (rows + piece - 1) / piece : 1, 0, carry, carry_decay};
     if ((C + cols - 1) / cols > 65535 || R > 256 || (piece > 0 && segments > 65535)) return (int)hipErrorInvalidValue;
     if (cols == 4) return cisr_scan_launch_c4(p, segments, vec, stream);
     if (cols == 8) return cisr_scan_launch_c8(p, segments, vec, stream);

@@ -293,7 +293,8 @@ def fused_merge_splits(splits, rows, accepts):
 
 def kernel_units(head_dim, dtype, law="softmax"):
     """Names of the shared objects that attention with this head size needs beside the core (library.ensure).
-    `law` "sigmoid": the build with sigmoid weights that are not normed over the keys."""
+    `law` "sigmoid": the build with sigmoid weights that are not normed over the keys; "distance": the one whose scores
+    fall with the distance."""
     from . import library
     if dtype == torch.bfloat16 and head_dim % 8 == 0 and 0 < head_dim <= 256:
         return [library.attention_unit(-(-head_dim // 32) * 32, law)]
@@ -306,7 +307,7 @@ def _split_workspace(ctx, rows, heads, splits, head_dim, dtype=torch.float32, ta
 
 
 def paged_attention(ctx, q, q_row_stride, kcache, vcache, view, out, heads, kv_heads, head_dim, window, scale,
-                    defer_merge=None, tuning=DEFAULT_TUNING, head_bias=None):
+                    defer_merge=None, tuning=DEFAULT_TUNING, head_bias=None, slopes=None, sink=None, keep_first=0):
     """out[r] = attention of row r's queries over its request's cached keys up to its own position (or the last
     `window` of them).  `ctx` is the step's context (rows, segments, positions, buffers, step arrays), `view` the
     cache group as the step sees it (block tables, page size).
@@ -314,18 +315,22 @@ def paged_attention(ctx, q, q_row_stride, kcache, vcache, view, out, heads, kv_h
     `head_bias` (float [heads]): the sigmoid law: a visible key weighs sigmoid(score + head_bias[head]) and the weights
     are not normed over the keys.  Same kernels, launch rules and step arrays, except that prompt rows always run as
     tiles (the forms through LDS have no such build) and no later product merges split keys.
+    `slopes` (float [heads]): slopes[head] times the distance is taken off a score; `keep_first`: that many first keys are
+    seen besides the window; `sink` (float [heads]): a score that joins the denominator and has no value.
 
     `defer_merge(splits) -> bool`: the caller's next product can merge the partial results of a decode step whose
     keys are split over `splits` blocks itself (ops.gemm_merged).  Where that is so, no merge kernel runs, `out`
     is left alone and (partial outputs bf16, statistics float, splits) is returned; otherwise None."""
     rows = out.shape[0]
-    span = ctx.span_hint if not window else min(ctx.span_hint, window + 31)
+    keep_first = int(keep_first) if window else 0
+    span = ctx.span_hint if not window else min(ctx.span_hint, window + 31 + keep_first)
+    law = dict(head_bias=head_bias, slopes=slopes, sink=sink, keep_first=keep_first)
     common = (q, q_row_stride, kcache, vcache, view.tables, ctx.seg_of_row, ctx.positions, out, heads, kv_heads, head_dim,
               view.page_size, window, scale)
     if not ops.mfma_attention_supported(out.dtype, head_dim, view.page_size):
         splits = rowwise_splits(rows * heads, span)
         workspace = _split_workspace(ctx, rows, heads, splits, head_dim) if splits > 1 else None
-        ops.attention_rowwise(*common, splits, workspace, head_bias=head_bias)
+        ops.attention_rowwise(*common, splits, workspace, **law)
         return None
     group = heads // kv_heads
     heads_per_chunk = min(group, 16)
@@ -343,14 +348,14 @@ def paged_attention(ctx, q, q_row_stride, kcache, vcache, view, out, heads, kv_h
             if fused is not None:
                 workspace = _split_workspace(ctx, rows, heads, fused, head_dim, torch.bfloat16, "attn.part_o16")
                 ops.attention_mfma(*common, None, fused, workspace, waves, merge=False,
-                                   stream_loads=stream(rows * chunks, waves, fused))
+                                   stream_loads=stream(rows * chunks, waves, fused), **law)
                 return workspace[0], workspace[1], fused
         workspace = _split_workspace(ctx, rows, heads, splits, head_dim) if splits > 1 else None
         order = None
         if splits == 1 and rows * chunks >= tuning.order_rows_from:
             order = ctx.step_array(RowsLongestFirst())[0][:rows]
         ops.attention_mfma(*common, None, splits, workspace, waves, row_ids=order, stream_loads=stream(rows * chunks, waves, splits),
-                           head_bias=head_bias)
+                           **law)
         return None
     singles = SingleRows(tuning.split_single_from)
     single_rows, n_single = ctx.step_array(singles)
@@ -359,15 +364,17 @@ def paged_attention(ctx, q, q_row_stride, kcache, vcache, view, out, heads, kv_h
         waves, splits = tuning.rows_launch or rows_launch(n_single * chunks, span, heads_per_chunk, head_dim)
         workspace = _split_workspace(ctx, n_single, heads, splits, head_dim) if splits > 1 else None
         ops.attention_mfma(*common, None, splits, workspace, waves, row_ids=single_rows[:n_single],
-                           stream_loads=stream(n_single * chunks, waves, splits), head_bias=head_bias)
+                           stream_loads=stream(n_single * chunks, waves, splits), **law)
     form = prompt_form(rows, ctx.n_segments, span, heads, kv_heads, head_dim, view.page_size, tuning)
     if head_bias is not None and form[0] != "tiles":
         form = ("tiles", 2 if tuning.item_tiles == 2 and head_dim <= 64 else 1, 1)
+    if (slopes is not None or keep_first) and form[0] == "block":
+        form = ("square", form[1], 1)         # (that law's build has no block tiles on the 16 x 16 instruction)
     kind, item_tiles, halves = form
     tasks, _ = ctx.step_array(TileTasks(rows_per_tile_of(form, heads, kv_heads), singles))
     ops.attention_mfma(*common, tasks.view(-1, 4), waves=tuning.tile_waves,
                        block_tiles={"tiles": False, "block": True, "square": 32}[kind], item_tiles=item_tiles, key_groups=halves,
-                       head_bias=head_bias)
+                       **law)
     return None
 
 

@@ -52,14 +52,15 @@ def _log(msg):
 
 def attention_unit(dpad, law="softmax"):
     """The unit of the matrix-core attention of a padded head size; `law` "sigmoid": weights sigmoid(score + a bias a
-    head) that are not normed over the keys."""
-    return f"attn_sig_d{dpad}" if law == "sigmoid" else f"attn_d{dpad}"
+    head) that are not normed over the keys; "distance": softmax of scores that fall with the distance, the first keys
+    kept beside the window."""
+    return {"sigmoid": "attn_sig_d", "distance": "attn_dist_d"}.get(law, "attn_d") + str(dpad)
 
 
 def units():
     """The shared objects the kernels are built into: the core, and one per padded head size of the
     matrix-core attention (a model needs only its own, so a first call compiles only that one)."""
-    return [CORE, *OWN_UNITS, TALKING] + [attention_unit(d, law) for law in ("softmax", "sigmoid") for d in ATTENTION_PADS]
+    return [CORE, *OWN_UNITS, TALKING] + [attention_unit(d, law) for law in ("softmax", "sigmoid", "distance") for d in ATTENTION_PADS]
 
 
 def sources(unit=CORE):

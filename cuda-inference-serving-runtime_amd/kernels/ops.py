@@ -47,7 +47,7 @@ def _declare(h):
         "cisr_page_copy": [p, p, p, i, i, ll, ll, p],
         "cisr_f32_to_bf16": [p, p, ll, p],
         "cisr_bias_add": [p, p, ll, i, i, i, p],
-        "cisr_attn_rowwise": [p, i, p, p, p, p, p, p, p, p, i, i, i, i, i, i, i, f, i, i, p],
+        "cisr_attn_rowwise": [p, i, p, p, p, p, p, p, p, p, i, i, i, i, i, i, i, f, i, i, p, p, i, p],
         "cisr_gemm_f32": [p, i, p, i, p, i, p, i, i, i, i, p],
         "cisr_gemm_bf16": [p, i, p, i, p, i, p, i, i, i, i, i, p],
         "cisr_gemm_bf16_swiglu": [p, i, p, i, p, i, i, i, i, i, p],
@@ -71,8 +71,8 @@ def _declare(h):
         "cisr_gemm_bf16_gated": [p, i, p, i, p, i, i, i, i, i, f, f, f, p],
         "cisr_post_norm_add": [p, p, p, p, p, p, i, i, f, f, p, f, p, i, i, i, f, f, p, p],
         "cisr_glu_clamped": [p, p, i, i, f, f, f, i, p],
-        "cisr_qk_norm_scatter": [p, i, p, p, p, p, p, p, p, i, i, i, i, i, i, i, f, i, i, i, i, p],
-        "cisr_head_gate": [p, p, i, p, i, i, i, i, i, p],
+        "cisr_qk_norm_scatter": [p, i, p, p, p, p, p, p, p, i, i, i, i, i, i, i, f, i, i, i, i, p, f, i, p],
+        "cisr_head_gate": [p, p, i, i, p, i, i, i, i, i, i, p],
         "cisr_layernorm": [p, p, p, p, p, i, i, f, i, p],
         "cisr_rms_slice": [p, i, i, p, p, i, i, f, i, p],
         "cisr_latent_keys": [p, i, i, p, p, i, p, p, p, p, p, p, p, i, i, i, i, i, i, i, i, i, i, f, i, p],
@@ -90,7 +90,11 @@ def _declare(h):
         "cisr_experts_route": [p, i, p, p, p, i, i, i, i, p, p, p],
         "cisr_experts_gemm": [p, i, p, p, p, i, i, p, i, i, i, i, i, i, i, p],
         "cisr_experts_rows": [p, i, p, p, i, p, i, i, i, i, i, i, i, p],
-        "cisr_experts_route_scored": [p, i, p, p, p, i, i, i, i, i, i, i, p, p, p],
+        "cisr_experts_route_scored": [p, i, p, p, p, i, i, i, i, i, i, i, i, f, i, p, p, p],
+        "cisr_experts_add": [p, p, p, p, p, p, i, i, i, i, i, p, f, p, i, p],
+        "cisr_experts_rows_gated": [p, i, p, p, i, p, i, i, i, i, i, f, f, f, p],
+        "cisr_embedding_sinusoid": [p, p, p, p, p, p, f, p, i, i, i, f, i, i, p],
+        "cisr_side_gate": [p, i, p, p, i, i, p, i, i, i, i, i, p],
         "cisr_experts_combine": [p, p, p, p, i, p, p, i, i, i, i, p],
         "cisr_bias_act": [p, p, p, ll, i, i, i, p],
         "cisr_experts_rows_ok": [i, i, i],
@@ -117,13 +121,14 @@ _attention_entries = {}
 def _attention_entry(dpad, law="softmax"):
     """The matrix-core attention entry point for a padded head size (its shared object is built and loaded
     at the first use of that size).  `law` "sigmoid": the build whose weights are sigmoid(score + a bias a head), not
-    normed over the keys; its entry takes the biases as a last argument."""
+    normed over the keys; its entry takes the biases as a last argument.  "distance": the softmax build whose scores fall
+    with the distance and whose window keeps the first keys (last arguments: sinks, slopes, number of keys kept; the
+    plain build's last argument: sinks)."""
     fn = _attention_entries.get((dpad, law))
     if fn is None:
         p, i, f = C.c_void_p, C.c_int, C.c_float
-        sigmoid = law == "sigmoid"
-        fn = getattr(library.load_attention(dpad, law), f"cisr_attn_mfma_sig_d{dpad}" if sigmoid else f"cisr_attn_mfma_d{dpad}")
-        fn.argtypes = [p, i, p, p, p, i, p, i, p, p, p, p, p, i, i, i, i, i, f, i, i, i, i, p] + ([p] if sigmoid else [])
+        fn = getattr(library.load_attention(dpad, law), {"sigmoid": "cisr_attn_mfma_sig_d", "distance": "cisr_attn_mfma_dist_d"}.get(law, "cisr_attn_mfma_d") + str(dpad))
+        fn.argtypes = [p, i, p, p, p, i, p, i, p, p, p, p, p, i, i, i, i, i, f, i, i, i, i, p] + ([p, p, i] if law == "distance" else [p])
         fn.restype = C.c_int
         _attention_entries[(dpad, law)] = fn
     return fn
@@ -323,12 +328,18 @@ ROWWISE_MAX_HEAD = 640     # the row-wise attention kernel's largest head (the m
 
 
 def attention_rowwise(q, q_row_stride, kcache, vcache, tables, seg_of_row, positions, out, heads, kv_heads, dim,
-                      page_size, window, scale, splits=1, workspace=None, head_bias=None):
+                      page_size, window, scale, splits=1, workspace=None, head_bias=None, slopes=None, sink=None, keep_first=0):
     """Each row attends to its request's cached keys lo..position.  q is a view
     into a row-major buffer with `q_row_stride` elements per row; out [T, heads*dim].
     `head_bias` (float [heads]): the weight of a visible key is sigmoid(score + head_bias[head]) instead of its share
-    of a softmax, and the weights are not normed over the keys."""
+    of a softmax, and the weights are not normed over the keys.  Of the softmax law: `slopes` (float [heads]):
+    slopes[head] * (position - key) is taken off a score; `sink` (float [heads]): a score that joins the denominator and
+    has no value; `keep_first`: the first keys that are seen besides the window."""
     rows = out.shape[0]
+    if keep_first and (not window or head_bias is not None):
+        raise KernelError("attention: keys are kept beside a window of the softmax law")
+    if head_bias is not None and (slopes is not None or sink is not None):
+        raise KernelError("attention: the sigmoid law has no slopes and no sink")
     dt = _storage(out, "out")
     if dim % 2 or dim > ROWWISE_MAX_HEAD:
         raise KernelError(f"attention: head size {dim} must be even and at most {ROWWISE_MAX_HEAD}")
@@ -357,7 +368,9 @@ def attention_rowwise(q, q_row_stride, kcache, vcache, tables, seg_of_row, posit
     if head_bias is not None:
         _check(lib().cisr_attn_rowwise_sigmoid(*args, _dev(head_bias, "head_bias", torch.float32, (heads,)), _stream()), "attention_rowwise")
     else:
-        _check(lib().cisr_attn_rowwise(*args, _stream()), "attention_rowwise")
+        _check(lib().cisr_attn_rowwise(*args, None if slopes is None else _dev(slopes, "slopes", torch.float32, (heads,)),
+                                       None if sink is None else _dev(sink, "sink", torch.float32, (heads,)), int(keep_first), _stream()),
+               "attention_rowwise")
     return out
 
 
@@ -852,7 +865,8 @@ def qkv_rope(a, w, q_out, positions, slots, cos, sin, kcache, vcache, heads, kv_
 
 def attention_mfma(q, q_row_stride, kcache, vcache, tables, seg_of_row, positions, out, heads, kv_heads, dim,
                    page_size, window, scale, tasks=None, splits=1, workspace=None, waves=4, block_tiles=False,
-                   item_tiles=1, row_ids=None, merge=True, key_groups=1, stream_loads=False, head_bias=None):
+                   item_tiles=1, row_ids=None, merge=True, key_groups=1, stream_loads=False, head_bias=None, slopes=None, sink=None,
+                   keep_first=0):
     """Matrix-core attention (bf16).  tasks int32 [n, 4] = (segment, first row, rows, 0) runs tiles of
     prompt rows: one tile of 16/GC rows a block whose waves share the keys (with item_tiles=2, head sizes up to
     64: 32/GC rows, two item tiles a wave), or with `block_tiles` (head sizes up to 128) one tile of
@@ -866,8 +880,17 @@ def attention_mfma(q, q_row_stride, kcache, vcache, tables, seg_of_row, position
     halves that take the even and the odd 32-key steps of its items and merge at the end.  `stream_loads` (rows mode):
     keys and values are read with non-temporal loads, which the caches do not keep.
     `head_bias` (float [heads]): the sigmoid law (see attention_rowwise); the tile and row forms have it, the block
-    tiles do not, and the partial results of split keys are plain sums that only this function merges."""
+    tiles do not, and the partial results of split keys are plain sums that only this function merges.
+    `slopes`, `sink`, `keep_first`: as in attention_rowwise; with slopes or kept keys every form but the block tiles of 64 and
+    128 items on the 16 x 16 instruction runs (a build of its own)."""
     rows = out.shape[0]
+    law_name = "sigmoid" if head_bias is not None else "distance" if slopes is not None or keep_first else "softmax"
+    if law_name == "sigmoid" and (sink is not None or slopes is not None or keep_first):
+        raise KernelError("attention_mfma: the sigmoid law has no slopes, no sink and no kept keys")
+    if keep_first and not window:
+        raise KernelError("attention_mfma: keys are kept beside a window")
+    if law_name == "distance" and (slopes is None or (block_tiles and block_tiles != 32)):
+        raise KernelError("attention_mfma: the law with slopes takes slopes (zeros: none), as rows, tiles or 32 x 32 block tiles")
     if head_bias is not None and (block_tiles or not merge):
         raise KernelError("attention_mfma: the sigmoid law runs as tiles and rows, merged here")
     if not mfma_attention_supported(out.dtype, dim, page_size):
@@ -884,8 +907,10 @@ def attention_mfma(q, q_row_stride, kcache, vcache, tables, seg_of_row, position
     if kcache.numel() >= 2 ** 31 or vcache.numel() >= 2 ** 31:
         raise KernelError("attention_mfma: a layer's keys (or values) must be fewer than 2^31 elements (32-bit byte offsets)")
     dpad = -(-dim // 32) * 32
-    fn = _attention_entry(dpad, "softmax" if head_bias is None else "sigmoid")
-    law = () if head_bias is None else (_dev(head_bias, "head_bias", torch.float32, (heads,)),)
+    fn = _attention_entry(dpad, law_name)
+    sp = None if sink is None else _dev(sink, "sink", torch.float32, (heads,))
+    law = ((_dev(head_bias, "head_bias", torch.float32, (heads,)),) if law_name == "sigmoid" else
+           (sp, _dev(slopes, "slopes", torch.float32, (heads,)), int(keep_first)) if law_name == "distance" else (sp,))
     po = pm = tp = None
     if tasks is not None:
         if item_tiles not in ((1, 2, 3, 4) if block_tiles == 32 else (1, 2)) or (item_tiles == 2 and dim > 64 and not block_tiles):
@@ -1100,15 +1125,17 @@ def glu_clamped(gate_up, out, limit, slope=1.702, shift=1.0):
 
 
 def qk_norm_scatter(qkv, q_norm, k_norm, q_out, kcache, vcache, slots, heads, kv_heads, dim, vdim, pad, page_size, eps, bias=None,
-                    plain_norm=False):
+                    plain_norm=False, temperature=None):
     """Rows of a fused projection [q: heads x dim | k: kv_heads x dim | v: kv_heads x vdim | ...]: queries and keys
     RMS-normed per head (weights float [dim]; None: left as they are, or with `plain_norm` normed without a weight), queries
     into q_out [T, heads * pad], keys and values into the cache at `slots`, all as heads of `pad` coordinates whose rest is
     zero (keys [pages, kv_heads, page_size, pad], values transposed in a page, [pages, kv_heads, pad, page_size]).  qkv has
     the cache's dtype, or is float.  `bias`: float over the q, k and v columns, added before everything else.  kcache None:
-    the rows have queries only (a layer that reads another's cache)."""
+    the rows have queries only (a layer that reads another's cache).  `temperature` = (positions int32 [T], coef, every):
+    queries are multiplied by 1 + coef ln(floor((position + 1) / every) + 1) at the end."""
     rows, ld = qkv.shape
     has_kv = kcache is not None
+    at, coef, every = temperature if temperature is not None else (None, 0.0, 0)
     columns = heads * dim + (kv_heads * (dim + vdim) if has_kv else 0)
     if dim > pad or vdim > pad or pad > 256 or ld < columns:
         raise KernelError(f"qk_norm_scatter: heads of {dim} / {vdim} do not fit rows of {ld} or pages of {pad}")
@@ -1125,21 +1152,25 @@ def qk_norm_scatter(qkv, q_norm, k_norm, q_out, kcache, vcache, slots, heads, kv
         sp = _dev(slots, "slots", torch.int32, (rows,))
     _check(lib().cisr_qk_norm_scatter(_dev(qkv, "qkv"), ld, bp, wq, wk, _dev(q_out, "q_out", None, (rows, heads * pad)), kp, vp, sp,
                                       rows, heads, kv_heads, dim, vdim, pad, page_size, float(eps), int(bool(plain_norm)), int(has_kv),
-                                      _storage(qkv, "qkv"), _storage(q_out, "q_out"), _stream()), "qk_norm_scatter")
+                                      _storage(qkv, "qkv"), _storage(q_out, "q_out"),
+                                      None if at is None else _dev(at, "positions", torch.int32, (rows,)), float(coef), int(every),
+                                      _stream()), "qk_norm_scatter")
     return q_out
 
 
 def head_gate(attn, gates, out, heads, vdim, pad):
-    """out[t, h, :] = attn[t, h, :vdim] * sigmoid(gates[t, h]); attn [T, heads * pad], gates a view [T, heads] of a
-    row-major buffer (or None: no gate, the heads are only packed), out [T, heads * vdim]."""
+    """out[t, h, :] = attn[t, h, :vdim] * sigmoid(gates[t, h]), or, with gates [T, heads * vdim], element by element; attn
+    [T, heads * pad], gates a view of a row-major buffer with unit column stride, of the activations' type or float (None: no
+    gate, the heads are only packed), out [T, heads * vdim]."""
     rows = attn.shape[0]
-    gp, ldg = None, 0
+    gp, ldg, per_element, gdt = None, 0, 0, _storage(attn, "attn")
     if gates is not None:
-        if gates.dtype != attn.dtype or tuple(gates.shape) != (rows, heads) or gates.stride(1) != 1 or not gates.is_cuda:
-            raise KernelError("head_gate: gates must be [T, heads] of the activations' dtype with unit stride")
-        gp, ldg = gates.data_ptr(), gates.stride(0)
-    _check(lib().cisr_head_gate(_dev(attn, "attn", None, (rows, heads * pad)), gp, ldg,
-                                _dev(out, "out", attn.dtype, (rows, heads * vdim)), rows, heads, vdim, pad,
+        if (gates.dtype not in (attn.dtype, torch.float32) or gates.dim() != 2 or gates.shape[0] != rows or gates.shape[1] not in (heads, heads * vdim)
+                or gates.stride(1) != 1 or not gates.is_cuda):
+            raise KernelError("head_gate: gates must be [T, heads] or [T, heads * vdim] of the activations' dtype (or float) with unit stride")
+        gp, ldg, per_element, gdt = gates.data_ptr(), gates.stride(0), int(gates.shape[1] != heads), _storage(gates, "gates")
+    _check(lib().cisr_head_gate(_dev(attn, "attn", None, (rows, heads * pad)), gp, ldg, per_element,
+                                _dev(out, "out", attn.dtype, (rows, heads * vdim)), rows, heads, vdim, pad, gdt,
                                 _storage(attn, "attn"), _stream()), "head_gate")
     return out
 
@@ -1282,7 +1313,7 @@ def _rec():
         h = library.load(library.RECURRENCE)
         p, i, f, ll = C.c_void_p, C.c_int, C.c_float, C.c_longlong
         sig = {
-            "cisr_linear_scan": [p, i, p, i, p, i, p, i, i, p, i, p, i, p, ll, p, p, i, i, i, i, i, f, i, i, i, p, p, p],
+            "cisr_linear_scan": [p, i, p, i, p, i, p, i, i, p, i, p, i, p, ll, p, p, i, i, i, i, i, f, i, i, i, i, p, p, p],
             "cisr_conv_silu": [p, i, i, p, p, p, ll, p, p, p, p, i, i, i, i, i, i, p, p, p, p, i, p],
             "cisr_decay_gate": [p, i, p, p, i, i, f, p],
             "cisr_decay_gate_low_rank": [p, i, i, p, p, p, i, i, f, p],
@@ -1345,7 +1376,7 @@ def scan_carry(rows, piece, heads, rows_of_state, cols_of_state, vector):
 
 
 def linear_scan(q, k, v, decay, out, state, seg_start, state_slots, heads, rows_of_state, cols_of_state, share=1,
-                step=None, q_scale=1.0, columns=None, piece=0, carry=None):
+                step=None, q_scale=1.0, columns=None, piece=0, carry=None, silu=False):
     """Per segment and head: S_t = diag(a_t) S_(t-1) + k_t (v_t step_t)^T, o_t = q_scale S_t^T q_t over the segment's
     rows in order, S [rows_of_state, cols_of_state] read from and written back to the segment's state slot.
     q, k float views [T, heads / share * R]; v, out [T, heads * C]; decay [T, heads * R] (a vector a head) or
@@ -1353,7 +1384,10 @@ def linear_scan(q, k, v, decay, out, state, seg_start, state_slots, heads, rows_
     start with the state); seg_start int32 [S + 1]; state_slots int32 [S].
     `piece` > 0: segments longer than that many rows are walked in pieces side by side (three launches: the pieces'
     end states from zero, the states at their starts in order, the results), with `carry` = (float buffer, float
-    buffer) of at least scan_carry(...) elements."""
+    buffer) of at least scan_carry(...) elements.  `silu`: q, k and v are silu of what is stored (no step then).  Decays
+    that do not change from row to row may be an expanded [1, heads] (row stride 0)."""
+    if silu and step is not None:
+        raise KernelError("linear_scan: silu of the values comes without a step size")
     R, Cc = int(rows_of_state), int(cols_of_state)
     T = v.shape[0]
     segments = state_slots.shape[0]
@@ -1384,7 +1418,7 @@ def linear_scan(q, k, v, decay, out, state, seg_start, state_slots, heads, rows_
     _check(_rec().cisr_linear_scan(qp, ldq, kp, ldk, vp, ldv, ap, lda, int(vec), sp, lds, op, ldo, state.data_ptr(),
                                    state.stride(0), _dev(seg_start, "seg_start", torch.int32, (segments + 1,)),
                                    _dev(state_slots, "state_slots", torch.int32, (segments,)), segments, heads, R, Cc,
-                                   int(share), float(q_scale), cols, T, int(piece), cp, dp, _stream()), "linear_scan")
+                                   int(share), float(q_scale), int(bool(silu)), cols, T, int(piece), cp, dp, _stream()), "linear_scan")
     return out
 
 
@@ -1769,6 +1803,39 @@ def embedding_pairs(tokens, positions, seg_of_row, seg_start, state_slots, table
     return out
 
 
+# -- embedding with sinusoidal positions, table rows of the token inside the layers (csrc/elementwise_sided.hip) ----------
+
+def embedding_sinusoid(tokens, positions, table, turns, out, scale=1.0, norm=None):
+    """out[r] = table[tokens[r]] * scale + the position's vector, float [T, H]: columns 2i and 2i + 1 are sine and cosine of
+    2 pi positions[r] turns[i] (double [ceil(H / 2)]).  `norm` = (weight float [H], eps, rows [T, H]): the norm that reads
+    the rows first is made by the same kernel."""
+    rows = tokens.shape[0]
+    vocab, dim = table.shape
+    wp, eps, np_, ndt = None, 0.0, None, F32
+    if norm is not None:
+        weight, eps, normed = norm
+        wp = _dev(weight, "norm weight", torch.float32, (dim,))
+        np_, ndt = _dev(normed, "normed", None, (rows, dim)), _storage(normed, "normed")
+    _check(lib().cisr_embedding_sinusoid(_dev(tokens, "tokens", torch.int32), _dev(positions, "positions", torch.int32, (rows,)), _dev(table, "table"),
+                                         _dev(turns, "turns", torch.float64, ((dim + 1) // 2,)), _dev(out, "out", torch.float32, (rows, dim)),
+                                         wp, float(eps), np_, rows, dim, vocab, float(scale), _storage(table, "table"), ndt, _stream()),
+           "embedding_sinusoid")
+    return out
+
+
+def side_gate(z, tokens, side, first, width, act):
+    """act[r, c] = gelu_tanh(z[r, c]) * side[tokens[r], first + c] for c < width, 0 in the columns of `act` behind them; z a
+    float view [T, >= width] with unit column stride, side [vocab, n] and act [T, >= width] of one type."""
+    rows, padded = act.shape
+    vocab, ld_side = side.shape
+    zp, ldz = _rows_of(z, "z")
+    if z.shape[0] != rows or z.shape[1] < width or padded < width or first < 0 or first + width > ld_side:
+        raise KernelError("side_gate: sizes disagree")
+    _check(lib().cisr_side_gate(zp, ldz, _dev(tokens, "tokens", torch.int32, (rows,)), _dev(side, "side", act.dtype), ld_side, int(first),
+                                _dev(act, "act"), rows, int(width), padded, vocab, _storage(act, "act"), _stream()), "side_gate")
+    return act
+
+
 class WeightedRows:
     """A sublayer's result as `top` rows a step row, to be summed with weights by the kernel that reads it next
     (gate_post_norm): rows float [T * top, H], weights float [T, top]."""
@@ -1870,12 +1937,15 @@ def experts_route(logits, bias, top, chosen, weights, pair_of_pos=None, tile_exp
     return chosen, weights
 
 
-def experts_route_scored(logits, correction, top, chosen, weights, experts, groups=None, pair_of_pos=None, tile_expert=None):
+def experts_route_scored(logits, correction, top, chosen, weights, experts, groups=None, pair_of_pos=None, tile_expert=None,
+                         sigmoid=False, group_pairs=False, floor=None):
     """Routing by scores: logits a float view [T, outputs]; s = softmax over all outputs; the choice goes by s + correction
     (float [outputs] or None), held to the best `groups[1]` of `groups[0]` equal groups of neighbours (a group's score is
     its largest choice score); chosen int32 [T, top] (the lowest index wins a tie), weights float [T, top] = s of the
     chosen, not normed again.  The first `experts` outputs have matrices: only their pairs are ordered by expert into
-    pair_of_pos / tile_expert (as experts_route does), the others are left to the caller."""
+    pair_of_pos / tile_expert (as experts_route does), the others are left to the caller.
+    `sigmoid`: s is the sigmoid of each logit instead; `group_pairs`: a group's score is the sum of its two largest choice
+    scores; `floor` (None: not): the weights are divided by the sum of the chosen scores plus that number."""
     rows, outputs = logits.shape
     if logits.dtype != torch.float32 or logits.stride(1) != 1 or not logits.is_cuda:
         raise KernelError("experts_route_scored: float logits with contiguous rows")
@@ -1891,7 +1961,8 @@ def experts_route_scored(logits, correction, top, chosen, weights, experts, grou
     _check(lib().cisr_experts_route_scored(logits.data_ptr(), logits.stride(0),
                                            None if correction is None else _dev(correction, "correction", torch.float32, (outputs,)),
                                            _dev(chosen, "chosen", torch.int32, (rows, top)), _dev(weights, "weights", torch.float32, (rows, top)),
-                                           rows, outputs, int(experts), top, int(count), int(keep), tiles, pp, tp, _stream()), "experts_route_scored")
+                                           rows, outputs, int(experts), top, int(count), int(keep), int(bool(sigmoid)), int(bool(group_pairs)),
+                                           -1.0 if floor is None else float(floor), tiles, pp, tp, _stream()), "experts_route_scored")
     return chosen, weights
 
 
@@ -1906,6 +1977,40 @@ def experts_combine(down, weights, chosen, x, y, experts, shared=None):
                                       None if shared is None else _dev(shared, "shared", torch.float32, (rows, dim)),
                                       _dev(y, "y", torch.float32, (rows, dim)), rows, dim, top, int(experts), _stream()), "experts_combine")
     return y
+
+
+class ExpertSum:
+    """A mixture's result before its sum, for the kernel that adds it to the residual stream (experts_add): down float
+    [T * top, H], weights float [T, top], chosen int32 [T, top] (of `experts` experts with matrices), shared float [T, H] or
+    None, gate a float view [T, 1] (the shared part times sigmoid(gate)) or None."""
+
+    def __init__(self, down, weights, chosen, experts, shared=None, gate=None):
+        self.down, self.weights, self.chosen, self.experts, self.shared, self.gate = down, weights, chosen, int(experts), shared, gate
+
+
+EXPERTS_ADD_MAX_COLS = 16384
+
+
+def experts_add(x, y, following=None):
+    """x += the sum of an ExpertSum, in place (float [T, H]); `following` = (weight float [H] or None, eps, out [T, H]):
+    out = rmsnorm(x) * weight, or with a weight of None the new rows themselves, in out's type."""
+    rows, dim = x.shape
+    top = y.weights.shape[1]
+    if dim > EXPERTS_ADD_MAX_COLS:
+        raise KernelError(f"experts_add: rows of {dim}, at most {EXPERTS_ADD_MAX_COLS}")
+    gp, ldg = None, 0
+    if y.gate is not None:
+        gp, ldg = _rows_of(y.gate, "gate", 1)
+    np_, neps, op, odt = None, 0.0, None, F32
+    if following is not None:
+        nw, neps, out = following
+        np_ = None if nw is None else _dev(nw, "following weight", torch.float32, (dim,))
+        op, odt = _dev(out, "following out", None, (rows, dim)), _storage(out, "following out")
+    _check(lib().cisr_experts_add(_dev(x, "x", torch.float32), _dev(y.down, "down", torch.float32, (rows * top, dim)),
+                                  _dev(y.weights, "weights", torch.float32), _dev(y.chosen, "chosen", torch.int32, (rows, top)),
+                                  None if y.shared is None else _dev(y.shared, "shared", torch.float32, (rows, dim)), gp, ldg, rows, dim, top,
+                                  y.experts, np_, float(neps), op, odt, _stream()), "experts_add")
+    return x
 
 
 EXPERT_ROWS_PAIRS = 32     # steps of at most this many (row, choice) pairs stream each pair's matrices (experts_rows)
@@ -1929,6 +2034,21 @@ def experts_rows(a, w, chosen, out, top=0, act=False):
         raise KernelError("experts_rows: too few operand rows")
     _check(lib().cisr_experts_rows(a.data_ptr(), a.stride(0), _dev(w, "w"), _dev(chosen, "chosen", torch.int32), int(top), _dev(out, "out"),
                                    out.stride(0), pairs, n, k, int(bool(act)), _storage(out, "out"), int(experts), _stream()), "experts_rows")
+    return out
+
+
+def experts_rows_gated(a, w, chosen, out, law, top=0):
+    """experts_rows over experts whose matrix is [gate; up] (w [experts, 2 N, K]) with their gated activation as the
+    epilogue: out bf16 [pairs, N]; law = (limit, slope, shift), or (0, 0, 0): silu(gate) up."""
+    experts, n2, k = w.shape
+    pairs = chosen.numel()
+    if not experts_rows_ok(a, w, pairs) or a.shape[1] != k or n2 % 2 or tuple(out.shape) != (pairs, n2 // 2) or not out.is_contiguous():
+        raise KernelError("experts_rows_gated: shape not supported")
+    if a.shape[0] < (-(-pairs // top) if top > 0 else pairs):
+        raise KernelError("experts_rows_gated: too few operand rows")
+    _check(lib().cisr_experts_rows_gated(a.data_ptr(), a.stride(0), _dev(w, "w"), _dev(chosen, "chosen", torch.int32), int(top),
+                                         _dev(out, "out", torch.bfloat16), out.stride(0), pairs, n2 // 2, k, int(experts),
+                                         *(float(v) for v in law), _stream()), "experts_rows_gated")
     return out
 
 

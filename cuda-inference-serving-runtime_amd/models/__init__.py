@@ -5,3 +5,4 @@ from .ditazen import build_ditazen
 from .noresun import build_noresun
 from .zovozen import build_zovozen
 from .guduzen import build_guduzen
+from .movazen import build_movazen

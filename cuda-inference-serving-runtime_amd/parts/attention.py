@@ -17,7 +17,7 @@ import math
 
 import torch
 
-from ..cache.pages import ChunkNeed, KVNeed
+from ..cache.pages import ChunkNeed, KeptWindowNeed, KVNeed
 from ..kernels import attention as kernel, ops
 from .base import Mixer, TensorSpec, matrix_operand, register_part
 
@@ -136,6 +136,13 @@ class NormedGatedAttention(Mixer):
     `own_kv` False: the layer has no key and value tensors and reads the cache another layer wrote.  `keep`: the window
     the layer's own cache keeps, where layers that read it look further back than it does itself.
 
+    Further parameters, each on its own: `head_gate` "element": the gate is a projection of heads * vdim rows, one number
+    an element of the heads' results.  `slopes` (a number a head): slope * (i - j) is taken off the score of key j at
+    position i.  `keep_first`: besides the window a row sees the first keys of the sequence (the cache then keeps their
+    pages).  `sink` (a number a head): a score that joins the softmax's denominator and has no value.  `q_temp` = (coef,
+    every): the query at position p is multiplied by 1 + coef ln(floor((p + 1) / every) + 1).  `ride(weight)`: further rows
+    for the input product, whose float results are then `rider` (float rows only).
+
     The pages hold heads of `pad` = max(dim, vdim) coordinates (rounded up to a multiple of 8), the rest zero: zero
     coordinates add nothing to a score and give result coordinates that are not read, so the attention kernels
     of the framework serve as they are.  `names`: the tensors' names under `name` (q, k, v, o, gate, q norm, k norm)."""
@@ -143,7 +150,8 @@ class NormedGatedAttention(Mixer):
     NAMES = {"q": "q", "k": "k", "v": "v", "o": "o", "gate": "g", "q_norm": "q.norm", "k_norm": "k.norm"}
 
     def __init__(self, name, hidden, heads, kv_heads, dim, vdim, scale, eps, qk_norm=True, head_gate=True, window=None,
-                 names=None, tuning=None, bias=False, float_rows=None, own_kv=True, keep="own"):
+                 names=None, tuning=None, bias=False, float_rows=None, own_kv=True, keep="own", slopes=None, keep_first=0, sink=None,
+                 q_temp=None):
         if heads % kv_heads:
             raise ValueError(f"{heads} query heads are not a multiple of {kv_heads} key/value heads")
         self.pad = -(-max(dim, vdim) // 8) * 8
@@ -153,10 +161,22 @@ class NormedGatedAttention(Mixer):
             raise ValueError("the score scale must be positive")
         self.name, self.hidden, self.heads, self.kv_heads, self.dim, self.vdim = name, hidden, heads, kv_heads, dim, vdim
         self.scale, self.eps, self.qk_norm, self.head_gate, self.window = float(scale), float(eps), qk_norm, bool(head_gate), window
+        self.gate_rows = 0 if not head_gate else heads * vdim if head_gate == "element" else heads
         self.bias, self.own_kv = bool(bias), bool(own_kv)
         self.float_rows = self.bias if float_rows is None else bool(float_rows)
-        if self.float_rows and self.head_gate:
-            raise ValueError("the heads' gates are read in the activations' type: no float rows beside them")
+        for what, numbers in (("slopes", slopes), ("sink", sink)):
+            if numbers is not None and len(numbers) != heads:
+                raise ValueError(f"{what}: one number a head")
+        if keep_first < 0 or (keep_first and (window is None or not own_kv or keep != "own")):
+            raise ValueError("first keys are kept beside a window, by a layer with keys of its own that no other layer's window widens")
+        if q_temp is not None and not (q_temp[1] > 0 and int(q_temp[1]) == q_temp[1]):
+            raise ValueError("the query temperature's step is a positive whole number of positions")
+        self.slopes, self.sink = (None if n is None else [float(v) for v in n] for n in (slopes, sink))
+        self.keep_first = int(keep_first)
+        if self.keep_first and self.slopes is None:
+            self.slopes = [0.0] * heads          # (kept keys and slopes are one build of the kernels)
+        self.q_temp = None if q_temp is None else (float(q_temp[0]), int(q_temp[1]))
+        self.rider, self.rider_rows = None, 0
         self.keep = window if keep == "own" else keep
         if self.keep is not None and (window is None or window > self.keep):
             raise ValueError("a layer's cache keeps at least the keys the layer itself looks back over")
@@ -168,12 +188,14 @@ class NormedGatedAttention(Mixer):
         return f"{self.name}.{self.names[which]}"
 
     def kernel_units(self, dtype):
-        return kernel.kernel_units(self.pad, dtype)
+        return kernel.kernel_units(self.pad, dtype, "softmax" if self.slopes is None else "distance")
 
     def step_arrays(self):
         return [kernel.SingleRows(self.tuning.split_single_from), kernel.RowsLongestFirst()]
 
     def cache_need(self):
+        if self.keep_first:
+            return KeptWindowNeed(self.kv_heads, self.pad, self.keep, self.keep_first)
         return KVNeed(self.kv_heads, self.pad, self.keep) if self.own_kv else None
 
     def cache_read(self):
@@ -190,7 +212,7 @@ class NormedGatedAttention(Mixer):
             specs += [TensorSpec(self._tensor(p) + ".b", (rows,)) for p, rows in self._projections().items()]
         specs.append(TensorSpec(self._tensor("o"), (H, nh * V)))
         if self.head_gate:
-            specs.append(TensorSpec(self._tensor("gate"), (nh, H)))
+            specs.append(TensorSpec(self._tensor("gate"), (self.gate_rows, H)))
         if self.qk_norm and self.qk_norm != "plain":
             specs.append(TensorSpec(self._tensor("q_norm"), (D,), init="one_plus_normal"))
             if self.own_kv:
@@ -199,17 +221,30 @@ class NormedGatedAttention(Mixer):
 
     def bind(self, tensors, dtype):
         inputs = list(self._projections())
-        parts = [matrix_operand(tensors[self._tensor(p)], dtype) for p in inputs + (["gate"] if self.head_gate else [])]
-        rows = sum(p.shape[0] for p in parts)
-        if rows % 8:      # rows of the fused projection are a multiple of 16 bytes: zero rows at the end
-            parts.append(torch.zeros(8 - rows % 8, self.hidden, dtype=parts[0].dtype, device=parts[0].device))
-        self.w_in = torch.cat(parts, dim=0).contiguous()
+        self.w_own = [matrix_operand(tensors[self._tensor(p)], dtype) for p in inputs + (["gate"] if self.head_gate else [])]
+        self.own_rows = sum(p.shape[0] for p in self.w_own)
+        self._join()
+        device = self.w_in.device
+        self.slope_t, self.sink_t = (None if n is None else torch.tensor(n, dtype=torch.float32, device=device) for n in (self.slopes, self.sink))
         self.w_out = matrix_operand(tensors[self._tensor("o")], dtype)
         if self.bias:
             self.b_in = torch.cat([tensors[self._tensor(p) + ".b"].to(torch.float32) for p in inputs]).contiguous()
         if self.qk_norm and self.qk_norm != "plain":
             self.q_weight = tensors[self._tensor("q_norm")].to(torch.float32).contiguous()
             self.k_weight = tensors[self._tensor("k_norm")].to(torch.float32).contiguous() if self.own_kv else None
+
+    def _join(self, extra=None):
+        parts = list(self.w_own) + ([] if extra is None else [extra])
+        rows = sum(p.shape[0] for p in parts)
+        if rows % 8:      # rows of the fused projection are a multiple of 16 bytes: zero rows at the end
+            parts.append(torch.zeros(8 - rows % 8, self.hidden, dtype=parts[0].dtype, device=parts[0].device))
+        self.w_in = torch.cat(parts, dim=0).contiguous()
+
+    def ride(self, weight):
+        if not self.float_rows:
+            raise ValueError("rows that ride in the input product have float results")
+        self.rider_rows = weight.shape[0]
+        self._join(weight)
 
     def output(self, h, ctx, site):
         """The mixer's result, float [T, hidden], without the residual sum."""
@@ -219,18 +254,21 @@ class NormedGatedAttention(Mixer):
         view = ctx.kv[gid]
         qkv = ctx.buffer("gattn.qkv", (T, self.w_in.shape[0]), torch.float32 if self.float_rows else ctx.dtype)
         ops.gemm(h, self.w_in, qkv, scratch=ctx.scratch)
+        self.rider = qkv[:, self.own_rows:self.own_rows + self.rider_rows] if self.rider_rows else None
         written = (kcache, vcache, view.slots) if self.own_kv else (None, None, None)
         q = ops.qk_norm_scatter(qkv, self.q_weight, self.k_weight, ctx.buffer("gattn.q", (T, nh * pad), ctx.dtype), *written,
-                                nh, nkv, D, V, pad, view.page_size, self.eps, bias=self.b_in, plain_norm=self.qk_norm == "plain")
+                                nh, nkv, D, V, pad, view.page_size, self.eps, bias=self.b_in, plain_norm=self.qk_norm == "plain",
+                                temperature=None if self.q_temp is None else (ctx.positions, *self.q_temp))
         out = ctx.buffer("gattn.out", (T, nh * pad), ctx.dtype)
         # a decode step of few rows may leave the partial results of its split keys to the output projection
         merges = None if self.head_gate or pad != V else (lambda splits: ops.gemm_merged_ok(T, self.w_out, nh, V, splits))
         unmerged = kernel.paged_attention(ctx, q, nh * pad, kcache, vcache, view, out, nh, nkv, pad, self.window, self.scale,
-                                          defer_merge=merges, tuning=self.tuning)
+                                          defer_merge=merges, tuning=self.tuning, slopes=self.slope_t, sink=self.sink_t,
+                                          keep_first=self.keep_first)
         if unmerged is not None:
             return ops.gemm_merged(unmerged, nh, V, self.w_out, ctx.buffer("gattn.y", (T, self.hidden), torch.float32))
         first_gate = sum(self._projections().values())
-        gates = qkv[:, first_gate:first_gate + nh] if self.head_gate else None
+        gates = qkv[:, first_gate:first_gate + self.gate_rows] if self.head_gate else None
         act = out
         if gates is not None or pad != V:
             act = ops.head_gate(out, gates, ctx.buffer("gattn.act", (T, nh * V), ctx.dtype), nh, V, pad)

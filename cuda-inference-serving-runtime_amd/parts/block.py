@@ -1,7 +1,8 @@
 """Arrangement of parts in a layer.  PreNormBlock is the Llama arrangement
 (reference: runtime/model.py:106-119): x = x + mixer(norm1(x)); x = x + ffn(norm2(x)),
 the residual stream x kept in float.  SandwichBlock norms each sublayer's result as well
-and scales it: x = x + m norm1b(mixer(norm1(x))); x = x + m norm2b(ffn(norm2(x))); without the norms in front
+and scales it: x = x + m norm1b(mixer(norm1(x))); x = x + m norm2b(ffn(norm2(x))) (or adds it as it is, and then what a side
+sublayer reads of x itself and a norm makes of it: x = x + norm3(side(x))); without the norms in front
 (`reads_stream`) its sublayers read x itself: x = x + m norm1b(mixer(x)).  PostNormBlock norms after the
 sum, and its sublayers read the stream itself: x = norm1(a x + g1 mixer(x)); x = norm2(a x + g2 ffn(x)), with
 optional gates g = sigmoid(W x + b) element by element.  HyperConnectedBlock keeps several streams instead of one x,
@@ -105,6 +106,10 @@ def add_sublayer(residual, result, norm, mult, eps=None, following=None):
     then = None
     if following is not None:
         then = (None, 0.0, following[1]) if following[0] is CAST else (following[0].weight, following[0].eps, following[1])
+    if isinstance(result, ops.ExpertSum):
+        if weight is not None or mult != 1.0:
+            raise ValueError("a mixture's rows are added as they are (no norm after them, no factor)")
+        return ops.experts_add(residual, result, following=then)
     if isinstance(result, ScaledSum):
         return ops.post_norm_add(residual, result.first, weight, 0.0 if eps is None else eps, mult,
                                  second=(result.second, result.first_scale, result.second_scale), following=then)
@@ -121,14 +126,23 @@ class SandwichBlock(Part):
     Its mixer and feed-forward give their result without the residual sum (`output`); `ffn` None: a layer without
     a feed-forward.  The norms after the sublayers are RMS norms (`weight`, `eps`); the sum, the norm and the scale
     are one kernel.  `reads_stream`: there are no norms in front (`mixer_norm`, `ffn_norm` None) and the sublayers read
-    the residual stream itself, in the activations' type (that copy is made by the kernel that wrote the stream last)."""
+    the residual stream itself, in the activations' type (that copy is made by the kernel that wrote the stream last).
+    Both norms after the sublayers None (`mixer_post`, `ffn_post`, with `mult` 1): results are added as they are, and a
+    mixture's rows are summed on the way.  `side` with `side_post`: a last sublayer that reads the stream itself (no norm in
+    front) and whose result is normed before the sum."""
 
-    def __init__(self, mixer_norm, mixer, mixer_post, ffn_norm=None, ffn=None, ffn_post=None, mult=1.0, reads_stream=False):
+    def __init__(self, mixer_norm, mixer, mixer_post, ffn_norm=None, ffn=None, ffn_post=None, mult=1.0, reads_stream=False, side=None,
+                 side_post=None):
         self.reads_stream = bool(reads_stream)
+        self.plain = mixer_post is None
+        if self.plain and (ffn_post is not None or mult != 1.0 or reads_stream):
+            raise ValueError("results that are added as they are: no norms after the sublayers, no factor, norms in front")
+        if (side is None) != (side_post is None) or (side is not None and (not self.plain or getattr(side_post, "fusable_as", None) != "rms")):
+            raise ValueError("a side sublayer comes with the RMS norm after it, beside sublayers that are added as they are")
         if self.reads_stream:
             if mixer_norm is not None or ffn_norm is not None or (ffn is None) != (ffn_post is None):
                 raise ValueError("sublayers that read the stream itself have no norm in front; a feed-forward comes with the norm after it")
-        elif (ffn is None) != (ffn_norm is None) or (ffn is None) != (ffn_post is None):
+        elif (ffn is None) != (ffn_norm is None) or (not self.plain and (ffn is None) != (ffn_post is None)):
             raise ValueError("a feed-forward comes with the norms before and after it, or not at all")
         for post in (mixer_post, ffn_post):
             if post is not None and getattr(post, "fusable_as", None) != "rms":
@@ -138,9 +152,11 @@ class SandwichBlock(Part):
         self.mixer_norm, self.mixer, self.mixer_post = mixer_norm, mixer, mixer_post
         self.ffn_norm, self.ffn, self.ffn_post = ffn_norm, ffn, ffn_post
         self.mult = float(mult)
+        self.side, self.side_post = side, side_post
 
     def parts(self):
-        return [p for p in (self.mixer_norm, self.mixer, self.mixer_post, self.ffn_norm, self.ffn, self.ffn_post) if p is not None]
+        return [p for p in (self.mixer_norm, self.mixer, self.mixer_post, self.ffn_norm, self.ffn, self.ffn_post, self.side, self.side_post)
+                if p is not None]
 
     def tensor_specs(self):
         return [s for p in self.parts() for s in p.tensor_specs()]
@@ -223,22 +239,38 @@ class SandwichBlock(Part):
             h = self.mixer_norm.forward(residual, ctx)
             ctx.settle(residual)
         T = residual.shape[0]
-        last = self.ffn is None
-
-        def following(norm, tag):
-            return (norm, ctx.buffer(tag, (T, residual.shape[1]), ctx.dtype)) if self._plain_rms(norm) else None
-
-        then = following(after if last else self.ffn_norm, "norm.ahead" if last else "norm.inside")
-        add_sublayer(residual, self.mixer.output(h, ctx, site), self.mixer_post, self.mult, following=then)
-        if last:
-            if then is not None:
-                ctx.leave_normed(after, residual, then[1])
-            return residual
-        h = then[1] if then is not None else self.ffn_norm.forward(residual, ctx)
-        then = following(after, "norm.ahead")
-        add_sublayer(residual, self.ffn.output(h, ctx), self.ffn_post, self.mult, following=then)
-        if then is not None:
-            ctx.leave_normed(after, residual, then[1])
+        # the sublayers in order and who reads the stream after each: the next one's norm, CAST before a side sublayer
+        subs = [(self.mixer, self.mixer_post)]
+        readers = []
+        if self.ffn is not None:
+            readers.append(self.ffn_norm)
+            subs.append((self.ffn, self.ffn_post))
+        if self.side is not None:
+            readers.append(CAST)
+            subs.append((self.side, self.side_post))
+        readers.append(after)
+        for i, (sub, post) in enumerate(subs):
+            reader, last = readers[i], i == len(subs) - 1
+            then = None
+            if reader is CAST:
+                if ctx.dtype != torch.float32:
+                    then = (CAST, ctx.buffer("norm.inside", residual.shape, ctx.dtype))
+            elif self._plain_rms(reader):
+                then = (reader, ctx.buffer("norm.ahead" if last else "norm.inside", residual.shape, ctx.dtype))
+            if sub is self.mixer:
+                result = sub.output(h, ctx, site)
+            elif self.plain and getattr(sub, "leaves_rows", False):
+                result = sub.output(h, ctx, unsummed=True)
+            else:
+                result = sub.output(h, ctx)
+            add_sublayer(residual, result, post, self.mult, following=then)
+            if last:
+                if then is not None:
+                    ctx.leave_normed(after, residual, then[1])
+                elif reader is CAST:
+                    ctx.leave_normed(CAST, residual, residual)
+            else:
+                h = then[1] if then is not None else residual if reader is CAST else reader.forward(residual, ctx)
         return residual
 
 

@@ -1,10 +1,12 @@
 """Token embedding and output head.
 
 x0[r] = E[token_r] with no scaling (reference: runtime/model.py:105), or with PairHashEmbedding
-E[token_r] * scale + B[hash(token before, token_r)]; logits =
+E[token_r] * scale + B[hash(token before, token_r)], with SinusoidEmbedding E[token_r] * scale + a vector of the position; logits =
 h . W^T with W the head's own matrix or, when tied, the embedding matrix
 (reference: runtime/checkpoint.py:38-39).  Logits are always float.
 """
+import math
+
 import torch
 
 from ..kernels import ops
@@ -46,6 +48,40 @@ class StreamsEmbedding(TokenEmbedding):
         if read is not None:
             ctx.leave_normed(reader, x, read[3])
         return x
+
+
+class SinusoidEmbedding(TokenEmbedding):
+    """x[r] = E[token_r] * scale + a vector of the position, sines in its even columns and cosines in its odd ones: entries
+    2i and 2i + 1 turn by base^(-2i / hidden) a position.  The norm that reads the rows first is made by the same kernel.
+    `side` = (tensor name, columns): a second table of the tokens, in the activations' type, that layers read (TokenSide);
+    it is this part's tensor and is found as `side_table`."""
+
+    def __init__(self, name, vocab, hidden, scale=1.0, base=10000.0, tensor=None, side=None):
+        super().__init__(name, vocab, hidden, tensor=tensor)
+        self.scale, self.base, self.side, self.side_table = float(scale), float(base), side, None
+
+    def tensor_specs(self):
+        return super().tensor_specs() + ([] if self.side is None else [TensorSpec(self.side[0], (self.vocab, self.side[1]))])
+
+    def bind(self, tensors, dtype):
+        super().bind(tensors, dtype)
+        if self.side is not None:
+            self.side_table = matrix_operand(tensors[self.side[0]], dtype)
+
+    def prepare(self, device, dtype):
+        pairs = torch.arange((self.hidden + 1) // 2, dtype=torch.float64)
+        self.turns = (self.base ** (-2.0 * pairs / self.hidden) / (2.0 * math.pi)).to(device)
+
+    def forward(self, ctx):
+        T = ctx.tokens.shape[0]
+        out = ctx.buffer("residual", (T, self.hidden), torch.float32)
+        norm, reader = None, ctx.next_norm
+        if getattr(reader, "fusable_as", None) == "rms":
+            norm = (reader.weight, reader.eps, ctx.buffer("residual.normed", (T, self.hidden), ctx.dtype))
+        ops.embedding_sinusoid(ctx.tokens, ctx.positions, self.weight, self.turns, out, scale=self.scale, norm=norm)
+        if norm is not None:
+            ctx.leave_normed(reader, out, norm[2])
+        return out
 
 
 STATE_SITE = "embedding"      # the key of the embedding's state among the cache manager's state sites

@@ -102,17 +102,20 @@ class ClampedGLU(FeedForward):
         self.w_gate_up = torch.cat([gate, up], dim=0).contiguous()
         self.w_down = matrix_operand(tensors[self._tensor(2)], dtype)
 
-    def output(self, h, ctx):
-        """The feed-forward's result, float [T, hidden], without the residual sum."""
+    def output(self, h, ctx, tag="ffn", unfinished=True):
+        """The feed-forward's result, float [T, hidden], without the residual sum; `unfinished`: it may be left as partial
+        sums (ops.Partials) for a reader that adds them."""
         T = h.shape[0]
         law = (self.limit, self.slope, self.shift)
-        act = ctx.buffer("ffn.act", (T, self.intermediate), ctx.dtype)
+        act = ctx.buffer(tag + ".act", (T, self.intermediate), ctx.dtype)
         if ops.swiglu_fused_ok(h, self.w_gate_up):
             ops.gemm_swiglu(h, self.w_gate_up, act, scratch=ctx.scratch, law=law)      # the product and the activation are one kernel
         else:
-            ops.gemm_swiglu(h, self.w_gate_up, act, gate_up=ctx.buffer("ffn.gate_up", (T, 2 * self.intermediate), ctx.dtype),
+            ops.gemm_swiglu(h, self.w_gate_up, act, gate_up=ctx.buffer(tag + ".gate_up", (T, 2 * self.intermediate), ctx.dtype),
                             scratch=ctx.scratch, law=law)
-        return ctx.product_for_norm(act, self.w_down, "ffn.out")
+        if unfinished:
+            return ctx.product_for_norm(act, self.w_down, tag + ".out")
+        return ops.gemm(act, self.w_down, ctx.buffer(tag + ".out", (T, self.hidden), torch.float32), scratch=ctx.scratch)
 
     def forward(self, h, residual, ctx, norm=None):
         from .block import add_sublayer
@@ -241,19 +244,25 @@ class RoutedExperts(FeedForward):
 
 
 class ScoredExperts(FeedForward):
-    """A mixture of experts routed by scores: s = softmax(W_r h) over all router outputs, in float; the choice goes by
-    s + `correction` (a tensor; the weights use s without it), optionally held to the best `groups[1]` of `groups[0]`
-    equal groups of neighbouring outputs (a group's score is its largest choice score; the others count as minus
-    infinity); the `top` largest are chosen and weigh s itself, not normed again.  The first `experts` outputs are gated
-    feed-forwards W_down (silu(W_gate h) * (W_up h)) without biases; the last `identity` outputs have no tensors: their
-    result is the input itself.  `shared`: a feed-forward part (with `output`) that every row goes through, added.
+    """A mixture of experts routed by scores: s = softmax(W_r h) over all router outputs, in float (`scores` "sigmoid": the
+    sigmoid of each); the choice goes by s + `correction` (a tensor; the weights use s without it), optionally held to the
+    best `groups[1]` of `groups[0]` equal groups of neighbouring outputs (a group's score is its largest choice score, with
+    `group_pairs` the sum of its two largest; the others count as minus infinity); the `top` largest are chosen and weigh s
+    itself, or with `floor` s divided by the sum of the chosen s plus that number.  The first `experts` outputs are gated
+    feed-forwards without biases, W_down (silu(W_gate h) * (W_up h)), or with `law` = (limit, slope, shift) the clamped form of
+    ClampedGLU; the last `identity` outputs have no tensors: their result is the input itself.  `shared`: a feed-forward
+    part (with `output`) that every row goes through, added, with `shared_gate` (a tensor's name under `name`, [1, hidden])
+    times sigmoid of that row's product with h.
 
     The rows of a step are ordered by expert on the device and each expert's matrices meet only their own rows
     (ops.experts_gemm; steps of few rows stream each pair's matrices, ops.experts_rows); gate and up are one product over
-    [gate; up] a expert, followed by the activation.  `names`: (router, correction, expert prefix, gate, up, down)."""
+    [gate; up] a expert, followed by the activation (its epilogue in steps of few rows).  `names`: (router, correction, expert
+    prefix, gate, up, down)."""
+    leaves_rows = True       # `output` takes `unsummed`
 
     def __init__(self, name, hidden, intermediate, experts, top, identity=0, groups=None, shared=None, correction=True,
-                 names=("router", "correction", "e", "gate", "up", "down")):
+                 names=("router", "correction", "e", "gate", "up", "down"), scores="softmax", group_pairs=False, floor=None, law=None,
+                 shared_gate=None):
         outputs = experts + identity
         if not 0 < top <= min(outputs, 16) or experts <= 0 or identity < 0:
             raise ValueError(f"{top} of {experts} + {identity} router outputs: between 1 and min(outputs, 16)")
@@ -263,9 +272,18 @@ class ScoredExperts(FeedForward):
                 raise ValueError(f"{outputs} router outputs in {count} groups of which {keep} are kept, for {top} choices")
         if shared is not None and not hasattr(shared, "output"):
             raise ValueError("the shared feed-forward must give its result without the residual sum (output)")
+        if scores not in ("softmax", "sigmoid"):
+            raise ValueError(f"scores {scores!r} are neither softmax nor sigmoid")
+        if law is not None and not law[0] > 0:
+            raise ValueError("the clamp's limit must be positive")
+        if shared_gate is not None and (shared is None or identity):
+            raise ValueError("a gate of the shared feed-forward comes with one, and without identity outputs")
         self.name, self.hidden, self.intermediate = name, hidden, intermediate
         self.experts, self.identity, self.outputs, self.top = int(experts), int(identity), outputs, int(top)
         self.groups, self.shared, self.has_correction, self.names = groups, shared, bool(correction), tuple(names)
+        self.route = dict(sigmoid=scores == "sigmoid", group_pairs=bool(group_pairs), floor=floor)
+        self.law = None if law is None else tuple(float(v) for v in law)
+        self.shared_gate = None if shared_gate is None else f"{name}.{shared_gate}"
 
     def _expert(self, j, which):
         return f"{self.name}.{self.names[2]}{j}.{self.names[3 + which]}"
@@ -277,13 +295,19 @@ class ScoredExperts(FeedForward):
             specs.append(TensorSpec(f"{self.name}.{self.names[1]}", (self.outputs,)))
         for j in range(self.experts):
             specs += [TensorSpec(self._expert(j, 0), (I, H)), TensorSpec(self._expert(j, 1), (I, H)), TensorSpec(self._expert(j, 2), (H, I))]
+        if self.shared_gate is not None:
+            specs.append(TensorSpec(self.shared_gate, (1, H)))
         return specs + ([] if self.shared is None else self.shared.tensor_specs())
 
     def bind(self, tensors, dtype):
-        router = matrix_operand(tensors[f"{self.name}.{self.names[0]}"], dtype)
-        if router.shape[0] % 8:      # rows of the router's product are a multiple of 8: zero rows at the end
-            router = torch.cat([router, torch.zeros(8 - router.shape[0] % 8, self.hidden, dtype=router.dtype, device=router.device)])
-        self.w_router = router.contiguous()
+        # (the shared part's gate is one more row of the router's product)
+        rows = [matrix_operand(tensors[f"{self.name}.{self.names[0]}"], dtype)]
+        if self.shared_gate is not None:
+            rows.append(matrix_operand(tensors[self.shared_gate], dtype))
+        n = sum(r.shape[0] for r in rows)
+        if n % 8:      # rows of the router's product are a multiple of 8: zero rows at the end
+            rows.append(torch.zeros(8 - n % 8, self.hidden, dtype=rows[0].dtype, device=rows[0].device))
+        self.w_router = torch.cat(rows, dim=0).contiguous()
         self.correction = tensors[f"{self.name}.{self.names[1]}"].to(torch.float32).contiguous() if self.has_correction else None
         self.w_gate_up = torch.stack([torch.cat([matrix_operand(tensors[self._expert(j, 0)], dtype), matrix_operand(tensors[self._expert(j, 1)], dtype)])
                                       for j in range(self.experts)]).contiguous()
@@ -295,27 +319,76 @@ class ScoredExperts(FeedForward):
         if self.shared is not None:
             self.shared.prepare(device, dtype)
 
-    def output(self, h, ctx):
-        """The feed-forward's result, float [T, hidden], without the residual sum."""
+    def _activation(self, gate_up, act):
+        return ops.swiglu(gate_up, act) if self.law is None else ops.glu_clamped(gate_up, act, *self.law)
+
+    def rows(self, h, ctx):
+        """The feed-forward's result as an ops.ExpertSum: the chosen experts' rows and their weights, and the shared part's
+        rows, for a kernel that adds them all (no identity outputs)."""
         T, E, top, I = h.shape[0], self.experts, self.top, self.intermediate
         logits = ops.gemm(h, self.w_router, ctx.buffer("moe.logits", (T, self.w_router.shape[0]), torch.float32), scratch=ctx.scratch)
         chosen, weights = ctx.buffer("moe.chosen", (T, top), torch.int32), ctx.buffer("moe.weights", (T, top), torch.float32)
         down = ctx.buffer("moe.down", (T * top, self.hidden), torch.float32)
+        route = (logits[:, :self.outputs], self.correction, top, chosen, weights, E, self.groups)
         if ops.experts_rows_ok(h, self.w_gate_up, T * top) and ops.experts_rows_ok(h, self.w_down, T * top):
             # few rows (decoding): every (row, choice) pair streams its expert's matrices
-            ops.experts_route_scored(logits[:, :self.outputs], self.correction, top, chosen, weights, E, self.groups)
-            gate_up = ops.experts_rows(h, self.w_gate_up, chosen, ctx.buffer("moe.gate_up", (T * top, 2 * I), ctx.dtype), top=top)
-            act = ops.swiglu(gate_up, ctx.buffer("moe.act", (T * top, I), ctx.dtype))
+            ops.experts_route_scored(*route, **self.route)
+            act = ops.experts_rows_gated(h, self.w_gate_up, chosen, ctx.buffer("moe.act", (T * top, I), ctx.dtype), self.law or (0.0, 0.0, 0.0), top=top)
             ops.experts_rows(act, self.w_down, chosen, down)
         else:
             tiles = ops.expert_tiles(T, top, E)
             places, tile_expert = ctx.buffer("moe.places", (tiles * ops.EXPERT_TILE,), torch.int32), ctx.buffer("moe.tiles", (tiles,), torch.int32)
-            ops.experts_route_scored(logits[:, :self.outputs], self.correction, top, chosen, weights, E, self.groups, places, tile_expert)
+            ops.experts_route_scored(*route, places, tile_expert, **self.route)
             gate_up = ops.experts_gemm(h, self.w_gate_up, places, tile_expert, ctx.buffer("moe.gate_up", (tiles * ops.EXPERT_TILE, 2 * I), ctx.dtype), top=top)
-            act = ops.swiglu(gate_up, ctx.buffer("moe.act", (tiles * ops.EXPERT_TILE, I), ctx.dtype))
+            act = self._activation(gate_up, ctx.buffer("moe.act", (tiles * ops.EXPERT_TILE, I), ctx.dtype))
             ops.experts_gemm(act, self.w_down, places, tile_expert, down, scatter=True)
-        also = None if self.shared is None else self.shared.output(h, ctx, tag="moe.shared")
-        return ops.experts_combine(down, weights, chosen, h, ctx.buffer("moe.y", (T, self.hidden), torch.float32), E, shared=also)
+        also = None if self.shared is None else self.shared.output(h, ctx, tag="moe.shared", unfinished=False)
+        gate = None if self.shared_gate is None else logits[:, self.outputs:self.outputs + 1]
+        return ops.ExpertSum(down, weights, chosen, E, shared=also, gate=gate)
+
+    def output(self, h, ctx, unsummed=False):
+        """The feed-forward's result, float [T, hidden], without the residual sum; `unsummed`: it may be left as an
+        ops.ExpertSum for a reader that adds the rows to the residual stream itself."""
+        parts = self.rows(h, ctx)
+        if unsummed and self.identity == 0 and self.hidden <= ops.EXPERTS_ADD_MAX_COLS:
+            return parts
+        y = ctx.buffer("moe.y", (h.shape[0], self.hidden), torch.float32)
+        if parts.gate is not None:
+            y.zero_()
+            return ops.experts_add(y, parts)
+        return ops.experts_combine(parts.down, parts.weights, parts.chosen, h, y, self.experts, shared=parts.shared)
+
+    def forward(self, h, residual, ctx, norm=None):
+        from .block import add_sublayer
+        return add_sublayer(residual, self.output(h, ctx, unsummed=True), None, 1.0)
+
+
+class TokenSide(FeedForward):
+    """A sublayer that reads a table by the token: y = Wp (gelu_tanh(Wg h) * e), e the columns [first, first + width) of the
+    token's row in `source.side_table` (a part that owns the table of all layers).  `names`: (gate, projection)."""
+
+    def __init__(self, name, hidden, width, first, source, names=("gate", "proj")):
+        self.name, self.hidden, self.width, self.first, self.source, self.names = name, hidden, int(width), int(first), source, tuple(names)
+        self.padded = -(-self.width // 8) * 8
+        self.w_gate = self.w_proj = None
+
+    def tensor_specs(self):
+        return [TensorSpec(f"{self.name}.{self.names[0]}", (self.width, self.hidden)), TensorSpec(f"{self.name}.{self.names[1]}", (self.hidden, self.width))]
+
+    def bind(self, tensors, dtype):
+        gate, proj = (matrix_operand(tensors[f"{self.name}.{n}"], dtype) for n in self.names)
+        extra = self.padded - self.width          # (zero rows and columns: operands in whole 16-byte words)
+        if extra:
+            gate = torch.cat([gate, torch.zeros(extra, self.hidden, dtype=gate.dtype, device=gate.device)])
+            proj = torch.cat([proj, torch.zeros(self.hidden, extra, dtype=proj.dtype, device=proj.device)], dim=1)
+        self.w_gate, self.w_proj = gate.contiguous(), proj.contiguous()
+
+    def output(self, h, ctx, unfinished=True):
+        """The sublayer's result, float [T, hidden], without the residual sum."""
+        T = h.shape[0]
+        z = ops.gemm(h, self.w_gate, ctx.buffer("side.z", (T, self.padded), torch.float32), scratch=ctx.scratch)
+        act = ops.side_gate(z, ctx.tokens, self.source.side_table, self.first, self.width, ctx.buffer("side.act", (T, self.padded), ctx.dtype))
+        return ctx.product_for_norm(act, self.w_proj, "side.y")
 
     def forward(self, h, residual, ctx, norm=None):
         from .block import add_sublayer
@@ -332,6 +405,7 @@ def _add_weighted(residual, y):
 
 register_part("ffn", "routed_experts", RoutedExperts)
 register_part("ffn", "scored_experts", ScoredExperts)
+register_part("ffn", "token_side", TokenSide)
 register_part("ffn", "gated_mlp", GatedMLP)
 register_part("ffn", "dense_mlp", DenseMLP)
 register_part("ffn", "clamped_glu", ClampedGLU)

@@ -103,6 +103,11 @@ class RotaryEmbedding(Part):
         return self._tables
 
 
+def distance_slopes(heads):
+    """What the score of a key loses a position of distance, head by head: 2^(-8 (h + 1) / heads) (ALiBi's slopes)."""
+    return [2.0 ** (-8.0 * (h + 1) / heads) for h in range(heads)]
+
+
 class NoPosition(Part):
     """Identity: a one-pair table with angle zero."""
     pairing = "split_half"

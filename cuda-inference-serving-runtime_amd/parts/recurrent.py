@@ -1,12 +1,14 @@
 """Mixers that keep a state of fixed size per request instead of keys and values.
 
-Both are the same recurrence per head, S_t = diag(a_t) S_(t-1) + k_t v_t^T, o_t = S_t^T q_t, run by one kernel
+The first three are the same recurrence per head, S_t = diag(a_t) S_(t-1) + k_t v_t^T, o_t = S_t^T q_t, run by one kernel
 (ops.linear_scan) over the rows of a step as they come (portions and single tokens of several requests), with
 the state in the cache manager's state slots, in float in every mode:
 
   GatedLinearAttention   a_t a vector over the key channels, sigmoid(z_t)^(1/tau), z_t from a low-rank projection
                          with a bias; q scaled by dim^(-1/2); each head's result RMS-normed over vdim with a weight
                          shared by the heads, times silu of a gate projection, then the output projection.
+  LightningAttention     a_t one number a head that never changes; q, k and v silu of their projections; the heads' results
+                         RMS-normed together, times sigmoid of a gate projection, then the output projection.
   StateSpaceDuality      (Mamba-2) a_t one number a head, exp(-exp(A_log) dt_t) with dt_t = softplus(dt + dt_bias);
                          k = B_t, q = C_t (shared by the heads of a group), v = dt_t x_t; x, B and C come out of a short
                          causal convolution with silu whose last inputs are part of the state; y = o + D x, times
@@ -106,6 +108,71 @@ class GatedLinearAttention(Mixer):
         act = ops.group_norm_gate(o, proj[:, 2 * K + V:2 * K + 2 * V], self.norm_weight, ctx.buffer("gla.act", (T, V), ctx.dtype),
                                   self.heads, self.eps, gate_first=False, shared_weight=True)
         return ctx.product_for_norm(act, self.w_out, "gla.y")
+
+    def forward(self, h, residual, ctx, site, norm=None):
+        from .block import add_sublayer
+        return add_sublayer(residual, self.output(h, ctx, site), None, 1.0)
+
+
+class LightningAttention(Mixer):
+    """Linear attention with a decay a head that no input changes: S <- decay_h S + k v^T, o = S^T q, with q, k and v the silu
+    of their projections (no other scale).  The heads' results, side by side, are RMS-normed together (a weight an
+    element), multiplied by sigmoid(Wg h) element by element, and go through the output projection.  State: float
+    [heads, dim, vdim] a request, zero at the start."""
+
+    NAMES = {"q": "q", "k": "k", "v": "v", "gate": "g", "o": "o", "norm": "norm"}
+
+    def __init__(self, name, hidden, heads, dim, vdim, decay, eps, names=None):
+        if len(decay) != heads:
+            raise ValueError(f"{len(decay)} decays for {heads} heads")
+        if dim > 256:
+            raise ValueError(f"query/key heads of {dim}: at most 256")
+        self.name, self.hidden, self.heads, self.dim, self.vdim, self.eps = name, hidden, heads, dim, vdim, float(eps)
+        self.decay = [float(d) for d in decay]
+        self.names = {**self.NAMES, **(names or {})}
+
+    def _tensor(self, which):
+        return f"{self.name}.{self.names[which]}"
+
+    def kernel_units(self, dtype):
+        return [library.RECURRENCE]
+
+    def state_need(self):
+        return StateNeed((self.heads, self.dim, self.vdim), "float32")
+
+    def tensor_specs(self):
+        H, K, V, t = self.hidden, self.heads * self.dim, self.heads * self.vdim, self._tensor
+        return [TensorSpec(t("q"), (K, H)), TensorSpec(t("k"), (K, H)), TensorSpec(t("v"), (V, H)), TensorSpec(t("gate"), (V, H)),
+                TensorSpec(t("o"), (H, V)), TensorSpec(t("norm"), (V,), init="one_plus_normal")]
+
+    def bind(self, tensors, dtype):
+        t = self._tensor
+        parts = [matrix_operand(tensors[t(p)], dtype) for p in ("q", "k", "v", "gate")]
+        rows = sum(p.shape[0] for p in parts)
+        if rows % 8:
+            parts.append(torch.zeros(8 - rows % 8, self.hidden, dtype=parts[0].dtype, device=parts[0].device))
+        self.w_in = torch.cat(parts, dim=0).contiguous()
+        self.w_out = matrix_operand(tensors[t("o")], dtype)
+        self.norm_weight = _float(tensors[t("norm")])
+        self.decay_row = torch.tensor([self.decay], dtype=torch.float32, device=self.w_in.device)
+
+    def input_weight(self):
+        """The matrix of the input product, for a neighbour that reads the same h and makes both products as one (its
+        float results then come back as `proj` of `output`)."""
+        return self.w_in
+
+    def output(self, h, ctx, site, proj=None):
+        """The mixer's result, float [T, hidden], without the residual sum; moves the request's state on."""
+        T, K, V = h.shape[0], self.heads * self.dim, self.heads * self.vdim
+        if proj is None:
+            proj = ops.gemm(h, self.w_in, ctx.buffer("la.proj", (T, self.w_in.shape[0]), torch.float32), scratch=ctx.scratch)
+        state = ctx.cache.state_storage[site]
+        o = ctx.buffer("la.o", (T, V), torch.float32)
+        _scan(ctx, "la", proj[:, :K], proj[:, K:2 * K], proj[:, 2 * K:2 * K + V], self.decay_row.expand(T, self.heads), o,
+              state.view(state.shape[0], -1), self.heads, self.dim, self.vdim, silu=True)
+        act = ops.group_norm_gate(o, proj[:, 2 * K + V:2 * K + 2 * V], self.norm_weight, ctx.buffer("la.act", (T, V), ctx.dtype),
+                                  1, self.eps, gate_first=False, sigmoid=True)
+        return ctx.product_for_norm(act, self.w_out, "la.y")
 
     def forward(self, h, residual, ctx, site, norm=None):
         from .block import add_sublayer
@@ -534,6 +601,7 @@ class SideBySide(Mixer):
 
 
 register_part("mixer", "gated_linear_attention", GatedLinearAttention)
+register_part("mixer", "lightning_attention", LightningAttention)
 register_part("mixer", "state_space_duality", StateSpaceDuality)
 register_part("mixer", "side_by_side", SideBySide)
 register_part("mixer", "gated_delta_rule", GatedDeltaRule)
