@@ -283,7 +283,7 @@ def main():
     ap.add_argument("--check", type=int, default=1, choices=[0, 1], help="compare the timed way of running with the plain one first")
     ap.add_argument("--widths", default="1024,2048,4096", help="designs workload: model widths to time (comma separated)")
     ap.add_argument("--design-layers", type=int, default=4, help="designs workload: layers of each model")
-    ap.add_argument("--designs", default="llama,novosun,ditazen,noresun,zovozen,guduzen", help="designs workload: which designs to time (comma separated)")
+    ap.add_argument("--designs", default="llama,novosun,ditazen,noresun,zovozen,guduzen,movazen", help="designs workload: which designs to time (comma separated)")
     args = ap.parse_args()
     if args.gpus != 1:
         print(f"bench.py measures one GPU only; --gpus {args.gpus} is not run")
@@ -388,7 +388,7 @@ def main():
 
 
 def design_configs(width, layers, context):
-    """A Llama, a Novosun, a Ditazen, a Noresun, a Zovozen and a Guduzen configuration of the same width, depth and vocabulary.  The
+    """A Llama, a Novosun, a Ditazen, a Noresun, a Zovozen, a Guduzen and a Movazen configuration of the same width, depth and vocabulary.  The
     Novosun layers alternate: softmax attention (heads of 64 for keys, 128 for values, a quarter as many key/value heads) beside
     a state-space layer (inner size twice the width in heads of 64, 128 states, a convolution of 4 taps), then gated
     linear attention (key size half the width, value size the width, in heads of 128 x 256)."""
@@ -453,11 +453,26 @@ def design_configs(width, layers, context):
              {"type": "attention", "mixer": {**slide, "kv_from": 0}, "mlp": glu}]
     guduzen = {"architecture": "Guduzen", "vocab": vocab, "width": width, "streams": 4, "logit_softcap": 30.0, "norm": {"eps": 1e-5},
                "layers": [order[i % 4] for i in range(layers)], "max_positions": context}
-    return {"llama": llama, "novosun": novosun, "ditazen": ditazen, "noresun": noresun, "zovozen": zovozen, "guduzen": guduzen}
+    # Movazen: attention over a window of 1,024 keys and the first 64 (heads of 128, a quarter as many key/value heads, scores
+    # that fall with the distance, a gate an element), then attention over every earlier key with one in the denominator
+    # beside lightning attention (as many heads, keys of 64, values of 128); every layer with 16 gated experts of width / 2 in 4
+    # groups of which 2 are kept, 4 chosen, a shared expert of the width (9 width^2 active), and 256 columns a layer of a table
+    # of the tokens
+    near = {"heads": heads, "kv_heads": max(1, width // 512), "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "mask": {"size": 1024, "keep_first": 64}}
+    far = {"heads": heads, "kv_heads": max(1, width // 512), "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "q_temp": {"coef": 0.1, "every": 1024}}
+    lightning = {"heads": heads, "dim": 64, "vdim": 128, "decay": [1.0 - 2.0 ** (-2 - 6 * i / heads) for i in range(heads)]}
+    clamped = {"kind": "moe", "expert": {"ff": width // 2, "limit": 7.0}, "router": {"experts": 16, "top": 4, "groups": {"count": 4, "keep": 2}},
+               "shared": {"ff": width, "limit": 7.0}}
+    order = [{"type": "attention", "mixer": near, "mlp": clamped},
+             {"type": "parallel", "mixer": {"left": far, "right": lightning, "left_scale": 1.0, "right_scale": 1.0}, "mlp": clamped}]
+    movazen = {"architecture": "Movazen", "vocab": vocab, "width": width, "embedding": {"scale": 1.0}, "norm": {"eps": 1e-5},
+               "token_side": {"dim": 256}, "layers": [order[i % 2] for i in range(layers)], "max_positions": context}
+    return {"llama": llama, "novosun": novosun, "ditazen": ditazen, "noresun": noresun, "zovozen": zovozen, "guduzen": guduzen,
+            "movazen": movazen}
 
 
 def designs(args):
-    """Prompt steps and decode steps of the Novosun, Ditazen, Noresun, Zovozen and Guduzen designs beside the Llama design at equal width, depth
+    """Prompt steps and decode steps of the Novosun, Ditazen, Noresun, Zovozen, Guduzen and Movazen designs beside the Llama design at equal width, depth
     and vocabulary (random weights drawn on the device): tokens a second of a whole prompt of --prompt tokens and
     of decode steps of 1, 8 and 64 requests after such prompts, through the step function with captured programs and
     the greedy pick."""
@@ -512,7 +527,7 @@ def designs(args):
             result["prefill"] = {"tokens": prompt, "ms": round(pf * 1e3, 3), "tokens_per_s": round(prompt / pf, 1)}
             out.setdefault(str(width), {})[design] = result
             del runner, model
-    return {"metric": f"prompt and decode tokens/s of the Novosun, Ditazen, Noresun, Zovozen and Guduzen designs beside Llama at equal width, {args.design_layers} layers",
+    return {"metric": f"prompt and decode tokens/s of the Novosun, Ditazen, Noresun, Zovozen, Guduzen and Movazen designs beside Llama at equal width, {args.design_layers} layers",
             "unit": "tokens/s", "n_gpus": 1, "dtype": "bf16" if args.dtype == "bfloat16" else "fp32", "steps": steps,
             "data": "synthetic (random weights N(0,0.02), uniform-random token ids)", "prompt_len": prompt,
             "execution": args.execution, "widths": out}

@@ -228,3 +228,10 @@ def forward(config, w, tokens, layers_out=None, margins=None):
         if layers_out is not None:
             layers_out.append(x.copy())
     return linear(rms(x, eps) * (1.0 + w["final.norm"]), w["head"])
+
+
+def greedy(config, w, prompt, n):
+    tokens = list(prompt)
+    for _ in range(n):
+        tokens.append(int(np.argmax(forward(config, w, tokens)[-1])))
+    return tokens[len(prompt):]
