@@ -169,22 +169,26 @@ def plain_logits(folder, tokens):
 
 def decided_rows(folder, tokens):
     """Which positions of a sequence have no close call of their own: True where every router's margin is at least
-    CLOSE_CALL.  In bfloat16 a narrower margin may choose another expert than the float64 implementation does, which is no
+    CLOSE_CALL and no side's gate leaves next to nothing of a row (which the norm behind it would blow up, rounding and
+    all).  In bfloat16 a narrower margin may choose another expert than the float64 implementation does, which is no
     fault; such a position is compared in float32 only."""
     return _plain(folder, tokens)[1] >= CLOSE_CALL
 
 
-def decisive_tokens(folder, seed, n, vocab, margin=0.5 * CLOSE_CALL, tries=400):
-    """`n` token ids drawn from `seed` at none of whose positions a router of the plain model decides by less than `margin`:
-    the first position that does gets another token until none is left (a position's routers see only the tokens up to
-    it, so what is settled stays settled)."""
+def decisive_tokens(folder, seed, n, vocab, margin=2 * CLOSE_CALL, tries=200):
+    """`n` token ids drawn from `seed` at none of whose positions the plain model's margins are under `margin`: positions at
+    which they are get other tokens until none is left."""
+    kept = _PLAIN.get(("tokens", str(folder), seed, n, margin))
+    if kept is not None:
+        return list(kept)
     rng = np.random.default_rng(seed)
     tokens = [int(t) for t in rng.integers(0, vocab, n)]
     for _ in range(tries):
-        margins = _plain(folder, tokens)[1]
-        close = np.nonzero(margins < margin)[0]
+        close = np.nonzero(_plain(folder, tokens)[1] < margin)[0]
         if not len(close):
+            _PLAIN[("tokens", str(folder), seed, n, margin)] = list(tokens)
             return tokens
         _PLAIN.pop((str(folder), tuple(tokens)), None)
-        tokens[int(close[0])] = int(rng.integers(0, vocab))
+        for at in close:
+            tokens[int(at)] = int(rng.integers(0, vocab))
     raise AssertionError(f"no sequence of {n} tokens without a close call after {tries} tries")

@@ -198,10 +198,15 @@ def mixture(h, w, p, m, margins=None):
 
 # -- the whole ----------------------------------------------------------------------------------------------------
 
-def token_side(x, tokens, w, p, i, dim, eps):
-    """The part of a token's row that belongs to layer i, gated by the stream, projected, normed."""
+def token_side(x, tokens, w, p, i, dim, eps, margins=None):
+    """The part of a token's row that belongs to layer i, gated by the stream, projected, normed.  `margins` (a list)
+    receives how small the gate leaves a row, times 0.4: what is nearly gated away and then normed is mostly rounding."""
     e = np.asarray(w["side.embed"], np.float64)[tokens, i * dim:(i + 1) * dim]
-    y = linear(gelu_tanh(linear(x, w[p + ".side.gate"])) * e, w[p + ".side.proj"])
+    z = linear(x, w[p + ".side.gate"])
+    if margins is not None:
+        size = lambda a: np.sqrt(np.mean(a * a, axis=-1))
+        margins.append(0.4 * size(gelu_tanh(z) * e) / np.maximum(size(z * e), 1e-300))
+    y = linear(gelu_tanh(z) * e, w[p + ".side.proj"])
     return rms(y, eps) * w[p + ".side.norm"]
 
 
@@ -215,7 +220,7 @@ def read_folder(folder):
 
 def forward(config, w, tokens, layers_out=None, margins=None):
     """Logits [T, vocab] of one sequence; `layers_out` (a list) receives the residual stream after every layer, `margins`
-    (a list) how far every router's decisions are from turning round."""
+    (a list) how far every router's decisions are from turning round and how much of a row its side gates leave."""
     tokens = np.asarray(tokens, int)
     eps = config["norm"]["eps"]
     x = np.asarray(w["embed"], np.float64)[tokens] * config["embedding"]["scale"] + sinusoids(np.arange(len(tokens)), config["width"])
@@ -224,7 +229,7 @@ def forward(config, w, tokens, layers_out=None, margins=None):
         x = x + mixer(rms(x, eps) * (1.0 + w[p + ".norm1"]), w, p + ".mix", layer, eps)
         if layer.get("mlp"):
             x = x + mixture(rms(x, eps) * (1.0 + w[p + ".norm2"]), w, p + ".mlp", layer["mlp"], margins)
-        x = x + token_side(x, tokens, w, p, i, config["token_side"]["dim"], eps)
+        x = x + token_side(x, tokens, w, p, i, config["token_side"]["dim"], eps, margins)
         if layers_out is not None:
             layers_out.append(x.copy())
     return linear(rms(x, eps) * (1.0 + w["final.norm"]), w["head"])
