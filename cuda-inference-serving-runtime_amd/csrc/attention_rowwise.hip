@@ -150,10 +150,22 @@ __global__ void attn_merge_sum_kernel(const float* __restrict__ part_o, T* __res
 // keys at all (padding) gives zeros.  LOG2: the maxima are in units of log2.  MANY: more than sixteen splits
 // (a kernel of its own, so that the common few-split form keeps its registers and code to itself).
 // `row_ids`: the partials of block row i belong to output row row_ids[i] (negative: to none).
-template <typename T, bool LOG2, bool MANY>
+// GATED: the heads are packed and gated on the way: out[row, head, d] for d < vdim, times sigmoid(gate[row, head vdim + d]).
+struct MergeGate { const float* gate; int ld, vdim; };
+template <typename T, bool LOG2, bool MANY, bool GATED = false>
 __global__ void attn_merge_kernel(const float* __restrict__ part_o, const float* __restrict__ part_ml,
-                                  T* __restrict__ out, int heads, int dim, int splits, const int* __restrict__ row_ids = nullptr) {
+                                  T* __restrict__ out, int heads, int dim, int splits, const int* __restrict__ row_ids = nullptr,
+                                  MergeGate mg = MergeGate{nullptr, 0, 0}) {
     const int head = blockIdx.y;
+    auto finish = [&](int row, int d, float y) {
+        if (GATED) {
+            if (d >= mg.vdim) return;
+            const float z = mg.gate[(size_t)row * mg.ld + head * mg.vdim + d];
+            store_f32(out + ((size_t)row * heads + head) * mg.vdim + d, y / (1.0f + expf(-z)));
+        } else {
+            store_f32(out + ((size_t)row * heads + head) * dim + d, y);
+        }
+    };
     const size_t base = ((size_t)blockIdx.x * heads + head) * splits;
     const int row = row_ids ? row_ids[blockIdx.x] : (int)blockIdx.x;
     if (row < 0) return;
@@ -179,7 +191,7 @@ __global__ void attn_merge_kernel(const float* __restrict__ part_o, const float*
                 den += w;
                 num += w * os[s];
             }
-            store_f32(out + ((size_t)row * heads + head) * dim + d, den > 0.f ? num / den : 0.f);
+            finish(row, d, den > 0.f ? num / den : 0.f);
         }
         return;
     }
@@ -211,7 +223,7 @@ __global__ void attn_merge_kernel(const float* __restrict__ part_o, const float*
                 num += w * os[s];
             }
         }
-        store_f32(out + ((size_t)row * heads + head) * dim + d, den > 0.f ? num / den : 0.f);
+        finish(row, d, den > 0.f ? num / den : 0.f);
     }
 }
 
@@ -226,6 +238,18 @@ extern "C" int cisr_attn_merge(const float* part_o, const float* part_ml, void* 
     const int threads = merge_threads(dim);
     if (splits <= 16) attn_merge_kernel<bf16_t, true, false><<<dim3(rows, heads), threads, 0, stream>>>(part_o, part_ml, (bf16_t*)out, heads, dim, splits, row_ids);
     else attn_merge_kernel<bf16_t, true, true><<<dim3(rows, heads), threads, 0, stream>>>(part_o, part_ml, (bf16_t*)out, heads, dim, splits, row_ids);
+    return CISR_LAUNCH_CHECK();
+}
+
+// the same with the heads packed to vdim coordinates and gated element by element (float gates)
+extern "C" int cisr_attn_merge_gated(const float* part_o, const float* part_ml, void* out, int rows, int heads, int dim, int splits,
+                                     const float* gate, int ld_gate, int vdim, hipStream_t stream) {
+    if (rows <= 0) return 0;
+    if (heads > 65535 || splits < 1 || !gate || vdim <= 0 || vdim > dim) return (int)hipErrorInvalidValue;
+    const MergeGate mg = {gate, ld_gate, vdim};
+    const int threads = merge_threads(dim);
+    if (splits <= 16) attn_merge_kernel<bf16_t, true, false, true><<<dim3(rows, heads), threads, 0, stream>>>(part_o, part_ml, (bf16_t*)out, heads, dim, splits, nullptr, mg);
+    else attn_merge_kernel<bf16_t, true, true, true><<<dim3(rows, heads), threads, 0, stream>>>(part_o, part_ml, (bf16_t*)out, heads, dim, splits, nullptr, mg);
     return CISR_LAUNCH_CHECK();
 }
 

@@ -21,11 +21,12 @@ embedding_sinusoid_kernel(const int* __restrict__ tokens, const int* __restrict_
     const TE* e = table + (size_t)tok * dim;
     float* o = out + (size_t)row * dim;
     float ss = 0.f;
+#pragma unroll 4
     for (int d = 2 * threadIdx.x; d < dim; d += 512) {
         double t = at * turns[d / 2];
-        t -= floor(t);
+        t -= rint(t);
         float s, c;
-        sincosf((float)(t * 6.283185307179586), &s, &c);
+        sincospif((float)(2.0 * t), &s, &c);
         const float v0 = load_f32(e + d) * scale + s;
         o[d] = v0;
         ss += v0 * v0;
@@ -70,6 +71,61 @@ side_gate_kernel(const float* __restrict__ z, int ldz, const int* __restrict__ t
         v = unary_activation(z[row * ldz + c], ACT_GELU_TANH) * load_f32(side + (size_t)tok * ld_side + first + c);
     }
     store_f32(act + i, v);
+}
+
+// Steps of few rows: the gate's product as well, z = h[r] . w[c] with bf16 operands.  grid (padded / 16, rows): a block of
+// four waves makes 16 columns of one row, a wave 4 of them, all loads of a row of w in flight together; hidden % 8 == 0 and
+// at most 64 x 8 x SIDE_CHUNKS.
+#define SIDE_CHUNKS 16
+typedef __attribute__((ext_vector_type(4))) uint32_t u32x4_side;
+__global__ void __launch_bounds__(256)
+side_rows_kernel(const bf16_t* __restrict__ h, int ldh, const bf16_t* __restrict__ w, const int* __restrict__ tokens,
+                 const bf16_t* __restrict__ side, int ld_side, int first, bf16_t* __restrict__ act, int hidden, int width, int padded, int vocab) {
+    const int row = blockIdx.y, wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
+    const int c0 = (blockIdx.x * 4 + wave) * 4;
+    if (c0 >= padded) return;
+    const bf16_t* hr = h + (size_t)row * ldh;
+    int tok = tokens[row];
+    tok = tok < 0 ? 0 : tok >= vocab ? vocab - 1 : tok;
+    const bool mine = lane < 4 && c0 + lane < width;
+    const float e = mine ? bf16_to_f32(side[(size_t)tok * ld_side + first + c0 + lane]) : 0.f;
+    const u32x4_side zero = {0u, 0u, 0u, 0u};
+    float sum[4] = {0.f, 0.f, 0.f, 0.f};
+    const int chunks = (hidden + 511) / 512;
+#pragma unroll
+    for (int c = 0; c < SIDE_CHUNKS; ++c) {
+        if (c >= chunks) continue;
+        const int k = (c * 64 + lane) * 8;
+        const u32x4_side a = k < hidden ? *(const u32x4_side*)(hr + k) : zero;
+        u32x4_side b[4];
+#pragma unroll
+        for (int j = 0; j < 4; ++j) b[j] = k < hidden ? *(const u32x4_side*)(w + (size_t)min(c0 + j, padded - 1) * hidden + k) : zero;
+        const uint32_t aw[4] = {a.x, a.y, a.z, a.w};
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            const uint32_t bw[4] = {b[j].x, b[j].y, b[j].z, b[j].w};
+#pragma unroll
+            for (int x = 0; x < 4; ++x) {
+                sum[j] = fmaf(__uint_as_float(aw[x] << 16), __uint_as_float(bw[x] << 16), sum[j]);
+                sum[j] = fmaf(__uint_as_float(aw[x] & 0xffff0000u), __uint_as_float(bw[x] & 0xffff0000u), sum[j]);
+            }
+        }
+    }
+#pragma unroll
+    for (int j = 0; j < 4; ++j) sum[j] = wave_sum(sum[j]);
+    if (lane < 4 && c0 + lane < padded)
+        act[(size_t)row * padded + c0 + lane] = f32_to_bf16(mine ? unary_activation(lane == 0 ? sum[0] : lane == 1 ? sum[1] : lane == 2 ? sum[2] : sum[3], ACT_GELU_TANH) * e : 0.f);
+}
+
+extern "C" int cisr_side_rows(const void* h, int ldh, const void* w, const int* tokens, const void* side, int ld_side, int first, void* act,
+                              int rows, int hidden, int width, int padded, int vocab, hipStream_t stream) {
+    if (rows <= 0) return 0;
+    if (hidden <= 0 || hidden % 8 || ldh % 8 || hidden > 512 * SIDE_CHUNKS || width <= 0 || padded < width || first < 0 || first + width > ld_side ||
+        vocab <= 0 || rows > 65535 || ((uintptr_t)h) % 16 || ((uintptr_t)w) % 16)
+        return (int)hipErrorInvalidValue;
+    side_rows_kernel<<<dim3((padded + 15) / 16, rows), 256, 0, stream>>>((const bf16_t*)h, ldh, (const bf16_t*)w, tokens, (const bf16_t*)side, ld_side, first,
+                                                                       (bf16_t*)act, hidden, width, padded, vocab);
+    return CISR_LAUNCH_CHECK();
 }
 
 extern "C" int cisr_side_gate(const float* z, int ldz, const int* tokens, const void* side, int ld_side, int first, void* act, int rows,

@@ -282,6 +282,128 @@ route_scored_wave_kernel(const float* __restrict__ logits, int ld, const float* 
     if (lane < top) weights[(size_t)row * top + lane] = law.floor >= 0.f ? mine_w / (total + law.floor) : mine_w;
 }
 
+// The router's product and the choice in one kernel, for bf16 rows and routers of at most 64 outputs (with the gate row):
+// logits = h . W^T in float, W [rows_w, K] the router's `outputs` rows and, if gate_out, one more whose logit goes there; the
+// choice as above.  A block of eight waves takes 16 rows: the waves share K in steps of 32 (step s to wave s mod 8), their
+// 16 x 16 tiles meet in LDS, then a wave routes two rows, a lane an output: an output's place among the choices is the
+// number of outputs that go before it, so no choice waits for the one before.
+typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8_route;
+typedef __attribute__((ext_vector_type(4))) float f32x4_route;
+#define ROUTE_WAVES 8
+template <int NT>
+__global__ void __launch_bounds__(ROUTE_WAVES * 64)
+route_product_kernel(const bf16_t* __restrict__ h, int ldh, const bf16_t* __restrict__ W, int rows_w, int K, const float* __restrict__ correction,
+                     int* __restrict__ chosen, float* __restrict__ weights, float* __restrict__ gate_out, int rows, int outputs, int top, int groups,
+                     int keep, ScoreLaw law) {
+    __shared__ float parts[ROUTE_WAVES][16][NT * 16 + 1];
+    __shared__ float cs[ROUTE_WAVES][64];
+    const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x / WAVE), lane = threadIdx.x % WAVE, r = lane % 16, g = lane / 16;
+    const int row0 = blockIdx.x * 16;
+    f32x4_route acc[NT];
+#pragma unroll
+    for (int j = 0; j < NT; ++j) acc[j] = (f32x4_route){0.f, 0.f, 0.f, 0.f};
+    const bf16_t* hr = h + (size_t)min(row0 + r, rows - 1) * ldh;
+    const int steps = (K + 31) / 32;
+#pragma unroll 4
+    for (int s = wave; s < steps; s += ROUTE_WAVES) {
+        const int k = s * 32 + g * 8;
+        const bool in = k < K;                                   // (K % 8 == 0: a lane's eight are all in or all out)
+        bf16x8_route a = {}, b[NT];
+        if (in) a = *(const bf16x8_route*)(hr + k);
+#pragma unroll
+        for (int j = 0; j < NT; ++j) b[j] = *(const bf16x8_route*)(W + (size_t)min(j * 16 + r, rows_w - 1) * K + (in ? k : 0));
+#pragma unroll
+        for (int j = 0; j < NT; ++j) acc[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b[j], acc[j], 0, 0, 0);
+    }
+#pragma unroll
+    for (int j = 0; j < NT; ++j)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) parts[wave][4 * g + e][j * 16 + r] = acc[j][e];
+    __syncthreads();
+    float* mine = cs[wave];
+    auto meet = [] {                                             // (the wave's own LDS writes, before its reads)
+        __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+        __builtin_amdgcn_wave_barrier();
+    };
+    for (int i = wave; i < 16; i += ROUTE_WAVES) {
+        const int row = row0 + i;
+        if (row >= rows) break;
+        float z = 0.f;
+        if (lane < NT * 16)
+            for (int w = 0; w < ROUTE_WAVES; ++w) z += parts[w][i][lane];
+        if (gate_out && lane == outputs) gate_out[row] = z;
+        const bool real = lane < outputs;
+        float s;
+        if (law.sigmoid) {
+            s = real ? logistic(z) : 0.f;
+        } else {
+            const float largest = wave_max(real ? z : -INFINITY);
+            s = real ? expf(z - largest) : 0.f;
+            s /= wave_sum(s);
+        }
+        float c = real ? s + (correction ? correction[lane] : 0.f) : -INFINITY;
+        if (groups > 0) {
+            const int per = outputs / groups;
+            meet();
+            mine[lane] = c;
+            meet();
+            float score = -INFINITY;
+            if (lane < groups) {
+                float first = -INFINITY, second = -INFINITY;
+                for (int j = 0; j < per; ++j) {
+                    const float v = mine[lane * per + j];
+                    second = fmaxf(second, fminf(first, v));
+                    first = fmaxf(first, v);
+                }
+                score = law.pairs && per > 1 ? first + second : first;
+            }
+            meet();
+            mine[lane] = score;
+            meet();
+            int before = 0;
+            for (int j = 0; j < groups; ++j) { const float v = mine[j]; before += v > score || (v == score && j < lane); }
+            const unsigned long long kept = __ballot(lane < groups && before < keep);
+            if (!(real && ((kept >> (lane / per)) & 1ull))) c = -INFINITY;
+        }
+        meet();
+        mine[lane] = c;
+        meet();
+        int place = 0;
+        for (int j = 0; j < outputs; ++j) { const float v = mine[j]; place += v > c || (v == c && j < lane); }
+        const bool taken = real && place < top;
+        const float total = wave_sum(taken ? s : 0.f);
+        if (taken) {
+            chosen[(size_t)row * top + place] = lane;
+            weights[(size_t)row * top + place] = law.floor >= 0.f ? s / (total + law.floor) : s;
+        }
+    }
+}
+
+extern "C" int cisr_experts_route_product(const void* h, int ldh, const void* W, int rows_w, int K, const float* correction, int* chosen, float* weights,
+                                          float* gate_out, int rows, int outputs, int experts, int top, int groups, int keep, int sigmoid,
+                                          int group_pairs, float floor, int max_tiles, int* pair_of_pos, int* tile_expert, hipStream_t stream) {
+    if (rows <= 0) return 0;
+    const bool arrange = pair_of_pos != nullptr;
+    const int used = outputs + (gate_out ? 1 : 0);
+    if (outputs <= 0 || used > 64 || rows_w < used || experts <= 0 || experts > outputs || top <= 0 || top > MAX_TOP || top > outputs || groups < 0 || groups > 64 ||
+        K <= 0 || K % 8 || ldh % 8 || ((uintptr_t)h) % 16 || ((uintptr_t)W) % 16 ||
+        (groups > 0 && (outputs % groups || keep <= 0 || keep > groups || keep * (outputs / groups) < top)) ||
+        (arrange && (!tile_expert || (long long)max_tiles * EX_TILE < (long long)rows * top + (long long)experts * (EX_TILE - 1))))
+        return (int)hipErrorInvalidValue;
+    const ScoreLaw law = {sigmoid, group_pairs, floor};
+#define ROUTE_PRODUCT(NT) route_product_kernel<NT><<<(rows + 15) / 16, ROUTE_WAVES * 64, 0, stream>>>((const bf16_t*)h, ldh, (const bf16_t*)W, rows_w, K, correction,         chosen, weights, gate_out, rows, outputs, top, groups, keep, law)
+    const int nt = (used + 15) / 16;
+    if (nt == 1) ROUTE_PRODUCT(1);
+    else if (nt == 2) ROUTE_PRODUCT(2);
+    else if (nt == 3) ROUTE_PRODUCT(3);
+    else ROUTE_PRODUCT(4);
+#undef ROUTE_PRODUCT
+    int err = CISR_LAUNCH_CHECK();
+    if (err || !arrange) return err;
+    arrange_kernel<<<1, 1024, 3 * experts * sizeof(int), stream>>>(chosen, rows * top, experts, max_tiles, pair_of_pos, tile_expert);
+    return CISR_LAUNCH_CHECK();
+}
+
 // `experts` of the router's `outputs` have matrices (the first ones): only their pairs are arranged into tiles.
 extern "C" int cisr_experts_route_scored(const float* logits, int ld, const float* correction, int* chosen, float* weights, int rows,
                                          int outputs, int experts, int top, int groups, int keep, int sigmoid, int group_pairs,
@@ -347,10 +469,10 @@ experts_add_kernel(float* __restrict__ x, const float* __restrict__ down, const 
                    const float* __restrict__ next_w, float next_eps, TO* __restrict__ out) {
     __shared__ float red[4];
     const size_t row = blockIdx.x;
-    float w[MAX_TOP];
-    for (int k = 0; k < top; ++k) {
-        const int e = chosen[row * top + k];
-        w[k] = e >= 0 && e < experts ? weights[row * top + k] : 0.f;
+    __shared__ float w[MAX_TOP];
+    if (threadIdx.x < top) {
+        const int e = chosen[row * top + threadIdx.x];
+        w[threadIdx.x] = e >= 0 && e < experts ? weights[row * top + threadIdx.x] : 0.f;
     }
     const float sg = shared && gate ? logistic(gate[row * ld_gate]) : 1.0f;
     float v[E], vx[E], ss = 0.f;
@@ -360,12 +482,26 @@ experts_add_kernel(float* __restrict__ x, const float* __restrict__ down, const 
         vx[e] = d < dim ? x[row * dim + d] : 0.f;
         v[e] = shared && d < dim ? sg * shared[row * dim + d] : 0.f;
     }
-    for (int k = 0; k < top; ++k)
+    __syncthreads();
+    // (four choices' rows on their way together where registers allow; a choice that adds nothing may never have been
+    // written: its row is read and dropped)
+    constexpr int KB = E <= 16 ? 4 : 1;
+    for (int k0 = 0; k0 < top; k0 += KB) {
+        float more[KB][E];
 #pragma unroll
-        for (int e = 0; e < E; ++e) {
-            const int d = threadIdx.x + 256 * e;
-            if (d < dim && w[k] != 0.f) v[e] += w[k] * down[(row * top + k) * dim + d];
+        for (int k = 0; k < KB; ++k)
+#pragma unroll
+            for (int e = 0; e < E; ++e) {
+                const int d = threadIdx.x + 256 * e;
+                more[k][e] = k0 + k < top && d < dim ? down[(row * top + k0 + k) * dim + d] : 0.f;
+            }
+#pragma unroll
+        for (int k = 0; k < KB; ++k) {
+            const float wk = k0 + k < top ? w[k0 + k] : 0.f;
+#pragma unroll
+            for (int e = 0; e < E; ++e) v[e] += wk != 0.f ? wk * more[k][e] : 0.f;
         }
+    }
 #pragma unroll
     for (int e = 0; e < E; ++e) {
         const int d = threadIdx.x + 256 * e;

@@ -306,8 +306,11 @@ def _split_workspace(ctx, rows, heads, splits, head_dim, dtype=torch.float32, ta
             ctx.buffer("attn.part_ml", (rows * heads * splits * 2,), torch.float32))
 
 
+GATED = "gated"       # paged_attention: the heads' results were packed and gated by the merge
+
+
 def paged_attention(ctx, q, q_row_stride, kcache, vcache, view, out, heads, kv_heads, head_dim, window, scale,
-                    defer_merge=None, tuning=DEFAULT_TUNING, head_bias=None, slopes=None, sink=None, keep_first=0):
+                    defer_merge=None, tuning=DEFAULT_TUNING, head_bias=None, slopes=None, sink=None, keep_first=0, merge_gate=None):
     """out[r] = attention of row r's queries over its request's cached keys up to its own position (or the last
     `window` of them).  `ctx` is the step's context (rows, segments, positions, buffers, step arrays), `view` the
     cache group as the step sees it (block tables, page size).
@@ -320,7 +323,10 @@ def paged_attention(ctx, q, q_row_stride, kcache, vcache, view, out, heads, kv_h
 
     `defer_merge(splits) -> bool`: the caller's next product can merge the partial results of a decode step whose
     keys are split over `splits` blocks itself (ops.gemm_merged).  Where that is so, no merge kernel runs, `out`
-    is left alone and (partial outputs bf16, statistics float, splits) is returned; otherwise None."""
+    is left alone and (partial outputs bf16, statistics float, splits) is returned; otherwise None.
+
+    `merge_gate` = (gates, packed, vdim): where the keys of a decode step are split, the merge packs and gates the heads
+    itself (ops.attention_mfma) and GATED is returned; otherwise `out` is written and the caller gates."""
     rows = out.shape[0]
     keep_first = int(keep_first) if window else 0
     span = ctx.span_hint if not window else min(ctx.span_hint, window + 31 + keep_first)
@@ -354,9 +360,10 @@ def paged_attention(ctx, q, q_row_stride, kcache, vcache, view, out, heads, kv_h
         order = None
         if splits == 1 and rows * chunks >= tuning.order_rows_from:
             order = ctx.step_array(RowsLongestFirst())[0][:rows]
+        gated = merge_gate if splits > 1 else None
         ops.attention_mfma(*common, None, splits, workspace, waves, row_ids=order, stream_loads=stream(rows * chunks, waves, splits),
-                           **law)
-        return None
+                           merge_gate=gated, **law)
+        return None if gated is None else GATED
     singles = SingleRows(tuning.split_single_from)
     single_rows, n_single = ctx.step_array(singles)
     if n_single:

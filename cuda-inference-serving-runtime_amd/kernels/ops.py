@@ -91,6 +91,9 @@ def _declare(h):
         "cisr_experts_gemm": [p, i, p, p, p, i, i, p, i, i, i, i, i, i, i, p],
         "cisr_experts_rows": [p, i, p, p, i, p, i, i, i, i, i, i, i, p],
         "cisr_experts_route_scored": [p, i, p, p, p, i, i, i, i, i, i, i, i, f, i, p, p, p],
+        "cisr_experts_route_product": [p, i, p, i, i, p, p, p, p, i, i, i, i, i, i, i, i, f, i, p, p, p],
+        "cisr_attn_merge_gated": [p, p, p, i, i, i, i, p, i, i, p],
+        "cisr_side_rows": [p, i, p, p, p, i, i, p, i, i, i, i, i, p],
         "cisr_experts_add": [p, p, p, p, p, p, i, i, i, i, i, p, f, p, i, p],
         "cisr_experts_rows_gated": [p, i, p, p, i, p, i, i, i, i, i, f, f, f, p],
         "cisr_embedding_sinusoid": [p, p, p, p, p, p, f, p, i, i, i, f, i, i, p],
@@ -866,7 +869,7 @@ def qkv_rope(a, w, q_out, positions, slots, cos, sin, kcache, vcache, heads, kv_
 def attention_mfma(q, q_row_stride, kcache, vcache, tables, seg_of_row, positions, out, heads, kv_heads, dim,
                    page_size, window, scale, tasks=None, splits=1, workspace=None, waves=4, block_tiles=False,
                    item_tiles=1, row_ids=None, merge=True, key_groups=1, stream_loads=False, head_bias=None, slopes=None, sink=None,
-                   keep_first=0):
+                   keep_first=0, merge_gate=None):
     """Matrix-core attention (bf16).  tasks int32 [n, 4] = (segment, first row, rows, 0) runs tiles of
     prompt rows: one tile of 16/GC rows a block whose waves share the keys (with item_tiles=2, head sizes up to
     64: 32/GC rows, two item tiles a wave), or with `block_tiles` (head sizes up to 128) one tile of
@@ -882,7 +885,9 @@ def attention_mfma(q, q_row_stride, kcache, vcache, tables, seg_of_row, position
     `head_bias` (float [heads]): the sigmoid law (see attention_rowwise); the tile and row forms have it, the block
     tiles do not, and the partial results of split keys are plain sums that only this function merges.
     `slopes`, `sink`, `keep_first`: as in attention_rowwise; with slopes or kept keys every form but the block tiles of 64 and
-    128 items on the 16 x 16 instruction runs (a build of its own)."""
+    128 items on the 16 x 16 instruction runs (a build of its own).  `merge_gate` = (gates float view [T, heads * vdim], packed
+    bf16 [T, heads * vdim], vdim) with splits > 1 and all rows: the merge packs the heads' first vdim coordinates, gates them
+    element by element and writes `packed`; `out` is not written."""
     rows = out.shape[0]
     law_name = "sigmoid" if head_bias is not None else "distance" if slopes is not None or keep_first else "softmax"
     if law_name == "sigmoid" and (sink is not None or slopes is not None or keep_first):
@@ -951,7 +956,14 @@ def attention_mfma(q, q_row_stride, kcache, vcache, tables, seg_of_row, position
               11 if mode == 1 and stream_loads else mode, int(waves),
               int(mode == 1 and splits > 1 and not merge), _stream(), *law), "attention_mfma")
     if mode == 1 and splits > 1 and merge:
-        if head_bias is not None:
+        if merge_gate is not None:
+            gates, packed, vdim = merge_gate
+            gp, ldg = _rows_of(gates, "gates", heads * vdim)
+            if head_bias is not None or tasks is not None or row_ids is not None or gates.shape[0] != rows or vdim > dim:
+                raise KernelError("attention_mfma: a gated merge is one of the softmax law over all rows")
+            _check(lib().cisr_attn_merge_gated(po, pm, _dev(packed, "packed", torch.bfloat16, (rows, heads * vdim)), n_tasks, heads, dim, int(splits),
+                                               gp, ldg, int(vdim), _stream()), "attention_merge")
+        elif head_bias is not None:
             _check(lib().cisr_attn_merge_sum(po, out.data_ptr(), n_tasks, heads, dim, int(splits), tp, _stream()), "attention_merge")
         else:
             _check(lib().cisr_attn_merge(po, pm, out.data_ptr(), n_tasks, heads, dim, int(splits), tp, _stream()), "attention_merge")
@@ -1314,6 +1326,8 @@ def _rec():
         p, i, f, ll = C.c_void_p, C.c_int, C.c_float, C.c_longlong
         sig = {
             "cisr_linear_scan": [p, i, p, i, p, i, p, i, i, p, i, p, i, p, ll, p, p, i, i, i, i, i, f, i, i, i, i, p, p, p],
+            "cisr_lightning_step": [p, i, p, i, p, i, p, p, i, p, ll, p, p, i, i, i, i, p],
+            "cisr_lightning_chunks": [p, i, p, i, p, i, p, p, i, p, ll, p, p, i, i, i, i, i, p, p],
             "cisr_conv_silu": [p, i, i, p, p, p, ll, p, p, p, p, i, i, i, i, i, i, p, p, p, p, i, p],
             "cisr_decay_gate": [p, i, p, p, i, i, f, p],
             "cisr_decay_gate_low_rank": [p, i, i, p, p, p, i, i, f, p],
@@ -1419,6 +1433,54 @@ def linear_scan(q, k, v, decay, out, state, seg_start, state_slots, heads, rows_
                                    state.stride(0), _dev(seg_start, "seg_start", torch.int32, (segments + 1,)),
                                    _dev(state_slots, "state_slots", torch.int32, (segments,)), segments, heads, R, Cc,
                                    int(share), float(q_scale), int(bool(silu)), cols, T, int(piece), cp, dp, _stream()), "linear_scan")
+    return out
+
+
+LIGHTNING_CHUNK = 64      # rows of a chunk (csrc/recurrence_lightning.hip)
+
+
+def lightning_form(q, v, out, state, rows, segments, decode_only, cols_of_state):
+    """Which form of the lightning recurrence a step takes: "step" (single rows), "chunks" (portions of sixteen rows and
+    more on the mean), or "scan" (ops.linear_scan: short portions, columns the step does not take).  Of a captured program
+    it depends on rows, segments and decode_only only."""
+    if decode_only:
+        aligned = (cols_of_state % 4 == 0 and cols_of_state <= 1024 and v.stride(0) % 4 == 0 and out.stride(0) % 4 == 0 and state.stride(0) % 4 == 0
+                   and all(t.data_ptr() % 16 == 0 for t in (v, out, state)))
+        return "step" if aligned else "scan"
+    return "chunks" if rows >= LIGHTNING_CHUNK and rows >= 16 * segments else "scan"
+
+
+def lightning_slots(rows, segments):
+    """Chunk slots (states [heads, R, C] each) that a step of so many rows and segments can need."""
+    return rows // LIGHTNING_CHUNK + segments
+
+
+def lightning(form, q, k, v, decay, out, state, seg_start, state_slots, heads, rows_of_state, cols_of_state, carry=None):
+    """Per segment and head: S <- decay[head] S + silu(k) silu(v)^T, out = S^T silu(q) over the segment's rows in order, S
+    [rows_of_state, cols_of_state] in the segment's state slot.  q, k float views [T, heads * R], v, out [T, heads * C], decay
+    float [heads]; state float [slots, >= heads * R * C].  `form` "step": every segment one row; "chunks": any portions,
+    with `carry` a float buffer of lightning_slots(T, segments) * heads * R * C elements."""
+    R, Cc = int(rows_of_state), int(cols_of_state)
+    segments, T = state_slots.shape[0], v.shape[0]
+    qp, ldq = _rows_of(q, "q", heads * R)
+    kp, ldk = _rows_of(k, "k", heads * R)
+    vp, ldv = _rows_of(v, "v", heads * Cc)
+    op, ldo = _rows_of(out, "out", heads * Cc)
+    if R > 256 or any(t.shape[0] != T for t in (q, k, out)):
+        raise KernelError("lightning: a state has at most 256 rows, operands as many rows as each other")
+    if state.dtype != torch.float32 or state.dim() != 2 or state.stride(1) != 1 or state.shape[1] < heads * R * Cc or not state.is_cuda:
+        raise KernelError("lightning: the state must be float [slots, >= heads * R * C]")
+    args = (qp, ldq, kp, ldk, vp, ldv, _dev(decay, "decay", torch.float32, (heads,)), op, ldo, state.data_ptr(), state.stride(0),
+            _dev(seg_start, "seg_start", torch.int32, (segments + 1,)), _dev(state_slots, "state_slots", torch.int32, (segments,)), segments, heads, R, Cc)
+    if form == "step":
+        _check(_rec().cisr_lightning_step(*args, _stream()), "lightning_step")
+    elif form == "chunks":
+        slots = lightning_slots(T, segments)
+        if carry is None or carry.numel() < slots * heads * R * Cc:
+            raise KernelError("lightning: the chunks' states do not fit their buffer")
+        _check(_rec().cisr_lightning_chunks(*args, slots, _dev(carry, "carry", torch.float32), _stream()), "lightning_chunks")
+    else:
+        raise KernelError(f"lightning: form {form!r}")
     return out
 
 
@@ -1823,6 +1885,26 @@ def embedding_sinusoid(tokens, positions, table, turns, out, scale=1.0, norm=Non
     return out
 
 
+SIDE_ROWS = 16        # steps of at most this many rows make the gate's product and the activation in one kernel
+
+
+def side_rows_ok(h, w):
+    return (h.dtype == torch.bfloat16 and w.dtype == torch.bfloat16 and 0 < h.shape[0] <= SIDE_ROWS and h.stride(1) == 1 and h.shape[1] % 8 == 0
+            and h.shape[1] <= 8192 and h.stride(0) % 8 == 0 and h.data_ptr() % 16 == 0 and w.data_ptr() % 16 == 0)
+
+
+def side_rows(h, w, tokens, side, first, width, act):
+    """side_gate of z = h . w^T, the product included (bf16, few rows: side_rows_ok); w [padded, hidden] with zero rows from
+    `width` on, act bf16 [T, padded]."""
+    rows, padded = act.shape
+    vocab, ld_side = side.shape
+    if not side_rows_ok(h, w) or tuple(w.shape) != (padded, h.shape[1]) or h.shape[0] != rows or padded < width or first < 0 or first + width > ld_side:
+        raise KernelError("side_rows: shape not supported")
+    _check(lib().cisr_side_rows(h.data_ptr(), h.stride(0), _dev(w, "w"), _dev(tokens, "tokens", torch.int32, (rows,)), _dev(side, "side", torch.bfloat16),
+                                ld_side, int(first), _dev(act, "act", torch.bfloat16), rows, h.shape[1], int(width), padded, vocab, _stream()), "side_rows")
+    return act
+
+
 def side_gate(z, tokens, side, first, width, act):
     """act[r, c] = gelu_tanh(z[r, c]) * side[tokens[r], first + c] for c < width, 0 in the columns of `act` behind them; z a
     float view [T, >= width] with unit column stride, side [vocab, n] and act [T, >= width] of one type."""
@@ -1977,6 +2059,35 @@ def experts_combine(down, weights, chosen, x, y, experts, shared=None):
                                       None if shared is None else _dev(shared, "shared", torch.float32, (rows, dim)),
                                       _dev(y, "y", torch.float32, (rows, dim)), rows, dim, top, int(experts), _stream()), "experts_combine")
     return y
+
+
+def experts_route_product_ok(h, w, used):
+    """Whether experts_route_product takes the router: bf16, at most 64 outputs (with the gate's), aligned rows."""
+    return (h.dtype == torch.bfloat16 and w.dtype == torch.bfloat16 and 0 < used <= 64 and used <= w.shape[0] and h.stride(1) == 1 and h.stride(0) % 8 == 0
+            and h.shape[1] % 8 == 0 and h.data_ptr() % 16 == 0 and w.data_ptr() % 16 == 0 and w.is_contiguous())
+
+
+def experts_route_product(h, w, correction, top, chosen, weights, outputs, experts, groups=None, pair_of_pos=None, tile_expert=None,
+                          sigmoid=False, group_pairs=False, floor=None, gate=None):
+    """experts_route_scored of the logits h . w[:outputs]^T, the product included (bf16, at most 64 outputs:
+    experts_route_product_ok).  `gate` float [T, 1]: receives the logit of row `outputs` of w."""
+    rows, k = h.shape
+    count, keep = groups or (0, 0)
+    if not experts_route_product_ok(h, w, outputs + (gate is not None)) or w.shape[1] != k or not 0 < top <= min(outputs, 16):
+        raise KernelError("experts_route_product: shape not supported")
+    tiles, pp, tp = 0, None, None
+    if pair_of_pos is not None:
+        tiles = tile_expert.shape[0]
+        if tiles < expert_tiles(rows, top, experts):
+            raise KernelError(f"experts_route_product: {tiles} tiles for {rows} rows x {top} of {experts} experts")
+        pp, tp = _dev(pair_of_pos, "pair_of_pos", torch.int32, (tiles * EXPERT_TILE,)), _dev(tile_expert, "tile_expert", torch.int32, (tiles,))
+    _check(lib().cisr_experts_route_product(h.data_ptr(), h.stride(0), _dev(w, "w"), w.shape[0], k,
+                                            None if correction is None else _dev(correction, "correction", torch.float32, (outputs,)),
+                                            _dev(chosen, "chosen", torch.int32, (rows, top)), _dev(weights, "weights", torch.float32, (rows, top)),
+                                            None if gate is None else _dev(gate, "gate", torch.float32, (rows, 1)), rows, outputs, int(experts), top,
+                                            int(count), int(keep), int(bool(sigmoid)), int(bool(group_pairs)), -1.0 if floor is None else float(floor),
+                                            tiles, pp, tp, _stream()), "experts_route_product")
+    return chosen, weights
 
 
 class ExpertSum:

@@ -160,7 +160,8 @@ class NormedGatedAttention(Mixer):
         if not scale > 0:
             raise ValueError("the score scale must be positive")
         self.name, self.hidden, self.heads, self.kv_heads, self.dim, self.vdim = name, hidden, heads, kv_heads, dim, vdim
-        self.scale, self.eps, self.qk_norm, self.head_gate, self.window = float(scale), float(eps), qk_norm, bool(head_gate), window
+        self.scale, self.eps, self.qk_norm, self.window = float(scale), float(eps), qk_norm, window
+        self.head_gate = head_gate if head_gate == "element" else bool(head_gate)
         self.gate_rows = 0 if not head_gate else heads * vdim if head_gate == "element" else heads
         self.bias, self.own_kv = bool(bias), bool(own_kv)
         self.float_rows = self.bias if float_rows is None else bool(float_rows)
@@ -261,17 +262,20 @@ class NormedGatedAttention(Mixer):
                                 temperature=None if self.q_temp is None else (ctx.positions, *self.q_temp))
         out = ctx.buffer("gattn.out", (T, nh * pad), ctx.dtype)
         # a decode step of few rows may leave the partial results of its split keys to the output projection
+        first_gate = sum(self._projections().values())
+        gates = qkv[:, first_gate:first_gate + self.gate_rows] if self.head_gate else None
+        act = ctx.buffer("gattn.act", (T, nh * V), ctx.dtype) if gates is not None or pad != V else out
+        merge_gate = (gates, act, V) if self.head_gate == "element" and self.float_rows and ctx.dtype == torch.bfloat16 else None
         merges = None if self.head_gate or pad != V else (lambda splits: ops.gemm_merged_ok(T, self.w_out, nh, V, splits))
         unmerged = kernel.paged_attention(ctx, q, nh * pad, kcache, vcache, view, out, nh, nkv, pad, self.window, self.scale,
                                           defer_merge=merges, tuning=self.tuning, slopes=self.slope_t, sink=self.sink_t,
-                                          keep_first=self.keep_first)
+                                          keep_first=self.keep_first, merge_gate=merge_gate)
+        if unmerged is kernel.GATED:
+            return ctx.product_for_norm(act, self.w_out, "gattn.y")
         if unmerged is not None:
             return ops.gemm_merged(unmerged, nh, V, self.w_out, ctx.buffer("gattn.y", (T, self.hidden), torch.float32))
-        first_gate = sum(self._projections().values())
-        gates = qkv[:, first_gate:first_gate + self.gate_rows] if self.head_gate else None
-        act = out
         if gates is not None or pad != V:
-            act = ops.head_gate(out, gates, ctx.buffer("gattn.act", (T, nh * V), ctx.dtype), nh, V, pad)
+            ops.head_gate(out, gates, act, nh, V, pad)
         return ctx.product_for_norm(act, self.w_out, "gattn.y")
 
     def forward(self, h, residual, ctx, site, norm=None):

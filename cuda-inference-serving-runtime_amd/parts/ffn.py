@@ -326,24 +326,33 @@ class ScoredExperts(FeedForward):
         """The feed-forward's result as an ops.ExpertSum: the chosen experts' rows and their weights, and the shared part's
         rows, for a kernel that adds them all (no identity outputs)."""
         T, E, top, I = h.shape[0], self.experts, self.top, self.intermediate
-        logits = ops.gemm(h, self.w_router, ctx.buffer("moe.logits", (T, self.w_router.shape[0]), torch.float32), scratch=ctx.scratch)
         chosen, weights = ctx.buffer("moe.chosen", (T, top), torch.int32), ctx.buffer("moe.weights", (T, top), torch.float32)
         down = ctx.buffer("moe.down", (T * top, self.hidden), torch.float32)
-        route = (logits[:, :self.outputs], self.correction, top, chosen, weights, E, self.groups)
+        gate = None
+        if ops.experts_route_product_ok(h, self.w_router, self.outputs + (self.shared_gate is not None)):
+            gate = None if self.shared_gate is None else ctx.buffer("moe.gate", (T, 1), torch.float32)      # the product and the choice in one kernel
+
+            def route(*layout):
+                ops.experts_route_product(h, self.w_router, self.correction, top, chosen, weights, self.outputs, E, self.groups, *layout, gate=gate, **self.route)
+        else:
+            logits = ops.gemm(h, self.w_router, ctx.buffer("moe.logits", (T, self.w_router.shape[0]), torch.float32), scratch=ctx.scratch)
+            gate = None if self.shared_gate is None else logits[:, self.outputs:self.outputs + 1]
+
+            def route(*layout):
+                ops.experts_route_scored(logits[:, :self.outputs], self.correction, top, chosen, weights, E, self.groups, *layout, **self.route)
         if ops.experts_rows_ok(h, self.w_gate_up, T * top) and ops.experts_rows_ok(h, self.w_down, T * top):
             # few rows (decoding): every (row, choice) pair streams its expert's matrices
-            ops.experts_route_scored(*route, **self.route)
+            route()
             act = ops.experts_rows_gated(h, self.w_gate_up, chosen, ctx.buffer("moe.act", (T * top, I), ctx.dtype), self.law or (0.0, 0.0, 0.0), top=top)
             ops.experts_rows(act, self.w_down, chosen, down)
         else:
             tiles = ops.expert_tiles(T, top, E)
             places, tile_expert = ctx.buffer("moe.places", (tiles * ops.EXPERT_TILE,), torch.int32), ctx.buffer("moe.tiles", (tiles,), torch.int32)
-            ops.experts_route_scored(*route, places, tile_expert, **self.route)
+            route(places, tile_expert)
             gate_up = ops.experts_gemm(h, self.w_gate_up, places, tile_expert, ctx.buffer("moe.gate_up", (tiles * ops.EXPERT_TILE, 2 * I), ctx.dtype), top=top)
             act = self._activation(gate_up, ctx.buffer("moe.act", (tiles * ops.EXPERT_TILE, I), ctx.dtype))
             ops.experts_gemm(act, self.w_down, places, tile_expert, down, scatter=True)
         also = None if self.shared is None else self.shared.output(h, ctx, tag="moe.shared", unfinished=False)
-        gate = None if self.shared_gate is None else logits[:, self.outputs:self.outputs + 1]
         return ops.ExpertSum(down, weights, chosen, E, shared=also, gate=gate)
 
     def output(self, h, ctx, unsummed=False):
@@ -386,8 +395,12 @@ class TokenSide(FeedForward):
     def output(self, h, ctx, unfinished=True):
         """The sublayer's result, float [T, hidden], without the residual sum."""
         T = h.shape[0]
-        z = ops.gemm(h, self.w_gate, ctx.buffer("side.z", (T, self.padded), torch.float32), scratch=ctx.scratch)
-        act = ops.side_gate(z, ctx.tokens, self.source.side_table, self.first, self.width, ctx.buffer("side.act", (T, self.padded), ctx.dtype))
+        act, table = ctx.buffer("side.act", (T, self.padded), ctx.dtype), self.source.side_table
+        if ops.side_rows_ok(h, self.w_gate):
+            ops.side_rows(h, self.w_gate, ctx.tokens, table, self.first, self.width, act)        # few rows: the gate's product as well
+        else:
+            z = ops.gemm(h, self.w_gate, ctx.buffer("side.z", (T, self.padded), torch.float32), scratch=ctx.scratch)
+            ops.side_gate(z, ctx.tokens, table, self.first, self.width, act)
         return ctx.product_for_norm(act, self.w_proj, "side.y")
 
     def forward(self, h, residual, ctx, norm=None):

@@ -168,8 +168,16 @@ class LightningAttention(Mixer):
             proj = ops.gemm(h, self.w_in, ctx.buffer("la.proj", (T, self.w_in.shape[0]), torch.float32), scratch=ctx.scratch)
         state = ctx.cache.state_storage[site]
         o = ctx.buffer("la.o", (T, V), torch.float32)
-        _scan(ctx, "la", proj[:, :K], proj[:, K:2 * K], proj[:, 2 * K:2 * K + V], self.decay_row.expand(T, self.heads), o,
-              state.view(state.shape[0], -1), self.heads, self.dim, self.vdim, silu=True)
+        state = state.view(state.shape[0], -1)
+        q, k, v, sizes = proj[:, :K], proj[:, K:2 * K], proj[:, 2 * K:2 * K + V], (self.heads, self.dim, self.vdim)
+        form = ops.lightning_form(q, v, o, state, T, ctx.n_segments, ctx.decode_only, self.vdim)
+        if form == "scan":
+            _scan(ctx, "la", q, k, v, self.decay_row.expand(T, self.heads), o, state, *sizes, silu=True)
+        else:
+            carry = None
+            if form == "chunks":
+                carry = ctx.buffer("la.carry", (ops.lightning_slots(T, ctx.n_segments), self.heads * self.dim * self.vdim), torch.float32)
+            ops.lightning(form, q, k, v, self.decay_row[0], o, state, ctx.seg_start, ctx.state_slots, *sizes, carry=carry)
         act = ops.group_norm_gate(o, proj[:, 2 * K + V:2 * K + 2 * V], self.norm_weight, ctx.buffer("la.act", (T, V), ctx.dtype),
                                   1, self.eps, gate_first=False, sigmoid=True)
         return ctx.product_for_norm(act, self.w_out, "la.y")

@@ -171,6 +171,14 @@ def test_matrix_core_attention_with_slopes_kept_keys_and_a_sink_in_every_form(he
         assert np.isfinite(got).all(), f"{kind} {n} {m}"
         err = np.abs(got - want).max() / np.abs(want).max()
         assert err < 1.5e-2, f"{kind} {n} {m} differs by {err:.3e}"
+        if kind == "rows" and n > 1:             # the merge packs part of a head and gates it element by element
+            vdim = max(1, dim - 3)
+            gates = torch.randn(T, heads * vdim + 4, device="cuda")
+            packed, untouched = torch.empty(T, heads * vdim, dtype=torch.bfloat16, device="cuda"), out.fill_(7.0)
+            ops.attention_mfma(*common, splits=n, workspace=work, waves=m, merge_gate=(gates[:, 4:], packed, vdim), **law)
+            expected = want.reshape(T, heads, dim)[:, :, :vdim].reshape(T, -1) * P.sigmoid(gates[:, 4:].double().cpu().numpy())
+            close(packed.float().cpu().numpy(), expected, 1.5e-2)
+            assert (untouched == 7.0).all()
     assert ran >= 4
 
 
@@ -298,6 +306,36 @@ def test_routing_by_sigmoid_scores_and_pairs_of_a_group(rows, experts, top, grou
     place, te, flat = places.cpu().numpy(), tile_expert.cpu().numpy(), got.reshape(-1)
     assert sorted(p for p in place if p >= 0) == list(range(rows * top))
     assert all(te[pos // 64] == flat[pair] for pos, pair in enumerate(place) if pair >= 0)
+
+
+@pytest.mark.parametrize("rows, hidden, outputs, top, groups, sigmoid", [(1, 64, 2, 2, None, True), (9, 1000, 6, 3, (3, 2), True), (300, 96, 16, 4, (4, 2), True),
+                                                                        (70, 2048, 63, 8, (9, 4), True), (33, 40, 5, 1, None, False), (17, 264, 48, 6, (8, 3), False),
+                                                                        (2000, 512, 33, 2, (11, 5), True), (16, 136, 32, 3, (32, 7), True)])
+def test_the_router_s_product_and_the_choice_in_one_kernel(rows, hidden, outputs, top, groups, sigmoid):
+    """Beside the product and the choice as two kernels, which another test holds against plain arithmetic."""
+    from runtime.kernels import ops
+    rng = np.random.default_rng(rows + outputs)
+    h, w = dev(rng.standard_normal((rows, hidden)), torch.bfloat16), dev(2.0 * rng.standard_normal((outputs + 1, hidden)) / math.sqrt(hidden), torch.bfloat16)
+    correction = dev(0.1 * rng.standard_normal(outputs) - 0.9)
+    law = dict(sigmoid=sigmoid, group_pairs=sigmoid, floor=1e-20 if sigmoid else None)
+    made = {}
+    for which in ("two", "one"):
+        tiles = ops.expert_tiles(rows, top, outputs)
+        chosen, weights = torch.full((rows, top), -9, dtype=torch.int32, device="cuda"), torch.full((rows, top), float("nan"), device="cuda")
+        places, tile_expert = torch.empty(tiles * 64, dtype=torch.int32, device="cuda"), torch.empty(tiles, dtype=torch.int32, device="cuda")
+        gate = torch.full((rows, 1), float("nan"), device="cuda")
+        if which == "one":
+            ops.experts_route_product(h, w, correction, top, chosen, weights, outputs, outputs, groups, places, tile_expert, gate=gate, **law)
+        else:
+            logits = (h.double() @ w.double().t()).float().contiguous()
+            gate = logits[:, outputs:].contiguous()
+            ops.experts_route_scored(logits[:, :outputs], correction, top, chosen, weights, outputs, groups, places, tile_expert, **law)
+        made[which] = (chosen.cpu().numpy(), weights.cpu().numpy(), gate.cpu().numpy(), np.sort(places.cpu().numpy()))
+    close(made["one"][2], made["two"][2], 1e-5)
+    same = (made["one"][0] == made["two"][0]).all(axis=1)
+    assert same.mean() > 0.98, "choices differ beyond close calls"
+    close(made["one"][1][same], made["two"][1][same], 2e-5)
+    np.testing.assert_array_equal(made["one"][3], made["two"][3])
 
 
 @pytest.mark.parametrize("hidden, ff, experts, top, shared, rows", [(64, 24, 6, 3, 40, 1), (64, 24, 6, 3, 40, 9), (90, 11, 3, 3, None, 5), (128, 48, 16, 4, 40, 200),
