@@ -8,7 +8,9 @@
 // One block a row.  Columns 2 i and 2 i + 1 of a position's vector are sine and cosine of 2 pi position turns[i]; the
 // turns are double, so that the angle of a far position keeps the bits that a float angle would have lost.  With
 // norm_w the norm that reads the rows first is made on the way: normed = rmsnorm(x) * norm_w.
-template <typename TE, typename TH>
+// P > 0: a thread's column pairs wait in registers (rows of up to 512 P columns), all their loads on their way together;
+// P 0: any width, the row is read back.
+template <typename TE, typename TH, int P>
 __global__ void __launch_bounds__(256)
 embedding_sinusoid_kernel(const int* __restrict__ tokens, const int* __restrict__ positions, const TE* __restrict__ table,
                           const double* __restrict__ turns, float* __restrict__ out, const float* __restrict__ norm_w, float eps,
@@ -20,26 +22,60 @@ embedding_sinusoid_kernel(const int* __restrict__ tokens, const int* __restrict_
     const double at = (double)positions[row];
     const TE* e = table + (size_t)tok * dim;
     float* o = out + (size_t)row * dim;
-    float ss = 0.f;
-#pragma unroll 4
-    for (int d = 2 * threadIdx.x; d < dim; d += 512) {
-        double t = at * turns[d / 2];
+    auto vector_of = [&](double turn, float& s, float& c) {
+        double t = at * turn;
         t -= rint(t);
-        float s, c;
         sincospif((float)(2.0 * t), &s, &c);
-        const float v0 = load_f32(e + d) * scale + s;
-        o[d] = v0;
-        ss += v0 * v0;
-        if (d + 1 < dim) {
-            const float v1 = load_f32(e + d + 1) * scale + c;
-            o[d + 1] = v1;
-            ss += v1 * v1;
+    };
+    float ss = 0.f;
+    if constexpr (P > 0) {
+        double turn[P];
+        float v[P][2], w[P][2];
+#pragma unroll
+        for (int i = 0; i < P; ++i) {
+            const int d = 2 * (threadIdx.x + 256 * i);
+            turn[i] = d < dim ? turns[d / 2] : 0.0;
+#pragma unroll
+            for (int j = 0; j < 2; ++j) {
+                const int dd = min(d + j, dim - 1);
+                v[i][j] = load_f32(e + dd);
+                w[i][j] = norm_w ? norm_w[dd] : 1.f;
+            }
         }
+#pragma unroll
+        for (int i = 0; i < P; ++i) {
+            const int d = 2 * (threadIdx.x + 256 * i);
+            float add[2];
+            vector_of(turn[i], add[0], add[1]);
+#pragma unroll
+            for (int j = 0; j < 2; ++j) {
+                v[i][j] = v[i][j] * scale + add[j];
+                if (d + j < dim) { o[d + j] = v[i][j]; ss += v[i][j] * v[i][j]; }
+            }
+        }
+        if (!norm_w) return;
+        const float rs = 1.0f / sqrtf(block_sum<256>(ss, red) / (float)dim + eps);
+#pragma unroll
+        for (int i = 0; i < P; ++i) {
+            const int d = 2 * (threadIdx.x + 256 * i);
+#pragma unroll
+            for (int j = 0; j < 2; ++j) if (d + j < dim) store_f32(normed + (size_t)row * dim + d + j, v[i][j] * rs * w[i][j]);
+        }
+    } else {
+        for (int d = 2 * threadIdx.x; d < dim; d += 512) {
+            float add[2];
+            vector_of(turns[d / 2], add[0], add[1]);
+            for (int j = 0; j < 2 && d + j < dim; ++j) {
+                const float v = load_f32(e + d + j) * scale + add[j];
+                o[d + j] = v;
+                ss += v * v;
+            }
+        }
+        if (!norm_w) return;
+        const float rs = 1.0f / sqrtf(block_sum<256>(ss, red) / (float)dim + eps);
+        for (int d = 2 * threadIdx.x; d < dim; d += 512)          // (a thread reads back what it wrote itself)
+            for (int j = 0; j < 2 && d + j < dim; ++j) store_f32(normed + (size_t)row * dim + d + j, o[d + j] * rs * norm_w[d + j]);
     }
-    if (!norm_w) return;
-    const float rs = 1.0f / sqrtf(block_sum<256>(ss, red) / (float)dim + eps);
-    for (int d = 2 * threadIdx.x; d < dim; d += 512)          // (a thread reads back what it wrote itself)
-        for (int j = 0; j < 2 && d + j < dim; ++j) store_f32(normed + (size_t)row * dim + d + j, o[d + j] * rs * norm_w[d + j]);
 }
 
 extern "C" int cisr_embedding_sinusoid(const int* tokens, const int* positions, const void* table, const double* turns, float* out,
@@ -47,10 +83,13 @@ extern "C" int cisr_embedding_sinusoid(const int* tokens, const int* positions, 
                                        int table_dtype, int normed_dtype, hipStream_t stream) {
     if (rows <= 0) return 0;
     if (dim <= 0 || vocab <= 0 || !turns || (norm_w && !normed)) return (int)hipErrorInvalidValue;
-#define EMB(TE, TH) embedding_sinusoid_kernel<TE, TH><<<rows, 256, 0, stream>>>(tokens, positions, (const TE*)table, turns, out, norm_w, eps, (TH*)normed, dim, vocab, scale)
+#define EMB_P(TE, TH, P) embedding_sinusoid_kernel<TE, TH, P><<<rows, 256, 0, stream>>>(tokens, positions, (const TE*)table, turns, out, norm_w, eps, (TH*)normed, dim, vocab, scale)
+#define EMB(TE, TH) do { if (dim <= 512) EMB_P(TE, TH, 1); else if (dim <= 1024) EMB_P(TE, TH, 2); else if (dim <= 2048) EMB_P(TE, TH, 4); \
+                         else if (dim <= 4096) EMB_P(TE, TH, 8); else EMB_P(TE, TH, 0); } while (0)
     if (table_dtype == DT_F32) { if (normed_dtype == DT_F32) EMB(float, float); else EMB(float, bf16_t); }
     else { if (normed_dtype == DT_F32) EMB(bf16_t, float); else EMB(bf16_t, bf16_t); }
 #undef EMB
+#undef EMB_P
     return CISR_LAUNCH_CHECK();
 }
 

@@ -329,8 +329,10 @@ route_product_kernel(const bf16_t* __restrict__ h, int ldh, const bf16_t* __rest
         const int row = row0 + i;
         if (row >= rows) break;
         float z = 0.f;
-        if (lane < NT * 16)
+        if (lane < NT * 16) {
+#pragma unroll
             for (int w = 0; w < ROUTE_WAVES; ++w) z += parts[w][i][lane];
+        }
         if (gate_out && lane == outputs) gate_out[row] = z;
         const bool real = lane < outputs;
         float s;
@@ -361,6 +363,7 @@ route_product_kernel(const bf16_t* __restrict__ h, int ldh, const bf16_t* __rest
             mine[lane] = score;
             meet();
             int before = 0;
+#pragma unroll 8
             for (int j = 0; j < groups; ++j) { const float v = mine[j]; before += v > score || (v == score && j < lane); }
             const unsigned long long kept = __ballot(lane < groups && before < keep);
             if (!(real && ((kept >> (lane / per)) & 1ull))) c = -INFINITY;
@@ -369,6 +372,7 @@ route_product_kernel(const bf16_t* __restrict__ h, int ldh, const bf16_t* __rest
         mine[lane] = c;
         meet();
         int place = 0;
+#pragma unroll 8
         for (int j = 0; j < outputs; ++j) { const float v = mine[j]; place += v > c || (v == c && j < lane); }
         const bool taken = real && place < top;
         const float total = wave_sum(taken ? s : 0.f);
@@ -629,11 +633,14 @@ typedef __attribute__((ext_vector_type(4))) uint32_t u32x4;
 // MT 2 (steps of many rows): the block of a tile that is the first, third, ... of its expert's run also takes the tile
 // after it if that is the same expert's (else its second half is padding), and the block of the other tile leaves at
 // once: every byte of the expert's matrix then meets twice the rows.
+// ACT_GATED: an expert's matrix is [gate; up] of N / 2 rows each; a block's 128 columns are 64 outputs' gates and ups in
+// turns of 16, so that a wave holds both of an output, and C (N / 2 columns) is their gated activation.
+#define ACT_GATED 2
 template <typename TC, int ACT, int MT>
 __global__ void __launch_bounds__(256)
 expert_gemm_mfma_kernel(const bf16_t* __restrict__ A, int lda, const bf16_t* __restrict__ W, const int* __restrict__ tile_expert,
                         const int* __restrict__ pair_of_pos, int gather_div, int scatter, TC* __restrict__ C, int ldc, int N, int K,
-                        int tiles) {
+                        int tiles, GateLaw law) {
     // The hardware deals consecutive blocks round-robin to the 8 XCDs, each with an L2 of its own.  Renumber so that an
     // XCD gets a contiguous run of (tile, column block) pairs, tiles fastest: the tiles of one expert follow each other,
     // so the blocks that read the same 128 rows of that expert's matrix run on one XCD at about the same time.
@@ -672,8 +679,13 @@ expert_gemm_mfma_kernel(const bf16_t* __restrict__ A, int lda, const bf16_t* __r
     }
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-        const int n = n0 + lr + 32 * i;
-        wp[i] = n < N ? W + ((size_t)e * N + n) * K : nullptr;
+        if (ACT == ACT_GATED) {
+            const int n = n0 / 2 + 16 * i + lr % 16;
+            wp[i] = n < N / 2 ? W + ((size_t)e * N + (lr < 16 ? 0 : N / 2) + n) * K : nullptr;
+        } else {
+            const int n = n0 + lr + 32 * i;
+            wp[i] = n < N ? W + ((size_t)e * N + n) * K : nullptr;
+        }
     }
     const u32x4 zero = {0u, 0u, 0u, 0u};
     // MT 1: two steps' operands are on their way at any time (two sets of registers taking turns: one step's arithmetic
@@ -731,10 +743,18 @@ expert_gemm_mfma_kernel(const bf16_t* __restrict__ A, int lda, const bf16_t* __r
         for (int x = 0; x < 4; ++x) {
             const int m = crow[wm * 32 * MT + i * 16 + g * 4 + x];
             if (m < 0) continue;
+            if (ACT == ACT_GATED) {
 #pragma unroll
-            for (int j = 0; j < 4; ++j) {
-                const int n = n0 + wn * 64 + j * 16 + r;
-                if (n < N) store_f32(C + (size_t)m * ldc + n, expert_act<ACT>(acc[i][j][x]));
+                for (int j = 0; j < 4; j += 2) {
+                    const int n = n0 / 2 + wn * 32 + j * 8 + r;
+                    if (n < N / 2) store_f32(C + (size_t)m * ldc + n, gated_activation(acc[i][j][x], acc[i][j + 1][x], law));
+                }
+            } else {
+#pragma unroll
+                for (int j = 0; j < 4; ++j) {
+                    const int n = n0 + wn * 64 + j * 16 + r;
+                    if (n < N) store_f32(C + (size_t)m * ldc + n, expert_act<ACT>(acc[i][j][x]));
+                }
             }
         }
 }
@@ -859,8 +879,8 @@ extern "C" int cisr_experts_gemm(const void* A, int lda, const void* W, const in
     if (vec) {
         // steps of many rows (an expert meets more than one tile as a rule): a block takes two tiles of one expert
 #define EX_MFMA(TC, ACT) \
-        do { if (max_tiles >= EX_PAIRED_FROM) expert_gemm_mfma_kernel<TC, ACT, 2><<<wide, 256, 0, stream>>>(a, lda, w, EX_ARGS, (TC*)C, ldc, N, K, max_tiles); \
-             else expert_gemm_mfma_kernel<TC, ACT, 1><<<wide, 256, 0, stream>>>(a, lda, w, EX_ARGS, (TC*)C, ldc, N, K, max_tiles); } while (0)
+        do { if (max_tiles >= EX_PAIRED_FROM) expert_gemm_mfma_kernel<TC, ACT, 2><<<wide, 256, 0, stream>>>(a, lda, w, EX_ARGS, (TC*)C, ldc, N, K, max_tiles, GateLaw{0.f, 0.f, 0.f}); \
+             else expert_gemm_mfma_kernel<TC, ACT, 1><<<wide, 256, 0, stream>>>(a, lda, w, EX_ARGS, (TC*)C, ldc, N, K, max_tiles, GateLaw{0.f, 0.f, 0.f}); } while (0)
         if (out_dtype == DT_F32) {
             if (act) EX_MFMA(float, 1);
             else EX_MFMA(float, 0);
@@ -879,5 +899,21 @@ extern "C" int cisr_experts_gemm(const void* A, int lda, const void* W, const in
         }
     }
 #undef EX_ARGS
+    return CISR_LAUNCH_CHECK();
+}
+
+// The gated form of the matrix-core tiles: W [experts, 2 N, K] = [gate; up] of every expert, C by place, bf16 [places, N].
+extern "C" int cisr_experts_gemm_gated(const void* A, int lda, const void* W, const int* tile_expert, const int* pair_of_pos, int gather_div,
+                                       void* C, int ldc, int max_tiles, int N, int K, float limit, float slope, float shift, hipStream_t stream) {
+    if (max_tiles <= 0 || N <= 0) return 0;
+    const long long blocks = (long long)max_tiles * ((2 * N + EX_BN - 1) / EX_BN);
+    if (K <= 0 || K % 8 || lda % 8 || ((uintptr_t)A) % 16 || ((uintptr_t)W) % 16 || max_tiles > 0x7fffff || blocks > 0x7ffffff0LL) return (int)hipErrorInvalidValue;
+    const dim3 grid((unsigned)((blocks + 7) / 8 * 8));
+    const GateLaw law = {limit, slope, shift};
+#define EX_GATED(MT) expert_gemm_mfma_kernel<bf16_t, ACT_GATED, MT><<<grid, 256, 0, stream>>>((const bf16_t*)A, lda, (const bf16_t*)W, tile_expert, pair_of_pos, \
+        gather_div, 0, (bf16_t*)C, ldc, 2 * N, K, max_tiles, law)
+    if (max_tiles >= EX_PAIRED_FROM) EX_GATED(2);
+    else EX_GATED(1);
+#undef EX_GATED
     return CISR_LAUNCH_CHECK();
 }

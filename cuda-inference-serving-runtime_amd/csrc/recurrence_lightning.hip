@@ -28,6 +28,9 @@ struct LightningArgs {
     float* carry;                     // [slots][heads][R][C]
 };
 
+// an element at a 32-bit byte offset from a base that is uniform over the wave (no 64-bit arithmetic a load)
+__device__ __forceinline__ float element_at(const float* base, uint32_t element) { return *(const float*)((const char*)base + (uint32_t)(element * 4u)); }
+
 __device__ __forceinline__ float silu_of(float z) { return z / (1.0f + expf(-z)); }
 
 __device__ __forceinline__ double power_of(double x, int n) {
@@ -60,50 +63,57 @@ __device__ __forceinline__ LightningChunk lightning_chunk(const LightningArgs& p
 // A block a (chunk, head, 128 columns): the keys, silu'd and decayed to the chunk's end, wait in LDS; a wave owns 16-column
 // tiles and all rows of the state, four row tiles at a time; its values come straight from memory.
 #define LCOLS 128
-__global__ void __launch_bounds__(256) lightning_end_kernel(LightningArgs p) {
+__global__ void __launch_bounds__(256, 4) lightning_end_kernel(LightningArgs p) {
     extern __shared__ __attribute__((aligned(16))) float lds[];
     __shared__ float pw[LCHUNK];
     const LightningChunk ch = lightning_chunk(p, blockIdx.x);
     if (ch.n <= 0) return;
     const int head = blockIdx.y, tid = threadIdx.x, wave = __builtin_amdgcn_readfirstlane(tid / WAVE), lane = tid % WAVE, r = lane % 16, g = lane / 16;
-    const int R = p.R, C = p.C, n = ch.n, Rp = (R + 15) / 16 * 16, RS = (Rp + 63) / 64 * 64 + 16;
+    const int R = p.R, C = p.C, n = ch.n, Rp = (R + 63) / 64 * 64, RS = Rp + 16;
+    const float* vh = p.v + (size_t)ch.t0 * p.ldv + (size_t)head * C;
+    // a wave's first tile's values are asked for before the keys' way into LDS, every following tile's during the one before
+    float b[LCHUNK / 4];
+    auto ask = [&](int ct) {
+        const int cc = min((int)blockIdx.z * LCOLS + ct * 16 + r, C - 1);
+#pragma unroll
+        for (int s = 0; s < LCHUNK / 4; ++s) b[s] = element_at(vh, (uint32_t)(min(4 * s + g, n - 1) * p.ldv + cc));
+    };
+    ask(wave);
     if (tid < n) pw[tid] = (float)power_of((double)p.decay[head], n - 1 - tid);
     __syncthreads();
     const float* kh = p.k + (size_t)ch.t0 * p.ldk + (size_t)head * R;
-    for (int idx = tid; idx < LCHUNK * Rp; idx += 256) {
-        const int i = idx / Rp, c = idx % Rp;
-        const float x = kh[(size_t)min(i, n - 1) * p.ldk + min(c, R - 1)];
-        lds[i * RS + c] = i < n && c < R ? silu_of(x) * pw[i] : 0.f;
-    }
+    for (int c = lane; c < Rp; c += 64)
+#pragma unroll 8
+        for (int i = wave; i < LCHUNK; i += 4) {
+            const float x = element_at(kh, (uint32_t)(min(i, n - 1) * p.ldk + min(c, R - 1)));
+            lds[i * RS + c] = i < n && c < R ? silu_of(x) * pw[i] : 0.f;
+        }
     __syncthreads();
-    const float* vh = p.v + (size_t)ch.t0 * p.ldv + (size_t)head * C;
     float* end = p.carry + ((size_t)blockIdx.x * p.heads + head) * R * C;
-    const int steps = (n + 3) / 4;
+#pragma unroll 1
     for (int ct = wave; ct < LCOLS / 16; ct += 4) {
-        const int c = blockIdx.z * LCOLS + ct * 16 + r, cc = min(c, C - 1);
+        const int c = blockIdx.z * LCOLS + ct * 16 + r;
         if (blockIdx.z * LCOLS + ct * 16 >= C) break;                // (uniform over the wave)
-        float b[LCHUNK / 4];
+        float val[LCHUNK / 4];
 #pragma unroll
-        for (int s = 0; s < LCHUNK / 4; ++s) b[s] = vh[(size_t)min(4 * s + g, n - 1) * p.ldv + cc];
-#pragma unroll
-        for (int s = 0; s < LCHUNK / 4; ++s) b[s] = silu_of(b[s]);     // (rows behind the last are the last: their keys are zero)
+        for (int s = 0; s < LCHUNK / 4; ++s) val[s] = silu_of(b[s]);   // (rows behind the last are the last: their keys are zero)
+        ask(ct + 4);
+#pragma unroll 1
         for (int rt0 = 0; rt0 < Rp / 16; rt0 += 4) {
             f32x4_t acc[4];
 #pragma unroll
             for (int j = 0; j < 4; ++j) acc[j] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
 #pragma unroll
             for (int s = 0; s < LCHUNK / 4; ++s) {
-                if (s >= steps) continue;
 #pragma unroll
-                for (int j = 0; j < 4; ++j)
-                    if (rt0 + j < Rp / 16) acc[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(lds[(4 * s + g) * RS + (rt0 + j) * 16 + r], b[s], acc[j], 0, 0, 0);
+                for (int j = 0; j < 4; ++j) acc[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(lds[(4 * s + g) * RS + (rt0 + j) * 16 + r], val[s], acc[j], 0, 0, 0);
             }
 #pragma unroll
             for (int j = 0; j < 4; ++j)
 #pragma unroll
                 for (int e = 0; e < 4; ++e) {
                     const int row = (rt0 + j) * 16 + 4 * g + e;
-                    if (row < R && c < C) end[(size_t)row * C + c] = acc[j][e];
+                    if (row < R && c < C) *(float*)((char*)end + (uint32_t)(row * C + c) * 4u) = acc[j][e];
                 }
         }
     }
@@ -141,30 +151,47 @@ __global__ void __launch_bounds__(256) lightning_carry_kernel(LightningArgs p) {
 // A block a (chunk, head, 128 columns).  Queries and keys wait in LDS; the wave w makes the 16 rows w of the decayed scores
 // P, which then take the keys' place; a wave owns 16-column tiles of the results and all four row tiles, with the state and
 // the values straight from memory (each read once a block).
-__global__ void __launch_bounds__(256) lightning_out_kernel(LightningArgs p) {
+__global__ void __launch_bounds__(256, 3) lightning_out_kernel(LightningArgs p) {
     extern __shared__ __attribute__((aligned(16))) float lds[];
     __shared__ float pw[LCHUNK + 1];
     const LightningChunk ch = lightning_chunk(p, blockIdx.x);
     if (ch.n <= 0) return;
     const int head = blockIdx.y, tid = threadIdx.x, wave = __builtin_amdgcn_readfirstlane(tid / WAVE), lane = tid % WAVE, r = lane % 16, g = lane / 16;
-    const int R = p.R, C = p.C, n = ch.n, Rp = (R + 3) / 4 * 4, RS = (Rp + 63) / 64 * 64 + 4, PS = LCHUNK + 4;
+    const int R = p.R, C = p.C, n = ch.n, Rp = (R + 63) / 64 * 64, RS = Rp + 4, PS = LCHUNK + 4;
     float* sq = lds;
+    const float* vh = p.v + (size_t)ch.t0 * p.ldv + (size_t)head * C;
+    const float* start = p.carry + ((size_t)blockIdx.x * p.heads + head) * R * C;
+    float b[LCHUNK / 4], s0[16];         // a tile's values, and sixteen rows of the state: a wave's first are asked for here
+    auto ask_values = [&](int ct) {
+        const int cc = min((int)blockIdx.z * LCOLS + ct * 16 + r, C - 1);
+#pragma unroll
+        for (int s = 0; s < LCHUNK / 4; ++s) b[s] = element_at(vh, (uint32_t)(min(4 * s + g, n - 1) * p.ldv + cc));
+    };
+    auto ask_state = [&](int ct, int k0) {
+        const int cc = min((int)blockIdx.z * LCOLS + ct * 16 + r, C - 1);
+#pragma unroll
+        for (int s = 0; s < 16; ++s) s0[s] = element_at(start, (uint32_t)(min(k0 + 4 * s + g, R - 1) * C + cc));
+    };
+    ask_state(wave, 0);
+    ask_values(wave);
     float* sk = lds + LCHUNK * RS;       // and P, [LCHUNK][PS], once the scores are made (RS >= PS)
     if (tid <= LCHUNK) pw[tid] = (float)power_of((double)p.decay[head], tid);
     const float* qh = p.q + (size_t)ch.t0 * p.ldq + (size_t)head * R;
     const float* kh = p.k + (size_t)ch.t0 * p.ldk + (size_t)head * R;
-    for (int idx = tid; idx < LCHUNK * Rp; idx += 256) {
-        const int i = idx / Rp, c = idx % Rp;
-        const size_t row = min(i, n - 1);
-        const float x = qh[row * p.ldq + min(c, R - 1)], y = kh[row * p.ldk + min(c, R - 1)];
-        const bool in = i < n && c < R;
-        sq[i * RS + c] = in ? silu_of(x) : 0.f;
-        sk[i * RS + c] = in ? silu_of(y) : 0.f;
-    }
+    for (int c = lane; c < Rp; c += 64)
+#pragma unroll 8
+        for (int i = wave; i < LCHUNK; i += 4) {
+            const int row = min(i, n - 1);
+            const float x = element_at(qh, (uint32_t)(row * p.ldq + min(c, R - 1))), y = element_at(kh, (uint32_t)(row * p.ldk + min(c, R - 1)));
+            const bool in = i < n && c < R;
+            sq[i * RS + c] = in ? silu_of(x) : 0.f;
+            sk[i * RS + c] = in ? silu_of(y) : 0.f;
+        }
     __syncthreads();
     f32x4_t sc[4];
 #pragma unroll
     for (int j = 0; j < 4; ++j) sc[j] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
     for (int k0 = 0; k0 < Rp; k0 += 4) {
         const float a = sq[(wave * 16 + r) * RS + k0 + g];
 #pragma unroll
@@ -180,25 +207,18 @@ __global__ void __launch_bounds__(256) lightning_out_kernel(LightningArgs p) {
             sk[row * PS + col] = col <= row ? sc[j][e] * pw[max(row - col, 0)] : 0.f;
         }
     __syncthreads();
-    const float* vh = p.v + (size_t)ch.t0 * p.ldv + (size_t)head * C;
-    const float* start = p.carry + ((size_t)blockIdx.x * p.heads + head) * R * C;
     const int row_tiles = (n + 15) / 16;
+#pragma unroll 1
     for (int ct = wave; ct < LCOLS / 16; ct += 4) {
-        const int c = blockIdx.z * LCOLS + ct * 16 + r, cc = min(c, C - 1);
+        const int c = blockIdx.z * LCOLS + ct * 16 + r;
         if (blockIdx.z * LCOLS + ct * 16 >= C) break;                // (uniform over the wave)
-        float b[LCHUNK / 4];
-#pragma unroll
-        for (int s = 0; s < LCHUNK / 4; ++s) b[s] = vh[(size_t)min(4 * s + g, n - 1) * p.ldv + cc];
         f32x4_t acc[4];
 #pragma unroll
         for (int j = 0; j < 4; ++j) acc[j] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
         for (int k0 = 0; k0 < Rp; k0 += 64) {                        // sixteen steps' loads of the state together
-            float s0[16];
-#pragma unroll
-            for (int s = 0; s < 16; ++s) s0[s] = start[(size_t)min(k0 + 4 * s + g, R - 1) * C + cc];
+            if (k0 > 0) ask_state(ct, k0);
 #pragma unroll
             for (int s = 0; s < 16; ++s) {
-                if (k0 + 4 * s >= Rp) continue;
 #pragma unroll
                 for (int j = 0; j < 4; ++j)
                     acc[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(sq[(j * 16 + r) * RS + k0 + 4 * s + g], s0[s], acc[j], 0, 0, 0);
@@ -208,6 +228,7 @@ __global__ void __launch_bounds__(256) lightning_out_kernel(LightningArgs p) {
         for (int j = 0; j < 4; ++j)
 #pragma unroll
             for (int e = 0; e < 4; ++e) acc[j][e] *= pw[j * 16 + 4 * g + e + 1];
+        ask_state(ct + 4, 0);
 #pragma unroll
         for (int s = 0; s < LCHUNK / 4; ++s) {
             const float value = silu_of(b[s]);
@@ -217,6 +238,7 @@ __global__ void __launch_bounds__(256) lightning_out_kernel(LightningArgs p) {
         }
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
+            if (j == 0) ask_values(ct + 4);
             if (j >= row_tiles) continue;
 #pragma unroll
             for (int e = 0; e < 4; ++e) {
@@ -303,10 +325,12 @@ extern "C" int cisr_lightning_chunks(const float* q, int ldq, const float* k, in
                                      int heads, int R, int C, int slots, float* carry, hipStream_t stream) {
     if (segments <= 0 || slots <= 0) return 0;
     const LightningArgs p{q, ldq, k, ldk, v, ldv, decay, out, ldo, state, slot_stride, seg_start, state_slots, R, C, heads, segments, carry};
+    if ((long long)LCHUNK * ldq >= (1 << 29) || (long long)LCHUNK * ldk >= (1 << 29) || (long long)LCHUNK * ldv >= (1 << 29) || (long long)R * C >= (1 << 29))
+        return (int)hipErrorInvalidValue;                       // (offsets inside a chunk's rows fit 32 bits)
     if (lightning_bad(p) || !carry || (C + LCOLS - 1) / LCOLS > 65535) return (int)hipErrorInvalidValue;
     const dim3 grid(slots, heads, (C + LCOLS - 1) / LCOLS);
-    const size_t end_lds = (size_t)LCHUNK * (((R + 15) / 16 * 16 + 63) / 64 * 64 + 16) * sizeof(float);
-    const size_t out_lds = (size_t)2 * LCHUNK * (((R + 3) / 4 * 4 + 63) / 64 * 64 + 4) * sizeof(float);
+    const size_t end_lds = (size_t)LCHUNK * ((R + 63) / 64 * 64 + 16) * sizeof(float);
+    const size_t out_lds = (size_t)2 * LCHUNK * ((R + 63) / 64 * 64 + 4) * sizeof(float);
     hipError_t e = hipSuccess;
     if (end_lds > 65536 - 1024) e = hipFuncSetAttribute((const void*)lightning_end_kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)end_lds);
     if (e == hipSuccess && out_lds > 65536 - 1024) e = hipFuncSetAttribute((const void*)lightning_out_kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)out_lds);

@@ -93,6 +93,7 @@ def _declare(h):
         "cisr_experts_route_scored": [p, i, p, p, p, i, i, i, i, i, i, i, i, f, i, p, p, p],
         "cisr_experts_route_product": [p, i, p, i, i, p, p, p, p, i, i, i, i, i, i, i, i, f, i, p, p, p],
         "cisr_attn_merge_gated": [p, p, p, i, i, i, i, p, i, i, p],
+        "cisr_experts_gemm_gated": [p, i, p, p, p, i, p, i, i, i, i, f, f, f, p],
         "cisr_side_rows": [p, i, p, p, p, i, i, p, i, i, i, i, i, p],
         "cisr_experts_add": [p, p, p, p, p, p, i, i, i, i, i, p, f, p, i, p],
         "cisr_experts_rows_gated": [p, i, p, p, i, p, i, i, i, i, i, f, f, f, p],
@@ -394,6 +395,11 @@ LIBRARY_GATED_MIN_ROWS, LIBRARY_GATED_MIN_BYTES = 33, 64 << 20
 # with 2 MB of weights: at 2,048 rows 1,792 x 2,048 takes 21 us there and 35 in the tiled kernel here (float results; the
 # same with bf16), 2,048 x 1,536 18 and 28, 1,024 x 1,024 10 and 14; at 128 rows 6.8 and 12.7, 5.8 and 9.9, 5.3 and 6.9.
 LIBRARY_PLAIN_MIN_BYTES = 2 << 20
+# Of those, float results go there with smaller weights still where the inner size is long (the tiled kernel does not cut it:
+# 256 x 2,048 at 128 rows 10.9 us here and 5.3 there, 64 x 2,048 10.7 and 5.5) or the rows are many (2,048 x 256 at 2,048 rows
+# 10.7 and 8.8, 1,024 x 256 6.9 and 6.3; at 128 rows 4.1 and 5.2, so not there).
+LIBRARY_FLOAT_LONG_K, LIBRARY_FLOAT_LONG_K_BYTES = 1024, 128 << 10
+LIBRARY_FLOAT_MANY_ROWS, LIBRARY_FLOAT_MANY_ROWS_BYTES = 1024, 512 << 10
 
 
 def attention_talking(q, q_row_stride, kcache, vcache, tables, seg_of_row, positions, out, heads, kv_heads, vdim, pad, page_size,
@@ -520,8 +526,8 @@ class ScratchPool:
 DEFAULT_SCRATCH = ScratchPool()
 
 
-def library_ok(m, w, gated=False, plain=False):
-    """`plain`: the product ends with its store.  `gated`: the product of gate and up, whose activation is a kernel of its own after the library's product.  With
+def library_ok(m, w, gated=False, plain=False, floats=False):
+    """`plain`: the product ends with its store (`floats`: of float results).  `gated`: the product of gate and up, whose activation is a kernel of its own after the library's product.  With
     weights of 64 MB and more it goes there from 33 rows on: 64 rows against the 8B sizes' 235 MB take 60.7 us there and
     69.7 in the wide kernel here (58.4 against 63.0 at 33 rows; 23.0 against 26.5 at the 1.7B sizes), the activation
     included; the other products of 33 to 64 rows are as fast here."""
@@ -529,6 +535,11 @@ def library_ok(m, w, gated=False, plain=False):
     if gated and w.numel() * 2 >= LIBRARY_GATED_MIN_BYTES:
         least = min(least, LIBRARY_GATED_MIN_ROWS)
     least_bytes = LIBRARY_PLAIN_MIN_BYTES if plain and w.shape[0] % 8 == 0 and w.shape[1] % 8 == 0 else LIBRARY_MIN_BYTES
+    if floats and plain and w.shape[0] % 8 == 0 and w.shape[1] % 8 == 0:
+        if w.shape[1] >= LIBRARY_FLOAT_LONG_K:
+            least_bytes = min(least_bytes, LIBRARY_FLOAT_LONG_K_BYTES)
+        if m >= LIBRARY_FLOAT_MANY_ROWS:
+            least_bytes = min(least_bytes, LIBRARY_FLOAT_MANY_ROWS_BYTES)
     return (LIBRARY_MIN_ROWS > 0 and m >= least and w.dtype == torch.bfloat16 and w.is_contiguous()
             and w.numel() * 2 >= least_bytes)
 
@@ -562,7 +573,7 @@ def gemm(a, w, out, residual=None, after_norm=False, scratch=None):
             raise KernelError("gemm: float operands need a float output")
         code = lib().cisr_gemm_f32(a.data_ptr(), a.stride(0), w.data_ptr(), w.stride(0), out.data_ptr(), out.stride(0),
                                    rp, ldr, m, n, k, _stream())
-    elif (a.dtype == torch.bfloat16 and library_ok(m, w, plain=residual is None) and a.is_contiguous() and out.is_contiguous()
+    elif (a.dtype == torch.bfloat16 and library_ok(m, w, plain=residual is None, floats=out.dtype == torch.float32) and a.is_contiguous() and out.is_contiguous()
           and (residual is None or residual is out)):
         if residual is None:
             # (float results are the library's float accumulators as they are: 2,048 rows against 10,240 x 2,048 take 83 us
@@ -2182,6 +2193,27 @@ def experts_gemm(a, w, pair_of_pos, tile_expert, out, top=0, scatter=False, act=
                                    _dev(tile_expert, "tile_expert", torch.int32), _dev(pair_of_pos, "pair_of_pos", torch.int32),
                                    int(top), int(bool(scatter)), _dev(out, "out"), out.stride(0), tiles, n, k, int(bool(act)),
                                    _storage(a, "a"), _storage(out, "out"), _stream()), "experts_gemm")
+    return out
+
+
+def experts_gemm_gated_ok(a, w):
+    return (a.dtype == torch.bfloat16 and w.dtype == torch.bfloat16 and a.stride(1) == 1 and w.shape[2] % 8 == 0 and a.stride(0) % 8 == 0
+            and a.data_ptr() % 16 == 0 and w.data_ptr() % 16 == 0)
+
+
+def experts_gemm_gated(a, w, pair_of_pos, tile_expert, out, law, top=0):
+    """experts_gemm by place over experts whose matrix is [gate; up] (w [experts, 2 N, K], bf16: experts_gemm_gated_ok) with
+    their gated activation as the epilogue: out bf16 [places, N]; law as in experts_rows_gated."""
+    experts, n2, k = w.shape
+    tiles = tile_expert.shape[0]
+    places = tiles * EXPERT_TILE
+    if not experts_gemm_gated_ok(a, w) or a.dim() != 2 or a.shape[1] != k or n2 % 2 or not w.is_contiguous() or pair_of_pos.numel() != places:
+        raise KernelError("experts_gemm_gated: shape not supported")
+    if out.dim() != 2 or out.shape[1] != n2 // 2 or out.shape[0] < places or (top <= 0 and a.shape[0] < places):
+        raise KernelError("experts_gemm_gated: operands and results by place need a row a place")
+    _check(lib().cisr_experts_gemm_gated(a.data_ptr(), a.stride(0), _dev(w, "w"), _dev(tile_expert, "tile_expert", torch.int32),
+                                         _dev(pair_of_pos, "pair_of_pos", torch.int32), int(top), _dev(out, "out", torch.bfloat16), out.stride(0),
+                                         tiles, n2 // 2, k, *(float(v) for v in law), _stream()), "experts_gemm_gated")
     return out
 
 

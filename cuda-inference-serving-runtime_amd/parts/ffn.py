@@ -256,7 +256,7 @@ class ScoredExperts(FeedForward):
 
     The rows of a step are ordered by expert on the device and each expert's matrices meet only their own rows
     (ops.experts_gemm; steps of few rows stream each pair's matrices, ops.experts_rows); gate and up are one product over
-    [gate; up] a expert, followed by the activation (its epilogue in steps of few rows).  `names`: (router, correction, expert
+    [gate; up] a expert with the activation as its epilogue (float32: a kernel after it).  `names`: (router, correction, expert
     prefix, gate, up, down)."""
     leaves_rows = True       # `output` takes `unsummed`
 
@@ -349,8 +349,12 @@ class ScoredExperts(FeedForward):
             tiles = ops.expert_tiles(T, top, E)
             places, tile_expert = ctx.buffer("moe.places", (tiles * ops.EXPERT_TILE,), torch.int32), ctx.buffer("moe.tiles", (tiles,), torch.int32)
             route(places, tile_expert)
-            gate_up = ops.experts_gemm(h, self.w_gate_up, places, tile_expert, ctx.buffer("moe.gate_up", (tiles * ops.EXPERT_TILE, 2 * I), ctx.dtype), top=top)
-            act = self._activation(gate_up, ctx.buffer("moe.act", (tiles * ops.EXPERT_TILE, I), ctx.dtype))
+            act = ctx.buffer("moe.act", (tiles * ops.EXPERT_TILE, I), ctx.dtype)
+            if ops.experts_gemm_gated_ok(h, self.w_gate_up):
+                ops.experts_gemm_gated(h, self.w_gate_up, places, tile_expert, act, self.law or (0.0, 0.0, 0.0), top=top)
+            else:
+                gate_up = ops.experts_gemm(h, self.w_gate_up, places, tile_expert, ctx.buffer("moe.gate_up", (tiles * ops.EXPERT_TILE, 2 * I), ctx.dtype), top=top)
+                self._activation(gate_up, act)
             ops.experts_gemm(act, self.w_down, places, tile_expert, down, scatter=True)
         also = None if self.shared is None else self.shared.output(h, ctx, tag="moe.shared", unfinished=False)
         return ops.ExpertSum(down, weights, chosen, E, shared=also, gate=gate)

@@ -1100,6 +1100,36 @@ def test_library_products_of_many_rows_also_in_captured_graphs(ops, monkeypatch)
         check(f"replay {i}")
 
 
+@pytest.mark.parametrize("M, N, K", [(65, 64, 1024), (128, 256, 2048), (512, 24, 4096), (1024, 512, 512), (2048, 2048, 128), (2048, 256, 2048), (3000, 128, 2048), (130, 4096, 256)])
+def test_float_results_of_small_weights_from_the_library_also_in_captured_graphs(ops, M, N, K):
+    """Float results against weights of less than 2 MB go to the library where the inner size is long or the rows are many
+    (library_ok): checked against double products, eagerly and on every replay of a captured graph, with new inputs,
+    eager work and synchronisations between the replays."""
+    torch.manual_seed(M + N)
+    w = (torch.randn(N, K, device=DEV) / K ** 0.5).bfloat16()
+    assert ops.library_ok(M, w, plain=True, floats=True) == (N * K * 2 >= (2 << 20) or (K >= 1024 and N * K >= 65536) or (M >= 1024 and N * K >= 262144))
+    assert not ops.library_ok(64, w, plain=True, floats=True)
+    a, out = torch.empty(M, K, dtype=torch.bfloat16, device=DEV), torch.empty(M, N, device=DEV)
+
+    def check(tag):
+        ref = a.double() @ w.double().T
+        assert ((out.double() - ref).abs().max() / ref.abs().max()).item() < 1e-5, tag
+
+    a.copy_(torch.randn(M, K, device=DEV))
+    ops.gemm(a, w, out)
+    check("eager")
+    graph = torch.cuda.CUDAGraph()
+    with torch.cuda.graph(graph):
+        ops.gemm(a, w, out)
+    for i in range(5):
+        a.copy_(torch.randn(M, K, device=DEV))
+        out.fill_(7)
+        (torch.randn(300, 300, device=DEV) @ torch.randn(300, 300, device=DEV)).sum().item()       # eager work between replays
+        graph.replay()
+        torch.cuda.synchronize()
+        check(f"replay {i}")
+
+
 @pytest.mark.parametrize("M, N, K", GEMM_SHAPES)
 def test_gemm_f32(ops, M, N, K):
     a, w, r = rnd(M, K, seed=1), rnd(N, K, seed=2), rnd(M, N, seed=3)
