@@ -127,15 +127,14 @@ class CacheManager:
             if n <= 0:
                 raise ValueError("a request must bring at least one token")
             seen.add(request)
-        if self.fast_decode and all(n == 1 for _, n in items) and all(g.need.window is None for g in self.groups):
-            return self._append_one_each(items, commit)
         # Windows first give back, for every request of the step, the pages that no later query can see; only then
         # are fresh pages counted and taken.  (Trimmed one request at a time, a request that needs a page could
         # come before the one whose window frees it, and run out in the middle of the step.)  Giving such a page
         # back changes nothing that a retry of the step would read.
-        for request, _ in items:
-            for group in self.groups:
-                group.trim(request, self.lengths[request])
+        for group in self.groups:
+            group.trim_each(items, self.lengths)
+        if self.fast_decode and all(n == 1 for _, n in items):
+            return self._append_one_each(items, commit)
         if not self.can_append(items):
             raise OutOfPages("not enough free KV pages for this step")
         result = []
@@ -178,8 +177,8 @@ class CacheManager:
                     group._touch(d.request)
 
     def _append_one_each(self, items, commit=True):
-        """append_many for the common step in which every request brings one token and no group has a
-        window: the same pages in the same order, with the counting and the placing done in line."""
+        """append_many, once windows have given back what they can, for the common step in which every request brings one
+        token: the same pages in the same order, with the counting and the placing done in line."""
         P = self.page_size
         lengths = self.lengths
         for group in self.groups:

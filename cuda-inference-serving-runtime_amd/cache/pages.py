@@ -126,13 +126,18 @@ class CacheGroup:
         self.page_size = page_size
         self.pool = PagePool(n_pages)
         self.tables = {}
+        self.given_back = {}  # request -> logical page before which every dead page has gone back already
         self.versions = {}   # request -> stamp of the last change of its table (stamps are never reused)
         self._stamp = 0
         self.storage = None  # device tensor of the shape the need states (storage_shape), set by the owner
 
     # -- planning -------------------------------------------------------
     def _dead_pages(self, request, length):
-        """Logical pages that no later query can see, a range (window groups only)."""
+        """Logical pages that no later query can see and that may still be held, a range (window groups only)."""
+        dead = self._unseen_pages(length)
+        return range(max(dead.start, self.given_back.get(request, 0)), min(dead.stop, len(self.tables[request])))
+
+    def _unseen_pages(self, length):
         P = self.page_size
         rule = getattr(self.need, "first_visible", None)
         if rule is not None:               # (a need with a rule of its own: blocks of positions)
@@ -154,8 +159,7 @@ class CacheGroup:
 
     def trimmable(self, request, length):
         table = self.tables[request]
-        return sum(1 for j in self._dead_pages(request, length)
-                   if j < len(table) and table[j] >= 0 and self.pool.refs[table[j]] == 1)
+        return sum(1 for j in self._dead_pages(request, length) if table[j] >= 0 and self.pool.refs[table[j]] == 1)
 
     # -- mutation -------------------------------------------------------
     def _touch(self, request):
@@ -164,11 +168,28 @@ class CacheGroup:
 
     def trim(self, request, length):
         table = self.tables[request]
-        for j in self._dead_pages(request, length):
-            if j < len(table) and table[j] >= 0:
+        dead = self._dead_pages(request, length)
+        for j in dead:
+            if table[j] >= 0:
                 self.pool.drop(table[j])
                 table[j] = -1
                 self._touch(request)
+        if dead:
+            self.given_back[request] = dead.stop
+
+    def trim_each(self, items, lengths):
+        """trim for every (request, _) of a step; with a window most requests have nothing new to give back, which costs a
+        comparison here."""
+        window = self.need.window
+        if window is None:
+            return
+        P, back = self.page_size, self.given_back
+        own_rule = hasattr(self.need, "first_visible")
+        kept = -(-getattr(self.need, "keep_first", 0) // P)
+        for request, _ in items:
+            length = lengths[request]
+            if own_rule or (length - window + 1) // P > back.get(request, kept):
+                self.trim(request, length)
 
     def append(self, request, length, n_new):
         """Slots of the n_new tokens at logical positions length.. and the page
@@ -197,6 +218,8 @@ class CacheGroup:
 
     def fork(self, source, target):
         self.tables[target] = list(self.tables[source])
+        if source in self.given_back:
+            self.given_back[target] = self.given_back[source]
         self._touch(target)
         for page in self.tables[target]:
             if page >= 0:
@@ -204,6 +227,7 @@ class CacheGroup:
 
     def release(self, request):
         self.versions.pop(request, None)
+        self.given_back.pop(request, None)
         for page in self.tables.pop(request):
             if page >= 0:
                 self.pool.drop(page)

@@ -5,6 +5,7 @@ import random
 import pytest
 
 from runtime.cache import CacheManager, KVNeed, OutOfPages, StateNeed, StateSlots
+from runtime.cache.pages import ChunkNeed, KeptWindowNeed
 
 
 def manager(pages=8, page_size=4, sites=2, window=None, max_requests=8, **kw):
@@ -263,14 +264,18 @@ def test_random_orders_keep_every_page_accounted_for(seed):
     assert all(free == 12 for free in m.free_pages()) and len(m.slots.free) == 5
 
 
+@pytest.mark.parametrize("windows", [False, True])
 @pytest.mark.parametrize("seed", range(4))
-def test_single_token_steps_take_the_same_pages_on_the_short_path(seed):
+def test_single_token_steps_take_the_same_pages_on_the_short_path(seed, windows):
     """Steps of one token a request run a short path; it must hand out exactly the pages, slots, copies and
     errors of the general path, also after forks (shared last pages) and when the pool runs dry."""
     def run(fast):
         rng = random.Random(seed)
         copies = []
-        m = CacheManager({0: KVNeed(2, 8, None), 1: KVNeed(2, 8, None), 2: KVNeed(1, 16, None)}, 10, 4, 6,
+        needs = {0: KVNeed(2, 8, None), 1: KVNeed(2, 8, None), 2: KVNeed(1, 16, None)}
+        if windows:
+            needs.update({2: KVNeed(1, 16, rng.choice([1, 6])), 3: KeptWindowNeed(1, 8, 5, 6), 4: ChunkNeed(1, 8, 7, 7)})
+        m = CacheManager(needs, 10, 4, 6,
                          copy_pages=lambda group, pairs: copies.append(list(pairs)))
         m.fast_decode = fast
         live, counter, log = [], 0, []

@@ -740,6 +740,33 @@ def test_command_line_serves_the_design(folders, tmp_path):
     assert out["runner"]["replays"] >= 1 and out["runner"]["cache"][0]["resident_pages"] == 0
 
 
+@pytest.mark.parametrize("dtype, execution", [("float32", "eager"), ("bfloat16", "eager"), ("bfloat16", "graph")])
+def test_a_long_window_whose_keys_are_split_over_blocks_in_decoding(tmp_path, dtype, execution):
+    """A window of several hundred keys with heads large enough that a decode step splits a row's keys over blocks (the
+    merge then packs and gates the heads, and the output projection of the other layer merges its own), after a prompt
+    that passes the window, beside a short second request."""
+    from movazen_models import attention, config, moe, parallel
+    from runtime.engine import StepEntry
+    from runtime.kernels import attention as rules
+    cfg = config(61, 64, 0.8, 1e-5, 16, [
+        attention(4, 2, 72, 80, 0.12, (400, 20), moe(24, 2.0, 4, 2, (2, 1), (16, 1.5))),
+        parallel((2, 1, 80, 80, 0.12, (0.3, 100)), (2, 16, 24, (0.9, 0.999)), 1.0, 0.8)])
+    assert rules.rows_launch(2 * 2, 451, 2, 80)[1] > 1
+    folder = write_folder(tmp_path / "m", cfg, 99)
+    first, second = decisive_tokens(folder, 5, 620, 61), decisive_tokens(folder, 6, 30, 61)
+    runner = make_runner(folder, dtype, pages=60, execution=execution)
+    runner.create("x"); runner.create("y")
+    got = [runner.step([StepEntry("x", first[:450], list(range(450)))]).cpu().numpy(), runner.step([StepEntry("x", first[450:600], list(range(150)))]).cpu().numpy()]
+    other = [runner.step([StepEntry("y", second[:10], list(range(10)))]).cpu().numpy()]
+    for i in range(20):
+        out = runner.step([StepEntry("x", [first[600 + i]], [0]), StepEntry("y", [second[10 + i]], [0])]).cpu().numpy()
+        got.append(out[:1])
+        other.append(out[1:])
+    assert_close(np.concatenate(got), plain_logits(folder, first), dtype, "a long window")
+    assert_close(np.concatenate(other), plain_logits(folder, second), dtype, "the short one")
+    runner.cache.check()
+
+
 # -- configurations drawn at random -----------------------------------------------------------------------------------
 
 def random_config(seed):
